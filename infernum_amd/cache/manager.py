@@ -9,7 +9,8 @@ shape; for attention [num_pages, nkv, page_size, d] for keys and the transposed 
 page_size] for values; the reference keeps [num_pages, page_size, nkv, d] per layer,
 infernum-cuda/src/inner/cuda/paged_kv_cache.rs:88-102, and has one group only).
 Pages go back to the pool when a request ends (infernum-runtime/src/scheduler.rs:
-289-305) or, in a window group, when every later query's window has passed them
+289-305) or, in a window group, when every later query's window has passed them (the pages of a request's first
+``keep_first`` positions stay where the mixer's CacheSpec asks for that)
 (the reference keeps them, TABNINE.md:53).
 
 State slots: a mixer that declares a StateSpec gets a [num_slots, *shape] tensor
@@ -38,8 +39,8 @@ class CacheGroup:
     """One group as the host sees it: what kind it is, which schedule entries own pages in it, and its pool
     (the tables themselves are kept natively by the manager)."""
 
-    def __init__(self, index: int, kind: str, window: int, page_size: int):
-        self.index, self.kind, self.window = index, kind, int(window)
+    def __init__(self, index: int, kind: str, window: int, page_size: int, keep_first: int = 0):
+        self.index, self.kind, self.window, self.keep_first = index, kind, int(window), int(keep_first)
         self.page_size = int(page_size)
         self.entries: List[int] = []         # schedule entries that own pages in this group
         self.allocator: Optional[PageAllocator] = None
@@ -55,7 +56,7 @@ class StateSlotPool:
         if _view is not None:
             self._h, self._owned = _view, False
         else:
-            self._h = ctypes.c_void_p(self._lib.ia_cache_create(0, None, None, 1, 1, self.num_slots))
+            self._h = ctypes.c_void_p(self._lib.ia_cache_create(0, None, None, None, 1, 1, self.num_slots))
             self._owned = True
 
     def __del__(self):
@@ -116,7 +117,7 @@ class CacheManager:
             key = cs.group_key()
             if key not in key_to_group:
                 key_to_group[key] = len(self.groups)
-                self.groups.append(CacheGroup(len(self.groups), cs.kind, cs.window, self.page_size))
+                self.groups.append(CacheGroup(len(self.groups), cs.kind, cs.window, self.page_size, cs.keep_first))
             g = key_to_group[key]
             self.groups[g].entries.append(i)
             self._entry_group.append(g)
@@ -125,7 +126,8 @@ class CacheManager:
         G = len(self.groups)
         kinds = (ctypes.c_int * max(G, 1))(*[_KINDS[g.kind] for g in self.groups])
         windows = (ctypes.c_int * max(G, 1))(*[g.window for g in self.groups])
-        self._h = ctypes.c_void_p(self._lib.ia_cache_create(G, kinds, windows, self.page_size, int(config.num_pages),
+        keeps = (ctypes.c_int * max(G, 1))(*[g.keep_first for g in self.groups])
+        self._h = ctypes.c_void_p(self._lib.ia_cache_create(G, kinds, windows, keeps, self.page_size, int(config.num_pages),
                                                             int(config.num_state_slots)))
         if not self._h:
             raise ValueError("the cache could not be created: page_size, num_pages must be positive, slots not negative")

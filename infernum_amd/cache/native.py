@@ -23,7 +23,7 @@ _SIGNATURES = {
     "ia_pool_allocate_many": (c_int, [c_void_p, c_int, POINTER(c_int)]),
     "ia_pool_free": (c_int, [c_void_p, c_int]),
     "ia_pool_is_used": (c_int, [c_void_p, c_int]),
-    "ia_cache_create": (c_void_p, [c_int, POINTER(c_int), POINTER(c_int), c_int, c_int, c_int]),
+    "ia_cache_create": (c_void_p, [c_int, POINTER(c_int), POINTER(c_int), POINTER(c_int), c_int, c_int, c_int]),
     "ia_cache_destroy": (None, [c_void_p]),
     "ia_cache_error": (c_char_p, [c_void_p]),
     "ia_cache_group_pool": (c_void_p, [c_void_p, c_int]),

@@ -79,14 +79,15 @@ def pages_for(num_tokens: int, page_size: int) -> int:
 
 class BlockTable:
     """Pages of one request in one group (a copy of the native table at the time it was asked for).
-    ``pages[i]`` holds positions [i * page_size, (i + 1) * page_size); NO_PAGE where a window has passed."""
+    ``pages[i]`` holds positions [i * page_size, (i + 1) * page_size); NO_PAGE where a window has passed
+    (in a group that keeps a request's first positions their pages stay)."""
 
     __slots__ = ("pages", "num_tokens", "first_live")
 
     def __init__(self, pages: Optional[List[int]] = None, num_tokens: int = 0, first_live: int = 0) -> None:
         self.pages: List[int] = list(pages or [])
         self.num_tokens = int(num_tokens)
-        self.first_live = int(first_live)      # pages before this index have been given back
+        self.first_live = int(first_live)      # pages before this index have been given back, but those kept for good
 
     def live_pages(self) -> List[int]:
-        return [p for p in self.pages[self.first_live:] if p != NO_PAGE]
+        return [p for p in self.pages if p != NO_PAGE]

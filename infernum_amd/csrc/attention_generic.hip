@@ -9,7 +9,9 @@
 // page_size]; block_tables[s, j / page_size] is the page of key j of sequence s.  The query of token n stands at positions[n] and
 // sees keys max(0, pos - window + 1) .. pos  (window 0: all keys from 0; window < 0: the keys of its own
 // chunk of -window positions, see ia_first_visible_key).  sinks (nullable, fp32 [nh]): exp(sinks[h]) is added to
-// the softmax's denominator of head h; it has no key and no value.
+// the softmax's denominator of head h; it has no key and no value.  Value heads may have another size, dv, than
+// query and key heads (value pages [num_pages, nkv, dv, page_size], out rows of nh dv values).  Under a window the
+// request's first `keep` keys stay visible; a softcap c > 0 turns a scaled score s into c tanh(s / c).
 #include "common.h"
 
 #define AG_MAX_D 640
@@ -21,8 +23,9 @@ __global__ __launch_bounds__(64) void attn_generic_kernel(const T* __restrict__ 
                                                           int out_row_stride, const int* __restrict__ token_seq,
                                                           const int* __restrict__ positions,
                                                           const int* __restrict__ block_tables, int bt_stride, int nh,
-                                                          int nkv, int d, int page_size, int num_pages, float scale,
-                                                          int window, const float* __restrict__ sinks) {
+                                                          int nkv, int d, int dv, int page_size, int num_pages,
+                                                          float scale, int window, const float* __restrict__ sinks,
+                                                          int keep, float softcap) {
   __shared__ float qs[AG_MAX_D];
   __shared__ float ps[64];
   __shared__ int rs[64];
@@ -42,8 +45,11 @@ __global__ __launch_bounds__(64) void attn_generic_kernel(const T* __restrict__ 
 #pragma unroll
   for (int c = 0; c < AG_MAX_D / 64; ++c) acc[c] = 0.f;
 
-  for (int j0 = j_lo; j0 <= j_hi; j0 += 64) {
-    const int j = j0 + lane;
+  // the keys in the order of their positions: the kept ones before the window, then the window's
+  const int kept = window > 0 ? (keep < j_lo ? keep : j_lo) : 0;
+  const int count = kept + (j_hi - j_lo + 1);
+  for (int j0 = 0; j0 < count; j0 += 64) {
+    const int j = j0 + lane < kept ? j0 + lane : j0 + lane - kept + j_lo;
     const bool valid = j <= j_hi;
     float sc = -INFINITY;
     int row = 0;
@@ -55,6 +61,7 @@ __global__ __launch_bounds__(64) void attn_generic_kernel(const T* __restrict__ 
         float dot = 0.f;
         for (int i = 0; i < d; ++i) dot = fmaf(qs[i], to_float(kr[i]), dot);
         sc = dot * scale;
+        if (softcap > 0.f) sc = softcap * tanhf(sc / softcap);
       } else {
         sc = __uint_as_float(0x7fc00000u);  // a block table without a page here: poison, never a stray read
       }
@@ -68,17 +75,17 @@ __global__ __launch_bounds__(64) void attn_generic_kernel(const T* __restrict__ 
     ps[lane] = p;
     rs[lane] = row;
     __syncthreads();
-    const int cnt = (j_hi - j0 + 1) < 64 ? (j_hi - j0 + 1) : 64;
+    const int cnt = (count - j0) < 64 ? (count - j0) : 64;
     for (int jj = 0; jj < cnt; ++jj) {
-      // rs = (page * nkv + g) * page_size + offset  ->  value (dim) at ((page*nkv+g) * d + dim) * page_size + offset
+      // rs = (page * nkv + g) * page_size + offset  ->  value (dim) at ((page*nkv+g) * dv + dim) * page_size + offset
       const int r = rs[jj];
       const int head_page = r / page_size, off = r - head_page * page_size;
-      const T* vr = v_pages + (size_t)head_page * d * page_size + off;
+      const T* vr = v_pages + (size_t)head_page * dv * page_size + off;
       const float pj = ps[jj];
 #pragma unroll
       for (int c = 0; c < AG_MAX_D / 64; ++c) {
         const int dim = lane + 64 * c;
-        if (dim < d) acc[c] = fmaf(pj, to_float(vr[(size_t)dim * page_size]), acc[c]);
+        if (dim < dv) acc[c] = fmaf(pj, to_float(vr[(size_t)dim * page_size]), acc[c]);
       }
     }
     __syncthreads();
@@ -92,21 +99,22 @@ __global__ __launch_bounds__(64) void attn_generic_kernel(const T* __restrict__ 
 #pragma unroll
     for (int c = 0; c < AG_MAX_D / 64; ++c) acc[c] *= corr;
   }
-  T* o = out + (size_t)n * out_row_stride + (size_t)h * d;
+  T* o = out + (size_t)n * out_row_stride + (size_t)h * dv;
   const float inv_l = 1.0f / l;
 #pragma unroll
   for (int c = 0; c < AG_MAX_D / 64; ++c) {
     const int dim = lane + 64 * c;
-    if (dim < d) o[dim] = from_float<T>(acc[c] * inv_l);
+    if (dim < dv) o[dim] = from_float<T>(acc[c] * inv_l);
   }
 }
 
 extern "C" int ia_attention_generic(const void* q, int q_row_stride, const void* k_pages, const void* v_pages,
                                     void* out, int out_row_stride, int dtype, const int* token_seq,
                                     const int* positions, const int* block_tables, int bt_stride, int N, int nh,
-                                    int nkv, int d, int page_size, int num_pages, float scale, int window,
-                                    const float* sinks, hipStream_t stream) {
-  if (N < 0 || nh <= 0 || nkv <= 0 || nh % nkv != 0 || d <= 0 || d > AG_MAX_D || page_size <= 0 || num_pages <= 0 ||
+                                    int nkv, int d, int dv, int page_size, int num_pages, float scale, int window,
+                                    const float* sinks, int keep, float softcap, hipStream_t stream) {
+  if (N < 0 || nh <= 0 || nkv <= 0 || nh % nkv != 0 || d <= 0 || d > AG_MAX_D || dv <= 0 || dv > AG_MAX_D || keep < 0 ||
+      !(softcap >= 0.f) || q_row_stride < nh * d || out_row_stride < nh * dv || page_size <= 0 || num_pages <= 0 ||
       bt_stride <= 0)
     return IA_ERR_BAD_ARG;
   if (nh > 65535) return IA_ERR_UNSUPPORTED;
@@ -115,13 +123,13 @@ extern "C" int ia_attention_generic(const void* q, int q_row_stride, const void*
   if (dtype == IA_F32)
     attn_generic_kernel<float><<<grid, 64, 0, stream>>>((const float*)q, q_row_stride, (const float*)k_pages,
                                                         (const float*)v_pages, (float*)out, out_row_stride, token_seq,
-                                                        positions, block_tables, bt_stride, nh, nkv, d, page_size,
-                                                        num_pages, scale, window, sinks);
+                                                        positions, block_tables, bt_stride, nh, nkv, d, dv, page_size,
+                                                        num_pages, scale, window, sinks, keep, softcap);
   else if (dtype == IA_BF16)
     attn_generic_kernel<bf16_t><<<grid, 64, 0, stream>>>((const bf16_t*)q, q_row_stride, (const bf16_t*)k_pages,
                                                          (const bf16_t*)v_pages, (bf16_t*)out, out_row_stride,
-                                                         token_seq, positions, block_tables, bt_stride, nh, nkv, d,
-                                                         page_size, num_pages, scale, window, sinks);
+                                                         token_seq, positions, block_tables, bt_stride, nh, nkv, d, dv,
+                                                         page_size, num_pages, scale, window, sinks, keep, softcap);
   else
     return IA_ERR_BAD_ARG;
   IA_LAUNCH_CHECK();

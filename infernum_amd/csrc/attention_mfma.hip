@@ -1,5 +1,10 @@
 // bf16 attention over the paged cache on the matrix cores (v_mfma_f32_16x16x16_bf16 and
-// v_mfma_f32_16x16x32_bf16), compiled for one head size, IA_HEAD_DIM (a multiple of 16, at most 256).
+// v_mfma_f32_16x16x32_bf16), compiled for one head size, IA_HEAD_DIM (a multiple of 16, at most 256), or with
+// IA_VALUE_DIM beside it for values of another size than queries and keys.
+//
+// With IA_ATTN_EXT=1 the kernels also take (other libraries refuse them): a softcap c > 0 on the scaled scores,
+// s <- c tanh(s / c); and, under a window, the first `keep` keys of the request, which every query goes on seeing.
+// The tiles that hold kept keys before the window come first, then the window's own; between them nothing is read.
 //
 // Both kernels work on the transposed problem:
 //   S^T[key, col] = K[key, :] . Q[col, :]      A operand = 16 keys of K, B operand = 16 columns of Q
@@ -30,9 +35,38 @@
 #ifndef IA_HEAD_DIM
 #error "compile with -DIA_HEAD_DIM=<head size>"
 #endif
+#ifndef IA_VALUE_DIM
+#define IA_VALUE_DIM IA_HEAD_DIM
+#endif
+#ifndef IA_ATTN_EXT
+#define IA_ATTN_EXT 0
+#endif
 #define HD IA_HEAD_DIM
 #define NS (HD / 16)
+#define VD IA_VALUE_DIM         // values of a value head
+#define NSV (VD / 16)
+#define IA_MAX_DIM (IA_HEAD_DIM > IA_VALUE_DIM ? IA_HEAD_DIM : IA_VALUE_DIM)
 static_assert(HD % 16 == 0 && HD >= 16 && HD <= 256, "head size must be a multiple of 16 up to 256");
+static_assert(VD % 16 == 0 && VD >= 16 && VD <= 256, "value size must be a multiple of 16 up to 256");
+constexpr bool EXT = IA_ATTN_EXT != 0;
+
+// The options that only a library with IA_ATTN_EXT takes.
+struct AttnExt {
+  int keep;                      // under a window: the request's first `keep` keys stay visible
+  float cap_in, cap_out;         // softcap c: raw score times cap_in = scale / c, tanh, times cap_out = c log2(e)
+  bool capped;
+};
+
+// tanh to about 1e-7: 1 - 2 / (1 + exp(2 x)), which runs into 1 and -1 at the ends
+__device__ __forceinline__ float attn_tanh(float x) {
+  return 1.0f - 2.0f * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(2.8853900817779268f * x));
+}
+
+// Tiles of `size` keys that hold kept keys before the first key lo of a window (0 when the window reaches the start).
+__device__ __forceinline__ int attn_keep_tiles(int keep, int lo, int size) {
+  const int kept = keep < lo ? keep : lo;
+  return kept > 0 ? (kept + size - 1) / size : 0;
+}
 
 typedef short s16x4 __attribute__((ext_vector_type(4)));
 typedef float f32x4 __attribute__((ext_vector_type(4)));
@@ -80,14 +114,14 @@ typedef float f32x2_t __attribute__((ext_vector_type(2)));
 // 2,151 against 2,130 tokens/s, at one 274.5 against 271.9; with more workgroups than compute units four waves are
 // ahead: 12,620 against 12,274 tokens/s at 64 requests).  Head sizes above 128 keep four (the waves' partial results
 // would not fit the LDS twice).
-#define DEC_WAVES_FEW (IA_HEAD_DIM <= 128 ? 8 : 4)
+#define DEC_WAVES_FEW (IA_MAX_DIM <= 128 ? 8 : 4)
 #define DEC_COMPUTE_UNITS 256
 static bool dec_wide(int B, int groups, int splits) { return (long long)B * groups * splits <= DEC_COMPUTE_UNITS; }
 #define DEC_BT_LDS 2048          // block-table entries kept in LDS (a longer slice is read from global memory)
 
 struct DecTile {                 // 16 keys as they come from memory: operands of the two products
   s16x4 k[NS];
-  uint2 v[NS];
+  uint2 v[NSV];
   uint32_t mlo, mhi;             // which of the lane's four values are of keys in range (16 bits each)
   bool bad;                      // a key that is needed has no page
 };
@@ -98,13 +132,14 @@ struct DecGeom {                 // what does not change from tile to tile
   const int* bt_global;
   const int* bt_lds;
   int bt_first, bt_count;        // the slice [bt_first, bt_first + bt_count) of the table lies in bt_lds
-  size_t page_elems;
+  size_t k_page, v_page;         // values of one page, all heads
   int ps, ps_shift, num_pages, key_lo, key_hi;
+  int keep;                      // EXT: keys below it are seen as well as key_lo .. key_hi
   // the token's own key and value, when the kernel made them itself: they replace what the loads of the
   // tile of key patch_key bring for that key (patch_key < 0: nothing to replace)
   int patch_key;
   const uint16_t* new_k;         // [HD] in LDS
-  const uint16_t* new_v;         // [HD] in LDS
+  const uint16_t* new_v;         // [VD] in LDS
 };
 
 // POW2: the page size is a power of two (a shift and a mask; a division by a size known only at run time costs
@@ -120,29 +155,41 @@ __device__ __forceinline__ int dec_offset(const DecGeom& G, int key) {
   return POW2 ? key & (G.ps - 1) : key % G.ps;
 }
 
+__device__ __forceinline__ bool dec_sees(const DecGeom& G, int key) {
+  return key <= G.key_hi && (key >= G.key_lo || (EXT && key < G.keep));
+}
+
 template <bool POW2>
 __device__ __forceinline__ void dec_load(const DecGeom& G, int t0, int j, int qd, DecTile& T) {
   const int key = t0 + j;
-  const int keyc = key < G.key_lo ? G.key_lo : (key > G.key_hi ? G.key_hi : key);
+  const int keyc = EXT ? (dec_sees(G, key) ? key : G.key_hi)
+                       : (key < G.key_lo ? G.key_lo : (key > G.key_hi ? G.key_hi : key));
   const int page = dec_page<POW2>(G, keyc);
   const bool page_ok = (unsigned)page < (unsigned)G.num_pages;
-  load_row_operand(G.k_base + (size_t)(page_ok ? page : 0) * G.page_elems + (size_t)dec_offset<POW2>(G, keyc) * HD, qd, T.k);
+  load_row_operand(G.k_base + (size_t)(page_ok ? page : 0) * G.k_page + (size_t)dec_offset<POW2>(G, keyc) * HD, qd, T.k);
   const int kg = t0 + 4 * qd;    // this lane brings the values of the keys kg .. kg+3 (one quad, one page)
-  const int kgc = kg < G.key_lo ? (G.key_lo & ~3) : (kg > G.key_hi ? (G.key_hi & ~3) : kg);
+  const bool quad = dec_sees(G, kg) || dec_sees(G, kg + 1) || dec_sees(G, kg + 2) || dec_sees(G, kg + 3);
+  const int kgc = EXT ? (quad ? kg : (G.key_hi & ~3))
+                      : (kg < G.key_lo ? (G.key_lo & ~3) : (kg > G.key_hi ? (G.key_hi & ~3) : kg));
   const int pagev = dec_page<POW2>(G, kgc);
   const bool pagev_ok = (unsigned)pagev < (unsigned)G.num_pages;
-  const uint16_t* vq = G.v_base + (size_t)(pagev_ok ? pagev : 0) * G.page_elems + dec_offset<POW2>(G, kgc);
+  const uint16_t* vq = G.v_base + (size_t)(pagev_ok ? pagev : 0) * G.v_page + dec_offset<POW2>(G, kgc);
   // keep the values of keys key_lo .. key_hi, zero the others (16 bits each)
   uint32_t mlo = 0u, mhi = 0u;
-  if (kg == kgc && pagev_ok) {
+  if (EXT) {
+    if (quad && pagev_ok) {
+      mlo = (dec_sees(G, kg) ? 0x0000ffffu : 0u) | (dec_sees(G, kg + 1) ? 0xffff0000u : 0u);
+      mhi = (dec_sees(G, kg + 2) ? 0x0000ffffu : 0u) | (dec_sees(G, kg + 3) ? 0xffff0000u : 0u);
+    }
+  } else if (kg == kgc && pagev_ok) {
     mlo = ((kg >= G.key_lo && kg <= G.key_hi) ? 0x0000ffffu : 0u) | ((kg + 1 >= G.key_lo && kg + 1 <= G.key_hi) ? 0xffff0000u : 0u);
     mhi = ((kg + 2 >= G.key_lo && kg + 2 <= G.key_hi) ? 0x0000ffffu : 0u) | ((kg + 3 >= G.key_lo && kg + 3 <= G.key_hi) ? 0xffff0000u : 0u);
   }
 #pragma unroll
-  for (int n = 0; n < NS; ++n) T.v[n] = *reinterpret_cast<const uint2*>(vq + (size_t)(n * 16 + j) * G.ps);
+  for (int n = 0; n < NSV; ++n) T.v[n] = *reinterpret_cast<const uint2*>(vq + (size_t)(n * 16 + j) * G.ps);
   T.mlo = mlo;
   T.mhi = mhi;
-  const bool k_needed = key == keyc, v_needed = kg + 3 >= G.key_lo && kg <= G.key_hi;
+  const bool k_needed = key == keyc, v_needed = EXT ? quad : kg + 3 >= G.key_lo && kg <= G.key_hi;
   T.bad = (k_needed && !page_ok) || (v_needed && !pagev_ok);
 }
 
@@ -151,13 +198,13 @@ __device__ __forceinline__ void dec_load(const DecGeom& G, int t0, int j, int qd
 // loads stay in flight until then.
 __device__ __forceinline__ void dec_finish(const DecGeom& G, int t0, int j, int qd, DecTile& T) {
 #pragma unroll
-  for (int n = 0; n < NS; ++n) T.v[n] = make_uint2(T.v[n].x & T.mlo, T.v[n].y & T.mhi);
+  for (int n = 0; n < NSV; ++n) T.v[n] = make_uint2(T.v[n].x & T.mlo, T.v[n].y & T.mhi);
   if (G.patch_key >= 0 && t0 == (G.patch_key & ~15)) {       // the same for all lanes of the wave
     if (j == (G.patch_key & 15)) load_row_operand(G.new_k, qd, T.k);
     const int e = G.patch_key - (t0 + 4 * qd);               // which of this lane's four keys, if any
     if (e >= 0 && e < 4) {
 #pragma unroll
-      for (int n = 0; n < NS; ++n) {
+      for (int n = 0; n < NSV; ++n) {
         const uint32_t nv = G.new_v[n * 16 + j];
         uint32_t lo = T.v[n].x, hi = T.v[n].y;
         if (e == 0) lo = (lo & 0xffff0000u) | nv;
@@ -171,9 +218,9 @@ __device__ __forceinline__ void dec_finish(const DecGeom& G, int t0, int j, int 
 }
 
 // One tile of 16 keys, t0 .. t0+15, against the 16 columns (heads) of this wave.
-//   pos, lo: this lane's column sees keys lo .. pos; pos < 0: no such column
+//   pos, lo: this lane's column sees keys lo .. pos (EXT: and those below X.keep); pos < 0: no such column
 __device__ __forceinline__ void dec_compute(int t0, const DecTile& T, const s16x4 (&q)[NS], int pos, int lo, int qd,
-                                            float scale_log2, f32x4 (&o)[NS], float& m, float& l) {
+                                            float scale_log2, f32x4 (&o)[NSV], float& m, float& l, const AttnExt& X) {
   // ---- S^T = K Q^T
   f32x4 s = (f32x4){0.f, 0.f, 0.f, 0.f};
 #pragma unroll
@@ -184,8 +231,9 @@ __device__ __forceinline__ void dec_compute(int t0, const DecTile& T, const s16x
 #pragma unroll
   for (int r = 0; r < 4; ++r) {
     const int kr = kg + r;
-    const bool ok = pos >= 0 && kr <= pos && kr >= lo;
-    sv[r] = ok ? s[r] * scale_log2 : -INFINITY;
+    const bool ok = pos >= 0 && kr <= pos && (kr >= lo || (EXT && kr < X.keep));
+    const float sl = (EXT && X.capped) ? X.cap_out * attn_tanh(s[r] * X.cap_in) : s[r] * scale_log2;
+    sv[r] = ok ? sl : -INFINITY;
   }
   float tmax = fmaxf(fmaxf(sv[0], sv[1]), fmaxf(sv[2], sv[3]));
   tmax = fmaxf(tmax, __shfl_xor(tmax, 16, IA_WAVE));
@@ -208,7 +256,7 @@ __device__ __forceinline__ void dec_compute(int t0, const DecTile& T, const s16x
   const s16x4 pb = as_s16x4(p0, p1);
   // ---- O^T = O^T corr + V^T P^T
 #pragma unroll
-  for (int n = 0; n < NS; ++n) {
+  for (int n = 0; n < NSV; ++n) {
     o[n] *= corr;
     o[n] = __builtin_amdgcn_mfma_f32_16x16x16bf16_1k(as_s16x4(T.v[n].x, T.v[n].y), pb, o[n], 0, 0, 0);
   }
@@ -229,16 +277,17 @@ struct DecFused {
 // include the token's own also make its key and value, use them from LDS (the loads from the page are replaced
 // in registers) and one of them (the first tile of heads) writes them to the page.
 template <bool FUSED, typename TS, bool POW2, int WAVES>
-__global__ __launch_bounds__(WAVES * 64, ((WAVES == 4 && HD <= 128) ? 3 : 1)) void attn_decode_kernel(
+__global__ __launch_bounds__(WAVES * 64, ((WAVES == 4 && IA_MAX_DIM <= 128) ? 3 : 1)) void attn_decode_kernel(
     const uint16_t* __restrict__ q, int q_row_stride, uint16_t* k_pages, uint16_t* v_pages,
     uint16_t* __restrict__ out, int out_row_stride, float* __restrict__ part_o, float* __restrict__ part_ml,
     const int* __restrict__ positions, const int* __restrict__ block_tables, int bt_stride, int nh, int nkv, int ps,
-    int num_pages, float scale_log2, int window, int num_splits, DecFused F, const float* __restrict__ sinks) {
+    int num_pages, float scale_log2, int window, int num_splits, DecFused F, const float* __restrict__ sinks,
+    AttnExt X) {
   __shared__ float s_m[WAVES][16], s_l[WAVES][16];
-  __shared__ f32x4 s_o[WAVES][NS][64];
+  __shared__ f32x4 s_o[WAVES][NSV][64];
   __shared__ int s_bt[DEC_BT_LDS];
   __shared__ __attribute__((aligned(16))) uint16_t s_q[FUSED ? 16 : 1][HD];
-  __shared__ __attribute__((aligned(16))) uint16_t s_newk[HD], s_newv[HD];
+  __shared__ __attribute__((aligned(16))) uint16_t s_newk[HD], s_newv[VD];
   __shared__ float s_cos[HD / 2], s_sin[HD / 2];
   const int b = blockIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6, j = lane & 15, qd = lane >> 4;
   const int G = nh / nkv, HT = (G + 15) / 16;
@@ -277,10 +326,13 @@ __global__ __launch_bounds__(WAVES * 64, ((WAVES == 4 && HD <= 128) ? 3 : 1)) vo
   const int bt_ahead = tid < bt_stride ? bt[tid] : -1;
   const int p = positions[b];
   const int lo0 = ia_first_visible_key(p, window);
-  const int t_first = lo0 / 16, t_last = p / 16;
-  const int per = (t_last - t_first + 1 + num_splits - 1) / num_splits;
-  const int ta = t_first + split * per;
+  // EXT: tiles are counted from t_first - n_keep on; the n_keep tiles before t_first stand for the request's first
+  const int n_keep = EXT ? attn_keep_tiles(X.keep, lo0, 16) : 0;
+  const int t_first = (EXT && lo0 / 16 < n_keep) ? n_keep : lo0 / 16, t_last = p / 16;
+  const int per = (t_last - t_first + 1 + n_keep + num_splits - 1) / num_splits;
+  const int ta = t_first - n_keep + split * per;
   const int tb = (ta + per < t_last + 1) ? ta + per : t_last + 1;
+  auto tile_at = [&](int t) { return (EXT && t < t_first) ? t - (t_first - n_keep) : t; };
 
   DecGeom geo;
   geo.ps = ps;
@@ -288,9 +340,11 @@ __global__ __launch_bounds__(WAVES * 64, ((WAVES == 4 && HD <= 128) ? 3 : 1)) vo
   geo.num_pages = num_pages;
   geo.key_lo = lo0;
   geo.key_hi = p;
-  geo.page_elems = (size_t)nkv * ps * HD;
+  geo.keep = EXT ? X.keep : 0;
+  geo.k_page = (size_t)nkv * ps * HD;
+  geo.v_page = (size_t)nkv * ps * VD;
   geo.k_base = k_pages + (size_t)g * ps * HD;
-  geo.v_base = v_pages + (size_t)g * HD * ps;
+  geo.v_base = v_pages + (size_t)g * VD * ps;
   geo.bt_global = bt;
   geo.bt_lds = s_bt;
   geo.patch_key = -1;
@@ -301,7 +355,7 @@ __global__ __launch_bounds__(WAVES * 64, ((WAVES == 4 && HD <= 128) ? 3 : 1)) vo
     const int k_from = ta * 16 < lo0 ? lo0 : ta * 16, k_to = tb * 16 - 1 > p ? p : tb * 16 - 1;
     const int first = POW2 ? k_from >> geo.ps_shift : k_from / ps;
     const int last = POW2 ? k_to >> geo.ps_shift : k_to / ps;
-    int count = ta < tb ? last - first + 1 : 0;
+    int count = ta < tb && last >= first ? last - first + 1 : 0;
     if (count > DEC_BT_LDS) count = DEC_BT_LDS;
     geo.bt_first = first;
     geo.bt_count = count;
@@ -312,9 +366,9 @@ __global__ __launch_bounds__(WAVES * 64, ((WAVES == 4 && HD <= 128) ? 3 : 1)) vo
     }
   }
   const int pos = col_ok ? p : -1;
-  f32x4 o[NS];
+  f32x4 o[NSV];
 #pragma unroll
-  for (int n = 0; n < NS; ++n) o[n] = (f32x4){0.f, 0.f, 0.f, 0.f};
+  for (int n = 0; n < NSV; ++n) o[n] = (f32x4){0.f, 0.f, 0.f, 0.f};
   float m = -INFINITY, l = 0.f;
   s16x4 qreg[NS];
   DecTile A, B;
@@ -330,14 +384,14 @@ __global__ __launch_bounds__(WAVES * 64, ((WAVES == 4 && HD <= 128) ? 3 : 1)) vo
         ka = load_split_sum_together(x, F.gsplits, F.split_stride);
         kb = load_split_sum_together(x + half, F.gsplits, F.split_stride);
       }
-      if (tid < HD) vv = load_split_sum_together(row + (size_t)(nh + nkv + g) * HD + tid, F.gsplits, F.split_stride);
+      if (tid < VD) vv = load_split_sum_together(row + (size_t)(nh + nkv) * HD + (size_t)g * VD + tid, F.gsplits, F.split_stride);
     }
     for (int i = tid; i < half; i += NT) rope_sincos(p, F.inv_freq, F.freq_f64, i, s_sin[i], s_cos[i]);
     // barriers without the fence of __syncthreads(), which would wait for every load in flight: only LDS
     // traffic has to be through
     asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
     __builtin_amdgcn_s_barrier();
-    if (t < tb) dec_load<POW2>(geo, t * 16, j, qd, A);             // the first tile's loads fly during the rotation
+    if (t < tb) dec_load<POW2>(geo, tile_at(t) * 16, j, qd, A);             // the first tile's loads fly during the rotation
 #pragma unroll
     for (int u = 0; u < QPT; ++u) {
       const int idx = tid + u * NT;
@@ -364,7 +418,7 @@ __global__ __launch_bounds__(WAVES * 64, ((WAVES == 4 && HD <= 128) ? 3 : 1)) vo
       }
       for (int i = F.rot + tid; i < HD; i += NT)
         s_newk[i] = float_to_bf16_bits(load_split_sum(row + (size_t)(nh + g) * HD + i, F.gsplits, F.split_stride));
-      if (tid < HD) s_newv[tid] = float_to_bf16_bits(vv);
+      if (tid < VD) s_newv[tid] = float_to_bf16_bits(vv);
       geo.patch_key = p;
     }
     asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
@@ -375,20 +429,20 @@ __global__ __launch_bounds__(WAVES * 64, ((WAVES == 4 && HD <= 128) ? 3 : 1)) vo
     if (col_ok) load_row_operand(q + (size_t)b * q_row_stride + (size_t)h * HD, qd, qreg);
     else zero_row_operand(qreg);
     __syncthreads();
-    if (t < tb) dec_load<POW2>(geo, t * 16, j, qd, A);
+    if (t < tb) dec_load<POW2>(geo, tile_at(t) * 16, j, qd, A);
   }
   // two tiles in flight: the loads of the next tile of this wave are issued before this one is worked on
   while (t < tb) {
     const bool more1 = t + WAVES < tb;
-    if (more1) dec_load<POW2>(geo, (t + WAVES) * 16, j, qd, B);
-    dec_finish(geo, t * 16, j, qd, A);
-    dec_compute(t * 16, A, qreg, pos, lo0, qd, scale_log2, o, m, l);
+    if (more1) dec_load<POW2>(geo, tile_at(t + WAVES) * 16, j, qd, B);
+    dec_finish(geo, tile_at(t) * 16, j, qd, A);
+    dec_compute(tile_at(t) * 16, A, qreg, pos, lo0, qd, scale_log2, o, m, l, X);
     t += WAVES;
     if (!more1) break;
     const bool more2 = t + WAVES < tb;
-    if (more2) dec_load<POW2>(geo, (t + WAVES) * 16, j, qd, A);
-    dec_finish(geo, t * 16, j, qd, B);
-    dec_compute(t * 16, B, qreg, pos, lo0, qd, scale_log2, o, m, l);
+    if (more2) dec_load<POW2>(geo, tile_at(t + WAVES) * 16, j, qd, A);
+    dec_finish(geo, tile_at(t) * 16, j, qd, B);
+    dec_compute(tile_at(t) * 16, B, qreg, pos, lo0, qd, scale_log2, o, m, l, X);
     t += WAVES;
     if (!more2) break;
   }
@@ -397,10 +451,10 @@ __global__ __launch_bounds__(WAVES * 64, ((WAVES == 4 && HD <= 128) ? 3 : 1)) vo
     if (slot >= 0 && slot < num_pages * ps) {
       const int page = slot / ps, off = slot - page * ps;
       uint16_t* kd = k_pages + (((size_t)page * nkv + g) * ps + off) * HD;
-      uint16_t* vd = v_pages + ((size_t)page * nkv + g) * HD * ps + off;
-      for (int i = tid; i < HD; i += NT) {
-        kd[i] = s_newk[i];
-        vd[(size_t)i * ps] = s_newv[i];
+      uint16_t* vd = v_pages + ((size_t)page * nkv + g) * VD * ps + off;
+      for (int i = tid; i < IA_MAX_DIM; i += NT) {
+        if (i < HD) kd[i] = s_newk[i];
+        if (i < VD) vd[(size_t)i * ps] = s_newv[i];
       }
     }
   }
@@ -418,11 +472,11 @@ __global__ __launch_bounds__(WAVES * 64, ((WAVES == 4 && HD <= 128) ? 3 : 1)) vo
   }
   const float f = (m == -INFINITY) ? 0.f : exp2f(m - M);
 #pragma unroll
-  for (int n = 0; n < NS; ++n) s_o[wave][n][lane] = o[n] * f;
+  for (int n = 0; n < NSV; ++n) s_o[wave][n][lane] = o[n] * f;
   __syncthreads();
   if (!col_ok) return;
   // wave w finishes the slices n = w, w + 4, ... of the head
-  for (int n = wave; n < NS; n += WAVES) {
+  for (int n = wave; n < NSV; n += WAVES) {
     f32x4 acc = s_o[0][n][lane];
 #pragma unroll
     for (int w = 1; w < WAVES; ++w) acc += s_o[w][n][lane];
@@ -432,10 +486,10 @@ __global__ __launch_bounds__(WAVES * 64, ((WAVES == 4 && HD <= 128) ? 3 : 1)) vo
       uint2 wv;
       wv.x = (uint32_t)float_to_bf16_bits(acc[0] * inv) | ((uint32_t)float_to_bf16_bits(acc[1] * inv) << 16);
       wv.y = (uint32_t)float_to_bf16_bits(acc[2] * inv) | ((uint32_t)float_to_bf16_bits(acc[3] * inv) << 16);
-      *reinterpret_cast<uint2*>(out + (size_t)b * out_row_stride + (size_t)h * HD + 4 * qd + n * 16) = wv;
+      *reinterpret_cast<uint2*>(out + (size_t)b * out_row_stride + (size_t)h * VD + 4 * qd + n * 16) = wv;
     } else {
       const size_t rec = ((size_t)b * nh + h) * num_splits + split;
-      *reinterpret_cast<f32x4*>(part_o + rec * HD + 4 * qd + n * 16) = acc;
+      *reinterpret_cast<f32x4*>(part_o + rec * VD + 4 * qd + n * 16) = acc;
     }
   }
   if (num_splits > 1 && wave == 0 && qd == 0) {
@@ -454,14 +508,14 @@ extern "C" __global__ __launch_bounds__(64) void attn_decode_reduce_kernel(
   const int b = blockIdx.x / nh, h = blockIdx.x - b * nh, lane = threadIdx.x;
   const size_t rec0 = (size_t)blockIdx.x * num_splits;
   // the first parts' outputs are asked for together with the statistics, not after them
-  constexpr int PRE = 4, NC = (HD + 63) / 64;
+  constexpr int PRE = 4, NC = (VD + 63) / 64;
   float pre[PRE][NC];
 #pragma unroll
   for (int j = 0; j < PRE; ++j)
 #pragma unroll
     for (int c = 0; c < NC; ++c) {
       const int dim = lane + 64 * c;
-      pre[j][c] = (j < num_splits && dim < HD) ? part_o[(rec0 + j) * HD + dim] : 0.f;
+      pre[j][c] = (j < num_splits && dim < VD) ? part_o[(rec0 + j) * VD + dim] : 0.f;
     }
   float M = -INFINITY;
   for (int s = lane; s < num_splits; s += 64) M = fmaxf(M, part_ml[(rec0 + s) * 2]);
@@ -497,16 +551,16 @@ extern "C" __global__ __launch_bounds__(64) void attn_decode_reduce_kernel(
       for (int c = 0; c < NC; ++c) {
         const int dim = lane + 64 * c;
         // every part was written (an empty one holds zeros), so the load needs no guard and does not wait
-        const float v = dim < HD ? part_o[(rec0 + s0 + j) * HD + dim] : 0.f;
+        const float v = dim < VD ? part_o[(rec0 + s0 + j) * VD + dim] : 0.f;
         acc[c] += (wj != 0.f) ? wj * v : 0.f;
       }
     }
   }
   const float inv = 1.0f / (sinks ? L + exp2f(sinks[h] * 1.4426950408889634f - M) : L);
 #pragma unroll
-  for (int c = 0; c < (HD + 63) / 64; ++c) {
+  for (int c = 0; c < (VD + 63) / 64; ++c) {
     const int dim = lane + 64 * c;
-    if (dim < HD) out[(size_t)b * out_row_stride + (size_t)h * HD + dim] = float_to_bf16_bits(acc[c] * inv);
+    if (dim < VD) out[(size_t)b * out_row_stride + (size_t)h * VD + dim] = float_to_bf16_bits(acc[c] * inv);
   }
 }
 
@@ -530,7 +584,7 @@ extern "C" __global__ __launch_bounds__(64) void attn_decode_reduce_kernel(
 // 16 + 4 qd .. 16 + 4 qd + 3; the values are laid into LDS in that order of keys, so the probabilities go
 // from registers to registers.
 typedef __bf16 bf16x8_t __attribute__((ext_vector_type(8)));
-#define PF_KT (HD <= 128 ? 64 : 32)   // keys per round of the main loop (one barrier), in parts of 32
+#define PF_KT (IA_MAX_DIM <= 128 ? 64 : 32)   // keys per round of the main loop (one barrier), in parts of 32
 #define PF_SUBS (PF_KT / 32)
 #define PF_QPT (PF_KT / 4)             // quads of 4 keys per round
 #define PF_KROW (HD + 8)        // bf16 per key row in LDS: 16 bytes of padding spread the banks
@@ -544,9 +598,9 @@ __global__ __launch_bounds__(4 * HGW * 64) void attn_prefill_kernel(
     const uint16_t* __restrict__ v_pages, uint16_t* __restrict__ out, int out_row_stride,
     const int* __restrict__ seq_starts, const int* __restrict__ seq_ctx, const int* __restrict__ block_tables,
     int bt_stride, const int* __restrict__ tiles, int nh, int nkv, int ps, int num_pages, float scale_log2,
-    int window, int paired, const float* __restrict__ sinks) {
+    int window, int paired, const float* __restrict__ sinks, AttnExt X) {
   __shared__ __attribute__((aligned(16))) uint16_t ks[2][PF_KT][PF_KROW];
-  __shared__ __attribute__((aligned(16))) uint16_t vs[2][PF_SUBS][HD][PF_VROW];
+  __shared__ __attribute__((aligned(16))) uint16_t vs[2][PF_SUBS][VD][PF_VROW];
   __shared__ int s_poison;
   constexpr int PF_THREADS = 4 * HGW * 64;
   const int tid = threadIdx.x, lane = tid & 63, j = lane & 15, qd = lane >> 4;
@@ -579,6 +633,7 @@ __global__ __launch_bounds__(4 * HGW * 64) void attn_prefill_kernel(
     last_row = (row0 + 64 < qlen ? row0 + 64 : qlen) - 1;
   }
   if (tid == 0) s_poison = 0;
+  const float to_log2 = (EXT && X.capped) ? 1.0f : scale_log2;      // capped scores are in the log2 domain already
 
   // ---- queries of this wave: CT heads x 16 rows, as B operands (col = row j of head c)
   // steps of 32 head dims; a head size that is an odd multiple of 16 ends with a step whose upper half
@@ -587,7 +642,7 @@ __global__ __launch_bounds__(4 * HGW * 64) void attn_prefill_kernel(
   constexpr bool HALF_LAST = (HD % 32) != 0;
   bf16x8_t q32[CT][NS32];
   int pos[CT], lo[CT];
-  f32x4 o[CT][NS];
+  f32x4 o[CT][NSV];
   float m[CT];
   f32x4 lacc[CT];           // sum of the probabilities of a column, from a product with a tile of ones
   const int row = rb + j;
@@ -607,7 +662,7 @@ __global__ __launch_bounds__(4 * HGW * 64) void attn_prefill_kernel(
     m[c] = ok ? -INFINITY : 0.f;       // a column without a row never asks for a reference point
     lacc[c] = (f32x4){0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-    for (int n = 0; n < NS; ++n) o[c][n] = (f32x4){0.f, 0.f, 0.f, 0.f};
+    for (int n = 0; n < NSV; ++n) o[c][n] = (f32x4){0.f, 0.f, 0.f, 0.f};
   }
   const bf16x8_t ones = __builtin_bit_cast(bf16x8_t, make_uint4(0x3f803f80u, 0x3f803f80u, 0x3f803f80u, 0x3f803f80u));
 
@@ -618,11 +673,16 @@ __global__ __launch_bounds__(4 * HGW * 64) void attn_prefill_kernel(
   const int wave_lo = ia_first_visible_key(ctx + rb, window);
   const int wave_lo_last = ia_first_visible_key(ctx + rb + 15, window);
   const int* bt = block_tables + (size_t)sidx * bt_stride;
-  const int t_begin = key_lo / PF_KT, t_end = key_hi / PF_KT;          // inclusive
+  // EXT: rounds are counted from t_begin - n_keep on; the n_keep rounds before t_begin are the request's first tiles
+  const int n_keep = EXT ? attn_keep_tiles(X.keep, key_lo, PF_KT) : 0;
+  const int t_begin = (EXT && key_lo / PF_KT < n_keep) ? 0 : key_lo / PF_KT - n_keep, t_end = key_hi / PF_KT;   // inclusive
+  const int t_gap = t_begin + n_keep;
+  auto tile_at = [&](int t) { return (EXT && t < t_gap) ? t - t_begin : t; };
+  auto any_row_sees = [&](int key) { return key <= key_hi && (key >= key_lo || key < X.keep); };
 
   // staging: K tile = 32 keys x HD/8 pieces of 16 bytes; V^T tile = HD dims x 8 quads of 4 keys (8 bytes)
   constexpr int KPIECES = PF_KT * (HD / 8), KPT = (KPIECES + PF_THREADS - 1) / (PF_THREADS);
-  constexpr int VPIECES = HD * PF_QPT, VPT = (VPIECES + PF_THREADS - 1) / (PF_THREADS);
+  constexpr int VPIECES = VD * PF_QPT, VPT = (VPIECES + PF_THREADS - 1) / (PF_THREADS);
   // two sets of registers: the loads of a tile are issued two rounds before the tile is used and wait in
   // registers for a round, then in LDS for another, so that a round is never shorter than a load takes
   uint4 kregs[2][KPT];
@@ -637,7 +697,7 @@ __global__ __launch_bounds__(4 * HGW * 64) void attn_prefill_kernel(
   // a page size that is a power of two (POW2) needs a shift and a mask, no division
   auto page_index = [&](int key) { return POW2 ? key >> ps_shift : key / ps; };
   auto page_offset = [&](int key) { return POW2 ? key & (ps - 1) : key % ps; };
-  const size_t page_elems = (size_t)nkv * ps * HD;                 // elements of one page (all heads)
+  const size_t k_page = (size_t)nkv * ps * HD, v_page = (size_t)nkv * ps * VD;      // elements of one page (all heads)
   // what does not change from tile to tile
   int k_row[KPT], k_col[KPT];
 #pragma unroll
@@ -648,8 +708,9 @@ __global__ __launch_bounds__(4 * HGW * 64) void attn_prefill_kernel(
   }
   const int v_quad = tid & (PF_QPT - 1);
   const uint16_t* k_base = k_pages + (size_t)g * ps * HD;
-  const uint16_t* v_base = v_pages + (size_t)g * HD * ps;
-  auto clampk = [&](int key) { return key < key_lo ? key_lo : (key > key_hi ? key_hi : key); };
+  const uint16_t* v_base = v_pages + (size_t)g * VD * ps;
+  // EXT: a key below the kept ones' end stands for itself
+  auto clampk = [&](int key) { return (key < key_lo && !(EXT && key < X.keep)) ? key_lo : (key > key_hi ? key_hi : key); };
   // per thread, once: where its pieces lie within a page row / a tile
   int k_off[KPT];                      // column of the piece within its key row
   size_t v_dim_off[VPT];
@@ -658,10 +719,10 @@ __global__ __launch_bounds__(4 * HGW * 64) void attn_prefill_kernel(
 #pragma unroll
   for (int i = 0; i < VPT; ++i) {
     const int dim = (tid + i * PF_THREADS) / PF_QPT;
-    v_dim_off[i] = (size_t)(dim < HD ? dim : HD - 1) * ps;
+    v_dim_off[i] = (size_t)(dim < VD ? dim : VD - 1) * ps;
   }
   auto load_pages = [&](int t) {
-    const int t0 = t * PF_KT;
+    const int t0 = tile_at(t) * PF_KT;
 #pragma unroll
     for (int i = 0; i < KPT; ++i) pgk[i] = bt[page_index(clampk(t0 + k_row[i]))];
     pgv = bt[page_index(clampk(t0 + v_quad * 4))];        // clamping stays within the quad's page when it is needed
@@ -669,7 +730,7 @@ __global__ __launch_bounds__(4 * HGW * 64) void attn_prefill_kernel(
   auto load_tile = [&](int t, auto set_c) {
     uint4* const kreg = kregs[decltype(set_c)::value];
     uint2* const vreg = vregs[decltype(set_c)::value];
-    const int t0 = t * PF_KT;
+    const int t0 = tile_at(t) * PF_KT;
     const int key0 = t0 + v_quad * 4;
     if (t0 >= key_lo && t0 + PF_KT - 1 <= key_hi) {
       // every key of the tile is one of the request's: no clamping, no masks
@@ -678,12 +739,12 @@ __global__ __launch_bounds__(4 * HGW * 64) void attn_prefill_kernel(
         const bool page_ok = (unsigned)pgk[i] < (unsigned)num_pages;
         bad |= !page_ok && (KPIECES % (PF_THREADS) == 0 || tid + i * PF_THREADS < KPIECES);
         const int key = t0 + (k_row[i] & (PF_KT - 1));
-        kreg[i] = *reinterpret_cast<const uint4*>(k_base + (size_t)(page_ok ? pgk[i] : 0) * page_elems +
+        kreg[i] = *reinterpret_cast<const uint4*>(k_base + (size_t)(page_ok ? pgk[i] : 0) * k_page +
                                                   page_offset(key) * HD + k_off[i]);
       }
       const bool vpage_ok = (unsigned)pgv < (unsigned)num_pages;
       bad |= !vpage_ok;
-      const uint16_t* vq = v_base + (size_t)(vpage_ok ? pgv : 0) * page_elems + page_offset(key0);
+      const uint16_t* vq = v_base + (size_t)(vpage_ok ? pgv : 0) * v_page + page_offset(key0);
 #pragma unroll
       for (int i = 0; i < VPT; ++i) vreg[i] = *reinterpret_cast<const uint2*>(vq + v_dim_off[i]);
       return;
@@ -694,21 +755,21 @@ __global__ __launch_bounds__(4 * HGW * 64) void attn_prefill_kernel(
       const bool need = key == keyc && (KPIECES % (PF_THREADS) == 0 || tid + i * PF_THREADS < KPIECES);
       const bool page_ok = (unsigned)pgk[i] < (unsigned)num_pages;
       bad |= need && !page_ok;
-      const uint4 v = *reinterpret_cast<const uint4*>(k_base + (size_t)(page_ok ? pgk[i] : 0) * page_elems +
+      const uint4 v = *reinterpret_cast<const uint4*>(k_base + (size_t)(page_ok ? pgk[i] : 0) * k_page +
                                                      page_offset(keyc) * HD + k_off[i]);
       kreg[i] = need && page_ok ? v : make_uint4(0u, 0u, 0u, 0u);
     }
-    const bool vneed = key0 + 3 >= key_lo && key0 <= key_hi;
+    const bool vneed = (key0 + 3 >= key_lo || (EXT && key0 < X.keep)) && key0 <= key_hi;
     const bool vpage_ok = (unsigned)pgv < (unsigned)num_pages;
     bad |= vneed && !vpage_ok;
     // keys outside the request's range are not its data: zero them (16 bits each)
-    const uint32_t m0 = (key0 >= key_lo && key0 <= key_hi) ? 0x0000ffffu : 0u;
-    const uint32_t m1 = (key0 + 1 >= key_lo && key0 + 1 <= key_hi) ? 0xffff0000u : 0u;
-    const uint32_t m2 = (key0 + 2 >= key_lo && key0 + 2 <= key_hi) ? 0x0000ffffu : 0u;
-    const uint32_t m3 = (key0 + 3 >= key_lo && key0 + 3 <= key_hi) ? 0xffff0000u : 0u;
+    const uint32_t m0 = (EXT ? any_row_sees(key0) : (key0 >= key_lo && key0 <= key_hi)) ? 0x0000ffffu : 0u;
+    const uint32_t m1 = (EXT ? any_row_sees(key0 + 1) : (key0 + 1 >= key_lo && key0 + 1 <= key_hi)) ? 0xffff0000u : 0u;
+    const uint32_t m2 = (EXT ? any_row_sees(key0 + 2) : (key0 + 2 >= key_lo && key0 + 2 <= key_hi)) ? 0x0000ffffu : 0u;
+    const uint32_t m3 = (EXT ? any_row_sees(key0 + 3) : (key0 + 3 >= key_lo && key0 + 3 <= key_hi)) ? 0xffff0000u : 0u;
     const uint32_t mx = vpage_ok ? (m0 | m1) : 0u, my = vpage_ok ? (m2 | m3) : 0u;
     // the quad lies within one page (the page size is a multiple of 4); its place there is the same for all dims
-    const uint16_t* vq = v_base + (size_t)(vpage_ok ? pgv : 0) * page_elems + page_offset(clampk(key0) & ~3);
+    const uint16_t* vq = v_base + (size_t)(vpage_ok ? pgv : 0) * v_page + page_offset(clampk(key0) & ~3);
 #pragma unroll
     for (int i = 0; i < VPT; ++i) {
       const uint2 v = *reinterpret_cast<const uint2*>(vq + v_dim_off[i]);
@@ -755,8 +816,8 @@ __global__ __launch_bounds__(4 * HGW * 64) void attn_prefill_kernel(
     }
 #pragma unroll
     for (int sub = 0; sub < PF_SUBS; ++sub) {
-    const int t0 = t * PF_KT + sub * 32;
-    if (wave_live && t0 <= wave_hi && t0 + 31 >= wave_lo && t0 <= key_hi) {
+    const int t0 = tile_at(t) * PF_KT + sub * 32;
+    if (wave_live && t0 <= wave_hi && (t0 + 31 >= wave_lo || (EXT && t0 < X.keep)) && t0 <= key_hi) {
       // ---- S^T = K Q^T for the two tiles of 16 keys
       f32x4 sc[CT][2];
 #pragma unroll
@@ -784,13 +845,17 @@ __global__ __launch_bounds__(4 * HGW * 64) void attn_prefill_kernel(
         for (int kt = 0; kt < 2; ++kt)
 #pragma unroll
           for (int r = 0; r < 4; ++r) sv[kt * 4 + r] = sc[c][kt][r];
+        if (EXT && X.capped) {
+#pragma unroll
+          for (int i = 0; i < 8; ++i) sv[i] = X.cap_out * attn_tanh(sv[i] * X.cap_in);
+        }
         if (need_mask) {
 #pragma unroll
           for (int kt = 0; kt < 2; ++kt)
 #pragma unroll
             for (int r = 0; r < 4; ++r) {
               const int kr = t0 + kt * 16 + 4 * qd + r;
-              const bool ok = pos[c] >= 0 && kr <= pos[c] && kr >= lo[c];
+              const bool ok = pos[c] >= 0 && kr <= pos[c] && (kr >= lo[c] || (EXT && kr < X.keep));
               sv[kt * 4 + r] = ok ? sv[kt * 4 + r] : -INFINITY;
             }
         }
@@ -806,10 +871,10 @@ __global__ __launch_bounds__(4 * HGW * 64) void attn_prefill_kernel(
         float m_safe = (m[c] == -INFINITY) ? 0.f : m[c];
         float e[8];
 #pragma unroll
-        for (int i = 0; i < 8; ++i) e[i] = __builtin_amdgcn_exp2f(fmaf(sv[i], scale_log2, -m_safe));
+        for (int i = 0; i < 8; ++i) e[i] = __builtin_amdgcn_exp2f(fmaf(sv[i], to_log2, -m_safe));
         const float emax = fmaxf(fmaxf(fmaxf(e[0], e[1]), fmaxf(e[2], e[3])), fmaxf(fmaxf(e[4], e[5]), fmaxf(e[6], e[7])));
         if (__any(emax > PF_LAZY_EXP || m[c] == -INFINITY)) {
-          const float lmax = scale_log2 * fmaxf(fmaxf(fmaxf(sv[0], sv[1]), fmaxf(sv[2], sv[3])),
+          const float lmax = to_log2 * fmaxf(fmaxf(fmaxf(sv[0], sv[1]), fmaxf(sv[2], sv[3])),
                                                 fmaxf(fmaxf(sv[4], sv[5]), fmaxf(sv[6], sv[7])));
           float tmax = fmaxf(lmax, __shfl_xor(lmax, 16, IA_WAVE));
           tmax = fmaxf(tmax, __shfl_xor(tmax, 32, IA_WAVE));
@@ -818,10 +883,10 @@ __global__ __launch_bounds__(4 * HGW * 64) void attn_prefill_kernel(
           const float corr = __builtin_amdgcn_exp2f(m[c] - m_safe);         // 1 where nothing moved, 0 at the start
           lacc[c] *= corr;
 #pragma unroll
-          for (int n = 0; n < NS; ++n) o[c][n] *= corr;
+          for (int n = 0; n < NSV; ++n) o[c][n] *= corr;
           m[c] = m_new;
 #pragma unroll
-          for (int i = 0; i < 8; ++i) e[i] = __builtin_amdgcn_exp2f(fmaf(sv[i], scale_log2, -m_safe));
+          for (int i = 0; i < 8; ++i) e[i] = __builtin_amdgcn_exp2f(fmaf(sv[i], to_log2, -m_safe));
         }
         // probabilities are rounded to bf16 by the hardware conversion (nearest even); their sum is taken by the
         // matrix cores of the same rounded values (a product with a tile of ones), so that numerator and
@@ -837,7 +902,7 @@ __global__ __launch_bounds__(4 * HGW * 64) void attn_prefill_kernel(
       }
       // ---- O^T += V^T P^T
 #pragma unroll
-      for (int n = 0; n < NS; ++n) {
+      for (int n = 0; n < NSV; ++n) {
         const bf16x8_t va = __builtin_bit_cast(bf16x8_t, *reinterpret_cast<const uint4*>(&vs[buf][sub][n * 16 + j][qd * 8]));
 #pragma unroll
         for (int c = 0; c < CT; ++c) o[c][n] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(va, pb[c], o[c][n], 0, 0, 0);
@@ -861,9 +926,9 @@ __global__ __launch_bounds__(4 * HGW * 64) void attn_prefill_kernel(
     if (sinks) lsum += exp2f(sinks[g * G + (hc * HGW + hgw) * CT + c] * 1.4426950408889634f - m[c]);
     const float inv = poison ? __uint_as_float(0x7fc00000u) : 1.0f / lsum;
     uint16_t* orow = out + (size_t)(qstart + row) * out_row_stride +
-                     (size_t)(g * G + (hc * HGW + hgw) * CT + c) * HD + 4 * qd;
+                     (size_t)(g * G + (hc * HGW + hgw) * CT + c) * VD + 4 * qd;
 #pragma unroll
-    for (int n = 0; n < NS; ++n) {
+    for (int n = 0; n < NSV; ++n) {
       uint2 w;
       w.x = (uint32_t)float_to_bf16_bits(o[c][n][0] * inv) | ((uint32_t)float_to_bf16_bits(o[c][n][1] * inv) << 16);
       w.y = (uint32_t)float_to_bf16_bits(o[c][n][2] * inv) | ((uint32_t)float_to_bf16_bits(o[c][n][3] * inv) << 16);
@@ -874,6 +939,20 @@ __global__ __launch_bounds__(4 * HGW * 64) void attn_prefill_kernel(
 
 // ------------------------------------------------------------------ C interface
 extern "C" int ia_attn_head_dim() { return HD; }
+
+// keep and softcap of a launch, and the scale the kernel multiplies raw scores with: with a softcap the scores it
+// sees are in the log2 domain already
+static int attn_ext(int window, int keep, float softcap, float scale, AttnExt& X, float& scale_log2) {
+  if (keep < 0 || !(softcap >= 0.f)) return IA_ERR_BAD_ARG;
+  if (!EXT && (keep > 0 || softcap > 0.f)) return IA_ERR_UNSUPPORTED;
+  if (window < 0 && keep > 0) return IA_ERR_UNSUPPORTED;
+  X.keep = window > 0 ? keep : 0;
+  X.capped = softcap > 0.f;
+  X.cap_in = X.capped ? scale / softcap : 0.f;
+  X.cap_out = softcap * 1.4426950408889634f;
+  scale_log2 = scale * 1.4426950408889634f;
+  return IA_OK;
+}
 
 static int dec_check(int B, int nh, int nkv, int ps, int num_pages, int bt_stride, int num_splits,
                      const float* part_o, const float* part_ml, int out_row_stride) {
@@ -890,18 +969,22 @@ static int dec_check(int B, int nh, int nkv, int ps, int num_pages, int bt_strid
 extern "C" int ia_attn_decode(const void* q, int q_row_stride, const void* k_pages, const void* v_pages, void* out,
                               int out_row_stride, float* part_o, float* part_ml, const int* positions,
                               const int* block_tables, int bt_stride, int B, int nh, int nkv, int ps, int num_pages,
-                              float scale, int window, int num_splits, const float* sinks, hipStream_t stream) {
+                              float scale, int window, int num_splits, const float* sinks, int keep, float softcap,
+                              hipStream_t stream) {
   const int rc = dec_check(B, nh, nkv, ps, num_pages, bt_stride, num_splits, part_o, part_ml, out_row_stride);
   if (rc != IA_OK) return rc;
   if (q_row_stride & 7) return IA_ERR_UNSUPPORTED;
   if (B == 0) return IA_OK;
   const int G = nh / nkv, HT = (G + 15) / 16;
-  const float scale_log2 = scale * 1.4426950408889634f;
+  AttnExt X;
+  float scale_log2;
+  const int xrc = attn_ext(window, keep, softcap, scale, X, scale_log2);
+  if (xrc != IA_OK) return xrc;
   dim3 grid(B, nkv * HT, num_splits);
 #define DEC_LAUNCH(P2, W)                                                                                          \
   attn_decode_kernel<false, bf16_t, P2, W><<<grid, W * 64, 0, stream>>>(                                             \
       (const uint16_t*)q, q_row_stride, (uint16_t*)k_pages, (uint16_t*)v_pages, (uint16_t*)out, out_row_stride, part_o, \
-      part_ml, positions, block_tables, bt_stride, nh, nkv, ps, num_pages, scale_log2, window, num_splits, DecFused{}, sinks)
+      part_ml, positions, block_tables, bt_stride, nh, nkv, ps, num_pages, scale_log2, window, num_splits, DecFused{}, sinks, X)
   const bool wide = dec_wide(B, nkv * HT, num_splits);
   if ((ps & (ps - 1)) == 0) {
     if (wide) DEC_LAUNCH(true, DEC_WAVES_FEW);
@@ -932,16 +1015,19 @@ extern "C" int ia_attn_decode_fused(const void* src, int src_dtype, int src_spli
                                     void* v_pages, void* out, int out_row_stride, float* part_o, float* part_ml,
                                     const int* positions, const int* block_tables, int bt_stride, int B, int nh,
                                     int nkv, int ps, int num_pages, float scale, int window, int num_splits,
-                                    const float* sinks, hipStream_t stream) {
+                                    const float* sinks, int keep, float softcap, hipStream_t stream) {
   const int rc = dec_check(B, nh, nkv, ps, num_pages, bt_stride, num_splits, part_o, part_ml, out_row_stride);
   if (rc != IA_OK) return rc;
   if (!src || src_splits < 1 || src_rows < B || rot < 0 || rot > HD || (rot & 1)) return IA_ERR_BAD_ARG;
-  if (row_stride < (nh + (slots ? 2 * nkv : 0)) * HD) return IA_ERR_BAD_ARG;
+  if (row_stride < nh * HD + (slots ? nkv * (HD + VD) : 0)) return IA_ERR_BAD_ARG;
   if (!(src_dtype == IA_F32 || (src_dtype == IA_BF16 && src_splits == 1))) return IA_ERR_BAD_ARG;
   if (B == 0) return IA_OK;
   if (!inv_freq) rot = 0;
   const int G = nh / nkv, HT = (G + 15) / 16;
-  const float scale_log2 = scale * 1.4426950408889634f;
+  AttnExt X;
+  float scale_log2;
+  const int xrc = attn_ext(window, keep, softcap, scale, X, scale_log2);
+  if (xrc != IA_OK) return xrc;
   DecFused F;
   F.src = src;
   F.split_stride = (size_t)src_rows * row_stride;
@@ -955,7 +1041,7 @@ extern "C" int ia_attn_decode_fused(const void* src, int src_dtype, int src_spli
 #define DEC_FUSED_LAUNCH(TS, P2, W)                                                                                 \
   attn_decode_kernel<true, TS, P2, W><<<grid, W * 64, 0, stream>>>(                                                 \
       nullptr, 0, (uint16_t*)k_pages, (uint16_t*)v_pages, (uint16_t*)out, out_row_stride, part_o, part_ml, positions, \
-      block_tables, bt_stride, nh, nkv, ps, num_pages, scale_log2, window, num_splits, F, sinks)
+      block_tables, bt_stride, nh, nkv, ps, num_pages, scale_log2, window, num_splits, F, sinks, X)
 #define DEC_FUSED_WAVES(TS, P2)                       \
   do {                                                \
     if (wide) DEC_FUSED_LAUNCH(TS, P2, DEC_WAVES_FEW); \
@@ -989,7 +1075,8 @@ extern "C" int ia_attn_decode_fused(const void* src, int src_dtype, int src_spli
 extern "C" int ia_attn_prefill(const void* q, int q_row_stride, const void* k_pages, const void* v_pages, void* out,
                                int out_row_stride, const int* seq_starts, const int* seq_ctx, const int* block_tables,
                                int bt_stride, const int* tiles, int num_tiles, int nh, int nkv, int ps, int num_pages,
-                               float scale, int window, int launch_shape, const float* sinks, hipStream_t stream) {
+                               float scale, int window, int launch_shape, const float* sinks, int keep, float softcap,
+                               hipStream_t stream) {
   if (launch_shape < 0 || (launch_shape & ~(0xff | IA_PREFILL_PAIRED))) return IA_ERR_BAD_ARG;
   // under a window the rows of the two ends share no keys, and the keys between them may have no page any more:
   // rows are not paired then, whatever was asked for
@@ -1006,22 +1093,25 @@ extern "C" int ia_attn_prefill(const void* q, int q_row_stride, const void* k_pa
   // that many times the rows of Q per tile of keys brought into LDS.  Four groups are 1024 threads, which
   // leaves 128 registers a wave: enough up to a head size of 160.  At head sizes up to 64 two groups measure
   // faster than four (the small tiles let several workgroups share a compute unit).
-  const int widest = (IA_HEAD_DIM >= 80 && IA_HEAD_DIM <= 160) ? 4 : 2;
+  const int widest = (IA_MAX_DIM >= 80 && IA_MAX_DIM <= 160) ? 4 : 2;
   int HGW = G >= 3 ? widest : (G == 2 ? 2 : 1);
   if (heads_per_workgroup != 0) {
     if (heads_per_workgroup != 1 && heads_per_workgroup != 2 && heads_per_workgroup != 4) return IA_ERR_BAD_ARG;
-    if (heads_per_workgroup == 4 && IA_HEAD_DIM > 160) return IA_ERR_UNSUPPORTED;
+    if (heads_per_workgroup == 4 && IA_MAX_DIM > 160) return IA_ERR_UNSUPPORTED;
     HGW = heads_per_workgroup;
   }
   const int HC = (G + HGW - 1) / HGW;
   if ((long long)nkv * HC > 65535) return IA_ERR_UNSUPPORTED;
-  const float scale_log2 = scale * 1.4426950408889634f;
+  AttnExt X;
+  float scale_log2;
+  const int xrc = attn_ext(window, keep, softcap, scale, X, scale_log2);
+  if (xrc != IA_OK) return xrc;
   dim3 grid(num_tiles, nkv * HC);
 #define PF_LAUNCH_P(C, W, P2)                                                                                     \
   attn_prefill_kernel<C, W, P2><<<grid, 4 * W * 64, 0, stream>>>(                                                 \
       (const uint16_t*)q, q_row_stride, (const uint16_t*)k_pages, (const uint16_t*)v_pages, (uint16_t*)out,       \
       out_row_stride, seq_starts, seq_ctx, block_tables, bt_stride, tiles, nh, nkv, ps, num_pages, scale_log2, window, \
-      paired, sinks)
+      paired, sinks, X)
 #define PF_LAUNCH(C, W)                      \
   do {                                       \
     if ((ps & (ps - 1)) == 0) PF_LAUNCH_P(C, W, true); \
@@ -1030,7 +1120,7 @@ extern "C" int ia_attn_prefill(const void* q, int q_row_stride, const void* k_pa
   if (HGW == 1) PF_LAUNCH(1, 1);
   else if (HGW == 2) PF_LAUNCH(1, 2);
   else {
-#if IA_HEAD_DIM <= 160
+#if IA_HEAD_DIM <= 160 && IA_VALUE_DIM <= 160
     PF_LAUNCH(1, 4);
 #else
     return IA_ERR_UNSUPPORTED;

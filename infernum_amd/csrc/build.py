@@ -45,6 +45,8 @@ CORE_SOURCES = [
     "activations.hip",
     "latent.hip",
     "moe.hip",
+    "hyper.hip",
+    "delta_rule.hip",
     "seqmix.hip",
     "linear_attention.hip",
     "sigmoid_attention.hip",
@@ -62,6 +64,8 @@ BLASLT_SOURCES = ["gemm_library.cpp"]
 # Head sizes whose attention library `build_all` compiles ahead of time.
 DEFAULT_HEAD_DIMS = (16, 32, 48, 64, 80, 96, 112, 128, 160, 192, 256)
 SUPPORTED_HEAD_DIMS = tuple(range(16, 257, 16))
+# (key size, value size, with kept first keys and a softcap) whose attention library `build_all` compiles ahead of time.
+DEFAULT_ATTENTION_SIZES = ((16, 32, False), (32, 16, False), (48, 32, False), (32, 32, True), (64, 64, True), (128, 128, True))
 # (key size, value size) pairs whose sigmoid-attention library `build_all` compiles ahead of time.
 DEFAULT_SIGATTN_SIZES = ((16, 32), (32, 64), (48, 16), (64, 64), (64, 128), (96, 32), (128, 32), (128, 64), (128, 128))
 # (key size, value size) pairs whose window-and-blocks attention library `build_all` compiles ahead of time.
@@ -142,7 +146,7 @@ def _fingerprint(sources: Sequence[str], defines: Sequence[str], host: bool = Fa
 
 
 def library_plan(name: str) -> Dict:
-    """Sources and defines of a library by its name ('core', 'attn_d<D>', 'sigattn_d<D>_v<V>', 'wpa_d<D>_v<V>', 'host'
+    """Sources and defines of a library by its name ('core', 'attn_d<D>[_v<V>][_x]', 'sigattn_d<D>_v<V>', 'wpa_d<D>_v<V>', 'host'
     or 'blaslt')."""
     if name == "host":
         return {"sources": _existing(HOST_SOURCES), "defines": [], "host": True}
@@ -155,13 +159,17 @@ def library_plan(name: str) -> Dict:
     if name == "core":
         return {"sources": _existing(CORE_SOURCES), "defines": []}
     if name.startswith("attn_d"):
-        d = int(name[len("attn_d"):])
-        if d not in SUPPORTED_HEAD_DIMS:
-            raise BuildError(f"no MFMA attention kernel for head size {d}: supported are multiples of 16 up to 256")
+        sizes, ext = (name[:-2], True) if name.endswith("_x") else (name, False)
+        d, _, v = sizes[len("attn_d"):].partition("_v")
+        v = v or d
+        if not (d.isdigit() and v.isdigit() and int(d) in SUPPORTED_HEAD_DIMS and int(v) in SUPPORTED_HEAD_DIMS):
+            raise BuildError(f"no MFMA attention kernel named {name!r}: head sizes are multiples of 16 up to 256")
         # accumulators of the matrix cores in ordinary vector registers: the softmax rescales them with
         # vector instructions, which cannot reach the accumulation registers
         return {"sources": ["attention_mfma.hip"],
-                "defines": [f"-DIA_HEAD_DIM={d}", "-mllvm", "-amdgpu-mfma-vgpr-form"]}
+                "defines": [f"-DIA_HEAD_DIM={int(d)}"]
+                + ([f"-DIA_VALUE_DIM={int(v)}"] if v != d else []) + (["-DIA_ATTN_EXT=1"] if ext else [])
+                + ["-mllvm", "-amdgpu-mfma-vgpr-form"]}
     if name.startswith("sigattn_d"):
         d, _, v = name[len("sigattn_d"):].partition("_v")
         if not (d.isdigit() and v.isdigit() and int(d) in SUPPORTED_HEAD_DIMS and int(v) in SUPPORTED_HEAD_DIMS):
@@ -177,6 +185,12 @@ def library_plan(name: str) -> Dict:
         return {"sources": ["window_pool_attention_mfma.hip"],
                 "defines": [f"-DWP_DIM={int(d)}", f"-DWP_VDIM={int(v)}", "-mllvm", "-amdgpu-mfma-vgpr-form"]}
     raise BuildError(f"unknown library {name!r}")
+
+
+def attention_library(d: int, dv: int, ext: bool = False) -> str:
+    """The name of the attention library for key heads of d and value heads of dv values; ``ext``: with kept first keys
+    under a window and a softcap."""
+    return f"attn_d{d}" + (f"_v{dv}" if dv != d else "") + ("_x" if ext else "")
 
 
 def library_path(name: str) -> str:
@@ -282,6 +296,7 @@ def build_all(head_dims: Sequence[int] = DEFAULT_HEAD_DIMS) -> List[str]:
     names = ["host", "blaslt", "core"]
     if os.path.isfile(os.path.join(CSRC_DIR, "attention_mfma.hip")):
         names += [f"attn_d{d}" for d in head_dims]
+        names += [attention_library(*sizes) for sizes in DEFAULT_ATTENTION_SIZES]
     if os.path.isfile(os.path.join(CSRC_DIR, "sigmoid_attention_mfma.hip")):
         names += [f"sigattn_d{d}_v{v}" for d, v in DEFAULT_SIGATTN_SIZES]
     if os.path.isfile(os.path.join(CSRC_DIR, "window_pool_attention_mfma.hip")):

@@ -63,17 +63,21 @@ struct Pool {
 struct Table {
   std::vector<int> pages;
   int64_t num_tokens = 0;
-  int first_live = 0;              // pages before this index have been given back
+  int first_live = 0;              // pages before this index have been given back (but a group's keep_pages first ones)
 };
 
 struct Group {
   int kind = KIND_FULL;
   int window = 0;
+  int keep_pages = 0;              // a window group's first pages of a request that never go back before it ends
   int page_size = 1;
   Pool pool;
   std::unordered_map<int64_t, Table> tables;
-  Group(int kind_, int window_, int page_size_, int num_pages) : kind(kind_), window(window_), page_size(page_size_), pool(num_pages) {}
+  Group(int kind_, int window_, int keep_first, int page_size_, int num_pages)
+      : kind(kind_), window(window_), keep_pages((keep_first + page_size_ - 1) / page_size_), page_size(page_size_), pool(num_pages) {}
 
+  // where a request's pages may begin that it still holds (those given back are NO_PAGE)
+  size_t first_held(const Table& t) const { return keep_pages > 0 ? 0 : (size_t)t.first_live; }
   int pages_for(int64_t tokens) const { return (int)((tokens + page_size - 1) / page_size); }
   int pages_missing(const Table& t, int64_t n_new) const {
     return std::max(0, pages_for(t.num_tokens + n_new) - (int)t.pages.size());
@@ -128,12 +132,14 @@ int ia_pool_is_used(void* h, int page) {
 }
 
 // ------------------------------------------------------------------------------------------- the cache
-// kinds[g]: 0 = all keys, 1 = a window of windows[g] keys, 2 = chunks of windows[g] positions (a query sees its own chunk).  Every group has num_pages pages of page_size.
-void* ia_cache_create(int n_groups, const int* kinds, const int* windows, int page_size, int num_pages, int num_slots) {
+// kinds[g]: 0 = all keys, 1 = a window of windows[g] keys, 2 = chunks of windows[g] positions (a query sees its own chunk).  keeps (nullable): a window group's
+// first keeps[g] positions of a request are kept as well.  Every group has num_pages pages of page_size.
+void* ia_cache_create(int n_groups, const int* kinds, const int* windows, const int* keeps, int page_size, int num_pages,
+                      int num_slots) {
   if (n_groups < 0 || page_size <= 0 || num_pages <= 0 || num_slots < 0) return nullptr;
   Cache* c = new Cache();
   c->page_size = page_size;
-  for (int g = 0; g < n_groups; ++g) c->groups.emplace_back(kinds[g], windows[g], page_size, num_pages);
+  for (int g = 0; g < n_groups; ++g) c->groups.emplace_back(kinds[g], windows[g], keeps ? std::max(keeps[g], 0) : 0, page_size, num_pages);
   c->num_slots = num_slots;
   c->slot_used.assign((size_t)num_slots, 0);
   for (int s = num_slots - 1; s >= 0; --s) c->free_slots.push_back(s);
@@ -267,7 +273,7 @@ int ia_cache_commit(void* h, int64_t req, int64_t n_new) {
       const int stop = (int)std::min<int64_t>(first_needed, (int64_t)t.pages.size());
       while (t.first_live < stop) {
         const int p = t.pages[(size_t)t.first_live];
-        if (p != NO_PAGE) {
+        if (p != NO_PAGE && t.first_live >= g.keep_pages) {
           g.pool.release(p);
           c->last_freed.push_back((int)gi);
           c->last_freed.push_back(p);
@@ -290,7 +296,7 @@ int ia_cache_release(void* h, int64_t req) {
   for (size_t gi = 0; gi < c->groups.size(); ++gi) {
     Group& g = c->groups[gi];
     Table& t = g.tables[req];
-    for (size_t i = (size_t)t.first_live; i < t.pages.size(); ++i)
+    for (size_t i = g.first_held(t); i < t.pages.size(); ++i)
       if (t.pages[i] != NO_PAGE) {
         g.pool.release(t.pages[i]);
         c->last_freed.push_back((int)gi);
@@ -407,7 +413,7 @@ int ia_cache_check(void* h) {
     std::unordered_map<int, int64_t> held;
     for (auto& kv : g.tables) {
       const Table& t = kv.second;
-      for (size_t i = (size_t)t.first_live; i < t.pages.size(); ++i) {
+      for (size_t i = g.first_held(t); i < t.pages.size(); ++i) {
         const int p = t.pages[i];
         if (p == NO_PAGE) continue;
         auto seen = held.find(p);

@@ -12,7 +12,8 @@
 //                       product D of its decays; a second kernel walks a request's tiles, S <- diag(D) S + U, and
 //                       leaves every tile the state before it; then every tile runs from that state and writes its
 //                       rows, the last one the request's slot.  All of it fp32, as the recurrence itself;
-//   ia_head_norm_gate   norm per head, weight, silu(gate), rounded once into the activations' type.
+//   ia_head_norm_gate   norm per head, weight (one for all heads or one a value of every head), silu(gate) or
+//                       sigmoid(gate), rounded once into the activations' type.
 //
 // The state of a head is kept in slices of GLA_PW value columns: slot[head][slice][n][GLA_PW], so that the workgroup
 // that owns (request, head, slice) reads and writes one stretch of memory.  log(alpha) = log_sigmoid(z) / tau and
@@ -404,12 +405,14 @@ extern "C" int ia_hgrn2_gates(void* proj, int code, int proj_stride, int q_col, 
   return IA_OK;
 }
 
-// One wave per (token, head): y = o / sqrt(mean(o^2) + eps) * w * silu(gate), o fp32 [N, nh vdim], w fp32 [vdim],
-// gate rows of gate_stride values in the activations' type (the head's vdim values from gate_col + head * vdim).
+// One wave per (token, head): y = o / sqrt(mean(o^2) + eps) * w * silu(gate), o fp32 [N, nh vdim], w fp32 [vdim]
+// (w_all: [nh vdim], a weight of its own for every head), gate rows of gate_stride values in the activations' type (the
+// head's vdim values from gate_col + head * vdim); plain_sigmoid: sigmoid(gate) in place of silu.  y: rows of y_stride.
 template <typename T>
 __global__ __launch_bounds__(256) void head_norm_gate_kernel(const float* __restrict__ o, const T* __restrict__ gate,
                                                              int gate_stride, int gate_col, const float* __restrict__ w,
-                                                             T* __restrict__ y, long pairs, int nh, int vdim, float eps) {
+                                                             T* __restrict__ y, int y_stride, long pairs, int nh,
+                                                             int vdim, float eps, int w_all, int plain_sigmoid) {
   const long pair = (long)blockIdx.x * 4 + (threadIdx.x >> 6);
   if (pair >= pairs) return;
   const int lane = threadIdx.x & 63;
@@ -420,20 +423,23 @@ __global__ __launch_bounds__(256) void head_norm_gate_kernel(const float* __rest
   for (int i = lane; i < vdim; i += 64) ss = fmaf(orow[i], orow[i], ss);
   ss = wave_sum(ss);
   const float inv = 1.0f / sqrtf(ss / (float)vdim + eps);
+  if (w_all) w += (size_t)hd * vdim;
+  T* yrow = y + (size_t)n * y_stride + (size_t)hd * vdim;
   if (!gate) {                       // no gate: the norm and the weight alone
-    for (int i = lane; i < vdim; i += 64) y[(size_t)pair * vdim + i] = from_float<T>(orow[i] * inv * w[i]);
+    for (int i = lane; i < vdim; i += 64) yrow[i] = from_float<T>(orow[i] * inv * w[i]);
     return;
   }
   const T* grow = gate + (size_t)n * gate_stride + gate_col + (size_t)hd * vdim;
   for (int i = lane; i < vdim; i += 64) {
     const float g = to_float(grow[i]);
-    y[(size_t)pair * vdim + i] = from_float<T>(orow[i] * inv * w[i] * (g / (1.0f + expf(-g))));
+    yrow[i] = from_float<T>(orow[i] * inv * w[i] * ((plain_sigmoid ? 1.0f : g) / (1.0f + expf(-g))));
   }
 }
 
 extern "C" int ia_head_norm_gate(const float* o, const void* gate, int code, int gate_stride, int gate_col,
-                                 const float* w, void* y, int N, int nh, int vdim, float eps, hipStream_t stream) {
-  if (N < 0 || nh <= 0 || vdim <= 0 || !(eps > 0.f) || (gate && (gate_col < 0 || gate_stride < gate_col + nh * vdim)))
+                                 const float* w, void* y, int y_stride, int N, int nh, int vdim, float eps, int w_all,
+                                 int plain_sigmoid, hipStream_t stream) {
+  if (N < 0 || y_stride < nh * vdim || nh <= 0 || vdim <= 0 || !(eps > 0.f) || (gate && (gate_col < 0 || gate_stride < gate_col + nh * vdim)))
     return IA_ERR_BAD_ARG;
   if (N == 0) return IA_OK;
   if (!o || !w || !y) return IA_ERR_BAD_ARG;
@@ -442,10 +448,12 @@ extern "C" int ia_head_norm_gate(const float* o, const void* gate, int code, int
   if (blocks > 0x7fffffffL) return IA_ERR_UNSUPPORTED;
   if (code == IA_F32)
     head_norm_gate_kernel<float><<<(unsigned)blocks, 256, 0, stream>>>(o, (const float*)gate, gate_stride, gate_col, w,
-                                                                       (float*)y, pairs, nh, vdim, eps);
+                                                                       (float*)y, y_stride, pairs, nh, vdim, eps, w_all,
+                                                                       plain_sigmoid);
   else if (code == IA_BF16)
     head_norm_gate_kernel<bf16_t><<<(unsigned)blocks, 256, 0, stream>>>(o, (const bf16_t*)gate, gate_stride, gate_col, w,
-                                                                        (bf16_t*)y, pairs, nh, vdim, eps);
+                                                                        (bf16_t*)y, y_stride, pairs, nh, vdim, eps, w_all,
+                                                                        plain_sigmoid);
   else
     return IA_ERR_BAD_ARG;
   IA_LAUNCH_CHECK();

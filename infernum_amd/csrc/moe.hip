@@ -3,7 +3,8 @@
 //                    over those alone;
 //   ia_moe_sort      the (token, choice) pairs grouped by expert: offsets[E + 1], perm[P];
 //   ia_moe_gate_up   per expert, over its pairs' tokens: g = min(Wg x, limit), u = clamp(Wu x, -limit, limit),
-//                    y = g sigmoid(alpha g) (u + 1); the rows of Wg and Wu alternate in the expert's matrix;
+//                    y = g sigmoid(alpha g) (u + shift); the rows of Wg and Wu alternate in the expert's matrix (limit
+//                    infinity, alpha 1, shift 0: y = silu(Wg x) (Wu x));
 //   ia_moe_down      per expert: Wd y times the pair's routing weight, as fp32 into parts[choice, token, :], which
 //                    the kernel that takes the feed-forward's result next adds in the order of the choices.
 // Only the chosen experts' weights are read.  A pair's result is one chain of operations over its own token and
@@ -136,7 +137,7 @@ template <typename T>
 __global__ __launch_bounds__(256) void moe_gate_up_kernel(const T* __restrict__ x, const T* __restrict__ Wgu,
                                                           T* __restrict__ y, const int* __restrict__ offsets,
                                                           const int* __restrict__ perm, int E, int top, int W,
-                                                          int ff, float limit, float alpha) {
+                                                          int ff, float limit, float alpha, float shift) {
   __shared__ TileFmaLds lds;
   int e, first, last;
   if (!moe_tile(offsets, E, blockIdx.y, e, first, last)) return;
@@ -154,7 +155,7 @@ __global__ __launch_bounds__(256) void moe_gate_up_kernel(const T* __restrict__ 
       // both products are rounded as a stored tensor would be, then the activation in fp32
       const float g = fminf(to_float(from_float<T>(v[j])), limit);
       const float u = fminf(fmaxf(to_float(from_float<T>(v[j + 1])), -limit), limit);
-      y[(size_t)p * ff + (c >> 1)] = from_float<T>(g * (1.0f / (1.0f + expf(-alpha * g))) * (u + 1.0f));
+      y[(size_t)p * ff + (c >> 1)] = from_float<T>(g * (1.0f / (1.0f + expf(-alpha * g))) * (u + shift));
     }
   });
 }
@@ -164,7 +165,7 @@ template <int BM, int BN>
 __global__ __launch_bounds__(BN == 256 ? 512 : 256) void moe_gate_up_big_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict__ Wgu,
                                                               bf16_t* __restrict__ y, const int* __restrict__ offsets,
                                                               const int* __restrict__ perm, int E, int top, int W,
-                                                              int ff, float limit, float alpha) {
+                                                              int ff, float limit, float alpha, float shift) {
   __shared__ TileBigLds<BM, BN> lds;
   int e, first, last;
   if (!moe_tile(offsets, E, blockIdx.y, e, first, last, BM)) return;
@@ -181,7 +182,7 @@ __global__ __launch_bounds__(BN == 256 ? 512 : 256) void moe_gate_up_big_kernel(
           if (c + 1 >= 2 * ff) continue;
           const float g = fminf(to_float(from_float<bf16_t>(v[j])), limit);
           const float u = fminf(fmaxf(to_float(from_float<bf16_t>(v[j + 1])), -limit), limit);
-          y[(size_t)p * ff + (c >> 1)] = from_float<bf16_t>(g * (1.0f / (1.0f + expf(-alpha * g))) * (u + 1.0f));
+          y[(size_t)p * ff + (c >> 1)] = from_float<bf16_t>(g * (1.0f / (1.0f + expf(-alpha * g))) * (u + shift));
         }
       });
 }
@@ -190,14 +191,15 @@ __global__ __launch_bounds__(BN == 256 ? 512 : 256) void moe_gate_up_big_kernel(
 static inline int moe_tile_rows(int P, int E) { return (long)P >= 48L * E ? 128 : 32; }
 
 extern "C" int ia_moe_gate_up(const void* x, const void* Wgu, void* y, const int* offsets, const int* perm, int dtype,
-                              int P, int E, int top, int W, int ff, float limit, float alpha, hipStream_t stream) {
+                              int P, int E, int top, int W, int ff, float limit, float alpha, float shift,
+                              hipStream_t stream) {
   if (P < 0 || E <= 0 || top <= 0 || W <= 0 || ff <= 0) return IA_ERR_BAD_ARG;
   if (P == 0) return IA_OK;
   dim3 grid((2 * ff + TF_T - 1) / TF_T, (P + TF_T - 1) / TF_T + E);
   if (grid.y > 65535u) return IA_ERR_UNSUPPORTED;
   if (dtype == IA_F32)
     moe_gate_up_kernel<float><<<grid, 256, 0, stream>>>((const float*)x, (const float*)Wgu, (float*)y, offsets,
-                                                               perm, E, top, W, ff, limit, alpha);
+                                                               perm, E, top, W, ff, limit, alpha, shift);
   else if (dtype == IA_BF16 && tile_rows_aligned(x, W) && tile_rows_aligned(Wgu, W)) {
     const int bm = moe_tile_rows(P, E);
     const int bn = bm == 128 ? 256 : TB_N;
@@ -205,14 +207,14 @@ extern "C" int ia_moe_gate_up(const void* x, const void* Wgu, void* y, const int
     if (big.y > 65535u) return IA_ERR_UNSUPPORTED;
     if (bm == 128)
       moe_gate_up_big_kernel<128, 256><<<big, 512, 0, stream>>>((const bf16_t*)x, (const bf16_t*)Wgu, (bf16_t*)y, offsets,
-                                                           perm, E, top, W, ff, limit, alpha);
+                                                           perm, E, top, W, ff, limit, alpha, shift);
     else
       moe_gate_up_big_kernel<32, TB_N><<<big, 256, 0, stream>>>((const bf16_t*)x, (const bf16_t*)Wgu, (bf16_t*)y, offsets,
-                                                          perm, E, top, W, ff, limit, alpha);
+                                                          perm, E, top, W, ff, limit, alpha, shift);
   }
   else if (dtype == IA_BF16)
     moe_gate_up_kernel<bf16_t><<<grid, 256, 0, stream>>>((const bf16_t*)x, (const bf16_t*)Wgu, (bf16_t*)y,
-                                                                offsets, perm, E, top, W, ff, limit, alpha);
+                                                                offsets, perm, E, top, W, ff, limit, alpha, shift);
   else
     return IA_ERR_BAD_ARG;
   IA_LAUNCH_CHECK();
@@ -309,8 +311,9 @@ extern "C" int ia_moe_down(const void* y, const void* Wd, float* parts, const fl
 // The tokens' rows are first brought into the order of the sort (an expert's rows one after the other), the two
 // products run expert by expert over those rows, and the activation and the routing weight are passes of their own:
 //   ia_moe_gather   xs[p, :] = x[perm[p] / top, :]
-//   ia_moe_glu      y[p, j] = g sigmoid(alpha g) (u + 1), g = min(gu[p, 2 j], limit), u = clamp(gu[p, 2 j + 1], +-limit)
-//   ia_moe_scatter  parts[choice, token, :] = float(o[p, :]) * weights[perm[p]]
+//   ia_moe_glu      y[p, j] = g sigmoid(alpha g) (u + shift), g = min(gu[p, 2 j], limit), u = clamp(gu[p, 2 j + 1], +-limit)
+//   ia_moe_scatter  parts[choice, token, :] = float(o[p, :]) * weights[perm[p]], for the places p below *last (nullable:
+//                   all of them)
 // All three in bfloat16 with rows that are read 16 bytes at a time.
 __global__ __launch_bounds__(256) void moe_gather_kernel(const uint4* __restrict__ x, const int* __restrict__ perm,
                                                          uint4* __restrict__ xs, int top, int pieces) {
@@ -330,7 +333,7 @@ extern "C" int ia_moe_gather(const void* x, const int* perm, void* xs, int P, in
 }
 
 __global__ __launch_bounds__(256) void moe_glu_kernel(const uint4* __restrict__ gu, uint2* __restrict__ y, size_t n4,
-                                                      float limit, float alpha) {
+                                                      float limit, float alpha, float shift) {
   const size_t stride = (size_t)gridDim.x * 256;
   for (size_t i = (size_t)blockIdx.x * 256 + threadIdx.x; i < n4; i += stride) {
     const uint4 v = gu[i];
@@ -340,7 +343,7 @@ __global__ __launch_bounds__(256) void moe_glu_kernel(const uint4* __restrict__ 
     for (int k = 0; k < 4; ++k) {
       const float g = fminf(__uint_as_float(w[k] << 16), limit);
       const float u = fminf(fmaxf(__uint_as_float(w[k] & 0xffff0000u), -limit), limit);
-      o[k] = g * (1.0f / (1.0f + expf(-alpha * g))) * (u + 1.0f);
+      o[k] = g * (1.0f / (1.0f + expf(-alpha * g))) * (u + shift);
     }
     uint2 r;
     r.x = (uint32_t)float_to_bf16_bits(o[0]) | ((uint32_t)float_to_bf16_bits(o[1]) << 16);
@@ -349,21 +352,22 @@ __global__ __launch_bounds__(256) void moe_glu_kernel(const uint4* __restrict__ 
   }
 }
 
-extern "C" int ia_moe_glu(const void* gu, void* y, int P, int ff, float limit, float alpha, hipStream_t stream) {
+extern "C" int ia_moe_glu(const void* gu, void* y, int P, int ff, float limit, float alpha, float shift, hipStream_t stream) {
   if (P < 0 || ff <= 0) return IA_ERR_BAD_ARG;
   if ((ff & 3) || ((reinterpret_cast<uintptr_t>(gu) | reinterpret_cast<uintptr_t>(y)) & 15)) return IA_ERR_UNSUPPORTED;
   const size_t n4 = (size_t)P * ff / 4;
   if (n4 == 0) return IA_OK;
   const unsigned grid = (unsigned)((n4 + 255) / 256 < 65536 ? (n4 + 255) / 256 : 65536);
-  moe_glu_kernel<<<grid, 256, 0, stream>>>((const uint4*)gu, (uint2*)y, n4, limit, alpha);
+  moe_glu_kernel<<<grid, 256, 0, stream>>>((const uint4*)gu, (uint2*)y, n4, limit, alpha, shift);
   IA_LAUNCH_CHECK();
   return IA_OK;
 }
 
 __global__ __launch_bounds__(256) void moe_scatter_kernel(const uint4* __restrict__ o, const int* __restrict__ perm,
                                                           const float* __restrict__ weights, float* __restrict__ parts,
-                                                          int N, int top, int W) {
+                                                          const int* __restrict__ last, int N, int top, int W) {
   const int p = blockIdx.x;
+  if (last && p >= *last) return;                  // a pair that went to no expert with tensors
   const int pair = perm[p];
   const int token = pair / top, choice = pair - token * top;
   const float wt = weights[pair];
@@ -378,19 +382,22 @@ __global__ __launch_bounds__(256) void moe_scatter_kernel(const uint4* __restric
   }
 }
 
-extern "C" int ia_moe_scatter(const void* o, const int* perm, const float* weights, float* parts, int N, int top,
-                              int W, hipStream_t stream) {
+extern "C" int ia_moe_scatter(const void* o, const int* perm, const float* weights, float* parts, const int* last, int N,
+                              int top, int W, hipStream_t stream) {
   if (N < 0 || top <= 0 || W <= 0) return IA_ERR_BAD_ARG;
   if ((W & 7) || ((reinterpret_cast<uintptr_t>(o) | reinterpret_cast<uintptr_t>(parts)) & 15)) return IA_ERR_UNSUPPORTED;
   if (N == 0) return IA_OK;
-  moe_scatter_kernel<<<N * top, 256, 0, stream>>>((const uint4*)o, perm, weights, parts, N, top, W);
+  moe_scatter_kernel<<<N * top, 256, 0, stream>>>((const uint4*)o, perm, weights, parts, last, N, top, W);
   IA_LAUNCH_CHECK();
   return IA_OK;
 }
 
 // ---- experts without a gate, and a router whose choice and weights go by different numbers ----
 //   ia_router_softmax_topk   s = softmax(z) over all experts; the `top` largest of s + correction are chosen (the
-//                            lowest index among equals); the weights are the chosen s over their sum (+ 1e-20);
+//                            lowest index among equals); the weights are the chosen s, with `renorm` over their sum
+//                            (+ 1e-20).  With `groups` > 1 the experts form that many groups of neighbours, a group's
+//                            score is its largest s + correction, and only experts of the `keep` best groups (the
+//                            lowest index among equals) can be chosen;
 //   ia_moe_up                per expert, over its pairs' tokens: y = act(Wu x), Wu [E, ff, W]; act by the codes of
 //                            ia_activation (2: the erf GELU, 3: the square of relu).
 __device__ __forceinline__ float moe_act(float z, int act) {
@@ -403,10 +410,12 @@ __device__ __forceinline__ float moe_act(float z, int act) {
 __global__ __launch_bounds__(256) void router_softmax_topk_kernel(const float* __restrict__ logits,
                                                                   const void* __restrict__ corr, int corr_dtype,
                                                                   int* __restrict__ ids, float* __restrict__ weights,
-                                                                  int N, int E, int top) {
+                                                                  int N, int E, int top, int z_stride, int groups,
+                                                                  int keep, int renorm) {
+  __shared__ float s_v[4][64 * RT_PER_LANE];       // a wave's choice scores, then (in place) its groups' scores
   const int n = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
   if (n >= N) return;
-  const float* z = logits + (size_t)n * E;
+  const float* z = logits + (size_t)n * z_stride;
   float s[RT_PER_LANE], v[RT_PER_LANE];
   unsigned taken = 0u;
   float zmax = -INFINITY;
@@ -431,6 +440,37 @@ __global__ __launch_bounds__(256) void router_softmax_topk_kernel(const float* _
     const int e = lane + 64 * c;
     s[c] *= inv_total;
     v[c] = e < E ? s[c] + (corr ? load_as_float(corr, corr_dtype, e) : 0.f) : -INFINITY;
+  }
+  if (groups > 1) {
+    // each wave works on its own part of LDS: a wave's accesses are in order, no barrier is needed between them
+    volatile float* mine = s_v[threadIdx.x >> 6];
+    const int size = E / groups;
+#pragma unroll
+    for (int c = 0; c < RT_PER_LANE; ++c)
+      if (lane + 64 * c < E) mine[lane + 64 * c] = (v[c] == v[c]) ? v[c] : -INFINITY;
+    float gs[RT_PER_LANE];                        // this lane's groups: lane, lane + 64, ...
+#pragma unroll
+    for (int c = 0; c < RT_PER_LANE; ++c) {
+      gs[c] = -INFINITY;
+      const int g = lane + 64 * c;
+      if (g < groups)
+        for (int i = 0; i < size; ++i) gs[c] = fmaxf(gs[c], mine[g * size + i]);
+    }
+    __builtin_amdgcn_wave_barrier();
+#pragma unroll
+    for (int c = 0; c < RT_PER_LANE; ++c)
+      if (lane + 64 * c < groups) mine[lane + 64 * c] = gs[c];
+    __builtin_amdgcn_wave_barrier();
+#pragma unroll
+    for (int c = 0; c < RT_PER_LANE; ++c) {
+      const int e = lane + 64 * c;
+      if (e >= E) continue;
+      const int g = e / size;
+      const float own = mine[g];
+      int better = 0;
+      for (int i = 0; i < groups; ++i) better += mine[i] > own || (mine[i] == own && i < g);
+      if (better >= keep) taken |= 1u << c;
+    }
   }
   float sum = 0.f;
   for (int k = 0; k < top; ++k) {
@@ -460,16 +500,19 @@ __global__ __launch_bounds__(256) void router_softmax_topk_kernel(const float* _
     }
   }
   const float inv = 1.0f / (sum + 1e-20f);
-  if (lane == 0)
+  if (lane == 0 && renorm)
     for (int k = 0; k < top; ++k) weights[(size_t)n * top + k] *= inv;
 }
 
 extern "C" int ia_router_softmax_topk(const float* logits, const void* corr, int corr_dtype, int* ids, float* weights,
-                                      int N, int E, int top, hipStream_t stream) {
-  if (N < 0 || E <= 0 || top <= 0 || top > E || !logits || !ids || !weights) return IA_ERR_BAD_ARG;
+                                      int N, int E, int top, int z_stride, int groups, int keep, int renorm,
+                                      hipStream_t stream) {
+  if (N < 0 || E <= 0 || top <= 0 || top > E || z_stride < E || groups < 1 || E % groups || keep < 1 || keep > groups ||
+      top > keep * (E / groups) || !logits || !ids || !weights) return IA_ERR_BAD_ARG;
   if (E > 64 * RT_PER_LANE) return IA_ERR_UNSUPPORTED;
   if (N == 0) return IA_OK;
-  router_softmax_topk_kernel<<<(N + 3) / 4, 256, 0, stream>>>(logits, corr, corr_dtype, ids, weights, N, E, top);
+  router_softmax_topk_kernel<<<(N + 3) / 4, 256, 0, stream>>>(logits, corr, corr_dtype, ids, weights, N, E, top, z_stride, groups,
+                                                                keep, renorm);
   IA_LAUNCH_CHECK();
   return IA_OK;
 }
@@ -549,7 +592,57 @@ extern "C" int ia_moe_up(const void* x, const void* Wu, void* y, const int* offs
   return IA_OK;
 }
 
+// ---- what a step adds beside its experts' products ----
+//   ia_moe_extras   for every pair whose expert is one of the last, without tensors (ids >= E: an expert whose result is
+//                   its input): parts[choice, token, :] = weight * x[token, :]; and for every token, with `shared`: its
+//                   result ([splits, shared_rows, W], added in the order of the parts) times sigmoid(gate[token]) into
+//                   parts[top, token, :], the part after the choices'.
+template <typename T, typename TS>
+__global__ __launch_bounds__(256) void moe_extras_kernel(const T* __restrict__ x, const int* __restrict__ ids,
+                                                         const float* __restrict__ weights, float* __restrict__ parts,
+                                                         const TS* __restrict__ shared, int splits, size_t split_stride,
+                                                         const float* __restrict__ gate, int gate_stride, int N, int E,
+                                                         int top, int W) {
+  const int n = blockIdx.x, choice = blockIdx.y;
+  float* o = parts + ((size_t)choice * N + n) * W;
+  if (choice == top) {
+    const float g = gate ? 1.0f / (1.0f + expf(-gate[(size_t)n * gate_stride])) : 1.0f;
+    const TS* s = shared + (size_t)n * W;
+    for (int i = threadIdx.x; i < W; i += 256) o[i] = g * load_split_sum(s + i, splits, split_stride);
+    return;
+  }
+  if (ids[(size_t)n * top + choice] < E) return;
+  const float wt = weights[(size_t)n * top + choice];
+  const T* xr = x + (size_t)n * W;
+  for (int i = threadIdx.x; i < W; i += 256) o[i] = wt * to_float(xr[i]);
+}
+
+// parts: fp32 [top (+ 1 with shared), N, W]; shared (nullable) of shared_dtype; gate (nullable): fp32, token n's logit
+// at gate[n gate_stride].
+extern "C" int ia_moe_extras(const void* x, int dtype, const int* ids, const float* weights, float* parts, const void* shared,
+                             int shared_dtype, int splits, int shared_rows, const float* gate, int gate_stride, int N, int E,
+                             int top, int W, hipStream_t stream) {
+  if (N < 0 || E < 0 || top <= 0 || W <= 0 || !x || !ids || !weights || !parts || top > 65534 ||
+      (shared && (splits < 1 || shared_rows < N)) || (dtype != IA_F32 && dtype != IA_BF16) ||
+      (shared && shared_dtype != IA_F32 && shared_dtype != IA_BF16))
+    return IA_ERR_BAD_ARG;
+  if (N == 0) return IA_OK;
+  const dim3 grid(N, top + (shared ? 1 : 0));
+  const size_t stride = (size_t)shared_rows * W;
+#define IA_MX(T, TS)                                                                                                  moe_extras_kernel<T, TS><<<grid, 256, 0, stream>>>((const T*)x, ids, weights, parts, (const TS*)shared, splits, stride,                                                      gate, gate_stride, N, E, top, W)
+  const bool sf = !shared || shared_dtype == IA_F32;
+  if (dtype == IA_F32) {
+    if (sf) IA_MX(float, float);
+    else return IA_ERR_BAD_ARG;
+  } else if (sf) IA_MX(bf16_t, float);
+  else IA_MX(bf16_t, bf16_t);
+#undef IA_MX
+  IA_LAUNCH_CHECK();
+  return IA_OK;
+}
+
 #include "op_call.h"
+IA_OP(ia_moe_extras)
 IA_OP(ia_router_topk)
 IA_OP(ia_moe_sort)
 IA_OP(ia_moe_gate_up)

@@ -330,6 +330,20 @@ extern "C" int ia_conv_state_update(const void* u, int u_code, int u_stride, con
 }
 
 // ------------------------------------------------------------------------------------------ queries and keys
+// What becomes of a value on its way to its page: v <- v_scale ((1 - lambda) v + lambda v_first), v_first the same
+// token's value of another layer (nullable: no mixing).
+struct ValueWay {
+  const void* first;             // rows of first_stride values in the activations' type, this token's value heads first
+  int first_stride;
+  float lambda, scale;
+};
+
+template <typename T>
+__device__ __forceinline__ float value_way(float v, const ValueWay& V, size_t row, int col) {
+  if (V.first) v = __builtin_fmaf(V.lambda, to_float(reinterpret_cast<const T*>(V.first)[row * V.first_stride + col]), (1.0f - V.lambda) * v);
+  return V.scale * v;
+}
+
 // One wave per (token, head).  Rows of x: nh query heads, nkv key heads, and nkv value heads when the values are
 // not the keys.  pairing 0: value i with value i + rot/2; 1: value 2i with value 2i+1.
 template <typename T>
@@ -337,7 +351,8 @@ __global__ __launch_bounds__(256) void qk_prepare_kernel(
     const T* __restrict__ x, int x_stride, T* __restrict__ q_out, int q_stride, const float* __restrict__ q_norm,
     const float* __restrict__ k_norm, float eps, const int* __restrict__ positions, const int* __restrict__ slots,
     const void* __restrict__ freq, int freq_f64, int rot, int pairing, float magnitude, T* __restrict__ k_pages,
-    T* __restrict__ v_pages, int N, int nh, int nkv, int d, int page_size, int num_pages, int values_are_keys) {
+    T* __restrict__ v_pages, int N, int nh, int nkv, int d, int dv, int page_size, int num_pages, int values_are_keys,
+    ValueWay V) {
   const int lane = threadIdx.x & 63;
   const int heads = nh + nkv;
   const long item = (long)blockIdx.x * 4 + (threadIdx.x >> 6);
@@ -364,9 +379,10 @@ __global__ __launch_bounds__(256) void qk_prepare_kernel(
     const int g = hd - nh;
     dst = k_pages + (((size_t)page * nkv + g) * page_size + off) * d;
     // the values: the value head of the row, or the key head as it came in; transposed within the page
-    const T* vsrc = values_are_keys ? src : x + (size_t)t * x_stride + (size_t)(heads + g) * d;
-    T* vdst = v_pages + ((size_t)page * nkv + g) * (size_t)d * page_size + off;
-    for (int i = lane; i < d; i += 64) vdst[(size_t)i * page_size] = vsrc[i];
+    const T* vsrc = values_are_keys ? src : x + (size_t)t * x_stride + (size_t)heads * d + (size_t)g * dv;
+    T* vdst = v_pages + ((size_t)page * nkv + g) * (size_t)dv * page_size + off;
+    for (int i = lane; i < dv; i += 64)
+      vdst[(size_t)i * page_size] = from_float<T>(value_way<T>(to_float(vsrc[i]), V, (size_t)t, g * dv + i));
   } else {
     dst = q_out + (size_t)t * q_stride + (size_t)hd * d;
   }
@@ -393,13 +409,47 @@ __global__ __launch_bounds__(256) void qk_prepare_kernel(
 
 // The same for bf16 heads of whole 16-byte pieces whose rotated pairs are neighbours (or that are not rotated):
 // a group of GL lanes (a power of two, at least d / 8) per (token, head), a lane takes 8 consecutive values, so a
-// pair lies within a lane and every access but the transposed values' is 16 bytes.
+// pair lies within a lane and every access is 16 bytes.  The workgroups from qk_blocks on write the values: a wave
+// takes 16 tokens and 32 values of a head, so that what it writes to the transposed pages are stretches of up to 16
+// positions.
 __global__ __launch_bounds__(256) void qk_prepare_vec_kernel(
     const bf16_t* __restrict__ x, int x_stride, bf16_t* __restrict__ q_out, int q_stride, const float* __restrict__ q_norm,
     const float* __restrict__ k_norm, float eps, const int* __restrict__ positions, const int* __restrict__ slots,
     const void* __restrict__ freq, int freq_f64, int rot, float magnitude, bf16_t* __restrict__ k_pages,
-    bf16_t* __restrict__ v_pages, int N, int nh, int nkv, int d, int page_size, int num_pages, int values_are_keys, int GL) {
+    bf16_t* __restrict__ v_pages, int N, int nh, int nkv, int d, int dv, int page_size, int num_pages, int values_are_keys,
+    int GL, int qk_blocks, ValueWay V) {
   const int heads = nh + nkv;
+  if ((int)blockIdx.x >= qk_blocks) {
+    const int pieces = nkv * dv / 8, groups = (pieces + 3) / 4;          // 8 values a lane, 4 lanes side by side
+    const long w = (long)((int)blockIdx.x - qk_blocks) * 4 + (threadIdx.x >> 6);
+    const int lane = threadIdx.x & 63;
+    const int t = (int)(w / groups) * 16 + (lane & 15), piece = (int)(w % groups) * 4 + (lane >> 4);
+    if (t >= N || piece >= pieces) return;
+    const int slot = slots[t], page = slot / page_size, off = slot - page * page_size;
+    if (page < 0 || page >= num_pages) return;
+    const int col = piece * 8, g = col / dv, c = col - g * dv;
+    const uint4 raw = *(const uint4*)(x + (size_t)t * x_stride + (size_t)(values_are_keys ? nh : heads) * d + col);
+    const uint32_t rw[4] = {raw.x, raw.y, raw.z, raw.w};
+    float v[8];
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      v[2 * e] = __uint_as_float(rw[e] << 16);
+      v[2 * e + 1] = __uint_as_float(rw[e] & 0xffff0000u);
+    }
+    if (V.first) {
+      const uint4 f = *(const uint4*)((const bf16_t*)V.first + (size_t)t * V.first_stride + col);
+      const uint32_t fw[4] = {f.x, f.y, f.z, f.w};
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        v[2 * e] = __builtin_fmaf(V.lambda, __uint_as_float(fw[e] << 16), (1.0f - V.lambda) * v[2 * e]);
+        v[2 * e + 1] = __builtin_fmaf(V.lambda, __uint_as_float(fw[e] & 0xffff0000u), (1.0f - V.lambda) * v[2 * e + 1]);
+      }
+    }
+    uint16_t* vdst = (uint16_t*)v_pages + ((size_t)page * nkv + g) * (size_t)dv * page_size + (size_t)c * page_size + off;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) vdst[(size_t)e * page_size] = float_to_bf16_bits(V.scale * v[e]);
+    return;
+  }
   const int per_block = 256 / GL;
   const long item = (long)blockIdx.x * per_block + threadIdx.x / GL;
   const int ch = threadIdx.x % GL;                        // which 8 values of the head
@@ -427,18 +477,6 @@ __global__ __launch_bounds__(256) void qk_prepare_vec_kernel(
   const int page = slot / page_size, off = slot - page * page_size;
   if (is_key && (page < 0 || page >= num_pages)) return;
   const int g = hd - nh;
-  if (is_key) {
-    // the values: the value head of the row, or the key head as it came in; transposed within the page
-    uint4 vr = raw;
-    if (!values_are_keys) vr = *(const uint4*)(x + (size_t)t * x_stride + (size_t)(heads + g) * d + 8 * ch);
-    const uint32_t vw[4] = {vr.x, vr.y, vr.z, vr.w};
-    uint16_t* vdst = (uint16_t*)v_pages + ((size_t)page * nkv + g) * (size_t)d * page_size + (size_t)(8 * ch) * page_size + off;
-#pragma unroll
-    for (int e = 0; e < 4; ++e) {
-      vdst[(size_t)(2 * e) * page_size] = (uint16_t)(vw[e] & 0xffffu);
-      vdst[(size_t)(2 * e + 1) * page_size] = (uint16_t)(vw[e] >> 16);
-    }
-  }
   if (wn) {
     const float inv = 1.0f / sqrtf(ss / (float)d + eps);
     const float4 w0 = *(const float4*)(wn + 8 * ch), w1 = *(const float4*)(wn + 8 * ch + 4);
@@ -467,30 +505,38 @@ __global__ __launch_bounds__(256) void qk_prepare_vec_kernel(
   *(uint4*)dst = make_uint4(o[0], o[1], o[2], o[3]);
 }
 
+// v_first (nullable): rows of v_first_stride values of x's type, the token's nkv value heads of dv from the row's start.
 extern "C" int ia_qk_prepare(const void* x, int code, int x_stride, void* q_out, int q_stride, const float* q_norm,
                              const float* k_norm, float eps, const int* positions, const int* slots, const void* freq,
                              int freq_f64, int rot, int pairing, float magnitude, void* k_pages, void* v_pages, int N,
-                             int nh, int nkv, int d, int page_size, int num_pages, int values_are_keys,
-                             hipStream_t stream) {
+                             int nh, int nkv, int d, int dv, int page_size, int num_pages, int values_are_keys,
+                             float v_scale, const void* v_first, int v_first_stride, float v_lambda, hipStream_t stream) {
   if (N == 0) return IA_OK;
-  const int write = k_pages != nullptr;
+  const bool write = k_pages != nullptr;
   if (!x || !q_out || !positions || N < 0 || nh <= 0 || nkv < 0 || d <= 0 || rot < 0 || rot > d || (rot & 1) ||
-      (rot > 0 && !freq) || (write && (!v_pages || !slots || page_size <= 0 || num_pages <= 0)) ||
-      x_stride < (nh + (write ? (values_are_keys ? nkv : 2 * nkv) : 0)) * d || q_stride < nh * d ||
-      (q_norm == nullptr) != (k_norm == nullptr))
+      (rot > 0 && !freq) || (write && (!v_pages || !slots || page_size <= 0 || num_pages <= 0 || dv <= 0)) ||
+      (write && values_are_keys && dv != d) ||
+      x_stride < (nh + (write ? nkv : 0)) * d + (write && !values_are_keys ? nkv * dv : 0) || q_stride < nh * d ||
+      (q_norm == nullptr) != (k_norm == nullptr) || (v_first && v_first_stride < nkv * dv))
     return IA_ERR_BAD_ARG;
   // the rotation reads its pair from the source and writes both places: in place only where source and
   // destination are the same element for element (q_out == x with equal strides), which this launch allows
   const long items = (long)N * (nh + nkv);
-  if (code == IA_BF16 && (pairing == 1 || rot == 0) && d % 8 == 0 && d <= 512 && x_stride % 8 == 0 && q_stride % 8 == 0 &&
-      !((uintptr_t)x & 15) && !((uintptr_t)q_out & 15) && !((uintptr_t)k_pages & 15) && !((uintptr_t)q_norm & 15) &&
-      !((uintptr_t)k_norm & 15)) {
+  const ValueWay V{v_first, v_first_stride, v_lambda, v_scale};
+  if (code == IA_BF16 && (pairing == 1 || rot == 0) && d % 8 == 0 && d <= 512 && (!write || dv % 8 == 0) && x_stride % 8 == 0 &&
+      q_stride % 8 == 0 && v_first_stride % 8 == 0 && !((uintptr_t)x & 15) && !((uintptr_t)q_out & 15) &&
+      !((uintptr_t)k_pages & 15) && !((uintptr_t)q_norm & 15) && !((uintptr_t)k_norm & 15) && !((uintptr_t)v_first & 15)) {
     int GL = 1;
     while (8 * GL < d) GL <<= 1;
     const int per_block = 256 / GL;
-    qk_prepare_vec_kernel<<<(unsigned)((items + per_block - 1) / per_block), 256, 0, stream>>>(
+    const long qk_blocks = (items + per_block - 1) / per_block;
+    const long v_waves = write ? (long)((N + 15) / 16) * ((nkv * dv / 8 + 3) / 4) : 0;
+    const long blocks = qk_blocks + (v_waves + 3) / 4;
+    if (blocks > 0x7fffffffL) return IA_ERR_UNSUPPORTED;
+    qk_prepare_vec_kernel<<<(unsigned)blocks, 256, 0, stream>>>(
         (const bf16_t*)x, x_stride, (bf16_t*)q_out, q_stride, q_norm, k_norm, eps, positions, slots, freq, freq_f64, rot,
-        magnitude, (bf16_t*)k_pages, (bf16_t*)v_pages, N, nh, nkv, d, page_size, num_pages, values_are_keys, GL);
+        magnitude, (bf16_t*)k_pages, (bf16_t*)v_pages, N, nh, nkv, d, dv, page_size, num_pages, values_are_keys, GL,
+        (int)qk_blocks, V);
     IA_LAUNCH_CHECK();
     return IA_OK;
   }
@@ -498,13 +544,13 @@ extern "C" int ia_qk_prepare(const void* x, int code, int x_stride, void* q_out,
   if (code == IA_F32)
     qk_prepare_kernel<float><<<grid, 256, 0, stream>>>((const float*)x, x_stride, (float*)q_out, q_stride, q_norm, k_norm,
                                                       eps, positions, slots, freq, freq_f64, rot, pairing, magnitude,
-                                                      (float*)k_pages, (float*)v_pages, N, nh, nkv, d, page_size,
-                                                      num_pages, values_are_keys);
+                                                      (float*)k_pages, (float*)v_pages, N, nh, nkv, d, dv, page_size,
+                                                      num_pages, values_are_keys, V);
   else if (code == IA_BF16)
     qk_prepare_kernel<bf16_t><<<grid, 256, 0, stream>>>((const bf16_t*)x, x_stride, (bf16_t*)q_out, q_stride, q_norm,
                                                        k_norm, eps, positions, slots, freq, freq_f64, rot, pairing,
-                                                       magnitude, (bf16_t*)k_pages, (bf16_t*)v_pages, N, nh, nkv, d,
-                                                       page_size, num_pages, values_are_keys);
+                                                       magnitude, (bf16_t*)k_pages, (bf16_t*)v_pages, N, nh, nkv, d, dv,
+                                                       page_size, num_pages, values_are_keys, V);
   else
     return IA_ERR_BAD_ARG;
   IA_LAUNCH_CHECK();

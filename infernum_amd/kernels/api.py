@@ -332,11 +332,13 @@ def moe_grouped_rows(N: int, E: int, top: int, W: int, ff: int, dtype: torch.dty
 
 
 def moe_experts(x: torch.Tensor, ids: torch.Tensor, weights: torch.Tensor, w_gate_up: torch.Tensor,
-                w_down: torch.Tensor, limit: float, alpha: float) -> SplitSum:
+                w_down: torch.Tensor, limit: float, alpha: float, shift: float = 1.0, total: int = 0,
+                parts: Optional[torch.Tensor] = None) -> SplitSum:
     """The chosen experts of every token: w_gate_up [E, 2 ff, W] with the gate's and up's rows alternating,
-    w_down [E, W, ff].  y = g sigmoid(alpha g) (u + 1) with g = min(gate, limit), u = clamp(up, -limit, limit).
-    Returns fp32 parts [top, N, W], each already times its routing weight."""
-    _dev(x, ids, weights, w_gate_up, w_down)
+    w_down [E, W, ff].  y = g sigmoid(alpha g) (u + shift) with g = min(gate, limit), u = clamp(up, -limit, limit).
+    Fills parts[:top] of fp32 ``parts`` [>= top, N, W], each already times its routing weight, and returns them as a sum.
+    ``total`` > E: ids go up to it, and those from E on are experts without tensors, whose pairs are left alone."""
+    _dev(x, ids, weights, w_gate_up, w_down, parts)
     N, W = x.shape
     E, two_ff, _ = w_gate_up.shape
     ff = two_ff // 2
@@ -345,27 +347,57 @@ def moe_experts(x: torch.Tensor, ids: torch.Tensor, weights: torch.Tensor, w_gat
     _need(tuple(w_gate_up.shape) == (E, 2 * ff, W) and tuple(w_down.shape) == (E, W, ff), "moe: weights' shapes")
     _need(ids.dtype == torch.int32 and tuple(ids.shape) == (N, top) and weights.dtype == torch.float32
           and tuple(weights.shape) == (N, top), "moe: ids int32 and weights fp32 [N, top]")
-    P = N * top
-    offsets = torch.empty(E + 1, dtype=torch.int32, device=x.device)
+    P, total = N * top, max(int(total), E)
+    offsets = torch.empty(total + 1, dtype=torch.int32, device=x.device)
     perm = torch.empty(max(P, 1), dtype=torch.int32, device=x.device)
     y = torch.empty((max(P, 1), ff), dtype=x.dtype, device=x.device)
-    parts = torch.empty((top, N, W), dtype=torch.float32, device=x.device)
+    if parts is None:
+        parts = torch.empty((top, N, W), dtype=torch.float32, device=x.device)
+    _need(parts.dtype == torch.float32 and parts.dim() == 3 and parts.shape[0] >= top and tuple(parts.shape[1:]) == (N, W),
+          "moe: parts fp32 [>= top, N, W]")
     code = DTYPE_CODE[x.dtype]
-    _ok(_core().ia_moe_sort(_p(ids), _p(offsets), _p(perm), P, E, _stream()), "moe_sort")
+    _ok(_core().ia_moe_sort(_p(ids), _p(offsets), _p(perm), P, total, _stream()), "moe_sort")
     if moe_grouped_rows(N, E, top, W, ff, x.dtype):
         # many rows an expert: the tokens' rows in the order of the sort, the LDS-tiled product expert by expert
         xs = torch.empty((P, W), dtype=x.dtype, device=x.device)
         gu = torch.empty((P, 2 * ff), dtype=x.dtype, device=x.device)
         _ok(_core().ia_moe_gather(_p(x), _p(perm), _p(xs), P, top, W, _stream()), "moe_gather")
         gemm_mfma_grouped(xs, w_gate_up, offsets, gu)
-        _ok(_core().ia_moe_glu(_p(gu), _p(y), P, ff, ctypes.c_float(limit), ctypes.c_float(alpha), _stream()), "moe_glu")
+        _ok(_core().ia_moe_glu(_p(gu), _p(y), P, ff, ctypes.c_float(limit), ctypes.c_float(alpha),
+                               ctypes.c_float(shift), _stream()), "moe_glu")
         gemm_mfma_grouped(y, w_down, offsets, xs)
-        _ok(_core().ia_moe_scatter(_p(xs), _p(perm), _p(weights), _p(parts), N, top, W, _stream()), "moe_scatter")
+        _ok(_core().ia_moe_scatter(_p(xs), _p(perm), _p(weights), _p(parts), _p(offsets[E:] if total > E else None), N, top,
+                                   W, _stream()), "moe_scatter")
         return SplitSum(parts)
     _ok(_core().ia_moe_gate_up(_p(x), _p(w_gate_up), _p(y), _p(offsets), _p(perm), code, P, E, top, W, ff,
-                               ctypes.c_float(limit), ctypes.c_float(alpha), _stream()), "moe_gate_up")
+                               ctypes.c_float(limit), ctypes.c_float(alpha), ctypes.c_float(shift), _stream()), "moe_gate_up")
     _ok(_core().ia_moe_down(_p(y), _p(w_down), _p(parts), _p(weights), _p(offsets), _p(perm), code, N, E, top, W, ff,
                             _stream()), "moe_down")
+    return SplitSum(parts)
+
+
+def moe_extras(x: torch.Tensor, ids: torch.Tensor, weights: torch.Tensor, parts: torch.Tensor, num_experts: int,
+               shared=None, gate: Optional[torch.Tensor] = None) -> SplitSum:
+    """What routed experts add beside their products: a pair whose id is ``num_experts`` or more goes to an expert whose
+    result is its input, parts[choice, token] = weight * x[token]; ``shared`` (a tensor [N, W] or a :class:`SplitSum`),
+    times sigmoid(gate[token]) when there is a ``gate`` (fp32 [N], any stride), becomes parts[top]."""
+    N, W = x.shape
+    top = ids.shape[1]
+    split = isinstance(shared, SplitSum)
+    sh = shared.parts if split else shared
+    _dev(x, ids, weights, parts, sh)
+    _need(parts.dtype == torch.float32 and parts.dim() == 3 and tuple(parts.shape[1:]) == (N, W)
+          and parts.shape[0] == top + (0 if sh is None else 1), "moe_extras: parts fp32 [top (+ 1 with shared), N, W]")
+    _need(ids.dtype == torch.int32 and tuple(ids.shape) == (N, top) and weights.dtype == torch.float32
+          and tuple(weights.shape) == (N, top), "moe_extras: ids int32 and weights fp32 [N, top]")
+    if sh is not None:
+        _need(tuple(sh.shape[-2:]) == (N, W) and sh.dtype in DTYPE_CODE, "moe_extras: shared of x's shape")
+    if gate is not None:
+        _need(gate.is_cuda and gate.dtype == torch.float32 and gate.dim() == 1 and gate.numel() == N, "moe_extras: gate fp32 [N]")
+    _ok(_core().ia_moe_extras(_p(x), DTYPE_CODE[x.dtype], _p(ids), _p(weights), _p(parts), _p(sh),
+                              DTYPE_CODE[sh.dtype] if sh is not None else 0, sh.shape[0] if split else 1, N, _p(gate),
+                              int(gate.stride(0)) if gate is not None else 0, N, int(num_experts), top, W, _stream()),
+        "moe_extras")
     return SplitSum(parts)
 
 
@@ -707,43 +739,57 @@ def gemm_skinny_rows(a: torch.Tensor, w: torch.Tensor, out: torch.Tensor, tiled:
 
 # ------------------------------------------------------------------------ attention
 def _check_paged(qkv, k_pages, v_pages, out, block_tables, nh, nkv, d, what):
-    _dev(qkv, k_pages, v_pages, out, block_tables)
+    _dev(k_pages, v_pages, block_tables)
+    _need(qkv.is_cuda and out.is_cuda and qkv.stride(-1) == 1 and out.stride(-1) == 1,
+          f"{what}: rows of q and out on the GPU, their values side by side")
     _need(qkv.dtype == out.dtype == k_pages.dtype == v_pages.dtype and qkv.dtype in DTYPE_CODE,
           f"{what}: q, pages and out must share one dtype")
     _need(qkv.dim() == 2 and qkv.shape[1] >= nh * d, f"{what}: q rows must hold nh*d values")
-    _need(out.dim() == 2 and out.shape[1] == nh * d and out.shape[0] == qkv.shape[0],
-          f"{what}: out must be [N, nh*d]")
-    _need(k_pages.dim() == 4 and k_pages.shape[1] == nkv and k_pages.shape[3] == d
-          and tuple(v_pages.shape) == (k_pages.shape[0], nkv, d, k_pages.shape[2]),
-          f"{what}: key pages must be [num_pages, nkv, page_size, d], value pages [num_pages, nkv, d, page_size]")
+    _need(k_pages.dim() == 4 and k_pages.shape[1] == nkv and k_pages.shape[3] == d and v_pages.dim() == 4
+          and tuple(v_pages.shape) == (k_pages.shape[0], nkv, v_pages.shape[2], k_pages.shape[2]),
+          f"{what}: key pages must be [num_pages, nkv, page_size, d], value pages [num_pages, nkv, dv, page_size]")
+    dv = v_pages.shape[2]
+    _need(out.dim() == 2 and out.shape[1] == nh * dv and out.shape[0] == qkv.shape[0],
+          f"{what}: out must be [N, nh*dv]")
     _need(block_tables.dtype == torch.int32 and block_tables.dim() == 2, f"{what}: block_tables int32 [B, MB]")
     _need(nh % nkv == 0, f"{what}: nh must be a multiple of nkv")
+    return dv
+
+
+def _rows_of(t: torch.Tensor) -> int:
+    """Values from a row to the next: a tensor of whole rows, or a range of columns of wider rows."""
+    _need(t.dim() == 2 and t.stride(1) == 1, "rows must lie one after the other, their values side by side")
+    return int(t.stride(0)) if t.shape[0] > 1 else max(int(t.stride(0)), int(t.shape[1]))
 
 
 def attention_generic(qkv: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.Tensor, out: torch.Tensor,
                       token_seq: torch.Tensor, positions: torch.Tensor, block_tables: torch.Tensor, nh: int,
-                      nkv: int, d: int, scale: float, window: int = 0, sinks: Optional[torch.Tensor] = None) -> None:
+                      nkv: int, d: int, scale: float, window: int = 0, sinks: Optional[torch.Tensor] = None,
+                      keep: int = 0, softcap: float = 0.0) -> None:
     """Causal paged attention, one wave per (token, head), fp32 arithmetic.  ``sinks`` fp32 [nh]: exp(sinks[h]) is
-    added to the softmax's denominator of head h.
+    added to the softmax's denominator of head h.  ``keep``: under a window the request's first ``keep`` keys stay
+    visible.  ``softcap`` c > 0: a scaled score s becomes c tanh(s / c).  The value heads' size is that of the pages.
 
     qkv [N, >= nh*d]: the q heads of token n are the first nh*d values of row n.
     token_seq[n] is the row of block_tables of token n; positions[n] its position.
     """
-    _check_paged(qkv, k_pages, v_pages, out, block_tables, nh, nkv, d, "attention")
+    dv = _check_paged(qkv, k_pages, v_pages, out, block_tables, nh, nkv, d, "attention")
     N = out.shape[0]
     _i32(token_seq, N, "attention token_seq")
     _i32(positions, N, "attention positions")
-    _need(0 < d <= GENERIC_MAX_HEAD_DIM, f"attention: head size must be at most {GENERIC_MAX_HEAD_DIM}")
+    _need(0 < max(d, dv) <= GENERIC_MAX_HEAD_DIM, f"attention: head size must be at most {GENERIC_MAX_HEAD_DIM}")
     _f32(sinks, nh, "attention sinks")
-    _ok(_core().ia_attention_generic(_p(qkv), qkv.shape[1], _p(k_pages), _p(v_pages), _p(out), nh * d,
+    _ok(_core().ia_attention_generic(_p(qkv), _rows_of(qkv), _p(k_pages), _p(v_pages), _p(out), _rows_of(out),
                                      DTYPE_CODE[out.dtype], _p(token_seq), _p(positions), _p(block_tables),
-                                     block_tables.shape[1], N, nh, nkv, d, k_pages.shape[2], k_pages.shape[0],
-                                     ctypes.c_float(scale), int(window), _p(sinks), _stream()), "attention_generic")
+                                     block_tables.shape[1], N, nh, nkv, d, dv, k_pages.shape[2], k_pages.shape[0],
+                                     ctypes.c_float(scale), int(window), _p(sinks), int(keep), ctypes.c_float(softcap),
+                                     _stream()), "attention_generic")
 
 
-def _attn(d: int) -> ctypes.CDLL:
-    lib = load_library(f"attn_d{d}")
-    return lib
+def _attn(d: int, dv: Optional[int] = None, ext: bool = False) -> ctypes.CDLL:
+    """The matrix-core attention library for key heads of d and value heads of dv values; ``ext``: the one that takes
+    kept first keys and a softcap."""
+    return load_library(_build.attention_library(d, dv or d, ext))
 
 
 _compute_units: Dict[int, int] = {}
@@ -789,12 +835,13 @@ def decode_splits(batch: int, nh: int, nkv: int, max_len: int, device: Optional[
 def attention_decode(qkv: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.Tensor, out: torch.Tensor,
                      positions: torch.Tensor, block_tables: torch.Tensor, nh: int, nkv: int, d: int, scale: float,
                      window: int, max_len: int, num_splits: Optional[int] = None,
-                     sinks: Optional[torch.Tensor] = None) -> None:
+                     sinks: Optional[torch.Tensor] = None, keep: int = 0, softcap: float = 0.0) -> None:
     """bf16 attention of B single tokens (row b of qkv: token b at positions[b]) over their pages, on MFMA.
 
-    ``max_len`` bounds the positions (host side), and sets how many parts the keys are split into.
+    ``max_len`` bounds the positions (host side), and sets how many parts the keys are split into.  ``keep`` and
+    ``softcap``: see :func:`attention_generic`.
     """
-    _check_paged(qkv, k_pages, v_pages, out, block_tables, nh, nkv, d, "attention_decode")
+    dv = _check_paged(qkv, k_pages, v_pages, out, block_tables, nh, nkv, d, "attention_decode")
     B = out.shape[0]
     _need(qkv.dtype == torch.bfloat16, "attention_decode: bf16 only")
     _i32(positions, B, "attention_decode positions")
@@ -802,15 +849,15 @@ def attention_decode(qkv: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.Te
     ps = k_pages.shape[2]
     _need(ps % 4 == 0, f"attention_decode: page size {ps} is not a multiple of 4")
     _need(block_tables.shape[1] * ps >= max_len, "attention_decode: block_tables are narrower than max_len")
-    splits = num_splits or decode_splits(B, nh, nkv, max_len, out.device, d)
+    splits = num_splits or decode_splits(B, nh, nkv, max_len, out.device, max(d, dv))
     part_o = part_ml = None
     if splits > 1:
-        part_o = torch.empty(B * nh * splits * d, dtype=torch.float32, device=out.device)
+        part_o = torch.empty(B * nh * splits * dv, dtype=torch.float32, device=out.device)
         part_ml = torch.empty(B * nh * splits * 2, dtype=torch.float32, device=out.device)
-    _ok(_attn(d).ia_attn_decode(_p(qkv), qkv.shape[1], _p(k_pages), _p(v_pages), _p(out), nh * d, _p(part_o),
-                                _p(part_ml), _p(positions), _p(block_tables), block_tables.shape[1], B, nh, nkv, ps,
-                                k_pages.shape[0], ctypes.c_float(scale), int(window), splits, _p(sinks), _stream()),
-        "attention_decode")
+    _ok(_attn(d, dv, keep > 0 or softcap > 0).ia_attn_decode(
+        _p(qkv), _rows_of(qkv), _p(k_pages), _p(v_pages), _p(out), _rows_of(out), _p(part_o), _p(part_ml),
+        _p(positions), _p(block_tables), block_tables.shape[1], B, nh, nkv, ps, k_pages.shape[0], ctypes.c_float(scale),
+        int(window), splits, _p(sinks), int(keep), ctypes.c_float(softcap), _stream()), "attention_decode")
 
 
 def attention_decode_rotating(qkv, positions: torch.Tensor, inv_freq: Optional[torch.Tensor], rot: int,
@@ -863,7 +910,7 @@ def attention_decode_rotating(qkv, positions: torch.Tensor, inv_freq: Optional[t
         1 if (inv_freq is not None and inv_freq.dtype == torch.float64) else 0, rot if inv_freq is not None else 0,
         _p(k_pages), _p(v_pages), _p(out), nh * d, _p(part_o), _p(part_ml), _p(positions), _p(block_tables),
         block_tables.shape[1], B, nh, nkv, ps, k_pages.shape[0], ctypes.c_float(scale), int(window), splits, _p(sinks),
-        _stream()), "attention_decode_rotating")
+        0, ctypes.c_float(0.0), _stream()), "attention_decode_rotating")
 
 
 PREFILL_TILE_ROWS = 64      # query rows of a workgroup's tile in attention_prefill
@@ -874,7 +921,7 @@ def attention_prefill(qkv: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.T
                       seq_starts: torch.Tensor, seq_ctx: torch.Tensor, block_tables: torch.Tensor,
                       tiles: torch.Tensor, num_tiles: int, nh: int, nkv: int, d: int, scale: float,
                       window: int, heads_per_workgroup: int = 0, paired: bool = False,
-                      sinks: Optional[torch.Tensor] = None) -> None:
+                      sinks: Optional[torch.Tensor] = None, keep: int = 0, softcap: float = 0.0) -> None:
     """bf16 causal attention of portions of prompts over their pages, on MFMA.
 
     Request s brings rows seq_starts[s] .. seq_starts[s+1]-1 of qkv and had seq_ctx[s] tokens cached
@@ -882,9 +929,10 @@ def attention_prefill(qkv: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.T
     0 for the kernel's own choice, or 1, 2, 4; ``paired``: a workgroup takes half a block of rows from each end of
     its request's new tokens, so that all workgroups of a request have the same work under the causal mask (every
     block of every request must be listed then; without effect under a window).  A value of :func:`prefill_launch_shape` may stand in
-    ``heads_per_workgroup`` for both.  The result has the same bits whatever the shape.
+    ``heads_per_workgroup`` for both.  The result has the same bits whatever the shape.  ``keep`` and ``softcap``: see
+    :func:`attention_generic`.
     """
-    _check_paged(qkv, k_pages, v_pages, out, block_tables, nh, nkv, d, "attention_prefill")
+    dv = _check_paged(qkv, k_pages, v_pages, out, block_tables, nh, nkv, d, "attention_prefill")
     _need(qkv.dtype == torch.bfloat16, "attention_prefill: bf16 only")
     B = block_tables.shape[0]
     _i32(seq_starts, B + 1, "attention_prefill seq_starts")
@@ -893,11 +941,11 @@ def attention_prefill(qkv: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.T
           "attention_prefill: tiles int32 [num_tiles, 2]")
     ps = k_pages.shape[2]
     _need(ps % 4 == 0, f"attention_prefill: page size {ps} is not a multiple of 4")
-    _ok(_attn(d).ia_attn_prefill(_p(qkv), qkv.shape[1], _p(k_pages), _p(v_pages), _p(out), nh * d, _p(seq_starts),
-                                 _p(seq_ctx), _p(block_tables), block_tables.shape[1], _p(tiles), num_tiles, nh, nkv,
-                                 ps, k_pages.shape[0], ctypes.c_float(scale), int(window),
-                                 int(heads_per_workgroup) | (PREFILL_PAIRED if paired else 0), _p(sinks), _stream()),
-        "attention_prefill")
+    _ok(_attn(d, dv, keep > 0 or softcap > 0).ia_attn_prefill(
+        _p(qkv), _rows_of(qkv), _p(k_pages), _p(v_pages), _p(out), _rows_of(out), _p(seq_starts), _p(seq_ctx),
+        _p(block_tables), block_tables.shape[1], _p(tiles), num_tiles, nh, nkv, ps, k_pages.shape[0],
+        ctypes.c_float(scale), int(window), int(heads_per_workgroup) | (PREFILL_PAIRED if paired else 0), _p(sinks),
+        int(keep), ctypes.c_float(softcap), _stream()), "attention_prefill")
 
 
 def prefill_launch_shape(nh: int, nkv: int, d: int, q_lens: Sequence[int], ctx_lens: Sequence[int],
@@ -1031,15 +1079,22 @@ def qk_prepare(x: torch.Tensor, q_out: torch.Tensor, nh: int, nkv: int, d: int, 
                q_norm: Optional[torch.Tensor] = None, k_norm: Optional[torch.Tensor] = None, eps: float = 0.0,
                freq: Optional[torch.Tensor] = None, rot: int = 0, pairing: str = "half", magnitude: float = 1.0,
                slots: Optional[torch.Tensor] = None, k_pages: Optional[torch.Tensor] = None,
-               v_pages: Optional[torch.Tensor] = None, values_are_keys: bool = False) -> torch.Tensor:
-    """Query and key heads between projection and attention.  ``x`` [N, (nh + nkv (+ nkv)) d]: nh query heads,
+               v_pages: Optional[torch.Tensor] = None, values_are_keys: bool = False, v_scale: float = 1.0,
+               v_first: Optional[torch.Tensor] = None, v_lambda: float = 0.0) -> torch.Tensor:
+    """Query and key heads between projection and attention.  ``x`` [N, (nh + nkv) d (+ nkv dv)]: nh query heads,
     nkv key heads, and nkv value heads unless ``values_are_keys`` (then a key head as it comes in is its value).
+    A value v goes to its page as ``v_scale`` ((1 - v_lambda) v + v_lambda v_first), ``v_first`` [N, nkv dv] (rows
+    may be columns of wider rows) the same tokens' values of another layer; without it as ``v_scale`` v.
     Per head: RMS norm over d with one weight for all heads (when given), rotation of the first ``rot`` values
     (``pairing`` "half": value i with i + rot/2; "neighbours": 2i with 2i+1) with sine and cosine times
     ``magnitude``.  Queries go to ``q_out`` [N, nh d], keys and values to their pages at ``slots``."""
     N = x.shape[0]
     write = k_pages is not None
-    _rows(x, (nh + (nkv if values_are_keys else 2 * nkv) * int(write)) * d, "qk_prepare input")
+    dv = v_pages.shape[2] if write else d
+    _rows(x, (nh + nkv * int(write)) * d + (nkv * dv if write and not values_are_keys else 0), "qk_prepare input")
+    if v_first is not None:
+        _rows(v_first, nkv * dv, "qk_prepare v_first")
+        _need(v_first.dtype == x.dtype and v_first.shape[0] == N, "qk_prepare: v_first of the input's dtype, a row a token")
     _rows(q_out, nh * d, "qk_prepare q_out")
     _need(q_out.dtype == x.dtype and q_out.shape[0] == N, "qk_prepare: q_out [N, nh d] of the input's dtype")
     _f32(q_norm, d, "qk_prepare q_norm")
@@ -1052,15 +1107,17 @@ def qk_prepare(x: torch.Tensor, q_out: torch.Tensor, nh: int, nkv: int, d: int, 
     if write:
         num_pages, ps = k_pages.shape[0], k_pages.shape[2]
         _need(slots is not None and v_pages is not None and k_pages.dtype == x.dtype and v_pages.dtype == x.dtype
-              and tuple(k_pages.shape) == (num_pages, nkv, ps, d) and tuple(v_pages.shape) == (num_pages, nkv, d, ps)
-              and k_pages.is_contiguous() and v_pages.is_contiguous(),
-              "qk_prepare: key pages [num_pages, nkv, page_size, d], value pages [num_pages, nkv, d, page_size]")
+              and tuple(k_pages.shape) == (num_pages, nkv, ps, d) and tuple(v_pages.shape) == (num_pages, nkv, dv, ps)
+              and (dv == d or not values_are_keys) and k_pages.is_contiguous() and v_pages.is_contiguous(),
+              "qk_prepare: key pages [num_pages, nkv, page_size, d], value pages [num_pages, nkv, dv, page_size]")
         _i32(slots, N, "qk_prepare slots")
     _ok(_core().ia_qk_prepare(_p(x), DTYPE_CODE[x.dtype], x.stride(0), _p(q_out), q_out.stride(0), _p(q_norm), _p(k_norm),
                               ctypes.c_float(eps), _p(positions), _p(slots), _p(freq if rot else None),
                               1 if (rot and freq.dtype == torch.float64) else 0, int(rot), PAIRINGS[pairing],
-                              ctypes.c_float(magnitude), _p(k_pages), _p(v_pages), N, nh, nkv if write else 0, d, ps,
-                              num_pages, int(bool(values_are_keys)), _stream()), "qk_prepare")
+                              ctypes.c_float(magnitude), _p(k_pages), _p(v_pages), N, nh, nkv if write else 0, d, dv,
+                              ps, num_pages, int(bool(values_are_keys)), ctypes.c_float(v_scale), _p(v_first),
+                              v_first.stride(0) if v_first is not None else 0, ctypes.c_float(v_lambda), _stream()),
+        "qk_prepare")
     return q_out
 
 
@@ -1253,12 +1310,17 @@ def gated_norm_add(h: torch.Tensor, delta, gate, gate_bias: Optional[torch.Tenso
     return h
 
 
-def router_softmax_topk(logits: torch.Tensor, correction: Optional[torch.Tensor], top: int):
+def router_softmax_topk(logits: torch.Tensor, correction: Optional[torch.Tensor], top: int, groups: int = 1, keep: int = 1,
+                        renorm: bool = True, experts: Optional[int] = None):
     """-> (ids int32 [N, top], weights fp32 [N, top]): s = softmax(logits) over all experts; the ``top`` largest of
-    s + correction are chosen (the lowest index among equals); the weights are the chosen s over their sum."""
+    s + correction are chosen (the lowest index among equals); the weights are the chosen s, with ``renorm`` over their
+    sum.  ``groups`` equal groups of neighbouring experts, of which only the ``keep`` with the largest s + correction
+    among their experts can be chosen from.  ``experts``: rows of ``logits`` hold more than the experts' (first)."""
     _dev(logits, correction)
     _need(logits.dtype == torch.float32 and logits.dim() == 2, "router_softmax_topk: fp32 logits [N, E]")
-    N, E = logits.shape
+    N, E = logits.shape[0], int(experts or logits.shape[1])
+    _need(E <= logits.shape[1] and groups >= 1 and E % groups == 0 and 1 <= keep <= groups and top <= keep * (E // groups),
+          "router_softmax_topk: equal groups, and as many experts in the kept ones as a token takes")
     _need(0 < top <= E, f"router_softmax_topk: top must be 1 .. {E}")
     _need(correction is None or (correction.dtype in DTYPE_CODE and correction.numel() == E),
           f"router_softmax_topk: {E} corrections")
@@ -1266,7 +1328,8 @@ def router_softmax_topk(logits: torch.Tensor, correction: Optional[torch.Tensor]
     weights = torch.empty((N, top), dtype=torch.float32, device=logits.device)
     _ok(_core().ia_router_softmax_topk(_p(logits), _p(correction),
                                        DTYPE_CODE[correction.dtype] if correction is not None else 0, _p(ids),
-                                       _p(weights), N, E, top, _stream()), "router_softmax_topk")
+                                       _p(weights), N, E, top, int(logits.shape[1]), int(groups), int(keep), int(bool(renorm)),
+                                       _stream()), "router_softmax_topk")
     return ids, weights
 
 
@@ -1299,7 +1362,7 @@ def moe_plain_experts(x: torch.Tensor, ids: torch.Tensor, weights: torch.Tensor,
         gemm_mfma_grouped(xs, w_up, offsets, y)
         activation(y, act)
         gemm_mfma_grouped(y, w_down, offsets, xs)
-        _ok(_core().ia_moe_scatter(_p(xs), _p(perm), _p(weights), _p(parts), N, top, W, _stream()), "moe_scatter")
+        _ok(_core().ia_moe_scatter(_p(xs), _p(perm), _p(weights), _p(parts), None, N, top, W, _stream()), "moe_scatter")
         return parts
     _ok(_core().ia_moe_up(_p(x), _p(w_up), _p(y), _p(offsets), _p(perm), code, P, E, top, W, ff, ACTIVATIONS[act],
                           _stream()), "moe_up")
@@ -1376,21 +1439,119 @@ def gla_chunked(proj: torch.Tensor, q_col: int, k_col: int, v_col: int, z: torch
 
 
 def head_norm_gate(o: torch.Tensor, gate: Optional[torch.Tensor], gate_col: int, w: torch.Tensor, eps: float, nh: int,
-                   vdim: int, out: torch.Tensor) -> torch.Tensor:
+                   vdim: int, out: torch.Tensor, per_head: bool = False, plain_sigmoid: bool = False) -> torch.Tensor:
     """out = o / sqrt(mean(o^2) + eps) * w * silu(gate) with the mean over each head's vdim values: o fp32 [N, nh vdim],
-    w fp32 [vdim] shared by the heads, gate rows holding nh vdim values from gate_col on."""
+    w fp32 [vdim] shared by the heads (``per_head``: [nh vdim], each head its own), gate rows holding nh vdim values
+    from gate_col on; ``plain_sigmoid``: sigmoid(gate) in place of silu.  ``out`` may be columns of wider rows."""
     N = o.shape[0]
     _need(o.is_cuda and o.dtype == torch.float32 and o.is_contiguous() and tuple(o.shape) == (N, nh * vdim),
           "head_norm_gate: o [N, nh vdim] fp32")
-    _f32(w, vdim, "head_norm_gate weight")
-    _need(out.is_cuda and out.is_contiguous() and tuple(out.shape) == (N, nh * vdim) and out.dtype in DTYPE_CODE,
+    _f32(w, nh * vdim if per_head else vdim, "head_norm_gate weight")
+    _need(out.is_cuda and tuple(out.shape) == (N, nh * vdim) and out.dtype in DTYPE_CODE,
           "head_norm_gate: out [N, nh vdim]")
     if gate is not None:           # without a gate: the norm and the weight alone
         _rows(gate, gate_col + nh * vdim, "head_norm_gate gate")
         _need(out.dtype == gate.dtype and gate.shape[0] == N, "head_norm_gate: out of the gate's dtype")
     _ok(_core().ia_head_norm_gate(_p(o), _p(gate), DTYPE_CODE[out.dtype], int(gate.stride(0)) if gate is not None else 0,
-                                  gate_col, _p(w), _p(out), N, nh, vdim, ctypes.c_float(eps), _stream()), "head_norm_gate")
+                                  gate_col, _p(w), _p(out), _rows_of(out), N, nh, vdim, ctypes.c_float(eps), int(bool(per_head)),
+                                  int(bool(plain_sigmoid)), _stream()), "head_norm_gate")
     return out
+
+
+# ------------------------------------------------------------ the generalized delta rule
+def delta_state_floats(nh: int, dim: int) -> int:
+    """fp32 values a request's slot holds for one run of a layer with nh heads."""
+    return nh * dim * dim
+
+
+DELTA_MAX_DIM = 256
+
+
+def tanh_rows(src: torch.Tensor, out: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """tanh of ``src`` [N, C] (columns of wider rows) as a tensor of its own."""
+    _rows(src, src.shape[1], "tanh_rows")
+    N, C = src.shape
+    if out is None:
+        out = torch.empty((N, C), dtype=src.dtype, device=src.device)
+    _need(out.dtype == src.dtype and out.is_contiguous() and tuple(out.shape) == (N, C), "tanh_rows: out like src")
+    _ok(_core().ia_delta_tanh_rows(_p(src), _rows_of(src), _p(out), DTYPE_CODE[src.dtype], N, C, _stream()), "tanh_rows")
+    return out
+
+
+def delta_prepare(proj: torch.Tensor, k_col: int, a_col: int, z: torch.Tensor, w0: torch.Tensor, a_bias: torch.Tensor,
+                  nh: int, dim: int, decay_scale: float, eps: float):
+    """What enters the delta rule beside the projections, in fp32: ``z`` [N, nh dim] becomes the decays
+    exp(-decay_scale sigmoid(z + w0)) in place; returns (a [N, nh dim], inv [N, nh]): a = sigmoid of the columns of
+    ``proj`` from a_col on plus a_bias, and 1 / sqrt(sum k^2 + eps) of every head's key (columns from k_col on)."""
+    N, n = proj.shape[0], nh * dim
+    _rows(proj, max(k_col, a_col) + n, "delta_prepare")
+    _f32(z, N * n, "delta_prepare z")
+    _f32(w0, n, "delta_prepare w0")
+    _f32(a_bias, n, "delta_prepare a_bias")
+    a = torch.empty((N, n), dtype=torch.float32, device=proj.device)
+    inv = torch.empty((N, nh), dtype=torch.float32, device=proj.device)
+    _ok(_core().ia_delta_prepare(_p(proj), DTYPE_CODE[proj.dtype], _rows_of(proj), k_col, a_col, _p(z), _p(w0), _p(a_bias),
+                                 _p(a), _p(inv), N, nh, dim, ctypes.c_float(decay_scale), ctypes.c_float(eps), _stream()),
+        "delta_prepare")
+    return a, inv
+
+
+def delta_scan(proj: torch.Tensor, r_col: int, k_col: int, v_col: int, w: torch.Tensor, a: torch.Tensor, inv: torch.Tensor,
+               state: torch.Tensor, out: torch.Tensor, seq_starts: torch.Tensor, state_slots: torch.Tensor, nh: int,
+               dim: int) -> torch.Tensor:
+    """S_t = diag(w_t) S - (a_t * u_t)(u_t^T S) + k_t v_t^T, o_t = S_t^T r_t with u = k inv, over the rows of every
+    request of the step: r, k, v from columns of ``proj``, w and a fp32 [N, nh dim], inv fp32 [N, nh], ``state``
+    [slots, >= nh dim dim] fp32 (moved on in place), ``out`` fp32 [N, nh dim]."""
+    N, n, B = proj.shape[0], nh * dim, state_slots.numel()
+    _rows(proj, max(r_col, k_col, v_col) + n, "delta_scan")
+    for t, size, what in ((w, N * n, "w"), (a, N * n, "a"), (inv, N * nh, "inv"), (out, out.shape[0] * n, "out")):
+        _f32(t, size, f"delta_scan {what}")
+    stride = _state_rows(state, delta_state_floats(nh, dim), "delta_scan")
+    _i32(seq_starts, B + 1, "delta_scan seq_starts")
+    _i32(state_slots, B, "delta_scan state_slots")
+    _ok(_core().ia_delta_scan(_p(proj), DTYPE_CODE[proj.dtype], _rows_of(proj), r_col, k_col, v_col, _p(w), _p(a), _p(inv),
+                              _p(state), ctypes.c_long(stride), _p(out), _p(seq_starts), _p(state_slots), B, nh, dim,
+                              _stream()), "delta_scan")
+    return out
+
+
+# ------------------------------------------------------------ several residual streams
+HYPER_MAX_STREAMS = 32
+
+
+def hyper_step(src: torch.Tensor, streams: int, new: Optional[torch.Tensor], delta, mix: Optional[torch.Tensor],
+               out_weights: Optional[torch.Tensor], in_weights: Optional[torch.Tensor], norm_weight: Optional[torch.Tensor],
+               eps: float, result: torch.Tensor) -> torch.Tensor:
+    """One pass over ``streams`` residual streams between two sublayers (fp32).  ``src``: [N, S, H], or [N, H] when all
+    streams are still equal.  With ``delta`` (a tensor [N, H], or a :class:`SplitSum`) the streams become
+    X_t = sum_s mix[s, t] X_s + out_weights[t] delta.  Then u = sum_s in_weights[s] X_s: normed (weight
+    ``norm_weight``) into ``result`` [N, H] in the activations' dtype, with the new streams in ``new`` [N, S, H] (may be
+    ``src``); or, without ``norm_weight``, unrounded into ``result`` fp32 [N, H], the streams left as they were
+    (in_weights None: their plain sum)."""
+    split = isinstance(delta, SplitSum)
+    d = delta.parts if split else delta
+    S, N, H = int(streams), src.shape[0], src.shape[-1]
+    _dev(src, new, d, mix, out_weights, in_weights, norm_weight, result)
+    _need(src.dtype == torch.float32 and tuple(src.shape) in ((N, H), (N, S, H)), "hyper_step: src fp32 [N, H] or [N, S, H]")
+    _need(1 <= S <= HYPER_MAX_STREAMS, f"hyper_step: 1 .. {HYPER_MAX_STREAMS} streams")
+    _f32(mix, S * S, "hyper_step mix")
+    _f32(out_weights, S, "hyper_step out_weights")
+    _f32(in_weights, S, "hyper_step in_weights")
+    normed = norm_weight is not None
+    _need(tuple(result.shape) == (N, H) and (result.dtype in DTYPE_CODE if normed else result.dtype == torch.float32),
+          "hyper_step: result [N, H]")
+    if d is not None:
+        _need(mix is not None and out_weights is not None, "hyper_step: a delta needs mix and out_weights")
+        _need(tuple(d.shape[-2:]) == (N, H) and d.dtype in DTYPE_CODE, "hyper_step: delta of the streams' shape")
+        if normed:
+            _need(new is not None and new.dtype == torch.float32 and tuple(new.shape) == (N, S, H), "hyper_step: new [N, S, H]")
+    act = result.dtype if normed else (torch.bfloat16 if d is not None and d.dtype == torch.bfloat16 else torch.float32)
+    _ok(_core().ia_hyper_step(
+        _p(src), S if src.dim() == 3 else 0, _p(new), _p(d), DTYPE_CODE[d.dtype] if d is not None else 0,
+        d.shape[0] if split else 1, N, _p(mix), _p(out_weights), _p(in_weights), _p(norm_weight),
+        DTYPE_CODE[norm_weight.dtype] if normed else 0, None if normed else _p(result), _p(result) if normed else None,
+        DTYPE_CODE[act], N, S, H, ctypes.c_float(eps), _stream()), "hyper_step")
+    return result
 
 
 # ------------------------------------------------------------ the recurrence with given decays (k = 1 - f)
@@ -1832,9 +1993,10 @@ def sample(logits: torch.Tensor, work: torch.Tensor, temperature: torch.Tensor, 
 
 
 # ---------------------------------------------------- which head sizes the MFMA kernels take
-def attention_mfma_available(d: int) -> bool:
-    """Whether the MFMA attention kernels take head size d (their library is built at its first use)."""
-    return d in _build.SUPPORTED_HEAD_DIMS
+def attention_mfma_available(d: int, dv: Optional[int] = None) -> bool:
+    """Whether the MFMA attention kernels take key heads of d and value heads of dv values (their library is built at
+    its first use)."""
+    return d in _build.SUPPORTED_HEAD_DIMS and (dv is None or dv in _build.SUPPORTED_HEAD_DIMS)
 
 
 # ------------------------------------------------- time per kernel, by the device's clock

@@ -21,7 +21,7 @@ from typing import Any, Dict, Mapping, Optional
 import torch
 
 from ..kernels import api as K
-from .base import (CacheSpec, CacheView, Mixer, PartSpec, Runtime, StepContext, WeightSpec, make_part,
+from .base import (CacheSpec, CacheView, Mixer, PageTensor, PartSpec, Runtime, StepContext, WeightSpec, make_part,
                    register_part)
 from .linear import emit_linear, linear, prepare_weights
 
@@ -50,18 +50,29 @@ class Attention(Mixer):
     def __init__(self, rt: Runtime, hidden_size: int, num_heads: int, num_kv_heads: int, head_dim: int,
                  position: Optional[Mapping[str, Any]] = None, window: Optional[int] = None,
                  scale: Optional[float] = None, kernels: str = "auto", init_std: float = 0.02,
-                 qk_transform: Optional[Mapping[str, Any]] = None, chunk: Optional[int] = None):
+                 qk_transform: Optional[Mapping[str, Any]] = None, chunk: Optional[int] = None,
+                 value_dim: Optional[int] = None, keep_first: int = 0, softcap: Optional[float] = None):
+        """``value_dim``: the size of a value head (default: the head size).  ``keep_first``: under a window, so many
+        first positions of a request that every later query goes on seeing.  ``softcap`` c: a scaled score s becomes
+        c tanh(s / c).  (This mixer's own projection has none of the three; mixers built on it do.)"""
         super().__init__(rt)
         if num_heads % num_kv_heads:
             raise ValueError(f"num_heads {num_heads} is not a multiple of num_kv_heads {num_kv_heads}")
         if head_dim > K.GENERIC_MAX_HEAD_DIM:
             raise ValueError(f"head size {head_dim} is above {K.GENERIC_MAX_HEAD_DIM}, the largest the attention kernels take")
         self.hidden_size, self.nh, self.nkv, self.d = int(hidden_size), int(num_heads), int(num_kv_heads), int(head_dim)
+        self.vd = int(value_dim) if value_dim else self.d
+        if not 0 < self.vd <= K.GENERIC_MAX_HEAD_DIM:
+            raise ValueError(f"value size {self.vd}: at most {K.GENERIC_MAX_HEAD_DIM}, the largest the attention kernels take")
         self.window = int(window) if window else 0
         # chunks of so many positions, counted from the request's start: a query sees the keys of its own chunk
         self.chunk = int(chunk) if chunk else 0
         if self.window < 0 or self.chunk < 0 or (self.window and self.chunk):
             raise ValueError("attention takes a window or chunks, each positive, not both")
+        self.keep_first = int(keep_first) if self.window else 0
+        self.score_cap = float(softcap) if softcap else 0.0
+        if self.keep_first < 0 or self.score_cap < 0:
+            raise ValueError("attention: keep_first and softcap must not be negative")
         # what the kernels are told: 0 all keys, w > 0 a window of w keys, -c chunks of c positions
         self.mask = self.window if self.window else -self.chunk
         self.scale = float(scale) if scale is not None else 1.0 / math.sqrt(self.d)
@@ -87,13 +98,19 @@ class Attention(Mixer):
         self.sinks: Optional[torch.Tensor] = None
         self.rotate_in_attention = _decode_rotation == "attention"
         self.use_mfma = (kernels == "auto" and rt.dtype == torch.bfloat16 and rt.device.type == "cuda"
-                         and K.attention_mfma_available(self.d))
+                         and K.attention_mfma_available(self.d, self.vd))
 
     # ---- what it needs ---------------------------------------------------
     def cache_spec(self) -> CacheSpec:
         if self.chunk:                  # pages of chunks that every later query has left go back to the pool
             return CacheSpec("chunk", self.nkv, self.d, self.chunk)
-        return CacheSpec("window" if self.window else "full", self.nkv, self.d, self.window)
+        payload = () if self.vd == self.d else (PageTensor("k", (self.nkv, self.d), token_axis=1),
+                                                PageTensor("v", (self.nkv, self.vd), token_axis=2))
+        return CacheSpec("window" if self.window else "full", self.nkv, self.d, self.window, payload, self.keep_first)
+
+    def _lib(self):
+        """The library of the matrix-core kernels for this mixer's sizes and options."""
+        return K._attn(self.d, self.vd, self.keep_first > 0 or self.score_cap > 0)
 
     def step_needs(self) -> Dict[str, Any]:
         # the MFMA kernel for portions of prompts works on tiles of 64 query rows
@@ -101,6 +118,8 @@ class Attention(Mixer):
 
     def weights(self) -> Dict[str, WeightSpec]:
         nh, nkv, d, H = self.nh, self.nkv, self.d, self.hidden_size
+        if self.vd != d or self.keep_first or self.score_cap:
+            raise ValueError("this mixer's values have the head size, and it has no kept positions and no softcap")
         init = ("normal", self.init_std)
         own = {
             "q_proj.weight": WeightSpec((nh * d, H), init),
@@ -230,7 +249,7 @@ class Attention(Mixer):
             fused = Guard.between(program.NPT, 0, 0) & Guard.between(N, 1, ROTATE_IN_ATTENTION_UP_TO)
         separate = ~fused
         if mfma:
-            lib = K._attn(d)
+            lib = self._lib()
             records = T + 1024      # requests x parts of their keys: what fills the GPU, or the requests themselves
             part_o = program.buffer("attention.part_o", records * nh * d * 4)
             part_ml = program.buffer("attention.part_ml", records * nh * 2 * 4)
@@ -242,7 +261,7 @@ class Attention(Mixer):
                 program.op(lib, "ia_attn_decode_fused",
                            [src, code, parts, N, row, slots, inv_freq, f64, rot, k, v, out, nh * d, part_o, part_ml,
                             program.positions, bt, bt_cols, N, nh, nkv, ps, num_pages, scale, window, splits, self.sinks,
-                            STREAM],
+                            self.keep_first, self.score_cap, STREAM],
                            alt.when & fused)
             q, q_stride = src, row
             if alt.splits:                   # partial sums: the rotated queries get a tensor of their own
@@ -257,7 +276,7 @@ class Attention(Mixer):
     def _attend_scalars(self, program, g: int, ps: int, records: int):
         """The two numbers that the host works out for the attention kernels once a step: into how many parts the
         keys of single tokens are cut, and the launch shape of the kernel for portions of prompts."""
-        nh, nkv, d, window, dev = self.nh, self.nkv, self.d, self.mask, self.rt.device
+        nh, nkv, big, window, dev = self.nh, self.nkv, max(self.d, self.vd), self.mask, self.rt.device
 
         def parts_of_the_keys(ctx: StepContext) -> int:
             nd = ctx.num_decode
@@ -265,7 +284,7 @@ class Attention(Mixer):
                 return 1
             if ctx.block_tables[g].shape[1] * ps < ctx.max_total_len:
                 raise K.KernelError("attention: the block tables are narrower than the longest request")
-            n = K.decode_splits(nd, nh, nkv, self._span(ctx.max_total_len), dev, d)
+            n = K.decode_splits(nd, nh, nkv, self._span(ctx.max_total_len), dev, big)
             if nd * n > records:
                 raise K.KernelError("attention: the parts of the keys do not fit the program's arena")
             return n
@@ -274,46 +293,53 @@ class Attention(Mixer):
             nd = ctx.num_decode
             if ctx.num_seqs == nd:
                 return 0
-            return K.prefill_launch_shape(nh, nkv, d, ctx.q_lens[nd:], ctx.ctx_lens[nd:], window, dev)
-        return (program.scalar(("attention: parts of the keys", nh, nkv, g, ps), parts_of_the_keys),
-                program.scalar(("attention: launch shape", nh, nkv, d, window), launch_shape))
+            return K.prefill_launch_shape(nh, nkv, big, ctx.q_lens[nd:], ctx.ctx_lens[nd:], window, dev)
+        return (program.scalar(("attention: parts of the keys", nh, nkv, big, g, ps, self._span(1 << 60)), parts_of_the_keys),
+                program.scalar(("attention: launch shape", nh, nkv, big, window), launch_shape))
 
-    def emit_attend(self, program, view: CacheView, q, q_stride: int, when, out=None):
+    def emit_attend(self, program, view: CacheView, q, q_stride: int, when, out=None, out_stride: Optional[int] = None):
         """The launches of :meth:`attend` alone, for queries ``q`` (rows of ``q_stride`` values, the heads first) that
         are rotated already and whose keys and values are in their pages: the kernel for single tokens on the first
-        rows and the one for portions of prompts on the rest, or the plain kernel on all rows.  Returns the buffer
-        [N, nh d] of the attended rows."""
+        rows and the one for portions of prompts on the rest, or the plain kernel on all rows.  ``out``: where the
+        attended rows go, ``out_stride`` values from a row to the next (default: a buffer [N, nh dv]).  Returns it."""
         from ..engine.program import STREAM, Guard
-        nh, nkv, d, window, rt = self.nh, self.nkv, self.d, self.mask, self.rt
+        nh, nkv, d, dv, window, rt = self.nh, self.nkv, self.d, self.vd, self.mask, self.rt
         k, v, g = view.k_pages, view.v_pages, view.group
         ps, num_pages = int(k.shape[2]), int(k.shape[0])
         T, act, scale = program.T, program.act_code, float(self.scale)
         program.keep(k, v, self.sinks)
         bt, bt_cols = program.block_table(g), program.bt_cols(g)
         if out is None:
-            out = program.buffer("attention.out", T * nh * d * program.act_bytes)
+            out = program.buffer("attention.out", T * nh * dv * program.act_bytes)
+        out_stride = int(out_stride) if out_stride else nh * dv
         if not (self.use_mfma and ps % 4 == 0):
             program.op("core", "ia_attention_generic",
-                       [q, q_stride, k, v, out, nh * d, act, program.token_seq, program.positions, bt, bt_cols, program.N,
-                        nh, nkv, d, ps, num_pages, scale, window, self.sinks, STREAM], when)
+                       [q, q_stride, k, v, out, out_stride, act, program.token_seq, program.positions, bt, bt_cols,
+                        program.N, nh, nkv, d, dv, ps, num_pages, scale, window, self.sinks, self.keep_first, self.score_cap,
+                        STREAM], when)
             return out
-        lib = K._attn(d)
+        lib = self._lib()
         records = T + 1024
-        part_o = program.buffer("attention.part_o", records * nh * d * 4)
+        part_o = program.buffer("attention.part_o", records * nh * dv * 4)
         part_ml = program.buffer("attention.part_ml", records * nh * 2 * 4)
         splits, shape = self._attend_scalars(program, g, ps, records)
         tiles, num_tiles = program.row_tiles(K.PREFILL_TILE_ROWS)
         program.op(lib, "ia_attn_decode",
-                   [q, q_stride, k, v, out, nh * d, part_o, part_ml, program.positions, bt, bt_cols, program.ND, nh,
-                    nkv, ps, num_pages, scale, window, splits, self.sinks, STREAM], when & Guard.between(program.ND, 1))
+                   [q, q_stride, k, v, out, out_stride, part_o, part_ml, program.positions, bt, bt_cols, program.ND, nh,
+                    nkv, ps, num_pages, scale, window, splits, self.sinks, self.keep_first, self.score_cap, STREAM],
+                   when & Guard.between(program.ND, 1))
         program.op(lib, "ia_attn_prefill",
-                   [q, q_stride, k, v, out, nh * d, program.seq_starts, program.seq_ctx, bt, bt_cols, tiles, num_tiles,
-                    nh, nkv, ps, num_pages, scale, window, shape, self.sinks, STREAM], when & Guard.between(program.NP, 1))
+                   [q, q_stride, k, v, out, out_stride, program.seq_starts, program.seq_ctx, bt, bt_cols, tiles, num_tiles,
+                    nh, nkv, ps, num_pages, scale, window, shape, self.sinks, self.keep_first, self.score_cap, STREAM],
+                   when & Guard.between(program.NP, 1))
         return out
 
     def _span(self, max_len: int) -> int:
         """The most keys a query can see, given the longest request: what the decode kernel's choice of parts
-        goes by (under chunks a query never sees more than its chunk)."""
+        goes by (under chunks a query never sees more than its chunk; with kept first positions no more than those
+        and its window)."""
+        if self.keep_first:
+            return min(max_len, self.window + self.keep_first)
         return min(max_len, self.chunk) if self.chunk else max_len
 
     def attend(self, qkv: torch.Tensor, out: torch.Tensor, ctx: StepContext, cache: CacheView) -> None:
@@ -321,21 +347,24 @@ class Attention(Mixer):
         bt = ctx.block_tables[cache.group]
         if not self.use_mfma or cache.k_pages.shape[2] % 4:
             K.attention_generic(qkv, cache.k_pages, cache.v_pages, out, ctx.token_seq, ctx.positions, bt, nh, nkv, d,
-                                self.scale, self.mask, sinks=self.sinks)
+                                self.scale, self.mask, sinks=self.sinks, keep=self.keep_first, softcap=self.score_cap)
             return
         nd = ctx.num_decode
         if nd > 0:
             K.attention_decode(qkv[:nd], cache.k_pages, cache.v_pages, out[:nd], ctx.positions[:nd], bt[:nd], nh, nkv,
-                               d, self.scale, self.mask, self._span(ctx.max_total_len), sinks=self.sinks)
+                               d, self.scale, self.mask, self._span(ctx.max_total_len), sinks=self.sinks,
+                               keep=self.keep_first, softcap=self.score_cap)
         if ctx.num_seqs > nd:
-            key = ("prefill_launch_shape", nh, nkv, d, self.mask)
+            big = max(d, self.vd)
+            key = ("prefill_launch_shape", nh, nkv, big, self.mask)
             hpw = ctx.extras.get(key)
             if hpw is None:             # once per step for all layers of this shape
-                hpw = ctx.extras[key] = K.prefill_launch_shape(nh, nkv, d, ctx.q_lens[nd:], ctx.ctx_lens[nd:],
+                hpw = ctx.extras[key] = K.prefill_launch_shape(nh, nkv, big, ctx.q_lens[nd:], ctx.ctx_lens[nd:],
                                                                self.mask, qkv.device)
             tiles, num_tiles = ctx.row_tiles(K.PREFILL_TILE_ROWS)
             K.attention_prefill(qkv, cache.k_pages, cache.v_pages, out, ctx.seq_starts, ctx.seq_ctx, bt,
-                                tiles, num_tiles, nh, nkv, d, self.scale, self.mask, hpw, sinks=self.sinks)
+                                tiles, num_tiles, nh, nkv, d, self.scale, self.mask, hpw, sinks=self.sinks,
+                                keep=self.keep_first, softcap=self.score_cap)
 
 
 register_part("mixer", "attention", Attention)

@@ -69,7 +69,7 @@ class PageTensor:
 @dataclass(frozen=True)
 class CacheSpec:
     """What a mixer needs of the paged cache: which positions are kept (all of them, 'full', or the last
-    ``window``, 'window'), and what a page holds for them (``payload``: named tensors with a per-token shape).
+    ``window``, 'window', and with ``keep_first`` a request's first positions beside them), and what a page holds for them (``payload``: named tensors with a per-token shape).
     With ``num_kv_heads`` and ``head_dim`` and no payload it is keys and values as the attention kernels read
     them: "k" [nkv, page_size, d] and "v", transposed within the page, [nkv, d, page_size]."""
 
@@ -78,6 +78,7 @@ class CacheSpec:
     head_dim: int = 0
     window: int = 0
     payload: Tuple[PageTensor, ...] = ()
+    keep_first: int = 0            # 'window': so many first positions of a request that are kept as well
 
     def __post_init__(self) -> None:
         if not self.payload:
@@ -93,7 +94,7 @@ class CacheSpec:
 
     def group_key(self) -> Tuple:
         """Layers with equal keys share page tables (one group of the cache manager)."""
-        return (self.kind, self.window)
+        return (self.kind, self.window, self.keep_first)
 
 
 @dataclass(frozen=True)

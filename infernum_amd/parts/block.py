@@ -20,6 +20,12 @@ feed_forward(f)).  The norms after the sublayers and the gates are extra parts (
 the branch, normalises it, adds it into the fp32 stream and, after the mixer, leaves the feed-forward's normalised
 input as well (``kernels.api.gated_norm_add``).
 
+``hyper``: several copies of the stream side by side (hyper-connections).  Each sublayer reads a weighted sum of the
+streams behind its norm, and its result goes back to all of them while they are mixed by a small matrix; the weights
+belong to extra parts ``mixer_hyper`` and ``feed_forward_hyper`` (category ``hyper``).  What a sublayer returned waits, as
+a pending delta does elsewhere, until one kernel writes it back, forms the next sublayer's sum and norms it
+(``kernels.api.hyper_step``).
+
 ``parallel``: h' = h + mixer(norm1(h)) + feed_forward(norm2(h)), both norms of the same stream; optionally a part
 that rewrites the stream at a later pass's entry and one that adds a token's own input after the sublayers.
 """
@@ -244,7 +250,43 @@ class ParallelBlock(Block):
             side.native(program, None, x_ready=True)
 
 
+class HyperBlock(Block):
+    graph_safe = True
+
+    def __init__(self, rt, mixer, feed_forward, mixer_norm, feed_forward_norm, extra):
+        super().__init__(rt, mixer, feed_forward, mixer_norm, feed_forward_norm, extra)
+        from .hyper import HyperConnection
+        from .rmsnorm import RMSNorm
+        self.sublayers = [("mixer", mixer_norm)] + ([("feed_forward", feed_forward_norm)] if feed_forward is not None else [])
+        for name, norm in self.sublayers:
+            if not isinstance(self.extra.get(name + "_hyper"), HyperConnection):
+                raise ValueError(f"the hyper arrangement needs a hyper_connection as {name + '_hyper'!r}")
+            if type(norm) is not RMSNorm:
+                raise ValueError("the hyper arrangement's norms are rmsnorms")
+
+    def forward(self, h: torch.Tensor, pending, ctx: StepContext, cache: CacheView):
+        for name, norm in self.sublayers:
+            hyper = self.extra[name + "_hyper"]
+            x = hyper.enter(h, pending, ctx, norm)
+            pending = self.mixer.forward(x, ctx, cache) if name == "mixer" else self.feed_forward.forward(x, ctx)
+            pending = hyper.leave(h, pending, ctx)
+        return pending
+
+    def native(self, program, view: CacheView) -> None:
+        if type(self).forward is not HyperBlock.forward:
+            return super().native(program, view)
+        for name, norm in self.sublayers:
+            hyper = self.extra[name + "_hyper"]
+            hyper.emit_enter(program, norm)
+            if name == "mixer":
+                self.mixer.native(program, view)
+            else:
+                self.feed_forward.native(program, None)
+            hyper.emit_leave(program)
+
+
 register_part("block", "prenorm", PreNormBlock)
+register_part("block", "hyper", HyperBlock)
 register_part("block", "parallel", ParallelBlock)
 register_part("block", "branchnorm", BranchNormBlock)
 register_part("block", "sandwich", SandwichBlock)

@@ -131,7 +131,8 @@ class ConvAttention(Attention):
                    [y, act, C, q, nh * d, self.q_norm, self.k_norm, float(self.norm_eps), program.positions,
                     program.slots(g), pos.inv_freq if rot else None,
                     int(bool(rot) and pos.inv_freq.dtype == torch.float64), rot, K.PAIRINGS[pos.pairing],
-                    float(pos.magnitude), k, v, N, nh, nkv, d, int(k.shape[2]), int(k.shape[0]), 1, STREAM])
+                    float(pos.magnitude), k, v, N, nh, nkv, d, d, int(k.shape[2]), int(k.shape[0]), 1,
+                    1.0, None, 0, 0.0, STREAM])
         out = self.emit_attend(program, view, q, nh * d, ALWAYS)
         o = emit_linear(program, out, N, self.w_o, rt.dtype, None, False, "conv_attention.out", "conv_attention.o")
         program.op("core", "ia_add_bias", [o.tensor(), act, self.b_o, N, self.hidden_size, STREAM])

@@ -130,8 +130,8 @@ class GatedLinearAttention(Mixer):
                                               floats,
                                               decay, self.nh, self.dim, self.vdim, STREAM], Guard.between(program.NP, 1))
         gated = program.buffer("gla.gated", T * nv * ab)
-        program.op("core", "ia_head_norm_gate", [o, proj, act, self.row, self.g_col, self.w_norm, gated, N, self.nh,
-                                                 self.vdim, float(self.norm_eps), STREAM])
+        program.op("core", "ia_head_norm_gate", [o, proj, act, self.row, self.g_col, self.w_norm, gated, nv, N,
+                                                 self.nh, self.vdim, float(self.norm_eps), 0, 0, STREAM])
         program.pending = emit_linear(program, gated, N, self.w_o, rt.dtype, None, True, "gla.out", "gla.o_proj")
 
 

@@ -115,8 +115,8 @@ class Hgrn2(Mixer):
                                                 num_tiles, program.ND, N, records, floats, decay, self.nh, self.dim,
                                                 self.vdim, STREAM], Guard.between(program.NP, 1))
         normed = program.buffer("hgrn2.normed", T * self.nv * ab)
-        program.op("core", "ia_head_norm_gate", [o, None, act, 0, 0, self.w_norm, normed, N, self.nh, self.vdim,
-                                                 float(self.norm_eps), STREAM])
+        program.op("core", "ia_head_norm_gate", [o, None, act, 0, 0, self.w_norm, normed, self.nv, N, self.nh,
+                                                 self.vdim, float(self.norm_eps), 0, 0, STREAM])
         program.pending = emit_linear(program, normed, N, self.w_o, rt.dtype, None, True, "hgrn2.out", "hgrn2.o_proj")
 
 

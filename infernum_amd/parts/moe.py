@@ -18,9 +18,18 @@ s = softmax(z) over ALL experts, the ``top`` largest of s + correction are chose
 moves the choice only), and the weights are the chosen s over their sum (+ 1e-20).  ``shared_ff``: one more expert of
 that middle width (``shared.up``, ``shared.down``; same form, no gate) that every token takes with weight 1; its
 result is added into the first choice's part.
+
+More options of gated experts: without ``limit`` nothing is clamped; ``up_shift`` stands in place of the 1 that is
+added to u (0 with alpha 1: D_e (silu(G_e x) * (U_e x))).  Of the ``softmax_top`` router: ``renorm=False`` leaves the
+chosen s as they are; ``groups`` and ``keep_groups``: the experts form equal groups of neighbours, a group's score is its
+largest s + correction, and only experts of the best groups can be chosen; ``identity`` n: the last n of
+num_experts + n experts have no tensors, and their result is their input.  ``shared_ff`` with gated experts: the shared
+expert is D (silu(G x) * (U x)) (``shared.gate``, ``shared.up``, ``shared.down``), with ``shared_gate`` (a local tensor
+name, [1, W]) times the sigmoid of one number per token; its result is a part of its own after the choices'.
 """
 from __future__ import annotations
 
+import math
 from typing import Dict, Optional
 
 import torch
@@ -37,24 +46,37 @@ class RoutedExperts(FeedForward):
                  limit: Optional[float] = None, alpha: float = 1.702, router_bias: bool = True,
                  router_name: str = "router", expert_prefix: str = "e", init_std: float = 0.02, gated: bool = True,
                  activation: str = "relu_squared", router: str = "top_softmax", correction_name: str = "correction",
-                 shared_ff: Optional[int] = None):
+                 shared_ff: Optional[int] = None, up_shift: float = 1.0, renorm: bool = True, groups: int = 1,
+                 keep_groups: int = 1, identity: int = 0, shared_gate: Optional[str] = None):
         super().__init__(rt)
         self.hidden_size, self.ff = int(hidden_size), int(intermediate_size)
         self.num_experts, self.top = int(num_experts), int(top)
-        if not 0 < self.top <= self.num_experts:
-            raise ValueError(f"a token takes {top} of {num_experts} experts")
+        self.identity = int(identity)
+        self.total = self.num_experts + self.identity           # what the router chooses among
+        self.groups, self.keep_groups, self.renorm = int(groups), int(keep_groups), bool(renorm)
+        if not 0 < self.top <= self.total or self.identity < 0:
+            raise ValueError(f"a token takes {top} of {self.total} experts")
+        if self.groups < 1 or self.total % self.groups or not 1 <= self.keep_groups <= self.groups \
+                or self.top > self.keep_groups * (self.total // self.groups):
+            raise ValueError(f"{self.total} experts in {groups} groups, {keep_groups} of them kept, cannot give a token {top}")
         self.gated, self.activation, self.router = bool(gated), str(activation), str(router)
         if self.router not in ("top_softmax", "softmax_top"):
             raise ValueError(f"router {router!r}: 'top_softmax' or 'softmax_top'")
         if not self.gated and self.activation not in K.ACTIVATIONS:
             raise ValueError(f"activation {activation!r}: one of {sorted(K.ACTIVATIONS)}")
-        self.limit, self.alpha = float(limit) if limit is not None else 0.0, float(alpha)
+        self.limit, self.alpha = float(limit) if limit is not None else math.inf, float(alpha)
+        self.up_shift = float(up_shift)
         if self.gated and not self.limit > 0:
             raise ValueError("the experts' limit must be positive")
+        if self.router != "softmax_top" and (self.groups > 1 or self.identity or not self.renorm):
+            raise ValueError("groups, identity experts and weights as they are go with the 'softmax_top' router")
+        if self.identity and not self.gated:
+            raise ValueError("identity experts go with gated experts")
         self.correction_name = correction_name
         self.shared_ff = int(shared_ff) if shared_ff else 0
-        if self.shared_ff and self.gated:
-            raise ValueError("a shared expert goes with experts without a gate")
+        self.shared_gate = str(shared_gate) if shared_gate else None
+        if self.shared_gate and not (self.shared_ff and self.gated):
+            raise ValueError("a gate on the shared expert needs a shared expert, of gated experts")
         self.router_bias, self.router_name, self.expert_prefix = bool(router_bias), router_name, expert_prefix
         self.init_std = init_std
         self.w_router: Optional[torch.Tensor] = None
@@ -65,11 +87,15 @@ class RoutedExperts(FeedForward):
     def weights(self) -> Dict[str, WeightSpec]:
         H, I, E = self.hidden_size, self.ff, self.num_experts
         init = ("normal", self.init_std)
-        out = {self.router_name: WeightSpec((E, H), init)}
+        out = {self.router_name: WeightSpec((self.total, H), init)}
         if self.router == "softmax_top":
-            out[self.correction_name] = WeightSpec((E,), ("normal", 0.05), follows_compute_dtype=False)
+            out[self.correction_name] = WeightSpec((self.total,), ("normal", 0.05), follows_compute_dtype=False)
         elif self.router_bias:
             out[self.router_name + ".b"] = WeightSpec((E,), ("normal", 0.5), follows_compute_dtype=False)
+        if self.shared_ff and self.gated:
+            out["shared.gate"] = WeightSpec((self.shared_ff, H), init)
+        if self.shared_gate:
+            out[self.shared_gate] = WeightSpec((1, H), init)
         if self.shared_ff:
             out["shared.up"] = WeightSpec((self.shared_ff, H), init)
             out["shared.down"] = WeightSpec((H, self.shared_ff), init)
@@ -84,6 +110,8 @@ class RoutedExperts(FeedForward):
     def load(self, tensors: Dict[str, torch.Tensor]) -> None:
         H, I, E = self.hidden_size, self.ff, self.num_experts
         self.w_router = tensors[self.router_name].contiguous()
+        if self.shared_gate:                  # the shared expert's gate is one more row of the router's product
+            self.w_router = torch.cat([self.w_router, tensors[self.shared_gate]], dim=0).contiguous()
         if self.router == "softmax_top":
             self.b_router = tensors[self.correction_name].contiguous()
         else:
@@ -99,17 +127,36 @@ class RoutedExperts(FeedForward):
             else:
                 self.w_gate_up[e] = tensors[p + "up"]
             self.w_down[e] = tensors[p + "down"]
-        if self.shared_ff:
+        if self.shared_ff and self.gated:
+            from .linear import prepare_weights
+            self.w_shared_gate_up = torch.cat([tensors["shared.gate"], tensors["shared.up"]], dim=0).contiguous()
+            self.w_shared_down = tensors["shared.down"].contiguous()
+            prepare_weights(self.rt, [(self.w_shared_gate_up, "swiglu", False), (self.w_shared_down, None, True)])
+        elif self.shared_ff:
             from .linear import prepare_weights
             self.w_shared_up, self.w_shared_down = tensors["shared.up"].contiguous(), tensors["shared.down"].contiguous()
             prepare_weights(self.rt, [(self.w_shared_up, None, False), (self.w_shared_down, None, False)])
 
     def forward(self, x: torch.Tensor, ctx: Optional[StepContext] = None):
         z = linear(x, self.w_router, out_dtype=torch.float32, kernels=self.rt.kernels)
-        choose = K.router_softmax_topk if self.router == "softmax_top" else K.router_topk
-        ids, weights = choose(z, self.b_router, self.top)
+        if self.router == "softmax_top":
+            ids, weights = K.router_softmax_topk(z, self.b_router, self.top, self.groups, self.keep_groups, self.renorm,
+                                                 self.total)
+        else:
+            ids, weights = K.router_topk(z, self.b_router, self.top)
         if self.gated:
-            return K.moe_experts(x, ids, weights, self.w_gate_up, self.w_down, self.limit, self.alpha)
+            extras = bool(self.identity or self.shared_ff)
+            parts = torch.empty((self.top + bool(self.shared_ff), x.shape[0], self.hidden_size), dtype=torch.float32,
+                                device=x.device)
+            out = K.moe_experts(x, ids, weights, self.w_gate_up, self.w_down, self.limit, self.alpha, self.up_shift,
+                                self.total, parts)
+            if not extras:
+                return out
+            shared = None
+            if self.shared_ff:
+                act = linear(x, self.w_shared_gate_up, epilogue="swiglu", kernels=self.rt.kernels)
+                shared = linear(act, self.w_shared_down, keep_split=True, kernels=self.rt.kernels)
+            return K.moe_extras(x, ids, weights, parts, self.num_experts, shared, z[:, self.total] if self.shared_gate else None)
         parts = K.moe_plain_experts(x, ids, weights, self.w_gate_up, self.w_down, self.activation)
         if self.shared_ff:
             u = K.activation(linear(x, self.w_shared_up, kernels=self.rt.kernels), self.activation)
@@ -121,19 +168,24 @@ class RoutedExperts(FeedForward):
             return super().native(program, view)
         from ..engine.program import ALWAYS, STREAM, Alt, Value
         H, I, E, top, T, N = self.hidden_size, self.ff, self.num_experts, self.top, program.T, program.N
+        total = self.total
         program.keep(self.w_router, self.b_router, self.w_gate_up, self.w_down)
         z = emit_linear(program, program.x, N, self.w_router, torch.float32, None, False, "moe.logits", "moe.router")
         ids = program.buffer("moe.ids", T * top * 4)
         wts = program.buffer("moe.weights", T * top * 4)
-        offsets = program.buffer("moe.offsets", (E + 1) * 4)
+        offsets = program.buffer("moe.offsets", (total + 1) * 4)
         perm = program.buffer("moe.perm", T * top * 4)
         y = program.buffer("moe.y", T * top * I * program.act_bytes)
-        parts = program.buffer("moe.parts", top * T * H * 4)
+        parts = program.buffer("moe.parts", (top + bool(self.gated and self.shared_ff)) * T * H * 4)
         b = self.b_router
-        choose = "ia_router_softmax_topk" if self.router == "softmax_top" else "ia_router_topk"
-        program.op("core", choose, [z.tensor(), b, K.DTYPE_CODE[b.dtype] if b is not None else 0, ids, wts,
-                                    N, E, top, STREAM])
-        program.op("core", "ia_moe_sort", [ids, offsets, perm, N * top, E, STREAM])
+        b_code = K.DTYPE_CODE[b.dtype] if b is not None else 0
+        if self.router == "softmax_top":
+            program.op("core", "ia_router_softmax_topk", [z.tensor(), b, b_code, ids, wts, N, total, top,
+                                                          int(self.w_router.shape[0]), self.groups, self.keep_groups,
+                                                          int(self.renorm), STREAM])
+        else:
+            program.op("core", "ia_router_topk", [z.tensor(), b, b_code, ids, wts, N, total, top, STREAM])
+        program.op("core", "ia_moe_sort", [ids, offsets, perm, N * top, total, STREAM])
         if not self.gated:
             return self._native_plain(program, ids, wts, offsets, perm, y, parts)
         from ..engine.program import NEVER, Guard
@@ -141,7 +193,7 @@ class RoutedExperts(FeedForward):
         grouped = Guard.between(N, first) if first > 0 else NEVER
         tiled = ~grouped
         program.op("core", "ia_moe_gate_up", [program.x, self.w_gate_up, y, offsets, perm, program.act_code, N * top,
-                                              E, top, H, I, self.limit, self.alpha, STREAM], tiled)
+                                              E, top, H, I, self.limit, self.alpha, self.up_shift, STREAM], tiled)
         program.op("core", "ia_moe_down", [y, self.w_down, parts, wts, offsets, perm, program.act_code, N, E, top, H,
                                            I, STREAM], tiled)
         if first > 0 and first <= T:
@@ -151,11 +203,29 @@ class RoutedExperts(FeedForward):
             program.op("core", "ia_moe_gather", [program.x, perm, xs, N * top, top, H, STREAM], grouped)
             program.op("core", "ia_gemm_mfma_grouped", [xs, self.w_gate_up, gu, offsets, E, N * top, 2 * I, H, STREAM],
                        grouped)
-            program.op("core", "ia_moe_glu", [gu, y, N * top, I, self.limit, self.alpha, STREAM], grouped)
+            program.op("core", "ia_moe_glu", [gu, y, N * top, I, self.limit, self.alpha, self.up_shift, STREAM], grouped)
             program.op("core", "ia_gemm_mfma_grouped", [y, self.w_down, xs, offsets, E, N * top, H, I, STREAM], grouped)
-            program.op("core", "ia_moe_scatter", [xs, perm, wts, parts, N, top, H, STREAM], grouped)
-        program.pending = Value(H, [Alt(ALWAYS, parts, top, torch.float32)])
+            program.op("core", "ia_moe_scatter", [xs, perm, wts, parts, offsets.at(E * 4) if self.identity else None, N, top, H,
+                                                  STREAM], grouped)
+        if self.identity or self.shared_ff:
+            self._native_extras(program, z.tensor(), ids, wts, parts)
+        program.pending = Value(H, [Alt(ALWAYS, parts, top + bool(self.shared_ff), torch.float32)])
 
+    def _native_extras(self, program, z, ids, wts, parts) -> None:
+        """Identity experts' pairs and the shared expert of gated experts."""
+        from ..engine.program import ALWAYS, STREAM, Alt
+        H, E, top, N, code = self.hidden_size, self.num_experts, self.top, program.N, program.act_code
+        alts = [Alt(ALWAYS, None, 0, self.rt.dtype)]
+        if self.shared_ff:
+            act = emit_linear(program, program.x, N, self.w_shared_gate_up, self.rt.dtype, "swiglu", False, "moe.shared.act",
+                              "moe.shared.gate_up").tensor()
+            alts = emit_linear(program, act, N, self.w_shared_down, self.rt.dtype, None, True, "moe.shared.out",
+                               "moe.shared.down").alts
+        for alt in alts:
+            program.op("core", "ia_moe_extras",
+                       [program.x, code, ids, wts, parts, alt.where, K.DTYPE_CODE[torch.float32 if alt.splits else alt.dtype],
+                        alt.splits or 1, N, z.at(self.total * 4) if self.shared_gate else None, int(self.w_router.shape[0]), N,
+                        E, top, H, STREAM], alt.when)
 
     def _native_plain(self, program, ids, wts, offsets, perm, y, parts) -> None:
         """The launches of ``kernels.api.moe_plain_experts`` and of the shared expert."""
@@ -176,7 +246,7 @@ class RoutedExperts(FeedForward):
             program.op("core", "ia_gemm_mfma_grouped", [xs, self.w_gate_up, y, offsets, E, N * top, I, H, STREAM], grouped)
             program.op("core", "ia_activation", [y, y, code, N * (top * I), act, STREAM], grouped)
             program.op("core", "ia_gemm_mfma_grouped", [y, self.w_down, xs, offsets, E, N * top, H, I, STREAM], grouped)
-            program.op("core", "ia_moe_scatter", [xs, perm, wts, parts, N, top, H, STREAM], grouped)
+            program.op("core", "ia_moe_scatter", [xs, perm, wts, parts, None, N, top, H, STREAM], grouped)
         if self.shared_ff:
             program.keep(self.w_shared_up, self.w_shared_down)
             u = emit(program, program.x, N, self.w_shared_up, self.rt.dtype, None, False, "moe.shared.act",

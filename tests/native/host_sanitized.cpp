@@ -12,7 +12,7 @@
 #include <vector>
 
 extern "C" {
-void* ia_cache_create(int, const int*, const int*, int, int, int);
+void* ia_cache_create(int, const int*, const int*, const int*, int, int, int);
 void ia_cache_destroy(void*);
 const char* ia_cache_error(void*);
 int ia_cache_admit(void*, int64_t);
@@ -51,7 +51,7 @@ static long g_calls = 0;
 static void cache_under_random_requests(unsigned seed) {
   std::mt19937 rng(seed);
   const int kinds[2] = {0, 1}, windows[2] = {0, 10};
-  void* c = ia_cache_create(2, kinds, windows, 4, 40, 6);
+  void* c = ia_cache_create(2, kinds, windows, nullptr, 4, 40, 6);
   CHECK(c);
   std::vector<int64_t> live;
   int64_t next = 0;
