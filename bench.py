@@ -651,6 +651,61 @@ def rogizen_bench(a) -> int:
                               rogizen_active_params, batches)
 
 
+# ---- the Pamazen design beside the Llama decoder at equal sizes -------------------------------------------------
+# Eight layers of one width over four residual streams: a layer with two mixers side by side (window attention whose values
+# are its keys, with four kept positions, sinks and capped scores, 16 or 32 heads of 128 over 4 or 8; the generalized delta
+# rule, as many heads of 128, decays through a middle of 64), then three of attention over all keys with rotated pairs and
+# values mixed with the first of them, twice; every layer sixteen experts and two identities in two groups of which one is
+# kept, two chosen, and a gated shared expert: together as many feed-forward weights a token as the twin has (when no
+# identity is chosen).  The Llama twin has the same width, layers, vocabulary and heads.
+PAMAZEN_SIZES = {
+    "2k": dict(width=2048, layers=8, vocab=32000, ff=5504, heads=16, kv_heads=4, dim=128, window=1024, keep=4, rank=64,
+               streams=4, experts=16, identity=2, top=2, expert_ff=1408, shared_ff=2688),
+    "4k": dict(width=4096, layers=8, vocab=32000, ff=9600, heads=32, kv_heads=8, dim=128, window=2048, keep=4, rank=64,
+               streams=4, experts=16, identity=2, top=2, expert_ff=2432, shared_ff=4736),
+}
+
+
+def pamazen_configs(size: dict):
+    from infernum_amd.config import LlamaConfig
+    from infernum_amd.config.pamazen import PamazenConfig
+    d = size["dim"]
+    heads = {"heads": size["heads"], "kv_heads": size["kv_heads"], "dim": d, "vdim": d, "scale": d ** -0.5}
+    attention = dict(heads, v_mix=True, rot={"base": 10000.0, "dims": d // 2, "scaling": {"factor": 4.0}})
+    side = {"left": dict(heads, softcap=30.0, mask={"size": size["window"], "keep_first": size["keep"]}),
+            "right": {"heads": size["heads"], "dim": d, "rank": size["rank"]}, "left_scale": 1.0, "right_scale": 0.5}
+    mlp = {"kind": "moe", "expert": {"ff": size["expert_ff"]}, "shared": {"ff": size["shared_ff"]},
+           "router": {"experts": size["experts"], "identity": size["identity"], "top": size["top"],
+                      "groups": {"count": 2, "keep": 1}}}
+    pam = PamazenConfig.from_dict({
+        "architecture": "Pamazen", "vocab": size["vocab"], "width": size["width"], "norm": {"eps": 1e-6},
+        "streams": size["streams"], "residual_mult": 0.5, "logit_softcap": 15.0,
+        "layers": [{"type": "attention" if i % 4 else "parallel", "mixer": attention if i % 4 else side, "mlp": mlp}
+                   for i in range(size["layers"])]})
+    llama = LlamaConfig.from_dict(dict(
+        model_type="llama", num_hidden_layers=size["layers"], hidden_size=size["width"],
+        num_attention_heads=size["heads"], num_key_value_heads=size["kv_heads"], intermediate_size=size["ff"],
+        vocab_size=size["vocab"], rope_theta=10000.0, rms_norm_eps=1e-6, tie_word_embeddings=True,
+        max_position_embeddings=8192))
+    return pam, llama
+
+
+def pamazen_active_params(size: dict) -> int:
+    """Weights that a token multiplies with in the Pamazen model of these sizes when it takes no identity expert (the
+    head included)."""
+    W, n, hd, kvd = size["width"], size["layers"], size["heads"] * size["dim"], size["kv_heads"] * size["dim"]
+    attention = W * (hd + 2 * kvd) + hd * W
+    side = W * (hd + kvd) + hd * W + W * (5 * hd + size["rank"]) + hd * size["rank"] + hd * W
+    moe = W * (size["experts"] + size["identity"] + 1) + 3 * W * (size["top"] * size["expert_ff"] + size["shared_ff"])
+    return (n // 4) * side + (n - n // 4) * attention + n * moe + size["vocab"] * W
+
+
+def pamazen_bench(a) -> int:
+    batches = [int(b) for b in a.pamazen_batches.split(",") if b]
+    return beside_llama_bench(a, "Pamazen", [(n, PAMAZEN_SIZES[n]) for n in a.pamazen.split(",")], pamazen_configs,
+                              pamazen_active_params, batches)
+
+
 def beside_llama_bench(a, design, sizes, configs, active_params, batches) -> int:
     """Prefill of 2,048 tokens and decode steps at batch 8 and 64 of a design and of the Llama decoder at equal
     sizes, random weights, through the same engine and generation loop; one JSON line of its own."""
@@ -755,6 +810,11 @@ def main() -> int:
                          "parallel sublayers) beside the Llama decoder at equal sizes: names of "
                          + ", ".join(SIKAZEN_SIZES) + " with commas")
     ap.add_argument("--sikazen-batches", default="8,64", help="decode batches of --sikazen")
+    ap.add_argument("--pamazen", default="", metavar="SIZES",
+                    help="the Pamazen design (several residual streams, window attention beside the generalized delta rule, "
+                         "mixed values, grouped experts with identities) beside the Llama decoder at equal sizes: names of "
+                         + ", ".join(PAMAZEN_SIZES) + " with commas")
+    ap.add_argument("--pamazen-batches", default="8,64", help="decode batches of --pamazen")
     a = ap.parse_args()
     if a.gpus != 1:
         print(f"bench.py measures one GPU: this engine has no multi-GPU path (asked for --gpus {a.gpus})")
@@ -766,6 +826,8 @@ def main() -> int:
         return malinex_bench(a)
     if a.sikazen:
         return sikazen_bench(a)
+    if a.pamazen:
+        return pamazen_bench(a)
     if a.rogizen:
         return rogizen_bench(a)
     if a.decode_kernels:

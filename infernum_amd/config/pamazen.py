@@ -4,7 +4,7 @@ The file names its design in ``architecture`` and describes every layer by itsel
   vocab, width, norm.eps, streams, residual_mult, logit_softcap,
   layers[i].type   the mixer: "parallel" | "attention",
   layers[i].mixer  parallel: {left: {heads, kv_heads, dim, vdim, scale, softcap, mask: {size, keep_first}},
-                   right: {heads, dim}, left_scale, right_scale};
+                   right: {heads, dim, rank (only random weights need it)}, left_scale, right_scale};
                    attention: {heads, kv_heads, dim, vdim, scale, v_mix, rot: {base, dims, scaling: {factor}}},
   layers[i].mlp    null | {kind: "moe", expert: {ff}, router: {experts, identity, top, groups: {count, keep}},
                    shared: {ff}}.
@@ -121,13 +121,17 @@ class WindowAttentionConfig:
 class DeltaConfig:
     heads: int
     dim: int
+    rank: Optional[int] = None  # the middle of the decays' two products; None: read off a file's tensors
 
     @staticmethod
     def from_reader(r: KeyReader) -> "DeltaConfig":
-        return DeltaConfig(r.integer("heads", minimum=1), r.integer("dim", minimum=1))
+        return DeltaConfig(r.integer("heads", minimum=1), r.integer("dim", minimum=1), r.integer("rank", None, minimum=1))
 
     def to_dict(self) -> dict:
-        return {"heads": self.heads, "dim": self.dim}
+        out = {"heads": self.heads, "dim": self.dim}
+        if self.rank is not None:
+            out["rank"] = self.rank
+        return out
 
 
 @dataclass(frozen=True)

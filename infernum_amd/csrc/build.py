@@ -65,7 +65,9 @@ BLASLT_SOURCES = ["gemm_library.cpp"]
 DEFAULT_HEAD_DIMS = (16, 32, 48, 64, 80, 96, 112, 128, 160, 192, 256)
 SUPPORTED_HEAD_DIMS = tuple(range(16, 257, 16))
 # (key size, value size, with kept first keys and a softcap) whose attention library `build_all` compiles ahead of time.
-DEFAULT_ATTENTION_SIZES = ((16, 32, False), (32, 16, False), (48, 32, False), (32, 32, True), (64, 64, True), (128, 128, True))
+DEFAULT_ATTENTION_SIZES = ((16, 32, False), (16, 48, False), (32, 16, False), (32, 256, False), (48, 16, False), (48, 32, False),
+                           (64, 32, False), (128, 64, False), (16, 16, True), (32, 32, True), (48, 48, True), (64, 64, True),
+                           (80, 16, True), (128, 64, True), (128, 128, True), (160, 32, True))
 # (key size, value size) pairs whose sigmoid-attention library `build_all` compiles ahead of time.
 DEFAULT_SIGATTN_SIZES = ((16, 32), (32, 64), (48, 16), (64, 64), (64, 128), (96, 32), (128, 32), (128, 64), (128, 128))
 # (key size, value size) pairs whose window-and-blocks attention library `build_all` compiles ahead of time.

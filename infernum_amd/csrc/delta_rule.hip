@@ -125,15 +125,43 @@ __device__ __forceinline__ void dr_read(const float* p, float (&v)[VEC]) {
   }
 }
 
-// grid (heads, requests, groups of DR_COLS columns), 64 DR_WAVES threads.
-template <typename T, int VEC, int J>
+// The vectors of one token as a lane needs them.
+template <int VEC, int J>
+struct DrToken {
+  float u[J][VEC], w[J][VEC], au[J][VEC], k[J][VEC], r[J][VEC], v;
+};
+
+// L values side by side from memory, as they are stored there (converted when they go to LDS: nothing waits here).
+template <typename T, int L> struct DrRaw;
+template <> struct DrRaw<float, 1> { typedef float type; };
+template <> struct DrRaw<float, 4> { typedef float4 type; };
+template <> struct DrRaw<bf16_t, 1> { typedef bf16_t type; };
+template <> struct DrRaw<bf16_t, 4> { typedef uint2 type; };
+__device__ __forceinline__ void dr_values(float x, float (&o)[1]) { o[0] = x; }
+__device__ __forceinline__ void dr_values(bf16_t x, float (&o)[1]) { o[0] = to_float(x); }
+__device__ __forceinline__ void dr_values(float4 x, float (&o)[4]) { o[0] = x.x; o[1] = x.y; o[2] = x.z; o[3] = x.w; }
+__device__ __forceinline__ void dr_values(uint2 x, float (&o)[4]) {
+  o[0] = __uint_as_float(x.x << 16);
+  o[1] = __uint_as_float(x.x & 0xffff0000u);
+  o[2] = __uint_as_float(x.y << 16);
+  o[3] = __uint_as_float(x.y & 0xffff0000u);
+}
+__device__ __forceinline__ void dr_put(float* at, const float (&v)[1]) { at[0] = v[0]; }
+__device__ __forceinline__ void dr_put(float* at, const float (&v)[4]) {
+  *reinterpret_cast<float4*>(at) = make_float4(v[0], v[1], v[2], v[3]);
+}
+
+// grid (heads, requests, groups of DR_COLS columns), 64 DR_WAVES threads.  L: channels of a load when vectors are staged
+// (4 where every row and column begins on a multiple of four values, else 1).
+template <typename T, int VEC, int J, int L>
 __global__ __launch_bounds__(64 * DR_WAVES) void delta_scan_kernel(
     const T* __restrict__ proj, int proj_stride, int r_col, int k_col, int v_col, const float* __restrict__ w,
     const float* __restrict__ a, const float* __restrict__ inv, float* __restrict__ state, long state_stride,
     float* __restrict__ out, const int* __restrict__ seq_starts, const int* __restrict__ state_slots, int nh, int dim) {
   constexpr int P = 16 * VEC * J;                     // the channels with those that pad them
   constexpr int NT = 64 * DR_WAVES;
-  constexpr int PER = (DR_TB * P + NT - 1) / NT;      // channel values a thread stages, of each vector
+  constexpr int PER = (DR_TB * P / L + NT - 1) / NT;  // pieces of L channels a thread stages, of each vector
+  static_assert(P % L == 0 && DR_TB * DR_COLS <= NT, "pieces fit the rows; a thread stages at most one value of v");
   __shared__ __attribute__((aligned(16))) float s_w[DR_TB][P], s_au[DR_TB][P], s_u[DR_TB][P], s_k[DR_TB][P], s_r[DR_TB][P];
   __shared__ float s_v[DR_TB][DR_COLS];
   const int hd = blockIdx.x, s = blockIdx.y, c0 = blockIdx.z * DR_COLS;
@@ -143,100 +171,147 @@ __global__ __launch_bounds__(64 * DR_WAVES) void delta_scan_kernel(
   const int col = c0 + grp;                           // this lane's column of the state
   const bool col_ok = col < dim;
   float* st = state + (size_t)state_slots[s] * state_stride + ((size_t)hd * dim + (col_ok ? col : 0)) * dim;
+  // the vectors of up to DR_TB tokens on their way to LDS: every load is made, from a place of this head's own rows where
+  // there is no such token or channel (those values are replaced by zeros on the way into LDS)
+  typename DrRaw<float, L>::type fw[PER], fa[PER];
+  typename DrRaw<T, L>::type fk[PER], fr[PER];
+  float fi[PER];
+  T fv;
+  auto fetch = [&](int t0) {
+#pragma unroll
+    for (int x = 0; x < PER; ++x) {
+      const int idx = tid + x * NT, t = idx / (P / L), n = (idx - t * (P / L)) * L;
+      const int tc = t0 + t < count ? t0 + t : count - 1, nc = n < dim ? n : 0;
+      const size_t row = (size_t)(first + tc), at = (row * nh + hd) * dim + nc;
+      const T* pr = proj + row * proj_stride + hd * dim + nc;
+      fw[x] = *reinterpret_cast<const typename DrRaw<float, L>::type*>(w + at);
+      fa[x] = *reinterpret_cast<const typename DrRaw<float, L>::type*>(a + at);
+      fk[x] = *reinterpret_cast<const typename DrRaw<T, L>::type*>(pr + k_col);
+      fr[x] = *reinterpret_cast<const typename DrRaw<T, L>::type*>(pr + r_col);
+      fi[x] = inv[row * nh + hd];
+    }
+    const int t = tid / DR_COLS, c = c0 + tid % DR_COLS;
+    fv = proj[(size_t)(first + (t0 + t < count ? t0 + t : count - 1)) * proj_stride + v_col + hd * dim + (c < dim ? c : 0)];
+  };
+  fetch(0);
   float S[J][VEC];
 #pragma unroll
   for (int j = 0; j < J; ++j)
 #pragma unroll
-    for (int e = 0; e < VEC; ++e) {
-      const int n = 16 * VEC * j + VEC * q + e;
-      S[j][e] = (col_ok && n < dim) ? st[n] : 0.f;
-    }
-  // the vectors of up to DR_TB tokens on their way to LDS
-  float fw[PER], fa[PER], fk[PER], fr[PER], fi[PER], fv = 0.f;
-  auto fetch = [&](int t0) {
+    for (int e = 0; e < VEC; ++e) S[j][e] = 0.f;
 #pragma unroll
-    for (int x = 0; x < PER; ++x) {
-      const int idx = tid + x * NT, t = idx / P, n = idx - t * P;
-      fw[x] = fa[x] = fk[x] = fr[x] = fi[x] = 0.f;
-      if (t < DR_TB && t0 + t < count && n < dim) {
-        const size_t row = (size_t)(first + t0 + t), at = (row * nh + hd) * dim + n;
-        const T* pr = proj + row * proj_stride + hd * dim + n;
-        fw[x] = w[at];
-        fa[x] = a[at];
-        fk[x] = to_float(pr[k_col]);
-        fr[x] = to_float(pr[r_col]);
-        fi[x] = inv[row * nh + hd];
+  for (int j = 0; j < J; ++j) {
+    const int n = 16 * VEC * j + VEC * q;
+    if (VEC == L && L == 4) {                         // channels in fours: all of them are there or none
+      if (col_ok && n < dim) dr_read<VEC>(st + n, S[j]);
+    } else {
+#pragma unroll
+      for (int e = 0; e < VEC; ++e)
+        if (col_ok && n + e < dim) S[j][e] = st[n + e];
+    }
+  }
+  DrToken<VEC, J> A, B;
+  auto load = [&](int t, DrToken<VEC, J>& X) {
+#pragma unroll
+    for (int j = 0; j < J; ++j) {
+      const int n = 16 * VEC * j + VEC * q;
+      dr_read<VEC>(&s_u[t][n], X.u[j]);
+      dr_read<VEC>(&s_w[t][n], X.w[j]);
+      dr_read<VEC>(&s_au[t][n], X.au[j]);
+      dr_read<VEC>(&s_k[t][n], X.k[j]);
+      dr_read<VEC>(&s_r[t][n], X.r[j]);
+    }
+    X.v = s_v[t][grp];
+  };
+  auto step = [&](const DrToken<VEC, J>& X) {
+    float d[J];
+#pragma unroll
+    for (int j = 0; j < J; ++j) {
+      d[j] = X.u[j][0] * S[j][0];
+#pragma unroll
+      for (int e = 1; e < VEC; ++e) d[j] = __builtin_fmaf(X.u[j][e], S[j][e], d[j]);
+    }
+#pragma unroll
+    for (int j = 1; j < J; ++j) d[0] += d[j];
+    const float dot = dr_sum16(d[0]);                 // u^T S of this column
+    float o[J];
+#pragma unroll
+    for (int j = 0; j < J; ++j) {
+      o[j] = 0.f;
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) {
+        const float add = __builtin_fmaf(X.k[j][e], X.v, -(X.au[j][e] * dot));
+        S[j][e] = __builtin_fmaf(X.w[j][e], S[j][e], add);
+        o[j] = __builtin_fmaf(X.r[j][e], S[j][e], o[j]);
       }
     }
-    const int t = tid / DR_COLS, c = c0 + tid % DR_COLS;
-    fv = 0.f;
-    if (t < DR_TB && t0 + t < count && c < dim) fv = to_float(proj[(size_t)(first + t0 + t) * proj_stride + v_col + hd * dim + c]);
+#pragma unroll
+    for (int j = 1; j < J; ++j) o[0] += o[j];
+    return dr_sum16(o[0]);
   };
-  static_assert(DR_TB * DR_COLS <= NT, "a thread stages at most one value of v");
-  fetch(0);
   for (int t0 = 0; t0 < count; t0 += DR_TB) {
     const int nt = count - t0 < DR_TB ? count - t0 : DR_TB;
     __syncthreads();                                  // the tokens before are read to their end
 #pragma unroll
     for (int x = 0; x < PER; ++x) {
-      const int idx = tid + x * NT, t = idx / P, n = idx - t * P;
+      const int idx = tid + x * NT, t = idx / (P / L), n = (idx - t * (P / L)) * L;
+      float vw[L], va[L], vk[L], vr[L], u[L];
+      dr_values(fw[x], vw);
+      dr_values(fa[x], va);
+      dr_values(fk[x], vk);
+      dr_values(fr[x], vr);
+      const bool real = n < dim && t < nt;
+#pragma unroll
+      for (int e = 0; e < L; ++e) {
+        u[e] = real ? vk[e] * fi[x] : 0.f;
+        va[e] = real ? va[e] * u[e] : 0.f;
+        vw[e] = real ? vw[e] : 0.f;
+        vk[e] = real ? vk[e] : 0.f;
+        vr[e] = real ? vr[e] : 0.f;
+      }
       if (t < DR_TB) {
-        const float u = fk[x] * fi[x];
-        s_w[t][n] = fw[x];
-        s_au[t][n] = fa[x] * u;
-        s_u[t][n] = u;
-        s_k[t][n] = fk[x];
-        s_r[t][n] = fr[x];
+        dr_put(&s_w[t][n], vw);
+        dr_put(&s_au[t][n], va);
+        dr_put(&s_u[t][n], u);
+        dr_put(&s_k[t][n], vk);
+        dr_put(&s_r[t][n], vr);
       }
     }
-    if (tid < DR_TB * DR_COLS) s_v[tid / DR_COLS][tid % DR_COLS] = fv;
+    if (tid < DR_TB * DR_COLS) s_v[tid / DR_COLS][tid % DR_COLS] = c0 + tid % DR_COLS < dim ? to_float(fv) : 0.f;
     __syncthreads();
     if (t0 + DR_TB < count) fetch(t0 + DR_TB);
     float mine = 0.f;                                 // lane q keeps token q's result of the column
+    load(0, A);
+    if (nt == DR_TB) {                                // the next token's vectors come in while this one is worked on
 #pragma unroll
-    for (int t = 0; t < DR_TB; ++t) {
-      if (t >= nt) break;
-      float u[J][VEC], x[J][VEC];
-      float dot = 0.f;
-#pragma unroll
-      for (int j = 0; j < J; ++j) {
-        dr_read<VEC>(&s_u[t][16 * VEC * j + VEC * q], u[j]);
-#pragma unroll
-        for (int e = 0; e < VEC; ++e) dot = __builtin_fmaf(u[j][e], S[j][e], dot);
+      for (int t = 0; t < DR_TB; t += 2) {
+        load(t + 1, B);
+        const float o0 = step(A);
+        mine = q == t ? o0 : mine;
+        if (t + 2 < DR_TB) load(t + 2, A);
+        const float o1 = step(B);
+        mine = q == t + 1 ? o1 : mine;
       }
-      dot = dr_sum16(dot);                            // u^T S of this column
-      const float v = s_v[t][grp];
-#pragma unroll
-      for (int j = 0; j < J; ++j) {
-        float au[VEC], k[VEC];
-        dr_read<VEC>(&s_w[t][16 * VEC * j + VEC * q], x[j]);
-        dr_read<VEC>(&s_au[t][16 * VEC * j + VEC * q], au);
-        dr_read<VEC>(&s_k[t][16 * VEC * j + VEC * q], k);
-#pragma unroll
-        for (int e = 0; e < VEC; ++e) {
-          const float add = __builtin_fmaf(k[e], v, -(au[e] * dot));
-          S[j][e] = __builtin_fmaf(x[j][e], S[j][e], add);
-        }
+    } else {
+      for (int t = 0; t < nt; ++t) {
+        const float o = step(A);
+        mine = q == t ? o : mine;
+        if (t + 1 < nt) load(t + 1, A);
       }
-      float o = 0.f;
-#pragma unroll
-      for (int j = 0; j < J; ++j) {
-        dr_read<VEC>(&s_r[t][16 * VEC * j + VEC * q], x[j]);
-#pragma unroll
-        for (int e = 0; e < VEC; ++e) o = __builtin_fmaf(x[j][e], S[j][e], o);
-      }
-      o = dr_sum16(o);
-      mine = q == t ? o : mine;
     }
     if (col_ok && q < nt) out[((size_t)(first + t0 + q) * nh + hd) * dim + col] = mine;
   }
 #pragma unroll
-  for (int j = 0; j < J; ++j)
+  for (int j = 0; j < J; ++j) {
+    const int n = 16 * VEC * j + VEC * q;
+    if (VEC == L && L == 4) {
+      if (col_ok && n < dim) *reinterpret_cast<float4*>(st + n) = make_float4(S[j][0], S[j][1 % VEC], S[j][2 % VEC], S[j][3 % VEC]);
+    } else {
 #pragma unroll
-    for (int e = 0; e < VEC; ++e) {
-      const int n = 16 * VEC * j + VEC * q + e;
-      if (col_ok && n < dim) st[n] = S[j][e];
+      for (int e = 0; e < VEC; ++e)
+        if (col_ok && n + e < dim) st[n + e] = S[j][e];
     }
+  }
 }
 
 // Floats a request's slot holds for one layer run.
@@ -255,10 +330,21 @@ extern "C" int ia_delta_scan(const void* proj, int code, int proj_stride, int r_
   const int groups = (dim + DR_COLS - 1) / DR_COLS;
   if (dim > 256 || B > 65535 || groups > 65535) return IA_ERR_UNSUPPORTED;
   const dim3 grid((unsigned)nh, (unsigned)B, (unsigned)groups);
-#define IA_DR(T, V, JJ)                                                                                                  \
-  delta_scan_kernel<T, V, JJ><<<grid, 64 * DR_WAVES, 0, stream>>>((const T*)proj, proj_stride, r_col, k_col, v_col, w, a, \
-                                                                  inv, state, state_stride, out, seq_starts,             \
-                                                                  state_slots, nh, dim)
+  // in fours where every address that a piece of four values is read from is a multiple of its size
+  const size_t el = code == IA_F32 ? 4 : 2;
+  const bool fours = ((dim | proj_stride | r_col | k_col) & 3) == 0 && ((uintptr_t)proj % (4 * el)) == 0 && (state_stride & 3) == 0 &&
+                     (((uintptr_t)w | (uintptr_t)a | (uintptr_t)state) & 15) == 0;
+#define IA_DR(T, V, JJ)                                                                                                    \
+  do {                                                                                                                     \
+    if (fours)                                                                                                             \
+      delta_scan_kernel<T, V, JJ, 4><<<grid, 64 * DR_WAVES, 0, stream>>>((const T*)proj, proj_stride, r_col, k_col, v_col, \
+                                                                         w, a, inv, state, state_stride, out, seq_starts,  \
+                                                                         state_slots, nh, dim);                            \
+    else                                                                                                                   \
+      delta_scan_kernel<T, V, JJ, 1><<<grid, 64 * DR_WAVES, 0, stream>>>((const T*)proj, proj_stride, r_col, k_col, v_col, \
+                                                                         w, a, inv, state, state_stride, out, seq_starts,  \
+                                                                         state_slots, nh, dim);                            \
+  } while (0)
 #define IA_DR_D(T)                         \
   do {                                     \
     if (dim <= 16) IA_DR(T, 1, 1);         \

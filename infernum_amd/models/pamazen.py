@@ -8,8 +8,6 @@ only, identity experts and a gated shared expert, or no feed-forward; capped log
 """
 from __future__ import annotations
 
-from typing import Optional
-
 from ..config.pamazen import PAMAZEN_MODEL_TYPE, AttentionConfig, PamazenConfig
 from ..config.registry import register_architecture
 from ..parts.base import LayerSpec, ModelSpec, PartSpec, ScheduleEntry
@@ -23,8 +21,7 @@ def _rope(rot, head_dim: int) -> dict:
                                        "pairing": "neighbours"}}
 
 
-def pamazen_model_spec(cfg: PamazenConfig, init_std: float = 0.05, decay_rank: Optional[int] = None) -> ModelSpec:
-    """``decay_rank``: the middle of the delta rule's decay logits, for random weights (a file's tensors have it)."""
+def pamazen_model_spec(cfg: PamazenConfig, init_std: float = 0.05) -> ModelSpec:
     W, last = cfg.width, len(cfg.layers) - 1
 
     def norm(prefix: str) -> PartSpec:
@@ -56,7 +53,7 @@ def pamazen_model_spec(cfg: PamazenConfig, init_std: float = 0.05, decay_rank: O
                     "init_std": init_std}},
                 "right": {"kind": "delta_rule", "scale": m.right_scale, "params": {
                     "hidden_size": W, "num_heads": right.heads, "head_dim": right.dim, "norm_eps": cfg.norm_eps,
-                    "decay_rank": decay_rank, "init_std": init_std}}}}, p + "mix.")
+                    "decay_rank": right.rank, "init_std": init_std}}}}, p + "mix.")
         ff, f = None, layer.mlp
         extra = {"mixer_hyper": hyper(p + "hc1.", i == last and f is None)}
         if f is not None:

@@ -99,7 +99,7 @@ def attention_mixer(a: torch.Tensor, w: Mapping[str, torch.Tensor], p: str, m: M
     H, G, d, dv = m["heads"], m["kv_heads"], m["dim"], m["vdim"]
     q = _r(a @ w[p + "q"].T, round_to).view(T, H, d)
     k = _r(a @ w[p + "k"].T, round_to).view(T, G, d)
-    v = _r(a @ w[p + "v"].T, round_to).view(T, G, dv)
+    v = _r(a @ w[p + "v"].T, round_to)
     rot = m.get("rot")
     if rot and rot["dims"]:
         ang = rotation_angles(torch.arange(T), rot["dims"], float(rot["base"]), float((rot.get("scaling") or {}).get("factor", 1.0)))
@@ -110,7 +110,7 @@ def attention_mixer(a: torch.Tensor, w: Mapping[str, torch.Tensor], p: str, m: M
             v = _r((1.0 - lam) * v + lam * shared["v_first"], round_to)
         else:
             shared["v_first"] = v
-    o = grouped_attention(q, k, v, m["scale"], seen_keys(T), torch.zeros(H, dtype=F64))
+    o = grouped_attention(q, k, v.view(T, G, dv), m["scale"], seen_keys(T), torch.zeros(H, dtype=F64))
     return _r(o, round_to) @ w[p + "o"].T
 
 
@@ -125,8 +125,9 @@ def window_attention(a: torch.Tensor, w: Mapping[str, torch.Tensor], p: str, m: 
     v = _r(k * scale, round_to)
     q = _r(unit_rms(q, eps) * w[p + "q.norm"], round_to)
     k = _r(unit_rms(k, eps) * w[p + "k.norm"], round_to)
-    o = grouped_attention(q, k, v, m["scale"], seen_keys(T, int(m["mask"]["size"]), int(m["mask"]["keep_first"])),
-                          w[p + "sink"], float(m["softcap"]))
+    mask = m.get("mask")
+    seen = seen_keys(T, int(mask["size"]), int(mask["keep_first"])) if mask else seen_keys(T)
+    o = grouped_attention(q, k, v, m["scale"], seen, w[p + "sink"], float(m["softcap"]) if m.get("softcap") else None)
     return _r(o, round_to) @ w[p + "o"].T
 
 
