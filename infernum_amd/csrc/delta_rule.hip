@@ -125,6 +125,14 @@ __device__ __forceinline__ void dr_read(const float* p, float (&v)[VEC]) {
   }
 }
 
+// A barrier for what goes through LDS alone: __syncthreads() would also wait for the results' stores on their way to
+// memory, which no other thread reads.
+__device__ __forceinline__ void dr_barrier() {
+  asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+  __builtin_amdgcn_s_barrier();
+  asm volatile("" ::: "memory");
+}
+
 // The vectors of one token as a lane needs them.
 template <int VEC, int J>
 struct DrToken {
@@ -193,7 +201,6 @@ __global__ __launch_bounds__(64 * DR_WAVES) void delta_scan_kernel(
     const int t = tid / DR_COLS, c = c0 + tid % DR_COLS;
     fv = proj[(size_t)(first + (t0 + t < count ? t0 + t : count - 1)) * proj_stride + v_col + hd * dim + (c < dim ? c : 0)];
   };
-  fetch(0);
   float S[J][VEC];
 #pragma unroll
   for (int j = 0; j < J; ++j)
@@ -210,6 +217,13 @@ __global__ __launch_bounds__(64 * DR_WAVES) void delta_scan_kernel(
         if (col_ok && n + e < dim) S[j][e] = st[n + e];
     }
   }
+  fetch(0);
+  // the state is in its registers from here on: a use of it inside the loop must not be taken for one that waits for a
+  // load, which would make every turn wait for the next tokens' vectors as well
+#pragma unroll
+  for (int j = 0; j < J; ++j)
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) asm volatile("" : "+v"(S[j][e]));
   DrToken<VEC, J> A, B;
   auto load = [&](int t, DrToken<VEC, J>& X) {
 #pragma unroll
@@ -251,7 +265,7 @@ __global__ __launch_bounds__(64 * DR_WAVES) void delta_scan_kernel(
   };
   for (int t0 = 0; t0 < count; t0 += DR_TB) {
     const int nt = count - t0 < DR_TB ? count - t0 : DR_TB;
-    __syncthreads();                                  // the tokens before are read to their end
+    dr_barrier();                                     // the tokens before are read to their end
 #pragma unroll
     for (int x = 0; x < PER; ++x) {
       const int idx = tid + x * NT, t = idx / (P / L), n = (idx - t * (P / L)) * L;
@@ -278,7 +292,7 @@ __global__ __launch_bounds__(64 * DR_WAVES) void delta_scan_kernel(
       }
     }
     if (tid < DR_TB * DR_COLS) s_v[tid / DR_COLS][tid % DR_COLS] = c0 + tid % DR_COLS < dim ? to_float(fv) : 0.f;
-    __syncthreads();
+    dr_barrier();
     if (t0 + DR_TB < count) fetch(t0 + DR_TB);
     float mine = 0.f;                                 // lane q keeps token q's result of the column
     load(0, A);

@@ -407,20 +407,22 @@ __device__ __forceinline__ float moe_act(float z, int act) {
   return z;
 }
 
+// PL: experts a lane holds (lane, lane + 64, ...)
+template <int PL>
 __global__ __launch_bounds__(256) void router_softmax_topk_kernel(const float* __restrict__ logits,
                                                                   const void* __restrict__ corr, int corr_dtype,
                                                                   int* __restrict__ ids, float* __restrict__ weights,
                                                                   int N, int E, int top, int z_stride, int groups,
                                                                   int keep, int renorm) {
-  __shared__ float s_v[4][64 * RT_PER_LANE];       // a wave's choice scores, then (in place) its groups' scores
+  __shared__ float s_v[4][64 * PL];       // a wave's choice scores, then (in place) its groups' scores
   const int n = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
   if (n >= N) return;
   const float* z = logits + (size_t)n * z_stride;
-  float s[RT_PER_LANE], v[RT_PER_LANE];
+  float s[PL], v[PL];
   unsigned taken = 0u;
   float zmax = -INFINITY;
 #pragma unroll
-  for (int c = 0; c < RT_PER_LANE; ++c) {
+  for (int c = 0; c < PL; ++c) {
     const int e = lane + 64 * c;
     s[c] = e < E ? z[e] : -INFINITY;
     zmax = fmaxf(zmax, s[c]);
@@ -429,14 +431,14 @@ __global__ __launch_bounds__(256) void router_softmax_topk_kernel(const float* _
   zmax = wave_max(zmax);
   float total = 0.f;
 #pragma unroll
-  for (int c = 0; c < RT_PER_LANE; ++c) {
+  for (int c = 0; c < PL; ++c) {
     s[c] = (lane + 64 * c) < E ? expf(s[c] - zmax) : 0.f;
     total += s[c];
   }
   total = wave_sum(total);
   const float inv_total = 1.0f / total;
 #pragma unroll
-  for (int c = 0; c < RT_PER_LANE; ++c) {
+  for (int c = 0; c < PL; ++c) {
     const int e = lane + 64 * c;
     s[c] *= inv_total;
     v[c] = e < E ? s[c] + (corr ? load_as_float(corr, corr_dtype, e) : 0.f) : -INFINITY;
@@ -446,11 +448,11 @@ __global__ __launch_bounds__(256) void router_softmax_topk_kernel(const float* _
     volatile float* mine = s_v[threadIdx.x >> 6];
     const int size = E / groups;
 #pragma unroll
-    for (int c = 0; c < RT_PER_LANE; ++c)
+    for (int c = 0; c < PL; ++c)
       if (lane + 64 * c < E) mine[lane + 64 * c] = (v[c] == v[c]) ? v[c] : -INFINITY;
-    float gs[RT_PER_LANE];                        // this lane's groups: lane, lane + 64, ...
+    float gs[PL];                        // this lane's groups: lane, lane + 64, ...
 #pragma unroll
-    for (int c = 0; c < RT_PER_LANE; ++c) {
+    for (int c = 0; c < PL; ++c) {
       gs[c] = -INFINITY;
       const int g = lane + 64 * c;
       if (g < groups)
@@ -458,11 +460,11 @@ __global__ __launch_bounds__(256) void router_softmax_topk_kernel(const float* _
     }
     __builtin_amdgcn_wave_barrier();
 #pragma unroll
-    for (int c = 0; c < RT_PER_LANE; ++c)
+    for (int c = 0; c < PL; ++c)
       if (lane + 64 * c < groups) mine[lane + 64 * c] = gs[c];
     __builtin_amdgcn_wave_barrier();
 #pragma unroll
-    for (int c = 0; c < RT_PER_LANE; ++c) {
+    for (int c = 0; c < PL; ++c) {
       const int e = lane + 64 * c;
       if (e >= E) continue;
       const int g = e / size;
@@ -477,7 +479,7 @@ __global__ __launch_bounds__(256) void router_softmax_topk_kernel(const float* _
     float best_v = -INFINITY, best_s = 0.f;
     int best_e = 0x7fffffff;
 #pragma unroll
-    for (int c = 0; c < RT_PER_LANE; ++c) {
+    for (int c = 0; c < PL; ++c) {
       const bool free_ = !((taken >> c) & 1u);
       const float x = (v[c] == v[c]) ? v[c] : -INFINITY;
       if (free_ && (best_e == 0x7fffffff || x > best_v)) { best_v = x; best_e = lane + 64 * c; best_s = s[c]; }
@@ -511,8 +513,13 @@ extern "C" int ia_router_softmax_topk(const float* logits, const void* corr, int
       top > keep * (E / groups) || !logits || !ids || !weights) return IA_ERR_BAD_ARG;
   if (E > 64 * RT_PER_LANE) return IA_ERR_UNSUPPORTED;
   if (N == 0) return IA_OK;
-  router_softmax_topk_kernel<<<(N + 3) / 4, 256, 0, stream>>>(logits, corr, corr_dtype, ids, weights, N, E, top, z_stride, groups,
-                                                                keep, renorm);
+#define IA_RT(PL)                                                                                                        \
+  router_softmax_topk_kernel<PL><<<(N + 3) / 4, 256, 0, stream>>>(logits, corr, corr_dtype, ids, weights, N, E, top, z_stride, \
+                                                                  groups, keep, renorm)
+  if (E <= 64) IA_RT(1);
+  else if (E <= 256) IA_RT(4);
+  else IA_RT(RT_PER_LANE);
+#undef IA_RT
   IA_LAUNCH_CHECK();
   return IA_OK;
 }
@@ -597,24 +604,49 @@ extern "C" int ia_moe_up(const void* x, const void* Wu, void* y, const int* offs
 //                   its input): parts[choice, token, :] = weight * x[token, :]; and for every token, with `shared`: its
 //                   result ([splits, shared_rows, W], added in the order of the parts) times sigmoid(gate[token]) into
 //                   parts[top, token, :], the part after the choices'.
-template <typename T, typename TS>
+// grid (N, top (+ 1), pieces of 256 V values of a row); V 4: rows of a multiple of four values, 16 (or 8) bytes an access.
+__device__ __forceinline__ void mx_load(const float* p, float (&v)[1]) { v[0] = p[0]; }
+__device__ __forceinline__ void mx_load(const bf16_t* p, float (&v)[1]) { v[0] = to_float(p[0]); }
+__device__ __forceinline__ void mx_load(const float* p, float (&v)[4]) {
+  const float4 t = *reinterpret_cast<const float4*>(p);
+  v[0] = t.x; v[1] = t.y; v[2] = t.z; v[3] = t.w;
+}
+__device__ __forceinline__ void mx_load(const bf16_t* p, float (&v)[4]) {
+  const uint2 t = *reinterpret_cast<const uint2*>(p);
+  v[0] = __uint_as_float(t.x << 16); v[1] = __uint_as_float(t.x & 0xffff0000u);
+  v[2] = __uint_as_float(t.y << 16); v[3] = __uint_as_float(t.y & 0xffff0000u);
+}
+__device__ __forceinline__ void mx_store(float* p, const float (&v)[1], float f) { p[0] = f * v[0]; }
+__device__ __forceinline__ void mx_store(float* p, const float (&v)[4], float f) {
+  *reinterpret_cast<float4*>(p) = make_float4(f * v[0], f * v[1], f * v[2], f * v[3]);
+}
+
+template <typename T, typename TS, int V>
 __global__ __launch_bounds__(256) void moe_extras_kernel(const T* __restrict__ x, const int* __restrict__ ids,
                                                          const float* __restrict__ weights, float* __restrict__ parts,
                                                          const TS* __restrict__ shared, int splits, size_t split_stride,
                                                          const float* __restrict__ gate, int gate_stride, int N, int E,
                                                          int top, int W) {
-  const int n = blockIdx.x, choice = blockIdx.y;
-  float* o = parts + ((size_t)choice * N + n) * W;
+  const int n = blockIdx.x, choice = blockIdx.y, i = (blockIdx.z * 256 + threadIdx.x) * V;
+  float* o = parts + ((size_t)choice * N + n) * W + i;
+  float v[V];
   if (choice == top) {
-    const float g = gate ? 1.0f / (1.0f + expf(-gate[(size_t)n * gate_stride])) : 1.0f;
-    const TS* s = shared + (size_t)n * W;
-    for (int i = threadIdx.x; i < W; i += 256) o[i] = g * load_split_sum(s + i, splits, split_stride);
+    if (i >= W) return;
+    const TS* s = shared + (size_t)n * W + i;
+    mx_load(s, v);
+#pragma unroll 4
+    for (int k = 1; k < splits; ++k) {                 // the parts in the order of their index
+      float p[V];
+      mx_load(s + k * split_stride, p);
+#pragma unroll
+      for (int e = 0; e < V; ++e) v[e] += p[e];
+    }
+    mx_store(o, v, gate ? 1.0f / (1.0f + expf(-gate[(size_t)n * gate_stride])) : 1.0f);
     return;
   }
-  if (ids[(size_t)n * top + choice] < E) return;
-  const float wt = weights[(size_t)n * top + choice];
-  const T* xr = x + (size_t)n * W;
-  for (int i = threadIdx.x; i < W; i += 256) o[i] = wt * to_float(xr[i]);
+  if (ids[(size_t)n * top + choice] < E || i >= W) return;
+  mx_load(x + (size_t)n * W + i, v);
+  mx_store(o, v, weights[(size_t)n * top + choice]);
 }
 
 // parts: fp32 [top (+ 1 with shared), N, W]; shared (nullable) of shared_dtype; gate (nullable): fp32, token n's logit
@@ -627,9 +659,17 @@ extern "C" int ia_moe_extras(const void* x, int dtype, const int* ids, const flo
       (shared && shared_dtype != IA_F32 && shared_dtype != IA_BF16))
     return IA_ERR_BAD_ARG;
   if (N == 0) return IA_OK;
-  const dim3 grid(N, top + (shared ? 1 : 0));
+  const bool vec = (W & 3) == 0 && (((uintptr_t)x | (uintptr_t)parts | (uintptr_t)shared) & 15) == 0;
+  const dim3 grid(N, top + (shared ? 1 : 0), (W + (vec ? 1024 : 256) - 1) / (vec ? 1024 : 256));
   const size_t stride = (size_t)shared_rows * W;
-#define IA_MX(T, TS)                                                                                                  moe_extras_kernel<T, TS><<<grid, 256, 0, stream>>>((const T*)x, ids, weights, parts, (const TS*)shared, splits, stride,                                                      gate, gate_stride, N, E, top, W)
+#define IA_MX_V(T, TS, V)                                                                                                    \
+  moe_extras_kernel<T, TS, V><<<grid, 256, 0, stream>>>((const T*)x, ids, weights, parts, (const TS*)shared, splits, stride, \
+                                                        gate, gate_stride, N, E, top, W)
+#define IA_MX(T, TS)                \
+  do {                              \
+    if (vec) IA_MX_V(T, TS, 4);     \
+    else IA_MX_V(T, TS, 1);         \
+  } while (0)
   const bool sf = !shared || shared_dtype == IA_F32;
   if (dtype == IA_F32) {
     if (sf) IA_MX(float, float);
@@ -637,6 +677,7 @@ extern "C" int ia_moe_extras(const void* x, int dtype, const int* ids, const flo
   } else if (sf) IA_MX(bf16_t, float);
   else IA_MX(bf16_t, bf16_t);
 #undef IA_MX
+#undef IA_MX_V
   IA_LAUNCH_CHECK();
   return IA_OK;
 }
