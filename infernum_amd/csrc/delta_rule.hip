@@ -10,8 +10,9 @@
 //   ia_delta_prepare     per token and head: z <- w in place, a, and 1 / sqrt(sum k^2 + eps); all fp32.
 //   ia_delta_scan        the recurrence token after token for the rows of every request of a step, from the request's
 //                        state slot, which it leaves moved on.
+//   ia_delta_chunked     the same for portions of prompts in chunks of DC_T tokens as matrix products (below).
 //
-// A column of S needs nothing of the other columns, so a wave takes four columns: sixteen lanes share a column's
+// Token after token: a column of S needs nothing of the other columns, so a wave takes four columns: sixteen lanes share a column's
 // channels (in registers, a lane dim / 16 of them), the sums over the channels are four rotations within the sixteen
 // lanes (every lane ends with the same bits), and a token costs no barrier and no trip through LDS but the reads of
 // the token's vectors, which DR_WAVES waves of a workgroup bring into LDS together, DR_TB tokens at a time, the next
@@ -19,6 +20,20 @@
 // steps and whatever else the step holds.
 //
 // A head's state is kept column by column: slot[head][column][channel].
+//
+// In chunks: with W_t the product of a chunk's decays up to its token t, S_t = diag(W_t) Z_t turns the recurrence into
+//     Z_t = Z_(t-1) - b_t (c_t^T Z_(t-1)) + d_t v_t^T,      b_t = a_t u_t / W_t,  c_t = u_t W_(t-1),  d_t = k_t / W_t,
+// so that with S_0 the state before the chunk and the 16 x 16 matrices A = (c_t . b_s), B = (c_t . d_s) below the diagonal
+// and F = (e_t . b_s), G = (e_t . d_s) up to it, e_t = r_t W_t, everything the chunk's tokens take from each other is known
+// without the state:
+//     p = C S_0 + B' V,   C = (I + A)^-1 c,  B' = (I + A)^-1 B;      o = E S_0 + D V,   E = e - F C,  D = G - F B';
+//     S_end = diag(W_T) S_0 - (b W_T)^T p + (d W_T)^T V.
+// One kernel makes C, E, B', D, -b W_T, d W_T and W_T of every chunk and head side by side; a second walks a request's
+// chunks, sixteen columns of a head a workgroup, its waves a tile of sixteen channels (or two) each, on the matrix cores in
+// fp32 (v_mfma_f32_16x16x4_f32).  A tile of the state stays in the accumulators: an accumulator's register r of lane
+// (q, j) is the state's channel 4 q + r, column j, which is what the second operand wants at a step whose four channels are
+// r, 4 + r, 8 + r, 12 + r, and the first operand's records are laid out so that a lane's values of the four steps are 16
+// bytes.  The chunks' decays stay above exp(-DC_T decay_scale), so that 1 / W is harmless.  All of it fp32.
 #include "common.h"
 
 #define DR_TB 8          // tokens whose vectors are staged together
@@ -377,7 +392,313 @@ extern "C" int ia_delta_scan(const void* proj, int code, int proj_stride, int r_
   return IA_OK;
 }
 
+// ------------------------------------------------------------------------------------------ in chunks
+#define DC_T 16          // tokens of a chunk
+#define DC_TILE 64       // rows of a tile of the host's list: four chunks
+#define DC_MAX_WAVES 8
+
+typedef float dc_f32x4 __attribute__((ext_vector_type(4)));
+
+// A record (one chunk of one head), in floats; `tiles` tiles of 16 channels: C and E [tile][token][16 channels], -b W_T and
+// d W_T [tile][channel][16 tokens], W_T [tile][16], B' and D [token][16 tokens].
+__host__ __device__ inline long dc_record_floats(int tiles) { return (long)tiles * (4 * 256 + 16) + 2 * 256; }
+
+// The first chunk's record of request s: chunks are counted in the order of the requests from first_request on, four to
+// every 64 rows begun.
+__device__ __forceinline__ int dc_first_chunk(const int* __restrict__ seq_starts, int first_request, int s) {
+  int tiles = 0;
+  for (int r = first_request; r < s; ++r) tiles += (seq_starts[r + 1] - seq_starts[r] + DC_TILE - 1) / DC_TILE;
+  return tiles * (DC_TILE / DC_T);
+}
+
+// grid (tiles x 4, heads), blockDim a multiple of 64: a thread a channel.
+template <typename T>
+__global__ __launch_bounds__(256, 3) void delta_chunk_prepare_kernel(
+    const T* __restrict__ proj, int proj_stride, int r_col, int k_col, const float* __restrict__ w, const float* __restrict__ a,
+    const float* __restrict__ inv, const int* __restrict__ seq_starts, const int* __restrict__ tiles_list, int first_request,
+    float* __restrict__ records, int nh, int dim) {
+  extern __shared__ __attribute__((aligned(16))) float lds[];
+  const int tiles = (dim + 15) / 16, DP = tiles * 16, LS = DP + 4;      // LS: a row in LDS
+  float* s_c = lds;
+  float* s_b = s_c + DC_T * LS;
+  float* s_d = s_b + DC_T * LS;
+  float* s_e = s_d + DC_T * LS;
+  float (*s_m)[16][16] = reinterpret_cast<float (*)[16][16]>(s_e + DC_T * LS);      // A, B, F, G
+  const int sub = blockIdx.x & 3, tile = blockIdx.x >> 2, hd = blockIdx.y;
+  const int s = tiles_list[2 * tile], row0 = tiles_list[2 * tile + 1] + sub * DC_T;
+  const int first = seq_starts[s], qlen = seq_starts[s + 1] - first;
+  if (row0 >= qlen) return;
+  const int count = qlen - row0 < DC_T ? qlen - row0 : DC_T;
+  const int chunk = dc_first_chunk(seq_starts, first_request, s) + row0 / DC_T;
+  float* rec = records + ((size_t)chunk * nh + hd) * dc_record_floats(tiles);
+  float* rec_c = rec;
+  float* rec_e = rec_c + tiles * 256;
+  float* rec_b = rec_e + tiles * 256;
+  float* rec_d = rec_b + tiles * 256;
+  float* rec_w = rec_d + tiles * 256;
+  float* rec_bp = rec_w + tiles * 16;
+  float* rec_dp = rec_bp + 256;
+  const int tid = threadIdx.x, nt = blockDim.x;
+  for (int n = tid; n < DP; n += nt) {
+    const bool real = n < dim;
+    const int nc = real ? n : 0;
+    float fw[DC_T], fa[DC_T], fi[DC_T];
+    T fk[DC_T], fr[DC_T];
+#pragma unroll
+    for (int t = 0; t < DC_T; ++t) {                  // rows past the end stand in for none: their values are not used
+      const size_t row = (size_t)(first + row0 + (t < count ? t : count - 1)), at = (row * nh + hd) * dim + nc;
+      fw[t] = w[at];
+      fa[t] = a[at];
+      fk[t] = proj[row * proj_stride + k_col + hd * dim + nc];
+      fr[t] = proj[row * proj_stride + r_col + hd * dim + nc];
+      fi[t] = inv[row * nh + hd];
+    }
+    float W = 1.f, b[DC_T], d[DC_T];
+#pragma unroll
+    for (int t = 0; t < DC_T; ++t) {
+      const bool ok = real && t < count;
+      const float k = ok ? to_float(fk[t]) : 0.f, u = k * fi[t];
+      s_c[t * LS + n] = ok ? u * W : 0.f;
+      W = ok ? W * fw[t] : W;
+      const float iw = 1.0f / W;
+      b[t] = ok ? fa[t] * u * iw : 0.f;
+      d[t] = k * iw;
+      s_b[t * LS + n] = b[t];
+      s_d[t * LS + n] = d[t];
+      s_e[t * LS + n] = ok ? to_float(fr[t]) * W : 0.f;
+    }
+    float* ob = rec_b + n * 16;                       // [tile][channel][token]: a channel's sixteen tokens side by side
+    float* od = rec_d + n * 16;
+#pragma unroll
+    for (int t = 0; t < DC_T; t += 4) {
+      *reinterpret_cast<float4*>(ob + t) = make_float4(-b[t] * W, -b[t + 1] * W, -b[t + 2] * W, -b[t + 3] * W);
+      *reinterpret_cast<float4*>(od + t) = make_float4(d[t] * W, d[t + 1] * W, d[t + 2] * W, d[t + 3] * W);
+    }
+    rec_w[n] = real ? W : 0.f;
+  }
+  __syncthreads();
+  // ---- A, B, F, G: rows of c or e against rows of b or d
+  const int lane = tid & 63, i = lane & 15, q = lane >> 4;
+  for (int m = tid >> 6; m < 4; m += nt >> 6) {
+    const float* x = (m < 2 ? s_c : s_e) + i * LS + 4 * q;
+    const float* y = ((m & 1) ? s_d : s_b) + i * LS + 4 * q;
+    dc_f32x4 acc = (dc_f32x4){0.f, 0.f, 0.f, 0.f};
+    for (int t = 0; t < tiles; ++t) {
+      const float4 xv = *reinterpret_cast<const float4*>(x + 16 * t), yv = *reinterpret_cast<const float4*>(y + 16 * t);
+      acc = __builtin_amdgcn_mfma_f32_16x16x4f32(xv.x, yv.x, acc, 0, 0, 0);
+      acc = __builtin_amdgcn_mfma_f32_16x16x4f32(xv.y, yv.y, acc, 0, 0, 0);
+      acc = __builtin_amdgcn_mfma_f32_16x16x4f32(xv.z, yv.z, acc, 0, 0, 0);
+      acc = __builtin_amdgcn_mfma_f32_16x16x4f32(xv.w, yv.w, acc, 0, 0, 0);
+    }
+#pragma unroll
+    for (int r = 0; r < 4; ++r) s_m[m][4 * q + r][i] = (i < 4 * q + r || (m >= 2 && i == 4 * q + r)) ? acc[r] : 0.f;
+  }
+  __syncthreads();
+  // ---- a thread a column of [c | B] and of [e | G]: forward substitution, then the product with F
+  for (int n = tid; n < DP + 16; n += nt) {
+    const bool ch = n < DP;
+    float y[DC_T];
+#pragma unroll
+    for (int t = 0; t < DC_T; ++t) {
+      float v = ch ? s_c[t * LS + n] : s_m[1][t][n - DP];
+#pragma unroll
+      for (int x = 0; x < t; ++x) v = __builtin_fmaf(-s_m[0][t][x], y[x], v);
+      y[t] = v;
+    }
+    float* o1 = ch ? rec_c + (n >> 4) * 256 + (n & 15) : rec_bp + (n - DP);       // [tile][token][channel]; [token][token]
+    float* o2 = ch ? rec_e + (n >> 4) * 256 + (n & 15) : rec_dp + (n - DP);
+#pragma unroll
+    for (int t = 0; t < DC_T; ++t) {
+      float v = ch ? s_e[t * LS + n] : s_m[3][t][n - DP];
+#pragma unroll
+      for (int x = 0; x <= t; ++x) v = __builtin_fmaf(-s_m[2][t][x], y[x], v);
+      o1[t * 16] = y[t];
+      o2[t * 16] = v;
+    }
+  }
+}
+
+// What a wave needs of one chunk.
+template <typename T, int TPW>
+struct DcOps {
+  dc_f32x4 c[TPW], e[TPW], b[TPW], d[TPW], w[TPW], bp, dp;
+  T v[4];
+};
+
+// grid (heads, requests, slices of 16 columns), blockDim 64 x waves; wave x takes the tiles of channels x TPW ...
+template <typename T, int TPW>
+__global__ __launch_bounds__(64 * DC_MAX_WAVES) void delta_chunk_scan_kernel(
+    const T* __restrict__ proj, int proj_stride, int v_col, float* __restrict__ state, long state_stride,
+    float* __restrict__ out, const int* __restrict__ seq_starts, const int* __restrict__ state_slots, int first_request,
+    const float* __restrict__ records, int nh, int dim) {
+  __shared__ dc_f32x4 part[2][2][DC_MAX_WAVES][64];
+  const int hd = blockIdx.x, s = first_request + blockIdx.y, c0 = blockIdx.z * 16;
+  const int first = seq_starts[s], count = seq_starts[s + 1] - first;
+  if (count <= 0) return;
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, nw = blockDim.x >> 6, j = lane & 15, q = lane >> 4;
+  const int tiles = (dim + 15) / 16, col = c0 + j;
+  const bool col_ok = col < dim;
+  const size_t rec_floats = (size_t)dc_record_floats(tiles);
+  const float* rec0 = records + ((size_t)dc_first_chunk(seq_starts, first_request, s) * nh + hd) * rec_floats;
+  float* st = state + (size_t)state_slots[s] * state_stride + ((size_t)hd * dim + (col_ok ? col : 0)) * dim;
+  const bool fours = (dim & 3) == 0;
+  int tile[TPW];
+  dc_f32x4 S[TPW];
+#pragma unroll
+  for (int x = 0; x < TPW; ++x) {
+    tile[x] = wave * TPW + x;
+    S[x] = (dc_f32x4){0.f, 0.f, 0.f, 0.f};
+    const int n = tile[x] * 16 + 4 * q;
+    if (fours) {
+      if (col_ok && n < dim) S[x] = *reinterpret_cast<const dc_f32x4*>(st + n);
+    } else {
+#pragma unroll
+      for (int r = 0; r < 4; ++r)
+        if (col_ok && n + r < dim) S[x][r] = st[n + r];
+    }
+  }
+  const int chunks = (count + DC_T - 1) / DC_T;
+  const T* vp = proj + v_col + hd * dim + (col_ok ? col : 0);
+  auto load = [&](int c, DcOps<T, TPW>& O) {
+    const float* rec = rec0 + (size_t)c * nh * rec_floats;
+    const int at = j * 16 + 4 * q;
+#pragma unroll
+    for (int x = 0; x < TPW; ++x) {
+      const int t = tile[x] < tiles ? tile[x] : tiles - 1;            // a tile past the head's last: its state stays zero
+      O.c[x] = *reinterpret_cast<const dc_f32x4*>(rec + (size_t)t * 256 + at);
+      O.e[x] = *reinterpret_cast<const dc_f32x4*>(rec + (size_t)(tiles + t) * 256 + at);
+      O.b[x] = *reinterpret_cast<const dc_f32x4*>(rec + (size_t)(2 * tiles + t) * 256 + at);
+      O.d[x] = *reinterpret_cast<const dc_f32x4*>(rec + (size_t)(3 * tiles + t) * 256 + at);
+      O.w[x] = *reinterpret_cast<const dc_f32x4*>(rec + (size_t)4 * tiles * 256 + t * 16 + 4 * q);
+    }
+    const float* sq = rec + (size_t)tiles * (4 * 256 + 16);
+    O.bp = *reinterpret_cast<const dc_f32x4*>(sq + at);
+    O.dp = *reinterpret_cast<const dc_f32x4*>(sq + 256 + at);
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int t = c * DC_T + 4 * q + r;                             // rows past the end meet zeros in every operand
+      O.v[r] = vp[(size_t)(first + (t < count ? t : count - 1)) * proj_stride];
+    }
+  };
+  auto work = [&](int c, const DcOps<T, TPW>& O, int buf) {
+    float v[4];
+#pragma unroll
+    for (int r = 0; r < 4; ++r) v[r] = to_float(O.v[r]);
+    dc_f32x4 P = (dc_f32x4){0.f, 0.f, 0.f, 0.f}, Y = (dc_f32x4){0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int x = 0; x < TPW; ++x)
+      if (tile[x] < tiles) {
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          P = __builtin_amdgcn_mfma_f32_16x16x4f32(O.c[x][r], S[x][r], P, 0, 0, 0);
+          Y = __builtin_amdgcn_mfma_f32_16x16x4f32(O.e[x][r], S[x][r], Y, 0, 0, 0);
+        }
+      }
+    if (wave == 0) {
+#pragma unroll
+      for (int r = 0; r < 4; ++r) P = __builtin_amdgcn_mfma_f32_16x16x4f32(O.bp[r], v[r], P, 0, 0, 0);
+    }
+    if (wave == nw - 1) {
+#pragma unroll
+      for (int r = 0; r < 4; ++r) Y = __builtin_amdgcn_mfma_f32_16x16x4f32(O.dp[r], v[r], Y, 0, 0, 0);
+    }
+    part[buf][0][wave][lane] = P;
+    part[buf][1][wave][lane] = Y;
+    dr_barrier();                                     // the other buffer's readers are past it: they met at the chunk before
+    P = part[buf][0][0][lane];
+    for (int x = 1; x < nw; ++x) P += part[buf][0][x][lane];
+#pragma unroll
+    for (int x = 0; x < TPW; ++x)
+      if (tile[x] < tiles) {
+        S[x] *= O.w[x];
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          S[x] = __builtin_amdgcn_mfma_f32_16x16x4f32(O.b[x][r], P[r], S[x], 0, 0, 0);
+          S[x] = __builtin_amdgcn_mfma_f32_16x16x4f32(O.d[x][r], v[r], S[x], 0, 0, 0);
+        }
+      }
+    if (wave == c % nw) {
+      Y = part[buf][1][0][lane];
+      for (int x = 1; x < nw; ++x) Y += part[buf][1][x][lane];
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int t = c * DC_T + 4 * q + r;
+        if (t < count && col_ok) out[((size_t)(first + t) * nh + hd) * dim + col] = Y[r];
+      }
+    }
+  };
+  DcOps<T, TPW> A, B;
+  load(0, A);
+#pragma unroll
+  for (int x = 0; x < TPW; ++x) asm volatile("" : "+v"(S[x]));        // the state has come (see delta_scan_kernel)
+  for (int c = 0; c < chunks; c += 2) {               // the next chunk's operands come in while this one is worked on
+    if (c + 1 < chunks) load(c + 1, B);
+    work(c, A, 0);
+    if (c + 1 >= chunks) break;
+    if (c + 2 < chunks) load(c + 2, A);
+    work(c + 1, B, 1);
+  }
+#pragma unroll
+  for (int x = 0; x < TPW; ++x) {
+    const int n = tile[x] * 16 + 4 * q;
+    if (fours) {
+      if (col_ok && n < dim) *reinterpret_cast<dc_f32x4*>(st + n) = S[x];
+    } else {
+#pragma unroll
+      for (int r = 0; r < 4; ++r)
+        if (col_ok && n + r < dim) st[n + r] = S[x][r];
+    }
+  }
+}
+
+// Floats of one chunk's records (all heads): what ia_delta_chunked wants of scratch for every chunk, four chunks to every
+// tile of the host's list.
+extern "C" long ia_delta_chunk_floats(int nh, int dim) { return (long)nh * dc_record_floats((dim + 15) / 16); }
+
+// ia_delta_scan for the `requests` requests from first_request on, whose rows tiles names: tiles[i] = (request, first row of
+// a tile of DC_TILE among its rows), every tile of those requests once, in any order.
+extern "C" int ia_delta_chunked(const void* proj, int code, int proj_stride, int r_col, int k_col, int v_col, const float* w,
+                                const float* a, const float* inv, float* state, long state_stride, float* out,
+                                const int* seq_starts, const int* state_slots, const int* tiles, int num_tiles,
+                                int first_request, int requests, float* records, int nh, int dim, hipStream_t stream) {
+  if (num_tiles == 0 || requests == 0) return IA_OK;
+  if (!proj || !w || !a || !inv || !state || !out || !seq_starts || !state_slots || !tiles || !records || num_tiles < 0 ||
+      first_request < 0 || requests < 0 || nh <= 0 || dim <= 0 || r_col < 0 || k_col < 0 || v_col < 0 ||
+      proj_stride < r_col + nh * dim || proj_stride < k_col + nh * dim || proj_stride < v_col + nh * dim ||
+      state_stride < ia_delta_state_floats(nh, dim) || (code != IA_F32 && code != IA_BF16) ||
+      (((uintptr_t)records | (uintptr_t)state) & 15) || ((dim & 3) == 0 && (state_stride & 3)))
+    return IA_ERR_BAD_ARG;
+  if (dim > 256 || requests > 65535 || nh > 65535 || num_tiles > 0x1fffffff) return IA_ERR_UNSUPPORTED;
+  const int t16 = (dim + 15) / 16, DP = t16 * 16;
+  const int threads = (DP + 63) / 64 * 64;
+  const size_t lds = sizeof(float) * (4 * (size_t)DC_T * (DP + 4) + 4 * 256);
+  const int tpw = t16 > DC_MAX_WAVES ? 2 : 1, waves = (t16 + tpw - 1) / tpw;
+  const dim3 pgrid((unsigned)num_tiles * 4, (unsigned)nh), sgrid((unsigned)nh, (unsigned)requests, (unsigned)t16);
+#define IA_DC(T)                                                                                                             \
+  do {                                                                                                                       \
+    if (lds > 64 * 1024)                                                                                                     \
+      (void)hipFuncSetAttribute((const void*)delta_chunk_prepare_kernel<T>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds); \
+    delta_chunk_prepare_kernel<T><<<pgrid, threads, lds, stream>>>((const T*)proj, proj_stride, r_col, k_col, w, a, inv,      \
+                                                                   seq_starts, tiles, first_request, records, nh, dim);      \
+    IA_LAUNCH_CHECK();                                                                                                       \
+    if (tpw == 1)                                                                                                            \
+      delta_chunk_scan_kernel<T, 1><<<sgrid, 64 * waves, 0, stream>>>((const T*)proj, proj_stride, v_col, state, state_stride, \
+                                                                      out, seq_starts, state_slots, first_request, records,  \
+                                                                      nh, dim);                                              \
+    else                                                                                                                     \
+      delta_chunk_scan_kernel<T, 2><<<sgrid, 64 * waves, 0, stream>>>((const T*)proj, proj_stride, v_col, state, state_stride, \
+                                                                      out, seq_starts, state_slots, first_request, records,  \
+                                                                      nh, dim);                                              \
+  } while (0)
+  if (code == IA_F32) IA_DC(float);
+  else IA_DC(bf16_t);
+#undef IA_DC
+  IA_LAUNCH_CHECK();
+  return IA_OK;
+}
+
 #include "op_call.h"
 IA_OP(ia_delta_tanh_rows)
 IA_OP(ia_delta_prepare)
 IA_OP(ia_delta_scan)
+IA_OP(ia_delta_chunked)

@@ -1515,6 +1515,41 @@ def delta_scan(proj: torch.Tensor, r_col: int, k_col: int, v_col: int, w: torch.
     return out
 
 
+def delta_chunk_floats(nh: int, dim: int) -> int:
+    """fp32 values of scratch that :func:`delta_chunked` wants for every chunk of 16 rows (four to every tile of
+    ``PREFILL_TILE_ROWS`` rows)."""
+    lib = _core()
+    lib.ia_delta_chunk_floats.restype = ctypes.c_long
+    return int(lib.ia_delta_chunk_floats(nh, dim))
+
+
+def delta_chunked(proj: torch.Tensor, r_col: int, k_col: int, v_col: int, w: torch.Tensor, a: torch.Tensor, inv: torch.Tensor,
+                  state: torch.Tensor, out: torch.Tensor, seq_starts: torch.Tensor, state_slots: torch.Tensor,
+                  tiles: torch.Tensor, num_tiles: int, first_request: int, requests: int, nh: int, dim: int,
+                  records: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """:func:`delta_scan` of the portions of prompts, the ``requests`` requests from ``first_request`` on, in chunks of 16
+    rows: tiles[i] = (request, first row of a tile of ``PREFILL_TILE_ROWS`` among its rows), every tile of those once."""
+    N, n, B = proj.shape[0], nh * dim, state_slots.numel()
+    _rows(proj, max(r_col, k_col, v_col) + n, "delta_chunked")
+    for t, size, what in ((w, N * n, "w"), (a, N * n, "a"), (inv, N * nh, "inv"), (out, out.shape[0] * n, "out")):
+        _f32(t, size, f"delta_chunked {what}")
+    stride = _state_rows(state, delta_state_floats(nh, dim), "delta_chunked")
+    _i32(seq_starts, B + 1, "delta_chunked seq_starts")
+    _i32(state_slots, B, "delta_chunked state_slots")
+    _need(tiles.dtype == torch.int32 and tiles.is_cuda and tiles.is_contiguous() and tiles.numel() >= 2 * num_tiles
+          and 0 <= first_request and first_request + requests <= B, "delta_chunked: int32 tiles [num_tiles, 2] and requests of the step")
+    floats = delta_chunk_floats(nh, dim)
+    if records is None:
+        records = torch.empty(max(num_tiles, 1) * 4 * floats, dtype=torch.float32, device=out.device)
+    _need(records.dtype == torch.float32 and records.is_contiguous() and records.numel() >= num_tiles * 4 * floats,
+          "delta_chunked: scratch for every chunk")
+    _ok(_core().ia_delta_chunked(_p(proj), DTYPE_CODE[proj.dtype], _rows_of(proj), r_col, k_col, v_col, _p(w), _p(a), _p(inv),
+                                 _p(state), ctypes.c_long(stride), _p(out), _p(seq_starts), _p(state_slots), _p(tiles),
+                                 int(num_tiles), int(first_request), int(requests), _p(records), nh, dim, _stream()),
+        "delta_chunked")
+    return out
+
+
 # ------------------------------------------------------------ several residual streams
 HYPER_MAX_STREAMS = 32
 

@@ -12,11 +12,12 @@ and with a state S of [dim, dim] that starts at zero
 Each head's o is divided by its root mean square, multiplied by a weight per value of every head and by sigmoid(g), and
 the heads, concatenated, are projected back.  Between steps a request keeps every head's S in one state slot of fp32
 values.  Decays, removal rates, unit norms, the state and the norm are fp32 whatever the activations' type.
+Single tokens run the recurrence itself, portions of prompts chunks of rows as matrix products (csrc/delta_rule.hip).
 """
 from __future__ import annotations
 
 import math
-from typing import Dict, Optional, Sequence
+from typing import Any, Dict, Optional, Sequence
 
 import torch
 
@@ -51,6 +52,9 @@ class DeltaRule(ProjectedMixer):
 
     def state_spec(self) -> StateSpec:
         return StateSpec((K.delta_state_floats(self.nh, self.dim),))
+
+    def step_needs(self) -> Dict[str, Any]:
+        return {"row_tiles": K.PREFILL_TILE_ROWS}
 
     def weights(self) -> Dict[str, WeightSpec]:
         H, n, rank, small = self.hidden_size, self.n, self.rank, dict(follows_compute_dtype=False)
@@ -93,13 +97,19 @@ class DeltaRule(ProjectedMixer):
         z = linear(mid, self.w_2, out_dtype=torch.float32, kernels=self.rt.kernels)
         a, inv = K.delta_prepare(proj, self.k_col, self.a_col, z, self.w_0, self.a_bias, self.nh, self.dim, DECAY_SCALE, KEY_EPS)
         o = torch.empty((n, self.n), dtype=torch.float32, device=dev)
-        K.delta_scan(proj, self.r_col, self.k_col, self.v_col, z, a, inv, state, o, ctx.seq_starts, ctx.state_slots, self.nh,
-                     self.dim)
+        nd = ctx.num_decode
+        if nd > 0:              # single tokens: the recurrence itself
+            K.delta_scan(proj, self.r_col, self.k_col, self.v_col, z, a, inv, state, o, ctx.seq_starts[:nd + 1],
+                         ctx.state_slots[:nd], self.nh, self.dim)
+        if ctx.num_seqs > nd:   # portions of prompts: chunks of rows as matrix products
+            tiles, num_tiles = ctx.row_tiles(K.PREFILL_TILE_ROWS)
+            K.delta_chunked(proj, self.r_col, self.k_col, self.v_col, z, a, inv, state, o, ctx.seq_starts, ctx.state_slots,
+                            tiles, num_tiles, nd, ctx.num_seqs - nd, self.nh, self.dim)
         K.head_norm_gate(o, proj, self.g_col, self.w_norm, self.norm_eps, self.nh, self.dim, out, per_head=True,
                          plain_sigmoid=True)
 
     def emit_mix(self, program, view: CacheView, proj, proj_row: int, out, out_row: int) -> None:
-        from ..engine.program import STREAM
+        from ..engine.program import STREAM, Guard
         from .softmax_attention import _at
         rt, N, T, act, ab, nh, dim = self.rt, program.N, program.T, program.act_code, program.act_bytes, self.nh, self.dim
         state = self._state(view)
@@ -113,8 +123,16 @@ class DeltaRule(ProjectedMixer):
                                                 N, nh, dim, DECAY_SCALE, KEY_EPS, STREAM])
         o = program.buffer("delta.o", T * self.n * 4)
         program.op("core", "ia_delta_scan", [proj, act, proj_row, self.r_col, self.k_col, self.v_col, z, a, inv, state,
-                                             int(state.stride(0)), o, program.seq_starts, program.state_slots, program.B, nh,
-                                             dim, STREAM])
+                                             int(state.stride(0)), o, program.seq_starts, program.state_slots, program.ND, nh,
+                                             dim, STREAM], Guard.between(program.ND, 1))
+        # a request holds a state slot, and a tile at least one row: so many tiles a step has at most
+        most = -(-T // K.PREFILL_TILE_ROWS) + int(state.shape[0])
+        records = program.buffer("delta.records", most * 4 * K.delta_chunk_floats(nh, dim) * 4)
+        tiles, num_tiles = program.row_tiles(K.PREFILL_TILE_ROWS)
+        program.op("core", "ia_delta_chunked", [proj, act, proj_row, self.r_col, self.k_col, self.v_col, z, a, inv, state,
+                                                int(state.stride(0)), o, program.seq_starts, program.state_slots, tiles,
+                                                num_tiles, program.ND, program.NP, records, nh, dim, STREAM],
+                   Guard.between(program.NP, 1))
         program.op("core", "ia_head_norm_gate", [o, proj, act, proj_row, self.g_col, self.w_norm, out, out_row, N, nh, dim,
                                                  float(self.norm_eps), 1, 1, STREAM])
 

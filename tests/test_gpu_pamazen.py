@@ -370,13 +370,13 @@ def test_delta_rule_at_many_head_sizes(dtype, dim, heads, T):
     rt = runtime(dtype)
     n = heads * dim
     g = torch.Generator().manual_seed(dim)
-    lens = [T, 1, 8, 2]
+    lens = [1, T, 8, 2, 75, 16]
     N = sum(lens)
     proj = (torch.randn(N, 3 * n + 5, generator=g) / math.sqrt(dim)).to(rt.dtype)
     w, a = 0.6 + 0.4 * torch.rand(N, n, generator=g), torch.rand(N, n, generator=g)
-    slots = torch.tensor([3, 0, 2, 4], dtype=torch.int32)
-    state = torch.randn(5, K.delta_state_floats(heads, dim), generator=g)
-    S0 = state.view(5, heads, dim, dim).transpose(2, 3)          # kept column by column
+    slots = torch.tensor([3, 0, 2, 4, 6, 5], dtype=torch.int32)
+    state = torch.randn(7, K.delta_state_floats(heads, dim), generator=g)
+    S0 = state.view(7, heads, dim, dim).transpose(2, 3)          # kept column by column
     r, k, v = (proj[:, i * n:(i + 1) * n].double().view(N, heads, dim) for i in range(3))
     inv = 1.0 / torch.sqrt((k * k).sum(-1) + 1e-6)
     out = torch.empty((N, n), device=DEV)
@@ -390,7 +390,7 @@ def test_delta_rule_at_many_head_sizes(dtype, dim, heads, T):
             c = slice(h * dim, (h + 1) * dim)
             o, S = PP.delta_recurrence(r[lo:hi, h], k[lo:hi, h], v[lo:hi, h], w[lo:hi, c].double(), a[lo:hi, c].double(), S0[s, h].double())
             assert rel_err(out[lo:hi, c], o) <= 2e-5
-            assert rel_err(st.cpu().view(5, heads, dim, dim)[s, h].T, S) <= 2e-5
+            assert rel_err(st.cpu().view(7, heads, dim, dim)[s, h].T, S) <= 2e-5
     assert torch.equal(st[1].cpu(), state[1])                    # a slot that no request holds
     # the same rows token by token: the same bits
     st2, out2 = state.clone().to(DEV), torch.empty_like(out)
@@ -405,6 +405,14 @@ def test_delta_rule_at_many_head_sizes(dtype, dim, heads, T):
         for i in live:
             done[i] += 1
     assert torch.equal(out, out2) and torch.equal(st, st2)
+    # the same rows in chunks, but for the first request's, whose tokens a step brings alone
+    st3, out3 = state.clone().to(DEV), torch.full_like(out, float("nan"))
+    tiles = torch.tensor([(i, r) for i, L in list(enumerate(lens))[1:] for r in range(0, L, K.PREFILL_TILE_ROWS)][::-1], dtype=torch.int32)
+    K.delta_chunked(proj.to(DEV), 0, n, 2 * n, *args, st3, out3, starts.to(DEV), slots.to(DEV), tiles.to(DEV), tiles.shape[0], 1,
+                    len(lens) - 1, heads, dim)
+    lo = lens[0]
+    assert rel_err(out3[lo:], out[lo:].double().cpu()) <= 2e-5
+    assert rel_err(st3, torch.where(torch.arange(7)[:, None] == slots[0], state, st.cpu()).double()) <= 2e-5
 
 
 @BOTH
