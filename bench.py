@@ -653,16 +653,16 @@ def rogizen_bench(a) -> int:
 
 # ---- the Pamazen design beside the Llama decoder at equal sizes -------------------------------------------------
 # Eight layers of one width over four residual streams: a layer with two mixers side by side (window attention whose values
-# are its keys, with four kept positions, sinks and capped scores, 16 or 32 heads of 128 over 4 or 8; the generalized delta
+# are its keys, with eight kept positions, sinks and capped scores, 16 or 32 heads of 128 over 4 or 8; the generalized delta
 # rule, as many heads of 128, decays through a middle of 64), then three of attention over all keys with rotated pairs and
-# values mixed with the first of them, twice; every layer sixteen experts and two identities in two groups of which one is
+# values mixed with the first of them, twice; every layer twenty experts and four identities in three groups of which two are
 # kept, two chosen, and a gated shared expert: together as many feed-forward weights a token as the twin has (when no
 # identity is chosen).  The Llama twin has the same width, layers, vocabulary and heads.
 PAMAZEN_SIZES = {
-    "2k": dict(width=2048, layers=8, vocab=32000, ff=5504, heads=16, kv_heads=4, dim=128, window=1024, keep=4, rank=64,
-               streams=4, experts=16, identity=2, top=2, expert_ff=1408, shared_ff=2688),
-    "4k": dict(width=4096, layers=8, vocab=32000, ff=9600, heads=32, kv_heads=8, dim=128, window=2048, keep=4, rank=64,
-               streams=4, experts=16, identity=2, top=2, expert_ff=2432, shared_ff=4736),
+    "2k": dict(width=2048, layers=8, vocab=32000, ff=5504, heads=16, kv_heads=4, dim=128, window=1024, keep=8, rank=64,
+               streams=4, experts=20, identity=4, top=2, expert_ff=1408, shared_ff=2688),
+    "4k": dict(width=4096, layers=8, vocab=32000, ff=9600, heads=32, kv_heads=8, dim=128, window=2048, keep=8, rank=64,
+               streams=4, experts=20, identity=4, top=2, expert_ff=2432, shared_ff=4736),
 }
 
 
@@ -671,15 +671,15 @@ def pamazen_configs(size: dict):
     from infernum_amd.config.pamazen import PamazenConfig
     d = size["dim"]
     heads = {"heads": size["heads"], "kv_heads": size["kv_heads"], "dim": d, "vdim": d, "scale": d ** -0.5}
-    attention = dict(heads, v_mix=True, rot={"base": 10000.0, "dims": d // 2, "scaling": {"factor": 4.0}})
+    attention = dict(heads, v_mix=True, rot={"base": 10000.0, "dims": d // 2, "scaling": {"factor": 2.0}})
     side = {"left": dict(heads, softcap=30.0, mask={"size": size["window"], "keep_first": size["keep"]}),
-            "right": {"heads": size["heads"], "dim": d, "rank": size["rank"]}, "left_scale": 1.0, "right_scale": 0.5}
+            "right": {"heads": size["heads"], "dim": d, "rank": size["rank"]}, "left_scale": 1.0, "right_scale": 0.8}
     mlp = {"kind": "moe", "expert": {"ff": size["expert_ff"]}, "shared": {"ff": size["shared_ff"]},
            "router": {"experts": size["experts"], "identity": size["identity"], "top": size["top"],
-                      "groups": {"count": 2, "keep": 1}}}
+                      "groups": {"count": 3, "keep": 2}}}
     pam = PamazenConfig.from_dict({
-        "architecture": "Pamazen", "vocab": size["vocab"], "width": size["width"], "norm": {"eps": 1e-6},
-        "streams": size["streams"], "residual_mult": 0.5, "logit_softcap": 15.0,
+        "architecture": "Pamazen", "vocab": size["vocab"], "width": size["width"], "norm": {"eps": 1e-5},
+        "streams": size["streams"], "residual_mult": 0.6, "logit_softcap": 25.0,
         "layers": [{"type": "attention" if i % 4 else "parallel", "mixer": attention if i % 4 else side, "mlp": mlp}
                    for i in range(size["layers"])]})
     llama = LlamaConfig.from_dict(dict(
