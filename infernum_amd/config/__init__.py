@@ -5,5 +5,6 @@ from .rogizen import RogizenConfig
 from .malinex import MalinexConfig
 from .sikazen import SikazenConfig
 from .pamazen import PamazenConfig
+from .mirovik import MirovikConfig
 from .registry import (config_from_dict, load_config, model_spec_for, register_architecture, registered_architectures,
                        resolve_architecture)

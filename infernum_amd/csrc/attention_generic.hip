@@ -11,10 +11,13 @@
 // chunk of -window positions, see ia_first_visible_key).  sinks (nullable, fp32 [nh]): exp(sinks[h]) is added to
 // the softmax's denominator of head h; it has no key and no value.  Value heads may have another size, dv, than
 // query and key heads (value pages [num_pages, nkv, dv, page_size], out rows of nh dv values).  Under a window the
-// request's first `keep` keys stay visible; a softcap c > 0 turns a scaled score s into c tanh(s / c).
+// request's first `keep` keys stay visible; a softcap c > 0 turns a scaled score s into c tanh(s / c).  bias (nullable,
+// fp32 [nh, span + 2 pad], the layout of attention_mfma.hip): a number added to the score by the key's distance; gate
+// (nullable, rows of gate_stride values): what a head leaves, times sigmoid(gate), value by value.
 #include "common.h"
 
 #define AG_MAX_D 640
+#define AG_BIAS_PAD 64
 
 template <typename T>
 __global__ __launch_bounds__(64) void attn_generic_kernel(const T* __restrict__ q, int q_row_stride,
@@ -25,7 +28,8 @@ __global__ __launch_bounds__(64) void attn_generic_kernel(const T* __restrict__ 
                                                           const int* __restrict__ block_tables, int bt_stride, int nh,
                                                           int nkv, int d, int dv, int page_size, int num_pages,
                                                           float scale, int window, const float* __restrict__ sinks,
-                                                          int keep, float softcap) {
+                                                          int keep, float softcap, const float* __restrict__ bias,
+                                                          int span, const T* __restrict__ gate, int gate_stride) {
   __shared__ float qs[AG_MAX_D];
   __shared__ float ps[64];
   __shared__ int rs[64];
@@ -62,6 +66,10 @@ __global__ __launch_bounds__(64) void attn_generic_kernel(const T* __restrict__ 
         for (int i = 0; i < d; ++i) dot = fmaf(qs[i], to_float(kr[i]), dot);
         sc = dot * scale;
         if (softcap > 0.f) sc = softcap * tanhf(sc / softcap);
+        if (bias) {
+          const int back = pos - j < span - 1 ? pos - j : span - 1;
+          sc += bias[(size_t)h * (span + 2 * AG_BIAS_PAD) + AG_BIAS_PAD + span - 1 - back];
+        }
       } else {
         sc = __uint_as_float(0x7fc00000u);  // a block table without a page here: poison, never a stray read
       }
@@ -104,7 +112,10 @@ __global__ __launch_bounds__(64) void attn_generic_kernel(const T* __restrict__ 
 #pragma unroll
   for (int c = 0; c < AG_MAX_D / 64; ++c) {
     const int dim = lane + 64 * c;
-    if (dim < dv) o[dim] = from_float<T>(acc[c] * inv_l);
+    if (dim >= dv) continue;
+    float v = acc[c] * inv_l;
+    if (gate) v *= 1.0f / (1.0f + expf(-to_float(gate[(size_t)n * gate_stride + (size_t)h * dv + dim])));
+    o[dim] = from_float<T>(v);
   }
 }
 
@@ -112,10 +123,11 @@ extern "C" int ia_attention_generic(const void* q, int q_row_stride, const void*
                                     void* out, int out_row_stride, int dtype, const int* token_seq,
                                     const int* positions, const int* block_tables, int bt_stride, int N, int nh,
                                     int nkv, int d, int dv, int page_size, int num_pages, float scale, int window,
-                                    const float* sinks, int keep, float softcap, hipStream_t stream) {
+                                    const float* sinks, int keep, float softcap, const float* bias, int span,
+                                    const void* gate, int gate_stride, hipStream_t stream) {
   if (N < 0 || nh <= 0 || nkv <= 0 || nh % nkv != 0 || d <= 0 || d > AG_MAX_D || dv <= 0 || dv > AG_MAX_D || keep < 0 ||
       !(softcap >= 0.f) || q_row_stride < nh * d || out_row_stride < nh * dv || page_size <= 0 || num_pages <= 0 ||
-      bt_stride <= 0)
+      bt_stride <= 0 || (bias && span < 1) || (gate && gate_stride < nh * dv))
     return IA_ERR_BAD_ARG;
   if (nh > 65535) return IA_ERR_UNSUPPORTED;
   if (N == 0) return IA_OK;
@@ -124,12 +136,14 @@ extern "C" int ia_attention_generic(const void* q, int q_row_stride, const void*
     attn_generic_kernel<float><<<grid, 64, 0, stream>>>((const float*)q, q_row_stride, (const float*)k_pages,
                                                         (const float*)v_pages, (float*)out, out_row_stride, token_seq,
                                                         positions, block_tables, bt_stride, nh, nkv, d, dv, page_size,
-                                                        num_pages, scale, window, sinks, keep, softcap);
+                                                        num_pages, scale, window, sinks, keep, softcap, bias, span,
+                                                        (const float*)gate, gate_stride);
   else if (dtype == IA_BF16)
     attn_generic_kernel<bf16_t><<<grid, 64, 0, stream>>>((const bf16_t*)q, q_row_stride, (const bf16_t*)k_pages,
                                                          (const bf16_t*)v_pages, (bf16_t*)out, out_row_stride,
                                                          token_seq, positions, block_tables, bt_stride, nh, nkv, d, dv,
-                                                         page_size, num_pages, scale, window, sinks, keep, softcap);
+                                                         page_size, num_pages, scale, window, sinks, keep, softcap,
+                                                         bias, span, (const bf16_t*)gate, gate_stride);
   else
     return IA_ERR_BAD_ARG;
   IA_LAUNCH_CHECK();

@@ -6,6 +6,13 @@
 // s <- c tanh(s / c); and, under a window, the first `keep` keys of the request, which every query goes on seeing.
 // The tiles that hold kept keys before the window come first, then the window's own; between them nothing is read.
 //
+// With IA_ATTN_EXT=2 they take (other libraries refuse them): a number added to the score by the key's distance, per
+// query head, and a gate on what a head leaves, out <- out * sigmoid(gate), one gate value per value.  The numbers come
+// as a table that runs backwards over the distance, so that keys in their order read it forwards: head h's row holds
+// ATTN_BIAS_PAD times the number of the furthest distance, span - 1, then those of span - 1, span - 2, ..., 0, then
+// ATTN_BIAS_PAD zeros; any distance from span - 1 on has the furthest one's number.  A tile of keys that are all that
+// far from all rows of a wave adds one number to its column and reads no table.  (3: all of them.)
+//
 // Both kernels work on the transposed problem:
 //   S^T[key, col] = K[key, :] . Q[col, :]      A operand = 16 keys of K, B operand = 16 columns of Q
 //   O^T[dim, col] += V^T[dim, key] P^T[key, col]
@@ -48,10 +55,17 @@
 #define IA_MAX_DIM (IA_HEAD_DIM > IA_VALUE_DIM ? IA_HEAD_DIM : IA_VALUE_DIM)
 static_assert(HD % 16 == 0 && HD >= 16 && HD <= 256, "head size must be a multiple of 16 up to 256");
 static_assert(VD % 16 == 0 && VD >= 16 && VD <= 256, "value size must be a multiple of 16 up to 256");
-constexpr bool EXT = IA_ATTN_EXT != 0;
+constexpr bool EXT = (IA_ATTN_EXT & 1) != 0;
+constexpr bool BIAS = (IA_ATTN_EXT & 2) != 0;
+#define ATTN_BIAS_PAD 64
+#define ATTN_LOG2E 1.4426950408889634f
 
 // The options that only a library with IA_ATTN_EXT takes.
 struct AttnExt {
+  const float* bias;             // BIAS (nullable): rows of span + 2 ATTN_BIAS_PAD numbers, one a query head
+  int span;
+  const uint16_t* gate;          // BIAS (nullable): token n's gate of value i of its row at gate[n * gate_stride + i]
+  int gate_stride;
   int keep;                      // under a window: the request's first `keep` keys stay visible
   float cap_in, cap_out;         // softcap c: raw score times cap_in = scale / c, tanh, times cap_out = c log2(e)
   bool capped;
@@ -60,6 +74,14 @@ struct AttnExt {
 // tanh to about 1e-7: 1 - 2 / (1 + exp(2 x)), which runs into 1 and -1 at the ends
 __device__ __forceinline__ float attn_tanh(float x) {
   return 1.0f - 2.0f * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(2.8853900817779268f * x));
+}
+
+// What four neighbouring values of a head become behind their gates, g the gates' place.
+__device__ __forceinline__ void attn_gate4(float (&v)[4], const uint16_t* g) {
+  const uint2 w = *reinterpret_cast<const uint2*>(g);
+  const uint32_t b[4] = {w.x << 16, w.x & 0xffff0000u, w.y << 16, w.y & 0xffff0000u};
+#pragma unroll
+  for (int r = 0; r < 4; ++r) v[r] *= 1.0f / (1.0f + __builtin_amdgcn_exp2f(-ATTN_LOG2E * __uint_as_float(b[r])));
 }
 
 // Tiles of `size` keys that hold kept keys before the first key lo of a window (0 when the window reaches the start).
@@ -219,8 +241,16 @@ __device__ __forceinline__ void dec_finish(const DecGeom& G, int t0, int j, int 
 
 // One tile of 16 keys, t0 .. t0+15, against the 16 columns (heads) of this wave.
 //   pos, lo: this lane's column sees keys lo .. pos (EXT: and those below X.keep); pos < 0: no such column
+//   brow, bfar, near_from (BIAS): key k's number for this lane's column at brow[k], that of a far key, times log2(e), and
+//   the first key that is not far
 __device__ __forceinline__ void dec_compute(int t0, const DecTile& T, const s16x4 (&q)[NS], int pos, int lo, int qd,
-                                            float scale_log2, f32x4 (&o)[NSV], float& m, float& l, const AttnExt& X) {
+                                            float scale_log2, f32x4 (&o)[NSV], float& m, float& l, const AttnExt& X,
+                                            const float* brow, float bfar, int near_from) {
+  float bv[4] = {bfar, bfar, bfar, bfar};
+  if (BIAS && X.bias && t0 + 15 >= near_from) {               // the same for all lanes of the wave
+#pragma unroll
+    for (int r = 0; r < 4; ++r) bv[r] = brow[t0 + 4 * qd + r] * ATTN_LOG2E;
+  }
   // ---- S^T = K Q^T
   f32x4 s = (f32x4){0.f, 0.f, 0.f, 0.f};
 #pragma unroll
@@ -233,7 +263,7 @@ __device__ __forceinline__ void dec_compute(int t0, const DecTile& T, const s16x
     const int kr = kg + r;
     const bool ok = pos >= 0 && kr <= pos && (kr >= lo || (EXT && kr < X.keep));
     const float sl = (EXT && X.capped) ? X.cap_out * attn_tanh(s[r] * X.cap_in) : s[r] * scale_log2;
-    sv[r] = ok ? sl : -INFINITY;
+    sv[r] = ok ? (BIAS ? sl + bv[r] : sl) : -INFINITY;
   }
   float tmax = fmaxf(fmaxf(sv[0], sv[1]), fmaxf(sv[2], sv[3]));
   tmax = fmaxf(tmax, __shfl_xor(tmax, 16, IA_WAVE));
@@ -366,6 +396,14 @@ __global__ __launch_bounds__(WAVES * 64, ((WAVES == 4 && IA_MAX_DIM <= 128) ? 3 
     }
   }
   const int pos = col_ok ? p : -1;
+  const float* brow = nullptr;
+  float bfar = 0.f;
+  const int near_from = p - (X.span - 1) + 1;       // BIAS: keys from here on have a distance below span - 1
+  if (BIAS && X.bias) {
+    const float* row0 = X.bias + (size_t)(col_ok ? h : g * G) * (X.span + 2 * ATTN_BIAS_PAD);
+    brow = row0 + (ATTN_BIAS_PAD + X.span - 1 - p);
+    bfar = row0[0] * ATTN_LOG2E;
+  }
   f32x4 o[NSV];
 #pragma unroll
   for (int n = 0; n < NSV; ++n) o[n] = (f32x4){0.f, 0.f, 0.f, 0.f};
@@ -436,13 +474,13 @@ __global__ __launch_bounds__(WAVES * 64, ((WAVES == 4 && IA_MAX_DIM <= 128) ? 3 
     const bool more1 = t + WAVES < tb;
     if (more1) dec_load<POW2>(geo, tile_at(t + WAVES) * 16, j, qd, B);
     dec_finish(geo, tile_at(t) * 16, j, qd, A);
-    dec_compute(tile_at(t) * 16, A, qreg, pos, lo0, qd, scale_log2, o, m, l, X);
+    dec_compute(tile_at(t) * 16, A, qreg, pos, lo0, qd, scale_log2, o, m, l, X, brow, bfar, near_from);
     t += WAVES;
     if (!more1) break;
     const bool more2 = t + WAVES < tb;
     if (more2) dec_load<POW2>(geo, tile_at(t + WAVES) * 16, j, qd, A);
     dec_finish(geo, tile_at(t) * 16, j, qd, B);
-    dec_compute(tile_at(t) * 16, B, qreg, pos, lo0, qd, scale_log2, o, m, l, X);
+    dec_compute(tile_at(t) * 16, B, qreg, pos, lo0, qd, scale_log2, o, m, l, X, brow, bfar, near_from);
     t += WAVES;
     if (!more2) break;
   }
@@ -483,9 +521,11 @@ __global__ __launch_bounds__(WAVES * 64, ((WAVES == 4 && IA_MAX_DIM <= 128) ? 3 
     if (num_splits == 1) {
       // a sink counts once, here or where the parts are joined
       const float inv = 1.0f / (sinks ? L + exp2f(sinks[h] * 1.4426950408889634f - M) : L);
+      float ov[4] = {acc[0] * inv, acc[1] * inv, acc[2] * inv, acc[3] * inv};
+      if (BIAS && X.gate) attn_gate4(ov, X.gate + (size_t)b * X.gate_stride + (size_t)h * VD + 4 * qd + n * 16);
       uint2 wv;
-      wv.x = (uint32_t)float_to_bf16_bits(acc[0] * inv) | ((uint32_t)float_to_bf16_bits(acc[1] * inv) << 16);
-      wv.y = (uint32_t)float_to_bf16_bits(acc[2] * inv) | ((uint32_t)float_to_bf16_bits(acc[3] * inv) << 16);
+      wv.x = (uint32_t)float_to_bf16_bits(ov[0]) | ((uint32_t)float_to_bf16_bits(ov[1]) << 16);
+      wv.y = (uint32_t)float_to_bf16_bits(ov[2]) | ((uint32_t)float_to_bf16_bits(ov[3]) << 16);
       *reinterpret_cast<uint2*>(out + (size_t)b * out_row_stride + (size_t)h * VD + 4 * qd + n * 16) = wv;
     } else {
       const size_t rec = ((size_t)b * nh + h) * num_splits + split;
@@ -504,7 +544,8 @@ __global__ __launch_bounds__(WAVES * 64, ((WAVES == 4 && IA_MAX_DIM <= 128) ? 3 
 // the loads of the partial outputs do not wait for each other.
 extern "C" __global__ __launch_bounds__(64) void attn_decode_reduce_kernel(
     const float* __restrict__ part_o, const float* __restrict__ part_ml, uint16_t* __restrict__ out,
-    int out_row_stride, int nh, int num_splits, const float* __restrict__ sinks) {
+    int out_row_stride, int nh, int num_splits, const float* __restrict__ sinks, const uint16_t* __restrict__ gate,
+    int gate_stride) {
   const int b = blockIdx.x / nh, h = blockIdx.x - b * nh, lane = threadIdx.x;
   const size_t rec0 = (size_t)blockIdx.x * num_splits;
   // the first parts' outputs are asked for together with the statistics, not after them
@@ -560,7 +601,11 @@ extern "C" __global__ __launch_bounds__(64) void attn_decode_reduce_kernel(
 #pragma unroll
   for (int c = 0; c < (VD + 63) / 64; ++c) {
     const int dim = lane + 64 * c;
-    if (dim < VD) out[(size_t)b * out_row_stride + (size_t)h * VD + dim] = float_to_bf16_bits(acc[c] * inv);
+    if (dim >= VD) continue;
+    float v = acc[c] * inv;
+    if (BIAS && gate)
+      v *= 1.0f / (1.0f + __builtin_amdgcn_exp2f(-ATTN_LOG2E * bf16_bits_to_float(gate[(size_t)b * gate_stride + (size_t)h * VD + dim])));
+    out[(size_t)b * out_row_stride + (size_t)h * VD + dim] = float_to_bf16_bits(v);
   }
 }
 
@@ -633,7 +678,7 @@ __global__ __launch_bounds__(4 * HGW * 64) void attn_prefill_kernel(
     last_row = (row0 + 64 < qlen ? row0 + 64 : qlen) - 1;
   }
   if (tid == 0) s_poison = 0;
-  const float to_log2 = (EXT && X.capped) ? 1.0f : scale_log2;      // capped scores are in the log2 domain already
+  const float to_log2_all = (EXT && X.capped) ? 1.0f : scale_log2;      // capped scores are in the log2 domain already
 
   // ---- queries of this wave: CT heads x 16 rows, as B operands (col = row j of head c)
   // steps of 32 head dims; a head size that is an odd multiple of 16 ends with a step whose upper half
@@ -665,6 +710,21 @@ __global__ __launch_bounds__(4 * HGW * 64) void attn_prefill_kernel(
     for (int n = 0; n < NSV; ++n) o[c][n] = (f32x4){0.f, 0.f, 0.f, 0.f};
   }
   const bf16x8_t ones = __builtin_bit_cast(bf16x8_t, make_uint4(0x3f803f80u, 0x3f803f80u, 0x3f803f80u, 0x3f803f80u));
+
+  // BIAS: the number of key k for row j of head c at brow[c][k], and that of a far key
+  const float* brow[CT];
+  float bfar[CT];
+#pragma unroll
+  for (int c = 0; c < CT; ++c) {
+    brow[c] = nullptr;
+    bfar[c] = 0.f;
+    if (BIAS && X.bias) {
+      const int hj = (hc * HGW + hgw) * CT + c;
+      const float* row0 = X.bias + (size_t)(g * G + (hj < G ? hj : 0)) * (X.span + 2 * ATTN_BIAS_PAD);
+      brow[c] = row0 + (ATTN_BIAS_PAD + X.span - 1 - (ctx + rb + j));
+      bfar[c] = row0[0] * ATTN_LOG2E;
+    }
+  }
 
   // ---- keys the workgroup needs: those its rows may see
   const int key_hi = ctx + last_row;
@@ -818,6 +878,15 @@ __global__ __launch_bounds__(4 * HGW * 64) void attn_prefill_kernel(
     for (int sub = 0; sub < PF_SUBS; ++sub) {
     const int t0 = tile_at(t) * PF_KT + sub * 32;
     if (wave_live && t0 <= wave_hi && (t0 + 31 >= wave_lo || (EXT && t0 < X.keep)) && t0 <= key_hi) {
+      // some key of the tile is nearer than the furthest distance of the table to some row of the wave
+      const bool near = BIAS && X.bias && t0 + 31 > ctx + rb - (X.span - 1);
+      float bv[CT][8];
+      if (near) {
+#pragma unroll
+        for (int c = 0; c < CT; ++c)
+#pragma unroll
+          for (int i = 0; i < 8; ++i) bv[c][i] = brow[c][t0 + (i >> 2) * 16 + 4 * qd + (i & 3)];
+      }
       // ---- S^T = K Q^T for the two tiles of 16 keys
       f32x4 sc[CT][2];
 #pragma unroll
@@ -849,6 +918,14 @@ __global__ __launch_bounds__(4 * HGW * 64) void attn_prefill_kernel(
 #pragma unroll
           for (int i = 0; i < 8; ++i) sv[i] = X.cap_out * attn_tanh(sv[i] * X.cap_in);
         }
+        // score in the log2 domain = sv * to_log2 + shift
+        float to_log2 = to_log2_all, shift = BIAS ? bfar[c] : 0.f;
+        if (near) {
+#pragma unroll
+          for (int i = 0; i < 8; ++i) sv[i] = fmaf(sv[i], to_log2_all, bv[c][i] * ATTN_LOG2E);
+          to_log2 = 1.0f;
+          shift = 0.f;
+        }
         if (need_mask) {
 #pragma unroll
           for (int kt = 0; kt < 2; ++kt)
@@ -871,11 +948,12 @@ __global__ __launch_bounds__(4 * HGW * 64) void attn_prefill_kernel(
         float m_safe = (m[c] == -INFINITY) ? 0.f : m[c];
         float e[8];
 #pragma unroll
-        for (int i = 0; i < 8; ++i) e[i] = __builtin_amdgcn_exp2f(fmaf(sv[i], to_log2, -m_safe));
+        for (int i = 0; i < 8; ++i) e[i] = __builtin_amdgcn_exp2f(fmaf(sv[i], to_log2, BIAS ? shift - m_safe : -m_safe));
         const float emax = fmaxf(fmaxf(fmaxf(e[0], e[1]), fmaxf(e[2], e[3])), fmaxf(fmaxf(e[4], e[5]), fmaxf(e[6], e[7])));
         if (__any(emax > PF_LAZY_EXP || m[c] == -INFINITY)) {
-          const float lmax = to_log2 * fmaxf(fmaxf(fmaxf(sv[0], sv[1]), fmaxf(sv[2], sv[3])),
-                                                fmaxf(fmaxf(sv[4], sv[5]), fmaxf(sv[6], sv[7])));
+          float lmax = to_log2 * fmaxf(fmaxf(fmaxf(sv[0], sv[1]), fmaxf(sv[2], sv[3])),
+                                          fmaxf(fmaxf(sv[4], sv[5]), fmaxf(sv[6], sv[7])));
+          if (BIAS) lmax += shift;
           float tmax = fmaxf(lmax, __shfl_xor(lmax, 16, IA_WAVE));
           tmax = fmaxf(tmax, __shfl_xor(tmax, 32, IA_WAVE));
           const float m_new = (tmax > m[c] + PF_LAZY) ? tmax : m[c];        // never moves to -inf
@@ -886,7 +964,7 @@ __global__ __launch_bounds__(4 * HGW * 64) void attn_prefill_kernel(
           for (int n = 0; n < NSV; ++n) o[c][n] *= corr;
           m[c] = m_new;
 #pragma unroll
-          for (int i = 0; i < 8; ++i) e[i] = __builtin_amdgcn_exp2f(fmaf(sv[i], to_log2, -m_safe));
+          for (int i = 0; i < 8; ++i) e[i] = __builtin_amdgcn_exp2f(fmaf(sv[i], to_log2, BIAS ? shift - m_safe : -m_safe));
         }
         // probabilities are rounded to bf16 by the hardware conversion (nearest even); their sum is taken by the
         // matrix cores of the same rounded values (a product with a tile of ones), so that numerator and
@@ -925,13 +1003,15 @@ __global__ __launch_bounds__(4 * HGW * 64) void attn_prefill_kernel(
     float lsum = lacc[c][0];
     if (sinks) lsum += exp2f(sinks[g * G + (hc * HGW + hgw) * CT + c] * 1.4426950408889634f - m[c]);
     const float inv = poison ? __uint_as_float(0x7fc00000u) : 1.0f / lsum;
-    uint16_t* orow = out + (size_t)(qstart + row) * out_row_stride +
-                     (size_t)(g * G + (hc * HGW + hgw) * CT + c) * VD + 4 * qd;
+    const size_t ocol = (size_t)(g * G + (hc * HGW + hgw) * CT + c) * VD + 4 * qd;
+    uint16_t* orow = out + (size_t)(qstart + row) * out_row_stride + ocol;
 #pragma unroll
     for (int n = 0; n < NSV; ++n) {
+      float ov[4] = {o[c][n][0] * inv, o[c][n][1] * inv, o[c][n][2] * inv, o[c][n][3] * inv};
+      if (BIAS && X.gate) attn_gate4(ov, X.gate + (size_t)(qstart + row) * X.gate_stride + ocol + n * 16);
       uint2 w;
-      w.x = (uint32_t)float_to_bf16_bits(o[c][n][0] * inv) | ((uint32_t)float_to_bf16_bits(o[c][n][1] * inv) << 16);
-      w.y = (uint32_t)float_to_bf16_bits(o[c][n][2] * inv) | ((uint32_t)float_to_bf16_bits(o[c][n][3] * inv) << 16);
+      w.x = (uint32_t)float_to_bf16_bits(ov[0]) | ((uint32_t)float_to_bf16_bits(ov[1]) << 16);
+      w.y = (uint32_t)float_to_bf16_bits(ov[2]) | ((uint32_t)float_to_bf16_bits(ov[3]) << 16);
       *reinterpret_cast<uint2*>(orow + n * 16) = w;
     }
   }
@@ -942,8 +1022,15 @@ extern "C" int ia_attn_head_dim() { return HD; }
 
 // keep and softcap of a launch, and the scale the kernel multiplies raw scores with: with a softcap the scores it
 // sees are in the log2 domain already
-static int attn_ext(int window, int keep, float softcap, float scale, AttnExt& X, float& scale_log2) {
-  if (keep < 0 || !(softcap >= 0.f)) return IA_ERR_BAD_ARG;
+static int attn_ext(int window, int keep, float softcap, float scale, const float* bias, int span, const void* gate,
+                    int gate_stride, int nh, AttnExt& X, float& scale_log2) {
+  if (keep < 0 || !(softcap >= 0.f) || (bias && span < 1) || (gate && gate_stride < nh * VD)) return IA_ERR_BAD_ARG;
+  if (!BIAS && (bias || gate)) return IA_ERR_UNSUPPORTED;
+  if (gate && ((gate_stride & 3) || ((uintptr_t)gate & 7))) return IA_ERR_UNSUPPORTED;
+  X.bias = bias;
+  X.span = bias ? span : 1;
+  X.gate = (const uint16_t*)gate;
+  X.gate_stride = gate_stride;
   if (!EXT && (keep > 0 || softcap > 0.f)) return IA_ERR_UNSUPPORTED;
   if (window < 0 && keep > 0) return IA_ERR_UNSUPPORTED;
   X.keep = window > 0 ? keep : 0;
@@ -970,7 +1057,7 @@ extern "C" int ia_attn_decode(const void* q, int q_row_stride, const void* k_pag
                               int out_row_stride, float* part_o, float* part_ml, const int* positions,
                               const int* block_tables, int bt_stride, int B, int nh, int nkv, int ps, int num_pages,
                               float scale, int window, int num_splits, const float* sinks, int keep, float softcap,
-                              hipStream_t stream) {
+                              const float* bias, int span, const void* gate, int gate_stride, hipStream_t stream) {
   const int rc = dec_check(B, nh, nkv, ps, num_pages, bt_stride, num_splits, part_o, part_ml, out_row_stride);
   if (rc != IA_OK) return rc;
   if (q_row_stride & 7) return IA_ERR_UNSUPPORTED;
@@ -978,7 +1065,7 @@ extern "C" int ia_attn_decode(const void* q, int q_row_stride, const void* k_pag
   const int G = nh / nkv, HT = (G + 15) / 16;
   AttnExt X;
   float scale_log2;
-  const int xrc = attn_ext(window, keep, softcap, scale, X, scale_log2);
+  const int xrc = attn_ext(window, keep, softcap, scale, bias, span, gate, gate_stride, nh, X, scale_log2);
   if (xrc != IA_OK) return xrc;
   dim3 grid(B, nkv * HT, num_splits);
 #define DEC_LAUNCH(P2, W)                                                                                          \
@@ -997,12 +1084,14 @@ extern "C" int ia_attn_decode(const void* q, int q_row_stride, const void* k_pag
   IA_LAUNCH_CHECK();
   if (num_splits > 1) {
     attn_decode_reduce_kernel<<<B * nh, 64, 0, stream>>>(part_o, part_ml, (uint16_t*)out, out_row_stride, nh,
-                                                         num_splits, sinks);
+                                                         num_splits, sinks, X.gate, X.gate_stride);
     IA_LAUNCH_CHECK();
   }
   return IA_OK;
 }
 
+// bias (nullable, fp32 [nh, span + 2 ATTN_BIAS_PAD], see the top of the file) and gate (nullable, rows of gate_stride
+// values of which the first nh * VD are read): only with IA_ATTN_EXT & 2.
 // sinks (nullable, fp32 [nh], in all three launchers): exp(sinks[h]) is added to the softmax's denominator of
 // head h, once, where the sum over all keys is known.
 // The same with the rotation in front: row b of src is the QKV product of token b, [nh q heads | nkv k heads |
@@ -1026,7 +1115,7 @@ extern "C" int ia_attn_decode_fused(const void* src, int src_dtype, int src_spli
   const int G = nh / nkv, HT = (G + 15) / 16;
   AttnExt X;
   float scale_log2;
-  const int xrc = attn_ext(window, keep, softcap, scale, X, scale_log2);
+  const int xrc = attn_ext(window, keep, softcap, scale, nullptr, 0, nullptr, 0, nh, X, scale_log2);
   if (xrc != IA_OK) return xrc;
   DecFused F;
   F.src = src;
@@ -1060,7 +1149,7 @@ extern "C" int ia_attn_decode_fused(const void* src, int src_dtype, int src_spli
   IA_LAUNCH_CHECK();
   if (num_splits > 1) {
     attn_decode_reduce_kernel<<<B * nh, 64, 0, stream>>>(part_o, part_ml, (uint16_t*)out, out_row_stride, nh,
-                                                         num_splits, sinks);
+                                                         num_splits, sinks, nullptr, 0);
     IA_LAUNCH_CHECK();
   }
   return IA_OK;
@@ -1076,7 +1165,7 @@ extern "C" int ia_attn_prefill(const void* q, int q_row_stride, const void* k_pa
                                int out_row_stride, const int* seq_starts, const int* seq_ctx, const int* block_tables,
                                int bt_stride, const int* tiles, int num_tiles, int nh, int nkv, int ps, int num_pages,
                                float scale, int window, int launch_shape, const float* sinks, int keep, float softcap,
-                               hipStream_t stream) {
+                               const float* bias, int span, const void* gate, int gate_stride, hipStream_t stream) {
   if (launch_shape < 0 || (launch_shape & ~(0xff | IA_PREFILL_PAIRED))) return IA_ERR_BAD_ARG;
   // under a window the rows of the two ends share no keys, and the keys between them may have no page any more:
   // rows are not paired then, whatever was asked for
@@ -1104,7 +1193,7 @@ extern "C" int ia_attn_prefill(const void* q, int q_row_stride, const void* k_pa
   if ((long long)nkv * HC > 65535) return IA_ERR_UNSUPPORTED;
   AttnExt X;
   float scale_log2;
-  const int xrc = attn_ext(window, keep, softcap, scale, X, scale_log2);
+  const int xrc = attn_ext(window, keep, softcap, scale, bias, span, gate, gate_stride, nh, X, scale_log2);
   if (xrc != IA_OK) return xrc;
   dim3 grid(num_tiles, nkv * HC);
 #define PF_LAUNCH_P(C, W, P2)                                                                                     \

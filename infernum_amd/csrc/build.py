@@ -49,6 +49,8 @@ CORE_SOURCES = [
     "delta_rule.hip",
     "seqmix.hip",
     "linear_attention.hip",
+    "retention.hip",
+    "selective_scan.hip",
     "sigmoid_attention.hip",
     "window_pool_attention.hip",
     "sampling.hip",
@@ -64,10 +66,11 @@ BLASLT_SOURCES = ["gemm_library.cpp"]
 # Head sizes whose attention library `build_all` compiles ahead of time.
 DEFAULT_HEAD_DIMS = (16, 32, 48, 64, 80, 96, 112, 128, 160, 192, 256)
 SUPPORTED_HEAD_DIMS = tuple(range(16, 257, 16))
-# (key size, value size, with kept first keys and a softcap) whose attention library `build_all` compiles ahead of time.
-DEFAULT_ATTENTION_SIZES = ((16, 32, False), (16, 48, False), (32, 16, False), (32, 256, False), (48, 16, False), (48, 32, False),
-                           (64, 32, False), (128, 64, False), (16, 16, True), (32, 32, True), (48, 48, True), (64, 64, True),
-                           (80, 16, True), (128, 64, True), (128, 128, True), (160, 32, True))
+# (key size, value size, options: 1 kept first keys and a softcap, 2 a number by distance and a gate) whose attention
+# library `build_all` compiles ahead of time.
+DEFAULT_ATTENTION_SIZES = ((16, 32, 0), (16, 48, 0), (32, 16, 0), (32, 256, 0), (48, 16, 0), (48, 32, 0), (64, 32, 0), (128, 64, 0),
+                           (16, 16, 1), (32, 32, 1), (48, 48, 1), (64, 64, 1), (80, 16, 1), (128, 64, 1), (128, 128, 1), (160, 32, 1),
+                           (16, 16, 2), (32, 16, 2), (48, 80, 2), (64, 64, 2), (80, 48, 2), (128, 128, 2), (160, 32, 2), (16, 32, 3))
 # (key size, value size) pairs whose sigmoid-attention library `build_all` compiles ahead of time.
 DEFAULT_SIGATTN_SIZES = ((16, 32), (32, 64), (48, 16), (64, 64), (64, 128), (96, 32), (128, 32), (128, 64), (128, 128))
 # (key size, value size) pairs whose window-and-blocks attention library `build_all` compiles ahead of time.
@@ -148,7 +151,7 @@ def _fingerprint(sources: Sequence[str], defines: Sequence[str], host: bool = Fa
 
 
 def library_plan(name: str) -> Dict:
-    """Sources and defines of a library by its name ('core', 'attn_d<D>[_v<V>][_x]', 'sigattn_d<D>_v<V>', 'wpa_d<D>_v<V>', 'host'
+    """Sources and defines of a library by its name ('core', 'attn_d<D>[_v<V>][_x|_b|_xb]', 'sigattn_d<D>_v<V>', 'wpa_d<D>_v<V>', 'host'
     or 'blaslt')."""
     if name == "host":
         return {"sources": _existing(HOST_SOURCES), "defines": [], "host": True}
@@ -161,7 +164,11 @@ def library_plan(name: str) -> Dict:
     if name == "core":
         return {"sources": _existing(CORE_SOURCES), "defines": []}
     if name.startswith("attn_d"):
-        sizes, ext = (name[:-2], True) if name.endswith("_x") else (name, False)
+        sizes, ext = name, 0
+        for tail, bits in ATTENTION_OPTION_NAMES:
+            if name.endswith(tail):
+                sizes, ext = name[:-len(tail)], bits
+                break
         d, _, v = sizes[len("attn_d"):].partition("_v")
         v = v or d
         if not (d.isdigit() and v.isdigit() and int(d) in SUPPORTED_HEAD_DIMS and int(v) in SUPPORTED_HEAD_DIMS):
@@ -170,7 +177,7 @@ def library_plan(name: str) -> Dict:
         # vector instructions, which cannot reach the accumulation registers
         return {"sources": ["attention_mfma.hip"],
                 "defines": [f"-DIA_HEAD_DIM={int(d)}"]
-                + ([f"-DIA_VALUE_DIM={int(v)}"] if v != d else []) + (["-DIA_ATTN_EXT=1"] if ext else [])
+                + ([f"-DIA_VALUE_DIM={int(v)}"] if v != d else []) + ([f"-DIA_ATTN_EXT={ext}"] if ext else [])
                 + ["-mllvm", "-amdgpu-mfma-vgpr-form"]}
     if name.startswith("sigattn_d"):
         d, _, v = name[len("sigattn_d"):].partition("_v")
@@ -189,10 +196,15 @@ def library_plan(name: str) -> Dict:
     raise BuildError(f"unknown library {name!r}")
 
 
-def attention_library(d: int, dv: int, ext: bool = False) -> str:
-    """The name of the attention library for key heads of d and value heads of dv values; ``ext``: with kept first keys
-    under a window and a softcap."""
-    return f"attn_d{d}" + (f"_v{dv}" if dv != d else "") + ("_x" if ext else "")
+# the tails of attention libraries' names and the options they stand for (longest first)
+ATTENTION_OPTION_NAMES = (("_xb", 3), ("_x", 1), ("_b", 2))
+
+
+def attention_library(d: int, dv: int, ext: int = 0) -> str:
+    """The name of the attention library for key heads of d and value heads of dv values; ``ext``: 1 with kept first keys
+    under a window and a softcap, 2 with a number by distance and a gate, 3 with all of them."""
+    tail = next((t for t, bits in ATTENTION_OPTION_NAMES if bits == int(ext)), "")
+    return f"attn_d{d}" + (f"_v{dv}" if dv != d else "") + tail
 
 
 def library_path(name: str) -> str:

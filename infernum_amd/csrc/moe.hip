@@ -7,6 +7,8 @@
 //                    infinity, alpha 1, shift 0: y = silu(Wg x) (Wu x));
 //   ia_moe_down      per expert: Wd y times the pair's routing weight, as fp32 into parts[choice, token, :], which
 //                    the kernel that takes the feed-forward's result next adds in the order of the choices.
+// A routing weight can stand on the expert's INPUT instead: ia_moe_gate_up (and ia_moe_glu) given the weights multiply
+// both products with it, in fp32 (G (w x) = w (G x)), and ia_moe_down (and ia_moe_scatter) given none leave theirs as it is.
 // Only the chosen experts' weights are read.  A pair's result is one chain of operations over its own token and
 // its expert's weights, whatever else the step holds and wherever the sort has put it.
 #include "common.h"
@@ -137,7 +139,8 @@ template <typename T>
 __global__ __launch_bounds__(256) void moe_gate_up_kernel(const T* __restrict__ x, const T* __restrict__ Wgu,
                                                           T* __restrict__ y, const int* __restrict__ offsets,
                                                           const int* __restrict__ perm, int E, int top, int W,
-                                                          int ff, float limit, float alpha, float shift) {
+                                                          int ff, float limit, float alpha, float shift,
+                                                          const float* __restrict__ in_w) {
   __shared__ TileFmaLds lds;
   int e, first, last;
   if (!moe_tile(offsets, E, blockIdx.y, e, first, last)) return;
@@ -148,13 +151,14 @@ __global__ __launch_bounds__(256) void moe_gate_up_kernel(const T* __restrict__ 
   tile_64(a_row, w_row, W, lds, [&](int i, int j0, const float* v) {
     const int p = first + i;
     if (p >= last) return;
+    const float wt = in_w ? in_w[perm[p]] : 1.0f;
 #pragma unroll
     for (int j = 0; j < 4; j += 2) {
       const int c = n0 + j0 + j;
       if (c + 1 >= 2 * ff) continue;
       // both products are rounded as a stored tensor would be, then the activation in fp32
-      const float g = fminf(to_float(from_float<T>(v[j])), limit);
-      const float u = fminf(fmaxf(to_float(from_float<T>(v[j + 1])), -limit), limit);
+      const float g = fminf(wt * to_float(from_float<T>(v[j])), limit);
+      const float u = fminf(fmaxf(wt * to_float(from_float<T>(v[j + 1])), -limit), limit);
       y[(size_t)p * ff + (c >> 1)] = from_float<T>(g * (1.0f / (1.0f + expf(-alpha * g))) * (u + shift));
     }
   });
@@ -165,7 +169,8 @@ template <int BM, int BN>
 __global__ __launch_bounds__(BN == 256 ? 512 : 256) void moe_gate_up_big_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict__ Wgu,
                                                               bf16_t* __restrict__ y, const int* __restrict__ offsets,
                                                               const int* __restrict__ perm, int E, int top, int W,
-                                                              int ff, float limit, float alpha, float shift) {
+                                                              int ff, float limit, float alpha, float shift,
+                                                              const float* __restrict__ in_w) {
   __shared__ TileBigLds<BM, BN> lds;
   int e, first, last;
   if (!moe_tile(offsets, E, blockIdx.y, e, first, last, BM)) return;
@@ -176,12 +181,13 @@ __global__ __launch_bounds__(BN == 256 ? 512 : 256) void moe_gate_up_big_kernel(
       [&](int i, int j0, const float* v) {
         const int p = first + i;
         if (p >= last) return;
+        const float wt = in_w ? in_w[perm[p]] : 1.0f;
 #pragma unroll
         for (int j = 0; j < 4; j += 2) {
           const int c = n0 + j0 + j;
           if (c + 1 >= 2 * ff) continue;
-          const float g = fminf(to_float(from_float<bf16_t>(v[j])), limit);
-          const float u = fminf(fmaxf(to_float(from_float<bf16_t>(v[j + 1])), -limit), limit);
+          const float g = fminf(wt * to_float(from_float<bf16_t>(v[j])), limit);
+          const float u = fminf(fmaxf(wt * to_float(from_float<bf16_t>(v[j + 1])), -limit), limit);
           y[(size_t)p * ff + (c >> 1)] = from_float<bf16_t>(g * (1.0f / (1.0f + expf(-alpha * g))) * (u + shift));
         }
       });
@@ -192,14 +198,14 @@ static inline int moe_tile_rows(int P, int E) { return (long)P >= 48L * E ? 128 
 
 extern "C" int ia_moe_gate_up(const void* x, const void* Wgu, void* y, const int* offsets, const int* perm, int dtype,
                               int P, int E, int top, int W, int ff, float limit, float alpha, float shift,
-                              hipStream_t stream) {
+                              const float* in_weights, hipStream_t stream) {
   if (P < 0 || E <= 0 || top <= 0 || W <= 0 || ff <= 0) return IA_ERR_BAD_ARG;
   if (P == 0) return IA_OK;
   dim3 grid((2 * ff + TF_T - 1) / TF_T, (P + TF_T - 1) / TF_T + E);
   if (grid.y > 65535u) return IA_ERR_UNSUPPORTED;
   if (dtype == IA_F32)
     moe_gate_up_kernel<float><<<grid, 256, 0, stream>>>((const float*)x, (const float*)Wgu, (float*)y, offsets,
-                                                               perm, E, top, W, ff, limit, alpha, shift);
+                                                               perm, E, top, W, ff, limit, alpha, shift, in_weights);
   else if (dtype == IA_BF16 && tile_rows_aligned(x, W) && tile_rows_aligned(Wgu, W)) {
     const int bm = moe_tile_rows(P, E);
     const int bn = bm == 128 ? 256 : TB_N;
@@ -207,14 +213,14 @@ extern "C" int ia_moe_gate_up(const void* x, const void* Wgu, void* y, const int
     if (big.y > 65535u) return IA_ERR_UNSUPPORTED;
     if (bm == 128)
       moe_gate_up_big_kernel<128, 256><<<big, 512, 0, stream>>>((const bf16_t*)x, (const bf16_t*)Wgu, (bf16_t*)y, offsets,
-                                                           perm, E, top, W, ff, limit, alpha, shift);
+                                                           perm, E, top, W, ff, limit, alpha, shift, in_weights);
     else
       moe_gate_up_big_kernel<32, TB_N><<<big, 256, 0, stream>>>((const bf16_t*)x, (const bf16_t*)Wgu, (bf16_t*)y, offsets,
-                                                          perm, E, top, W, ff, limit, alpha, shift);
+                                                          perm, E, top, W, ff, limit, alpha, shift, in_weights);
   }
   else if (dtype == IA_BF16)
     moe_gate_up_kernel<bf16_t><<<grid, 256, 0, stream>>>((const bf16_t*)x, (const bf16_t*)Wgu, (bf16_t*)y,
-                                                                offsets, perm, E, top, W, ff, limit, alpha, shift);
+                                                                offsets, perm, E, top, W, ff, limit, alpha, shift, in_weights);
   else
     return IA_ERR_BAD_ARG;
   IA_LAUNCH_CHECK();
@@ -239,7 +245,7 @@ __global__ __launch_bounds__(256) void moe_down_kernel(const T* __restrict__ y, 
     if (p >= last) return;
     const int pair = perm[p];
     const int token = pair / top, choice = pair - token * top;
-    const float wt = weights[pair];
+    const float wt = weights ? weights[pair] : 1.0f;
     float* o = parts + ((size_t)choice * N + token) * W;
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
@@ -266,7 +272,7 @@ __global__ __launch_bounds__(BN == 256 ? 512 : 256) void moe_down_big_kernel(con
         if (p >= last) return;
         const int pair = perm[p];
         const int token = pair / top, choice = pair - token * top;
-        const float wt = weights[pair];
+        const float wt = weights ? weights[pair] : 1.0f;
         float* o = parts + ((size_t)choice * N + token) * W;
 #pragma unroll
         for (int j = 0; j < 4; ++j) {
@@ -333,16 +339,18 @@ extern "C" int ia_moe_gather(const void* x, const int* perm, void* xs, int P, in
 }
 
 __global__ __launch_bounds__(256) void moe_glu_kernel(const uint4* __restrict__ gu, uint2* __restrict__ y, size_t n4,
-                                                      float limit, float alpha, float shift) {
+                                                      float limit, float alpha, float shift, const int* __restrict__ perm,
+                                                      const float* __restrict__ in_w, int quads) {
   const size_t stride = (size_t)gridDim.x * 256;
   for (size_t i = (size_t)blockIdx.x * 256 + threadIdx.x; i < n4; i += stride) {
     const uint4 v = gu[i];
     const uint32_t w[4] = {v.x, v.y, v.z, v.w};
     float o[4];
+    const float wt = in_w ? in_w[perm[i / quads]] : 1.0f;
 #pragma unroll
     for (int k = 0; k < 4; ++k) {
-      const float g = fminf(__uint_as_float(w[k] << 16), limit);
-      const float u = fminf(fmaxf(__uint_as_float(w[k] & 0xffff0000u), -limit), limit);
+      const float g = fminf(wt * __uint_as_float(w[k] << 16), limit);
+      const float u = fminf(fmaxf(wt * __uint_as_float(w[k] & 0xffff0000u), -limit), limit);
       o[k] = g * (1.0f / (1.0f + expf(-alpha * g))) * (u + shift);
     }
     uint2 r;
@@ -352,13 +360,14 @@ __global__ __launch_bounds__(256) void moe_glu_kernel(const uint4* __restrict__ 
   }
 }
 
-extern "C" int ia_moe_glu(const void* gu, void* y, int P, int ff, float limit, float alpha, float shift, hipStream_t stream) {
-  if (P < 0 || ff <= 0) return IA_ERR_BAD_ARG;
+extern "C" int ia_moe_glu(const void* gu, void* y, int P, int ff, float limit, float alpha, float shift, const int* perm,
+                          const float* in_weights, hipStream_t stream) {
+  if (P < 0 || ff <= 0 || (in_weights && !perm)) return IA_ERR_BAD_ARG;
   if ((ff & 3) || ((reinterpret_cast<uintptr_t>(gu) | reinterpret_cast<uintptr_t>(y)) & 15)) return IA_ERR_UNSUPPORTED;
   const size_t n4 = (size_t)P * ff / 4;
   if (n4 == 0) return IA_OK;
   const unsigned grid = (unsigned)((n4 + 255) / 256 < 65536 ? (n4 + 255) / 256 : 65536);
-  moe_glu_kernel<<<grid, 256, 0, stream>>>((const uint4*)gu, (uint2*)y, n4, limit, alpha, shift);
+  moe_glu_kernel<<<grid, 256, 0, stream>>>((const uint4*)gu, (uint2*)y, n4, limit, alpha, shift, perm, in_weights, ff / 4);
   IA_LAUNCH_CHECK();
   return IA_OK;
 }
@@ -370,7 +379,7 @@ __global__ __launch_bounds__(256) void moe_scatter_kernel(const uint4* __restric
   if (last && p >= *last) return;                  // a pair that went to no expert with tensors
   const int pair = perm[p];
   const int token = pair / top, choice = pair - token * top;
-  const float wt = weights[pair];
+  const float wt = weights ? weights[pair] : 1.0f;
   const uint4* src = o + (size_t)p * (W / 8);
   float4* dst = reinterpret_cast<float4*>(parts + ((size_t)choice * N + token) * W);
   for (int i = threadIdx.x; i < W / 8; i += 256) {
@@ -395,7 +404,8 @@ extern "C" int ia_moe_scatter(const void* o, const int* perm, const float* weigh
 // ---- experts without a gate, and a router whose choice and weights go by different numbers ----
 //   ia_router_softmax_topk   s = softmax(z) over all experts; the `top` largest of s + correction are chosen (the
 //                            lowest index among equals); the weights are the chosen s, with `renorm` over their sum
-//                            (+ 1e-20).  With `groups` > 1 the experts form that many groups of neighbours, a group's
+//                            (+ 1e-20).  With `sigmoid` s = sigmoid(z) instead, and without a correction the choice goes
+//                            by z itself (large z have equal s in fp32).  With `groups` > 1 the experts form that many groups of neighbours, a group's
 //                            score is its largest s + correction, and only experts of the `keep` best groups (the
 //                            lowest index among equals) can be chosen;
 //   ia_moe_up                per expert, over its pairs' tokens: y = act(Wu x), Wu [E, ff, W]; act by the codes of
@@ -413,7 +423,7 @@ __global__ __launch_bounds__(256) void router_softmax_topk_kernel(const float* _
                                                                   const void* __restrict__ corr, int corr_dtype,
                                                                   int* __restrict__ ids, float* __restrict__ weights,
                                                                   int N, int E, int top, int z_stride, int groups,
-                                                                  int keep, int renorm) {
+                                                                  int keep, int renorm, int sigmoid) {
   __shared__ float s_v[4][64 * PL];       // a wave's choice scores, then (in place) its groups' scores
   const int n = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
   if (n >= N) return;
@@ -440,8 +450,14 @@ __global__ __launch_bounds__(256) void router_softmax_topk_kernel(const float* _
 #pragma unroll
   for (int c = 0; c < PL; ++c) {
     const int e = lane + 64 * c;
-    s[c] *= inv_total;
-    v[c] = e < E ? s[c] + (corr ? load_as_float(corr, corr_dtype, e) : 0.f) : -INFINITY;
+    if (sigmoid) {
+      const float x = e < E ? z[e] : -INFINITY;
+      s[c] = 1.0f / (1.0f + expf(-x));
+      v[c] = e < E ? (corr ? s[c] + load_as_float(corr, corr_dtype, e) : x) : -INFINITY;
+    } else {
+      s[c] *= inv_total;
+      v[c] = e < E ? s[c] + (corr ? load_as_float(corr, corr_dtype, e) : 0.f) : -INFINITY;
+    }
   }
   if (groups > 1) {
     // each wave works on its own part of LDS: a wave's accesses are in order, no barrier is needed between them
@@ -508,14 +524,14 @@ __global__ __launch_bounds__(256) void router_softmax_topk_kernel(const float* _
 
 extern "C" int ia_router_softmax_topk(const float* logits, const void* corr, int corr_dtype, int* ids, float* weights,
                                       int N, int E, int top, int z_stride, int groups, int keep, int renorm,
-                                      hipStream_t stream) {
+                                      int sigmoid, hipStream_t stream) {
   if (N < 0 || E <= 0 || top <= 0 || top > E || z_stride < E || groups < 1 || E % groups || keep < 1 || keep > groups ||
       top > keep * (E / groups) || !logits || !ids || !weights) return IA_ERR_BAD_ARG;
   if (E > 64 * RT_PER_LANE) return IA_ERR_UNSUPPORTED;
   if (N == 0) return IA_OK;
 #define IA_RT(PL)                                                                                                        \
   router_softmax_topk_kernel<PL><<<(N + 3) / 4, 256, 0, stream>>>(logits, corr, corr_dtype, ids, weights, N, E, top, z_stride, \
-                                                                  groups, keep, renorm)
+                                                                  groups, keep, renorm, sigmoid)
   if (E <= 64) IA_RT(1);
   else if (E <= 256) IA_RT(4);
   else IA_RT(RT_PER_LANE);

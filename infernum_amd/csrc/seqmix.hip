@@ -9,6 +9,8 @@
 //                          for all heads), rotation of neighbouring or half-split pairs with a factor on sine and
 //                          cosine, the keys to their pages, and as values either the value heads of the row or the
 //                          key heads as they came in
+//   ia_qk_rows_prepare     the same for norms over ALL of a token's queries (and over all of its keys), a weight per value,
+//                          without rotation
 //   ia_ssd_scan            the selective state-space recurrence  S <- a S + dt B x^T,  y = S^T C + D x  per head,
 //                          the state [N, P] of every request in its slot (fp32), token after token
 //   ia_ssd_chunked         the same recurrence as matrix products over chunks of 64 tokens, for portions of prompts
@@ -16,6 +18,7 @@
 //   ia_concat_cast         rows [cast(a) | b]: the operand of a product over two streams side by side
 //   ia_stream_add         the fp32 stream += a tensor or the partial sums of a split product
 //   ia_stream_add2        the same for two of them one after the other, leaving the rounded stream as well
+//   ia_add_vector          one vector added to every row of the fp32 stream
 //   ia_add_bias, ia_softcap
 //
 // Everything between the loads and the stores is fp32: sums of squares, angles, decays, step sizes, the state.
@@ -553,6 +556,131 @@ extern "C" int ia_qk_prepare(const void* x, int code, int x_stride, void* q_out,
                                                        page_size, num_pages, values_are_keys, V);
   else
     return IA_ERR_BAD_ARG;
+  IA_LAUNCH_CHECK();
+  return IA_OK;
+}
+
+// Eight values of a value head to their transposed page: wave w of the value writers takes 16 tokens and 32 values, so that
+// what it writes are stretches of up to 16 positions.
+__device__ __forceinline__ void values_to_page(const bf16_t* __restrict__ rows, int x_stride, const int* __restrict__ slots,
+                                               bf16_t* __restrict__ v_pages, long w, int lane, int N, int nkv, int dv,
+                                               int page_size, int num_pages, float scale) {
+  const int pieces = nkv * dv / 8, groups = (pieces + 3) / 4;          // 8 values a lane, 4 lanes side by side
+  const int t = (int)(w / groups) * 16 + (lane & 15), piece = (int)(w % groups) * 4 + (lane >> 4);
+  if (t >= N || piece >= pieces) return;
+  const int slot = slots[t], page = slot / page_size, off = slot - page * page_size;
+  if (page < 0 || page >= num_pages) return;
+  const int col = piece * 8, g = col / dv, c = col - g * dv;
+  const uint4 raw = *(const uint4*)(rows + (size_t)t * x_stride + col);
+  const uint32_t rw[4] = {raw.x, raw.y, raw.z, raw.w};
+  uint16_t* vdst = (uint16_t*)v_pages + ((size_t)page * nkv + g) * (size_t)dv * page_size + (size_t)c * page_size + off;
+#pragma unroll
+  for (int e = 0; e < 4; ++e) {
+    vdst[(size_t)(2 * e) * page_size] = float_to_bf16_bits(scale * __uint_as_float(rw[e] << 16));
+    vdst[(size_t)(2 * e + 1) * page_size] = float_to_bf16_bits(scale * __uint_as_float(rw[e] & 0xffff0000u));
+  }
+}
+
+// One workgroup a token: the root mean square over all of its nh d queries, then over all of its nkv d keys, each value
+// times a weight of its own; queries to q_out, keys to their page.  VEC: bf16 rows of whole 16-byte pieces, whose values
+// the workgroups from N on write; without it a token's workgroup writes its values too.
+template <typename T, bool VEC>
+__global__ __launch_bounds__(256) void qk_rows_prepare_kernel(
+    const T* __restrict__ x, int x_stride, T* __restrict__ q_out, int q_stride, const float* __restrict__ wq,
+    const float* __restrict__ wk, float eps, const int* __restrict__ slots, T* __restrict__ k_pages, T* __restrict__ v_pages,
+    int N, int nh, int nkv, int d, int dv, int page_size, int num_pages, float v_scale) {
+  __shared__ float red[4];
+  const int tid = threadIdx.x, nq = nh * d, nk = nkv * d;
+  if constexpr (VEC) {
+    if ((int)blockIdx.x >= N) {
+      values_to_page(x + nq + nk, x_stride, slots, v_pages, (long)((int)blockIdx.x - N) * 4 + (tid >> 6), tid & 63, N, nkv,
+                     dv, page_size, num_pages, v_scale);
+      return;
+    }
+  }
+  const int n = blockIdx.x;
+  const T* row = x + (size_t)n * x_stride;
+  const int slot = slots[n], page = slot / page_size, off = slot - page * page_size;
+  const bool place = (unsigned)page < (unsigned)num_pages;            // a token without a place: its keys are not written
+#pragma unroll
+  for (int part = 0; part < 2; ++part) {
+    const int cols = part ? nk : nq;
+    const T* src = part ? row + nq : row;
+    const float* w = part ? wk : wq;
+    float ss = 0.f;
+    if constexpr (VEC) {
+      for (int i = tid * 8; i < cols; i += 2048) {
+        const uint4 v = *(const uint4*)(src + i);
+        const uint32_t u[4] = {v.x, v.y, v.z, v.w};
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          const float a = __uint_as_float(u[e] << 16), b = __uint_as_float(u[e] & 0xffff0000u);
+          ss = __builtin_fmaf(a, a, ss);
+          ss = __builtin_fmaf(b, b, ss);
+        }
+      }
+    } else {
+      for (int i = tid; i < cols; i += 256) {
+        const float v = to_float(src[i]);
+        ss = __builtin_fmaf(v, v, ss);
+      }
+    }
+    ss = block_sum<256>(ss, red);
+    const float inv = 1.0f / sqrtf(ss / (float)cols + eps);
+    if (part && !place) return;
+    if constexpr (VEC) {
+      for (int i = tid * 8; i < cols; i += 2048) {
+        const uint4 v = *(const uint4*)(src + i);
+        const uint32_t u[4] = {v.x, v.y, v.z, v.w};
+        const float4 w0 = *(const float4*)(w + i), w1 = *(const float4*)(w + i + 4);
+        const float wv[8] = {w0.x, w0.y, w0.z, w0.w, w1.x, w1.y, w1.z, w1.w};
+        uint32_t o[4];
+#pragma unroll
+        for (int e = 0; e < 4; ++e)
+          o[e] = (uint32_t)float_to_bf16_bits(__uint_as_float(u[e] << 16) * inv * wv[2 * e]) |
+                 ((uint32_t)float_to_bf16_bits(__uint_as_float(u[e] & 0xffff0000u) * inv * wv[2 * e + 1]) << 16);
+        const int g = part ? i / d : 0;
+        T* dst = part ? k_pages + (((size_t)page * nkv + g) * page_size + off) * d + (i - g * d) : q_out + (size_t)n * q_stride + i;
+        *(uint4*)dst = make_uint4(o[0], o[1], o[2], o[3]);
+      }
+    } else {
+      for (int i = tid; i < cols; i += 256) {
+        const int g = part ? i / d : 0;
+        T* dst = part ? k_pages + (((size_t)page * nkv + g) * page_size + off) * d + (i - g * d) : q_out + (size_t)n * q_stride + i;
+        *dst = from_float<T>(to_float(src[i]) * inv * w[i]);
+      }
+    }
+  }
+  if constexpr (!VEC) {
+    for (int i = tid; i < nkv * dv; i += 256) {
+      const int g = i / dv, c = i - g * dv;
+      v_pages[(((size_t)page * nkv + g) * dv + c) * page_size + off] = from_float<T>(v_scale * to_float(row[nq + nk + i]));
+    }
+  }
+}
+
+// x rows [nh d | nkv d | nkv dv | ...] of x_stride values; wq fp32 [nh d], wk fp32 [nkv d].
+extern "C" int ia_qk_rows_prepare(const void* x, int code, int x_stride, void* q_out, int q_stride, const float* wq,
+                                  const float* wk, float eps, const int* slots, void* k_pages, void* v_pages, int N, int nh,
+                                  int nkv, int d, int dv, int page_size, int num_pages, float v_scale, hipStream_t stream) {
+  if (N == 0) return IA_OK;
+  if (!x || !q_out || !wq || !wk || !slots || !k_pages || !v_pages || N < 0 || nh <= 0 || nkv <= 0 || d <= 0 || dv <= 0 ||
+      page_size <= 0 || num_pages <= 0 || !(eps > 0.f) || x_stride < (nh + nkv) * d + nkv * dv || q_stride < nh * d)
+    return IA_ERR_BAD_ARG;
+#define IA_QKR(T, VEC, GRID)                                                                                              \
+  qk_rows_prepare_kernel<T, VEC><<<(unsigned)(GRID), 256, 0, stream>>>((const T*)x, x_stride, (T*)q_out, q_stride, wq, wk, eps, \
+                                                                       slots, (T*)k_pages, (T*)v_pages, N, nh, nkv, d, dv,   \
+                                                                       page_size, num_pages, v_scale)
+  if (code == IA_F32) IA_QKR(float, false, N);
+  else if (code != IA_BF16) return IA_ERR_BAD_ARG;
+  else if (d % 8 == 0 && dv % 8 == 0 && x_stride % 8 == 0 && q_stride % 8 == 0 && !((uintptr_t)x & 15) && !((uintptr_t)q_out & 15) &&
+           !((uintptr_t)k_pages & 15) && !((uintptr_t)wq & 15) && !((uintptr_t)wk & 15)) {
+    const long v_waves = (long)((N + 15) / 16) * ((nkv * dv / 8 + 3) / 4);
+    const long blocks = N + (v_waves + 3) / 4;
+    if (blocks > 0x7fffffffL) return IA_ERR_UNSUPPORTED;
+    IA_QKR(bf16_t, true, blocks);
+  } else IA_QKR(bf16_t, false, N);
+#undef IA_QKR
   IA_LAUNCH_CHECK();
   return IA_OK;
 }
@@ -1143,6 +1271,21 @@ extern "C" int ia_stream_add2(float* h, const void* a, int a_code, int a_splits,
   return IA_OK;
 }
 
+// h [N, H] fp32 += v [H], the same vector for every row
+__global__ __launch_bounds__(256) void add_vector_kernel(float* __restrict__ h, const void* __restrict__ v, int v_code, size_t n, int H) {
+  const size_t i = (size_t)blockIdx.x * 256 + threadIdx.x;
+  if (i < n) h[i] += load_as_float(v, v_code, i % H);
+}
+
+extern "C" int ia_add_vector(float* h, const void* v, int v_code, int N, int H, hipStream_t stream) {
+  if (N == 0) return IA_OK;
+  if (!h || !v || N < 0 || H <= 0 || (v_code != IA_F32 && v_code != IA_BF16)) return IA_ERR_BAD_ARG;
+  const size_t n = (size_t)N * H;
+  add_vector_kernel<<<(unsigned)((n + 255) / 256), 256, 0, stream>>>(h, v, v_code, n, H);
+  IA_LAUNCH_CHECK();
+  return IA_OK;
+}
+
 // y [N, C] += bias (fp32 vector), rounded once
 template <typename T>
 __global__ __launch_bounds__(256) void add_bias_kernel(T* __restrict__ y, const float* __restrict__ bias, size_t n, int C) {
@@ -1185,6 +1328,8 @@ IA_OP(ia_causal_conv)
 IA_OP(ia_causal_conv_single)
 IA_OP(ia_conv_state_update)
 IA_OP(ia_qk_prepare)
+IA_OP(ia_qk_rows_prepare)
+IA_OP(ia_add_vector)
 IA_OP(ia_ssd_scan)
 IA_OP(ia_ssd_chunked)
 IA_OP(ia_gated_group_norm)

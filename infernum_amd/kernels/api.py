@@ -333,11 +333,13 @@ def moe_grouped_rows(N: int, E: int, top: int, W: int, ff: int, dtype: torch.dty
 
 def moe_experts(x: torch.Tensor, ids: torch.Tensor, weights: torch.Tensor, w_gate_up: torch.Tensor,
                 w_down: torch.Tensor, limit: float, alpha: float, shift: float = 1.0, total: int = 0,
-                parts: Optional[torch.Tensor] = None) -> SplitSum:
+                parts: Optional[torch.Tensor] = None, weights_on: str = "output") -> SplitSum:
     """The chosen experts of every token: w_gate_up [E, 2 ff, W] with the gate's and up's rows alternating,
     w_down [E, W, ff].  y = g sigmoid(alpha g) (u + shift) with g = min(gate, limit), u = clamp(up, -limit, limit).
     Fills parts[:top] of fp32 ``parts`` [>= top, N, W], each already times its routing weight, and returns them as a sum.
-    ``total`` > E: ids go up to it, and those from E on are experts without tensors, whose pairs are left alone."""
+    ``total`` > E: ids go up to it, and those from E on are experts without tensors, whose pairs are left alone.
+    ``weights_on`` "input": the weight multiplies what the expert reads (both of its first products), not what it leaves."""
+    in_w, out_w = (weights, None) if weights_on == "input" else (None, weights)
     _dev(x, ids, weights, w_gate_up, w_down, parts)
     N, W = x.shape
     E, two_ff, _ = w_gate_up.shape
@@ -364,14 +366,15 @@ def moe_experts(x: torch.Tensor, ids: torch.Tensor, weights: torch.Tensor, w_gat
         _ok(_core().ia_moe_gather(_p(x), _p(perm), _p(xs), P, top, W, _stream()), "moe_gather")
         gemm_mfma_grouped(xs, w_gate_up, offsets, gu)
         _ok(_core().ia_moe_glu(_p(gu), _p(y), P, ff, ctypes.c_float(limit), ctypes.c_float(alpha),
-                               ctypes.c_float(shift), _stream()), "moe_glu")
+                               ctypes.c_float(shift), _p(perm), _p(in_w), _stream()), "moe_glu")
         gemm_mfma_grouped(y, w_down, offsets, xs)
-        _ok(_core().ia_moe_scatter(_p(xs), _p(perm), _p(weights), _p(parts), _p(offsets[E:] if total > E else None), N, top,
+        _ok(_core().ia_moe_scatter(_p(xs), _p(perm), _p(out_w), _p(parts), _p(offsets[E:] if total > E else None), N, top,
                                    W, _stream()), "moe_scatter")
         return SplitSum(parts)
     _ok(_core().ia_moe_gate_up(_p(x), _p(w_gate_up), _p(y), _p(offsets), _p(perm), code, P, E, top, W, ff,
-                               ctypes.c_float(limit), ctypes.c_float(alpha), ctypes.c_float(shift), _stream()), "moe_gate_up")
-    _ok(_core().ia_moe_down(_p(y), _p(w_down), _p(parts), _p(weights), _p(offsets), _p(perm), code, N, E, top, W, ff,
+                               ctypes.c_float(limit), ctypes.c_float(alpha), ctypes.c_float(shift), _p(in_w), _stream()),
+        "moe_gate_up")
+    _ok(_core().ia_moe_down(_p(y), _p(w_down), _p(parts), _p(out_w), _p(offsets), _p(perm), code, N, E, top, W, ff,
                             _stream()), "moe_down")
     return SplitSum(parts)
 
@@ -765,13 +768,16 @@ def _rows_of(t: torch.Tensor) -> int:
 def attention_generic(qkv: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.Tensor, out: torch.Tensor,
                       token_seq: torch.Tensor, positions: torch.Tensor, block_tables: torch.Tensor, nh: int,
                       nkv: int, d: int, scale: float, window: int = 0, sinks: Optional[torch.Tensor] = None,
-                      keep: int = 0, softcap: float = 0.0) -> None:
+                      keep: int = 0, softcap: float = 0.0, bias: Optional[torch.Tensor] = None,
+                      gate: Optional[torch.Tensor] = None) -> None:
     """Causal paged attention, one wave per (token, head), fp32 arithmetic.  ``sinks`` fp32 [nh]: exp(sinks[h]) is
     added to the softmax's denominator of head h.  ``keep``: under a window the request's first ``keep`` keys stay
     visible.  ``softcap`` c > 0: a scaled score s becomes c tanh(s / c).  The value heads' size is that of the pages.
 
     qkv [N, >= nh*d]: the q heads of token n are the first nh*d values of row n.
     token_seq[n] is the row of block_tables of token n; positions[n] its position.
+    ``bias``: a table of :func:`distance_table`, a number added to the (scaled, capped) score by head and distance.
+    ``gate`` [N, >= nh dv] of out's dtype (columns of wider rows): what the heads leave, times sigmoid(gate), value by value.
     """
     dv = _check_paged(qkv, k_pages, v_pages, out, block_tables, nh, nkv, d, "attention")
     N = out.shape[0]
@@ -783,12 +789,41 @@ def attention_generic(qkv: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.T
                                      DTYPE_CODE[out.dtype], _p(token_seq), _p(positions), _p(block_tables),
                                      block_tables.shape[1], N, nh, nkv, d, dv, k_pages.shape[2], k_pages.shape[0],
                                      ctypes.c_float(scale), int(window), _p(sinks), int(keep), ctypes.c_float(softcap),
-                                     _stream()), "attention_generic")
+                                     *_bias_and_gate(bias, gate, nh, dv, out), _stream()), "attention_generic")
 
 
-def _attn(d: int, dv: Optional[int] = None, ext: bool = False) -> ctypes.CDLL:
-    """The matrix-core attention library for key heads of d and value heads of dv values; ``ext``: the one that takes
-    kept first keys and a softcap."""
+DISTANCE_PAD = 64           # numbers before and behind a head's own in a table of distances
+
+
+def distance_table(by_distance: torch.Tensor) -> torch.Tensor:
+    """by_distance fp32 [heads, span]: what is added to the score of a key so many places back, the last number for all
+    keys further back.  -> [heads, span + 2 DISTANCE_PAD] as the attention kernels read it: backwards over the distance,
+    with the furthest number before it and zeros behind it."""
+    t = by_distance.to(torch.float32).flip(1)
+    return torch.cat([t[:, :1].expand(-1, DISTANCE_PAD), t, t.new_zeros((t.shape[0], DISTANCE_PAD))], dim=1).contiguous()
+
+
+def _bias_and_gate(bias, gate, nh: int, dv: int, out: torch.Tensor) -> tuple:
+    span, stride = 0, 0
+    if bias is not None:
+        _need(bias.is_cuda and bias.dtype == torch.float32 and bias.is_contiguous() and bias.dim() == 2
+              and bias.shape[0] == nh and bias.shape[1] > 2 * DISTANCE_PAD, "attention: a table of distance_table for every head")
+        span = int(bias.shape[1]) - 2 * DISTANCE_PAD
+    if gate is not None:
+        _rows(gate, nh * dv, "attention gate")
+        _need(gate.dtype == out.dtype and gate.shape[0] >= out.shape[0], "attention: gates of out's dtype, a row a token")
+        stride = _rows_of(gate)
+    return _p(bias), span, _p(gate), stride
+
+
+def attention_options(keep: int = 0, softcap: float = 0.0, bias: bool = False, gate: bool = False) -> int:
+    """Which of its options a launch of the matrix-core kernels uses (csrc/build.attention_library)."""
+    return int(keep > 0 or softcap > 0) | (2 if bias or gate else 0)
+
+
+def _attn(d: int, dv: Optional[int] = None, ext: int = 0) -> ctypes.CDLL:
+    """The matrix-core attention library for key heads of d and value heads of dv values; ``ext``: the options it takes
+    (:func:`attention_options`)."""
     return load_library(_build.attention_library(d, dv or d, ext))
 
 
@@ -835,11 +870,12 @@ def decode_splits(batch: int, nh: int, nkv: int, max_len: int, device: Optional[
 def attention_decode(qkv: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.Tensor, out: torch.Tensor,
                      positions: torch.Tensor, block_tables: torch.Tensor, nh: int, nkv: int, d: int, scale: float,
                      window: int, max_len: int, num_splits: Optional[int] = None,
-                     sinks: Optional[torch.Tensor] = None, keep: int = 0, softcap: float = 0.0) -> None:
+                     sinks: Optional[torch.Tensor] = None, keep: int = 0, softcap: float = 0.0,
+                     bias: Optional[torch.Tensor] = None, gate: Optional[torch.Tensor] = None) -> None:
     """bf16 attention of B single tokens (row b of qkv: token b at positions[b]) over their pages, on MFMA.
 
-    ``max_len`` bounds the positions (host side), and sets how many parts the keys are split into.  ``keep`` and
-    ``softcap``: see :func:`attention_generic`.
+    ``max_len`` bounds the positions (host side), and sets how many parts the keys are split into.  ``keep``,
+    ``softcap``, ``bias`` and ``gate``: see :func:`attention_generic`.
     """
     dv = _check_paged(qkv, k_pages, v_pages, out, block_tables, nh, nkv, d, "attention_decode")
     B = out.shape[0]
@@ -854,10 +890,11 @@ def attention_decode(qkv: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.Te
     if splits > 1:
         part_o = torch.empty(B * nh * splits * dv, dtype=torch.float32, device=out.device)
         part_ml = torch.empty(B * nh * splits * 2, dtype=torch.float32, device=out.device)
-    _ok(_attn(d, dv, keep > 0 or softcap > 0).ia_attn_decode(
+    _ok(_attn(d, dv, attention_options(keep, softcap, bias is not None, gate is not None)).ia_attn_decode(
         _p(qkv), _rows_of(qkv), _p(k_pages), _p(v_pages), _p(out), _rows_of(out), _p(part_o), _p(part_ml),
         _p(positions), _p(block_tables), block_tables.shape[1], B, nh, nkv, ps, k_pages.shape[0], ctypes.c_float(scale),
-        int(window), splits, _p(sinks), int(keep), ctypes.c_float(softcap), _stream()), "attention_decode")
+        int(window), splits, _p(sinks), int(keep), ctypes.c_float(softcap), *_bias_and_gate(bias, gate, nh, dv, out), _stream()),
+        "attention_decode")
 
 
 def attention_decode_rotating(qkv, positions: torch.Tensor, inv_freq: Optional[torch.Tensor], rot: int,
@@ -921,7 +958,8 @@ def attention_prefill(qkv: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.T
                       seq_starts: torch.Tensor, seq_ctx: torch.Tensor, block_tables: torch.Tensor,
                       tiles: torch.Tensor, num_tiles: int, nh: int, nkv: int, d: int, scale: float,
                       window: int, heads_per_workgroup: int = 0, paired: bool = False,
-                      sinks: Optional[torch.Tensor] = None, keep: int = 0, softcap: float = 0.0) -> None:
+                      sinks: Optional[torch.Tensor] = None, keep: int = 0, softcap: float = 0.0,
+                      bias: Optional[torch.Tensor] = None, gate: Optional[torch.Tensor] = None) -> None:
     """bf16 causal attention of portions of prompts over their pages, on MFMA.
 
     Request s brings rows seq_starts[s] .. seq_starts[s+1]-1 of qkv and had seq_ctx[s] tokens cached
@@ -929,8 +967,8 @@ def attention_prefill(qkv: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.T
     0 for the kernel's own choice, or 1, 2, 4; ``paired``: a workgroup takes half a block of rows from each end of
     its request's new tokens, so that all workgroups of a request have the same work under the causal mask (every
     block of every request must be listed then; without effect under a window).  A value of :func:`prefill_launch_shape` may stand in
-    ``heads_per_workgroup`` for both.  The result has the same bits whatever the shape.  ``keep`` and ``softcap``: see
-    :func:`attention_generic`.
+    ``heads_per_workgroup`` for both.  The result has the same bits whatever the shape.  ``keep``, ``softcap``, ``bias``
+    and ``gate``: see :func:`attention_generic`.
     """
     dv = _check_paged(qkv, k_pages, v_pages, out, block_tables, nh, nkv, d, "attention_prefill")
     _need(qkv.dtype == torch.bfloat16, "attention_prefill: bf16 only")
@@ -941,11 +979,11 @@ def attention_prefill(qkv: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.T
           "attention_prefill: tiles int32 [num_tiles, 2]")
     ps = k_pages.shape[2]
     _need(ps % 4 == 0, f"attention_prefill: page size {ps} is not a multiple of 4")
-    _ok(_attn(d, dv, keep > 0 or softcap > 0).ia_attn_prefill(
+    _ok(_attn(d, dv, attention_options(keep, softcap, bias is not None, gate is not None)).ia_attn_prefill(
         _p(qkv), _rows_of(qkv), _p(k_pages), _p(v_pages), _p(out), _rows_of(out), _p(seq_starts), _p(seq_ctx),
         _p(block_tables), block_tables.shape[1], _p(tiles), num_tiles, nh, nkv, ps, k_pages.shape[0],
         ctypes.c_float(scale), int(window), int(heads_per_workgroup) | (PREFILL_PAIRED if paired else 0), _p(sinks),
-        int(keep), ctypes.c_float(softcap), _stream()), "attention_prefill")
+        int(keep), ctypes.c_float(softcap), *_bias_and_gate(bias, gate, nh, dv, out), _stream()), "attention_prefill")
 
 
 def prefill_launch_shape(nh: int, nkv: int, d: int, q_lens: Sequence[int], ctx_lens: Sequence[int],
@@ -1119,6 +1157,188 @@ def qk_prepare(x: torch.Tensor, q_out: torch.Tensor, nh: int, nkv: int, d: int, 
                               v_first.stride(0) if v_first is not None else 0, ctypes.c_float(v_lambda), _stream()),
         "qk_prepare")
     return q_out
+
+
+def qk_rows_prepare(x: torch.Tensor, q_out: torch.Tensor, nh: int, nkv: int, d: int, q_weight: torch.Tensor,
+                    k_weight: torch.Tensor, eps: float, slots: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.Tensor,
+                    v_scale: float = 1.0) -> torch.Tensor:
+    """Rows [nh d queries | nkv d keys | nkv dv values]: all of a token's queries divided by their root mean square and
+    multiplied by a weight each (``q_weight`` fp32 [nh d]) into ``q_out`` [N, nh d], all of its keys likewise
+    (``k_weight`` [nkv d]) and the values times ``v_scale`` into their pages at ``slots``."""
+    N, (num_pages, _, ps, _), dv = x.shape[0], k_pages.shape, v_pages.shape[2]
+    _rows(x, (nh + nkv) * d + nkv * dv, "qk_rows_prepare input")
+    _rows(q_out, nh * d, "qk_rows_prepare q_out")
+    _f32(q_weight, nh * d, "qk_rows_prepare q weight")
+    _f32(k_weight, nkv * d, "qk_rows_prepare k weight")
+    _i32(slots, N, "qk_rows_prepare slots")
+    _need(q_out.dtype == x.dtype and q_out.shape[0] == N and k_pages.dtype == x.dtype and v_pages.dtype == x.dtype
+          and tuple(k_pages.shape) == (num_pages, nkv, ps, d) and tuple(v_pages.shape) == (num_pages, nkv, dv, ps)
+          and k_pages.is_contiguous() and v_pages.is_contiguous(),
+          "qk_rows_prepare: key pages [num_pages, nkv, page_size, d], value pages [num_pages, nkv, dv, page_size]")
+    _ok(_core().ia_qk_rows_prepare(_p(x), DTYPE_CODE[x.dtype], _rows_of(x), _p(q_out), _rows_of(q_out), _p(q_weight),
+                                   _p(k_weight), ctypes.c_float(eps), _p(slots), _p(k_pages), _p(v_pages), N, nh, nkv, d, dv,
+                                   ps, num_pages, ctypes.c_float(v_scale), _stream()), "qk_rows_prepare")
+    return q_out
+
+
+def add_vector(h: torch.Tensor, v: torch.Tensor) -> torch.Tensor:
+    """h [N, H] fp32 += v [H], the same vector for every row."""
+    _dev(h, v)
+    N, H = h.shape
+    _need(h.dtype == torch.float32 and v.numel() == H and v.dtype in DTYPE_CODE and v.is_contiguous(),
+          "add_vector: h fp32 [N, H], a vector of H values")
+    _ok(_core().ia_add_vector(_p(h), _p(v), DTYPE_CODE[v.dtype], N, H, _stream()), "add_vector")
+    return h
+
+
+# ---- retention and the selective scan
+RETENTION_MAX_DIM = 1024        # head sizes of the kernel that runs token after token
+
+
+def rotation_table(positions: torch.Tensor, freq: torch.Tensor, out: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """fp32 [N, rot / 2, 2]: cosine and sine of positions[n] * freq[i]."""
+    N, half = positions.numel(), freq.numel()
+    _need(freq.is_cuda and freq.dtype in (torch.float32, torch.float64) and freq.is_contiguous(), "rotation_table: frequencies")
+    _i32(positions, N, "rotation_table positions")
+    if out is None:
+        out = torch.empty((N, half, 2), dtype=torch.float32, device=positions.device)
+    _need(out.dtype == torch.float32 and tuple(out.shape) == (N, half, 2) and out.is_contiguous(), "rotation_table: out")
+    _ok(_core().ia_rotation_table(_p(positions), _p(freq), int(freq.dtype == torch.float64), _p(out), N, half, _stream()),
+        "rotation_table")
+    return out
+
+
+def retention_state_floats(nh: int, dim: int, vdim: int) -> int:
+    """Floats of a request's state for one run of a retention layer: every head's S [dim, vdim]."""
+    return nh * dim * vdim
+
+
+def _retention_check(proj, cols, table, rot, decay, state, out, seq_starts, state_slots, B, nh, dim, vdim, what) -> int:
+    q_col, k_col, v_col, g_col = cols
+    N = proj.shape[0]
+    _rows(proj, max(q_col + nh * dim, k_col + nh * dim, v_col + nh * vdim, g_col + nh * vdim), what + " rows")
+    _rows(out, nh * vdim, what + " out")
+    _need(out.dtype == proj.dtype and out.shape[0] == N, f"{what}: out of proj's dtype, a row a token")
+    _f32(decay, 2 * nh, what + " decays and their logarithms")
+    if rot:
+        _need(table is not None and tuple(table.shape) == (N, rot // 2, 2) and rot % 2 == 0 and rot <= dim
+              and table.is_contiguous() and table.dtype == torch.float32, f"{what}: a rotation_table of rot / 2 pairs")
+    _dev(seq_starts, state_slots)
+    _need(seq_starts.dtype == torch.int32 and seq_starts.numel() >= B + 1 and state_slots.dtype == torch.int32
+          and state_slots.numel() >= B, f"{what}: int32 starts and slots")
+    return _state_rows(state, retention_state_floats(nh, dim, vdim), what)
+
+
+def retention_step(proj: torch.Tensor, cols: Sequence[int], table: Optional[torch.Tensor], rot: int, k_factor: float,
+                   decay: torch.Tensor, eps: float, o_factor: float, state: torch.Tensor, out: torch.Tensor,
+                   seq_starts: torch.Tensor, state_slots: torch.Tensor, nh: int, dim: int, vdim: int) -> torch.Tensor:
+    """Per request (as many as ``state_slots`` names) and head over the request's rows in order: q and k rotated by halves
+    (``table`` of :func:`rotation_table`), k times ``k_factor``, S <- g S + k v^T, o = S^T q;
+    out = o / sqrt(mean(o^2) + eps) * o_factor * silu(gate).  ``cols``: where q, k (nh dim values each), v and the gates
+    (nh vdim each) begin in the rows of ``proj``.  ``decay`` fp32 [2, nh]: g, then log2(g).  ``state`` [slots, >=
+    retention_state_floats] fp32 is read and left moved on.  ``out`` [N, nh vdim], possibly columns of wider rows."""
+    B = state_slots.numel()
+    stride = _retention_check(proj, cols, table, rot, decay, state, out, seq_starts, state_slots, B, nh, dim, vdim, "retention_step")
+    _ok(_core().ia_retention_step(_p(proj), DTYPE_CODE[proj.dtype], _rows_of(proj), *cols, _p(table), int(rot),
+                                  ctypes.c_float(k_factor), _p(decay), ctypes.c_float(eps), ctypes.c_float(o_factor), _p(state),
+                                  ctypes.c_long(stride), _p(out), _rows_of(out), _p(seq_starts), _p(state_slots), B, nh, dim,
+                                  vdim, _stream()), "retention_step")
+    return out
+
+
+def retention_chunked_takes(dtype: torch.dtype, nh: int, dim: int, vdim: int, proj_stride: int, cols: Sequence[int]) -> bool:
+    """Whether :func:`retention_chunked` has a kernel for these sizes: bf16 rows, head sizes of multiples of 16 up to 256
+    that fit the LDS."""
+    return dtype == torch.bfloat16 and bool(_core().ia_retention_chunked_takes(nh, dim, vdim, int(proj_stride), *cols[:3]))
+
+
+def retention_chunked(proj: torch.Tensor, cols: Sequence[int], table: Optional[torch.Tensor], rot: int, k_factor: float,
+                      decay: torch.Tensor, eps: float, o_factor: float, state: torch.Tensor, out: torch.Tensor,
+                      seq_starts: torch.Tensor, state_slots: torch.Tensor, tiles: torch.Tensor, num_tiles: int,
+                      first_request: int, nh: int, dim: int, vdim: int, records: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """:func:`retention_step` for the requests that ``tiles`` names (int32 [n, 2] of (request, first row of a tile of
+    PREFILL_TILE_ROWS among the request's rows) in any order: every tile of the requests from ``first_request`` on, once),
+    as matrix products over the tiles.  ``records`` fp32 [>= n, retention_state_floats] is scratch."""
+    floats = retention_state_floats(nh, dim, vdim)
+    stride = _retention_check(proj, cols, table, rot, decay, state, out, seq_starts, state_slots, state_slots.numel(), nh, dim,
+                              vdim, "retention_chunked")
+    _need(retention_chunked_takes(proj.dtype, nh, dim, vdim, _rows_of(proj), cols), "retention_chunked: sizes that it does not take")
+    _dev(tiles)
+    _need(tiles.dtype == torch.int32 and tiles.is_contiguous() and tiles.numel() >= 2 * num_tiles, "retention_chunked: int32 tiles")
+    if records is None:
+        records = torch.empty((max(num_tiles, 1), floats), dtype=torch.float32, device=out.device)
+    _need(records.dtype == torch.float32 and records.is_contiguous() and records.numel() >= num_tiles * floats,
+          "retention_chunked: scratch for every tile")
+    _ok(_core().ia_retention_chunked(_p(proj), DTYPE_CODE[proj.dtype], _rows_of(proj), *cols, _p(table), int(rot),
+                                     ctypes.c_float(k_factor), _p(decay), ctypes.c_float(eps), ctypes.c_float(o_factor),
+                                     _p(state), ctypes.c_long(stride), _p(out), _rows_of(out), _p(seq_starts), _p(state_slots),
+                                     _p(tiles), int(num_tiles), int(first_request), _p(records), ctypes.c_long(floats), nh, dim,
+                                     vdim, _stream()), "retention_chunked")
+    return out
+
+
+def selective_columns(states: int) -> int:
+    """Columns that B (and C) of a token take in a row for so many state values; 0: more than the kernel takes."""
+    for k in (8, 16, 32, 64, 128):
+        if states <= k:
+            return k
+    return 0
+
+
+SELECTIVE_SPLIT_FROM = 2.2      # so many times what a compute unit's share of the rows takes, a request's rows are cut
+SELECTIVE_WAVES = 2048          # waves that the segments of a cut step aim at
+
+
+def selective_segment(rows: Sequence[int], channels: int, device: Optional[torch.device] = None) -> int:
+    """Rows of a segment of :func:`selective_scan` for requests of so many rows each.  A request's rows run one after the
+    other, a wave for 64 channels; cut into segments side by side they cost twice the work, so they are cut where the
+    longest request would take more than that, in as many segments as fill the GPU."""
+    longest, total = max(rows, default=0), sum(rows)
+    waves = -(-channels // 64)
+    simds = 4 * compute_units(device)
+    if longest <= 64 or longest <= SELECTIVE_SPLIT_FROM * total * waves / simds:
+        return max(longest, 1)
+    segments = max(1, SELECTIVE_WAVES // waves)
+    return max(32, -(-(-(-total // segments)) // 16) * 16)
+
+
+def selective_scan(x: torch.Tensor, z: torch.Tensor, bc: torch.Tensor, b_col: int, c_col: int, dt_raw: torch.Tensor,
+                   dt_bias: torch.Tensor, a2: torch.Tensor, skip: torch.Tensor, state: torch.Tensor, out: torch.Tensor,
+                   seq_starts: torch.Tensor, state_slots: torch.Tensor, first_request: int, requests: int, max_rows: int,
+                   segment: Optional[int] = None) -> torch.Tensor:
+    """Per request first_request .. first_request + requests - 1 and channel over the request's rows in order:
+    dt = softplus(dt_raw + dt_bias), S[n] <- exp(dt A[n]) S[n] + dt x B[n], y = sum_n S[n] C[n] + skip x,
+    out = y silu(z).  ``x``, ``z``, ``out`` [N, C] (columns of wider rows); ``bc`` rows with :func:`selective_columns`
+    values of B from ``b_col`` and of C from ``c_col`` (zeros past the state's size); ``dt_raw`` fp32 [N, C]; ``a2`` fp32
+    [states, C]: A log2(e).  ``state`` [slots, >= states C] fp32 is read and left moved on.  ``max_rows``: the rows of the
+    longest of the requests; ``segment``: rows that run one after the other (more are cut into segments side by side)."""
+    N, C = x.shape
+    Ns = a2.shape[0]
+    kn = selective_columns(Ns)
+    _need(kn > 0, f"selective_scan: a state of {Ns} values, at most 128")
+    for t, cols, what in ((x, C, "x"), (z, C, "z"), (out, C, "out"), (bc, max(b_col, c_col) + kn, "B and C")):
+        _rows(t, cols, "selective_scan " + what)
+        _need(t.dtype == x.dtype and t.shape[0] == N, "selective_scan: rows of one dtype, one a token")
+    _need(dt_raw.is_cuda and dt_raw.dtype == torch.float32 and dt_raw.dim() == 2 and dt_raw.stride(1) == 1
+          and dt_raw.shape[0] == N and dt_raw.shape[1] >= C, "selective_scan: dt_raw fp32 [N, C]")
+    for t, what in ((dt_bias, "dt_bias"), (skip, "skip")):
+        _f32(t, C, "selective_scan " + what)
+    _f32(a2, Ns * C, "selective_scan a2")
+    _dev(seq_starts, state_slots)
+    _need(seq_starts.numel() > first_request + requests and state_slots.numel() >= first_request + requests,
+          "selective_scan: starts and slots of the requests")
+    stride = _state_rows(state, Ns * C, "selective_scan")
+    segment = int(segment or max_rows)
+    segs = -(-int(max_rows) // segment) if requests else 1
+    records = sums = None
+    if segs > 1:
+        records = torch.empty(requests * segs * Ns * C, dtype=torch.float32, device=x.device)
+        sums = torch.empty(requests * segs * C, dtype=torch.float32, device=x.device)
+    _ok(_core().ia_selective_scan(_p(x), DTYPE_CODE[x.dtype], _rows_of(x), _p(z), _rows_of(z), _p(bc), _rows_of(bc), b_col, c_col,
+                                  _p(dt_raw), _rows_of(dt_raw), _p(dt_bias), _p(a2), _p(skip), _p(state), ctypes.c_long(stride),
+                                  _p(out), _rows_of(out), _p(seq_starts), _p(state_slots), int(first_request), int(requests), C,
+                                  Ns, int(max_rows), segment, _p(records), _p(sums), _stream()), "selective_scan")
+    return out
 
 
 def ssd_scan(xbc: torch.Tensor, dt_raw: torch.Tensor, dt_bias: torch.Tensor, a_log: torch.Tensor, skip: torch.Tensor,
@@ -1311,11 +1531,12 @@ def gated_norm_add(h: torch.Tensor, delta, gate, gate_bias: Optional[torch.Tenso
 
 
 def router_softmax_topk(logits: torch.Tensor, correction: Optional[torch.Tensor], top: int, groups: int = 1, keep: int = 1,
-                        renorm: bool = True, experts: Optional[int] = None):
+                        renorm: bool = True, experts: Optional[int] = None, sigmoid: bool = False):
     """-> (ids int32 [N, top], weights fp32 [N, top]): s = softmax(logits) over all experts; the ``top`` largest of
     s + correction are chosen (the lowest index among equals); the weights are the chosen s, with ``renorm`` over their
     sum.  ``groups`` equal groups of neighbouring experts, of which only the ``keep`` with the largest s + correction
-    among their experts can be chosen from.  ``experts``: rows of ``logits`` hold more than the experts' (first)."""
+    among their experts can be chosen from.  ``experts``: rows of ``logits`` hold more than the experts' (first).
+    ``sigmoid``: s = sigmoid(logits) in place of the softmax."""
     _dev(logits, correction)
     _need(logits.dtype == torch.float32 and logits.dim() == 2, "router_softmax_topk: fp32 logits [N, E]")
     N, E = logits.shape[0], int(experts or logits.shape[1])
@@ -1329,7 +1550,7 @@ def router_softmax_topk(logits: torch.Tensor, correction: Optional[torch.Tensor]
     _ok(_core().ia_router_softmax_topk(_p(logits), _p(correction),
                                        DTYPE_CODE[correction.dtype] if correction is not None else 0, _p(ids),
                                        _p(weights), N, E, top, int(logits.shape[1]), int(groups), int(keep), int(bool(renorm)),
-                                       _stream()), "router_softmax_topk")
+                                       int(bool(sigmoid)), _stream()), "router_softmax_topk")
     return ids, weights
 
 

@@ -51,10 +51,13 @@ class Attention(Mixer):
                  position: Optional[Mapping[str, Any]] = None, window: Optional[int] = None,
                  scale: Optional[float] = None, kernels: str = "auto", init_std: float = 0.02,
                  qk_transform: Optional[Mapping[str, Any]] = None, chunk: Optional[int] = None,
-                 value_dim: Optional[int] = None, keep_first: int = 0, softcap: Optional[float] = None):
+                 value_dim: Optional[int] = None, keep_first: int = 0, softcap: Optional[float] = None,
+                 distance_bias: bool = False, output_gate: bool = False):
         """``value_dim``: the size of a value head (default: the head size).  ``keep_first``: under a window, so many
         first positions of a request that every later query goes on seeing.  ``softcap`` c: a scaled score s becomes
-        c tanh(s / c).  (This mixer's own projection has none of the three; mixers built on it do.)"""
+        c tanh(s / c).  ``distance_bias``: a number by head and distance on the score (``self.bias``, set when the mixer
+        loads); ``output_gate``: what the heads leave times sigmoid of a gate per value, which ``attend`` is handed.  (This
+        mixer's own projection has none of these; mixers built on it do.)"""
         super().__init__(rt)
         if num_heads % num_kv_heads:
             raise ValueError(f"num_heads {num_heads} is not a multiple of num_kv_heads {num_kv_heads}")
@@ -96,6 +99,9 @@ class Attention(Mixer):
         # fp32 [num_heads], or None: exp(sinks[h]) in the denominator of head h's softmax (a mixer that has sinks
         # sets it when it loads; every attention kernel takes it)
         self.sinks: Optional[torch.Tensor] = None
+        # a table of K.distance_table, or None
+        self.distance_bias, self.output_gate = bool(distance_bias), bool(output_gate)
+        self.bias: Optional[torch.Tensor] = None
         self.rotate_in_attention = _decode_rotation == "attention"
         self.use_mfma = (kernels == "auto" and rt.dtype == torch.bfloat16 and rt.device.type == "cuda"
                          and K.attention_mfma_available(self.d, self.vd))
@@ -110,7 +116,8 @@ class Attention(Mixer):
 
     def _lib(self):
         """The library of the matrix-core kernels for this mixer's sizes and options."""
-        return K._attn(self.d, self.vd, self.keep_first > 0 or self.score_cap > 0)
+        return K._attn(self.d, self.vd, K.attention_options(self.keep_first, self.score_cap, self.distance_bias,
+                                                            self.output_gate))
 
     def step_needs(self) -> Dict[str, Any]:
         # the MFMA kernel for portions of prompts works on tiles of 64 query rows
@@ -118,8 +125,8 @@ class Attention(Mixer):
 
     def weights(self) -> Dict[str, WeightSpec]:
         nh, nkv, d, H = self.nh, self.nkv, self.d, self.hidden_size
-        if self.vd != d or self.keep_first or self.score_cap:
-            raise ValueError("this mixer's values have the head size, and it has no kept positions and no softcap")
+        if self.vd != d or self.keep_first or self.score_cap or self.distance_bias or self.output_gate:
+            raise ValueError("this mixer's values have the head size, and it has no kept positions, softcap, bias or gate")
         init = ("normal", self.init_std)
         own = {
             "q_proj.weight": WeightSpec((nh * d, H), init),
@@ -297,17 +304,23 @@ class Attention(Mixer):
         return (program.scalar(("attention: parts of the keys", nh, nkv, big, g, ps, self._span(1 << 60)), parts_of_the_keys),
                 program.scalar(("attention: launch shape", nh, nkv, big, window), launch_shape))
 
-    def emit_attend(self, program, view: CacheView, q, q_stride: int, when, out=None, out_stride: Optional[int] = None):
+    def emit_attend(self, program, view: CacheView, q, q_stride: int, when, out=None, out_stride: Optional[int] = None,
+                    gate=None, gate_stride: int = 0):
         """The launches of :meth:`attend` alone, for queries ``q`` (rows of ``q_stride`` values, the heads first) that
         are rotated already and whose keys and values are in their pages: the kernel for single tokens on the first
         rows and the one for portions of prompts on the rest, or the plain kernel on all rows.  ``out``: where the
-        attended rows go, ``out_stride`` values from a row to the next (default: a buffer [N, nh dv]).  Returns it."""
+        attended rows go, ``out_stride`` values from a row to the next (default: a buffer [N, nh dv]); ``gate``: where the
+        gates of an ``output_gate`` lie, likewise.  Returns ``out``."""
         from ..engine.program import STREAM, Guard
         nh, nkv, d, dv, window, rt = self.nh, self.nkv, self.d, self.vd, self.mask, self.rt
         k, v, g = view.k_pages, view.v_pages, view.group
         ps, num_pages = int(k.shape[2]), int(k.shape[0])
         T, act, scale = program.T, program.act_code, float(self.scale)
-        program.keep(k, v, self.sinks)
+        program.keep(k, v, self.sinks, self.bias)
+        if (self.bias is None) == self.distance_bias or (gate is None) == self.output_gate:
+            raise K.KernelError("attention: the bias table and the gates are there exactly when the mixer has them")
+        more = [self.bias, int(self.bias.shape[1]) - 2 * K.DISTANCE_PAD if self.bias is not None else 0, gate,
+                int(gate_stride)]
         bt, bt_cols = program.block_table(g), program.bt_cols(g)
         if out is None:
             out = program.buffer("attention.out", T * nh * dv * program.act_bytes)
@@ -316,7 +329,7 @@ class Attention(Mixer):
             program.op("core", "ia_attention_generic",
                        [q, q_stride, k, v, out, out_stride, act, program.token_seq, program.positions, bt, bt_cols,
                         program.N, nh, nkv, d, dv, ps, num_pages, scale, window, self.sinks, self.keep_first, self.score_cap,
-                        STREAM], when)
+                        *more, STREAM], when)
             return out
         lib = self._lib()
         records = T + 1024
@@ -326,11 +339,11 @@ class Attention(Mixer):
         tiles, num_tiles = program.row_tiles(K.PREFILL_TILE_ROWS)
         program.op(lib, "ia_attn_decode",
                    [q, q_stride, k, v, out, out_stride, part_o, part_ml, program.positions, bt, bt_cols, program.ND, nh,
-                    nkv, ps, num_pages, scale, window, splits, self.sinks, self.keep_first, self.score_cap, STREAM],
+                    nkv, ps, num_pages, scale, window, splits, self.sinks, self.keep_first, self.score_cap, *more, STREAM],
                    when & Guard.between(program.ND, 1))
         program.op(lib, "ia_attn_prefill",
                    [q, q_stride, k, v, out, out_stride, program.seq_starts, program.seq_ctx, bt, bt_cols, tiles, num_tiles,
-                    nh, nkv, ps, num_pages, scale, window, shape, self.sinks, self.keep_first, self.score_cap, STREAM],
+                    nh, nkv, ps, num_pages, scale, window, shape, self.sinks, self.keep_first, self.score_cap, *more, STREAM],
                    when & Guard.between(program.NP, 1))
         return out
 
@@ -342,18 +355,23 @@ class Attention(Mixer):
             return min(max_len, self.window + self.keep_first)
         return min(max_len, self.chunk) if self.chunk else max_len
 
-    def attend(self, qkv: torch.Tensor, out: torch.Tensor, ctx: StepContext, cache: CacheView) -> None:
+    def attend(self, qkv: torch.Tensor, out: torch.Tensor, ctx: StepContext, cache: CacheView,
+               gate: Optional[torch.Tensor] = None) -> None:
         nh, nkv, d = self.nh, self.nkv, self.d
+        if (self.bias is None) == self.distance_bias or (gate is None) == self.output_gate:
+            raise K.KernelError("attention: the bias table and the gates are there exactly when the mixer has them")
         bt = ctx.block_tables[cache.group]
         if not self.use_mfma or cache.k_pages.shape[2] % 4:
             K.attention_generic(qkv, cache.k_pages, cache.v_pages, out, ctx.token_seq, ctx.positions, bt, nh, nkv, d,
-                                self.scale, self.mask, sinks=self.sinks, keep=self.keep_first, softcap=self.score_cap)
+                                self.scale, self.mask, sinks=self.sinks, keep=self.keep_first, softcap=self.score_cap,
+                                bias=self.bias, gate=gate)
             return
         nd = ctx.num_decode
         if nd > 0:
             K.attention_decode(qkv[:nd], cache.k_pages, cache.v_pages, out[:nd], ctx.positions[:nd], bt[:nd], nh, nkv,
                                d, self.scale, self.mask, self._span(ctx.max_total_len), sinks=self.sinks,
-                               keep=self.keep_first, softcap=self.score_cap)
+                               keep=self.keep_first, softcap=self.score_cap, bias=self.bias,
+                               gate=gate[:nd] if gate is not None else None)
         if ctx.num_seqs > nd:
             big = max(d, self.vd)
             key = ("prefill_launch_shape", nh, nkv, big, self.mask)
@@ -364,7 +382,7 @@ class Attention(Mixer):
             tiles, num_tiles = ctx.row_tiles(K.PREFILL_TILE_ROWS)
             K.attention_prefill(qkv, cache.k_pages, cache.v_pages, out, ctx.seq_starts, ctx.seq_ctx, bt,
                                 tiles, num_tiles, nh, nkv, d, self.scale, self.mask, hpw, sinks=self.sinks,
-                                keep=self.keep_first, softcap=self.score_cap)
+                                keep=self.keep_first, softcap=self.score_cap, bias=self.bias, gate=gate)
 
 
 register_part("mixer", "attention", Attention)

@@ -15,7 +15,8 @@ sublayer (``RMSNorm.add_normed``).
 
 ``sandwich``: a norm before and after each sublayer, and optionally a gate on the sublayer's result that reads what
 the sublayer read:  a = norm1(h); h' = h + norm1b(gate1(a) * mixer(a));  f = norm2(h'); h'' = h' + norm2b(gate2(f) *
-feed_forward(f)).  The norms after the sublayers and the gates are extra parts (``mixer_post_norm``,
+feed_forward(f)); the feed-forward (with its norms) may be absent, and an extra part ``stream_in`` rewrites the stream before
+the layer.  The norms after the sublayers and the gates are extra parts (``mixer_post_norm``,
 ``feed_forward_post_norm``: norms; ``mixer_gate``, ``feed_forward_gate``: category ``branch_gate``).  One kernel gates
 the branch, normalises it, adds it into the fp32 stream and, after the mixer, leaves the feed-forward's normalised
 input as well (``kernels.api.gated_norm_add``).
@@ -47,7 +48,7 @@ class PreNormBlock(Block):
                 cache: CacheView) -> torch.Tensor:
         stream_in = self.extra.get("stream_in")
         if stream_in is not None:
-            stream_in.forward(h, pending, ctx)
+            stream_in.forward(h, pending, ctx, cache.pass_index)
             pending = None
         n = self.mixer_norm.forward(h, pending)
         a = self.mixer.forward(n, ctx, cache)
@@ -60,7 +61,7 @@ class PreNormBlock(Block):
         if type(self).forward is not PreNormBlock.forward:
             return super().native(program, view)
         if self.extra.get("stream_in") is not None:
-            self.extra["stream_in"].native(program, None)
+            self.extra["stream_in"].native(program, view)
         self.mixer_norm.native(program, None)
         self.mixer.native(program, view)
         if self.feed_forward is not None:
@@ -136,6 +137,10 @@ class SandwichBlock(Block):
         return x
 
     def forward(self, h: torch.Tensor, pending, ctx: StepContext, cache: CacheView):
+        stream_in = self.extra.get("stream_in")
+        if stream_in is not None:
+            stream_in.forward(h, pending, ctx, cache.pass_index)
+            pending = None
         a = self.mixer_norm.forward(h, pending)
         y = self.mixer.forward(a, ctx, cache)
         nxt = self.feed_forward_norm if self._fuse_next else None
@@ -177,6 +182,8 @@ class SandwichBlock(Block):
     def native(self, program, view: CacheView) -> None:
         if type(self).forward is not SandwichBlock.forward:
             return super().native(program, view)
+        if self.extra.get("stream_in") is not None:
+            self.extra["stream_in"].native(program, view)
         self.mixer_norm.native(program, None)
         self.mixer.native(program, view)
         nxt = self.feed_forward_norm if self._fuse_next else None
@@ -201,7 +208,7 @@ class ParallelBlock(Block):
         from ..kernels import api as K
         stream_in = self.extra.get("stream_in")
         if stream_in is not None and cache.pass_index > 0:
-            stream_in.forward(h, pending, ctx)
+            stream_in.forward(h, pending, ctx, cache.pass_index)
             pending = None
         a = self.mixer.forward(self.mixer_norm.forward(h, pending), ctx, cache)
         f = None
@@ -234,7 +241,7 @@ class ParallelBlock(Block):
         if type(self).forward is not ParallelBlock.forward:
             return super().native(program, view)
         if self.extra.get("stream_in") is not None and view.pass_index > 0:
-            self.extra["stream_in"].native(program, None)
+            self.extra["stream_in"].native(program, view)
         self.mixer_norm.native(program, None)
         self.mixer.native(program, view)
         a, program.pending = program.pending, None

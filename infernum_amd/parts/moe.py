@@ -23,7 +23,9 @@ More options of gated experts: without ``limit`` nothing is clamped; ``up_shift`
 added to u (0 with alpha 1: D_e (silu(G_e x) * (U_e x))).  Of the ``softmax_top`` router: ``renorm=False`` leaves the
 chosen s as they are; ``groups`` and ``keep_groups``: the experts form equal groups of neighbours, a group's score is its
 largest s + correction, and only experts of the best groups can be chosen; ``identity`` n: the last n of
-num_experts + n experts have no tensors, and their result is their input.  ``shared_ff`` with gated experts: the shared
+num_experts + n experts have no tensors, and their result is their input.  ``scores="sigmoid"``: s = sigmoid(z) in place of
+the softmax; ``correction_name=None``: no correction.  ``weights_on="input"`` (gated experts): the weight multiplies what
+an expert reads, expert(w x), not what it leaves.  ``shared_ff`` with gated experts: the shared
 expert is D (silu(G x) * (U x)) (``shared.gate``, ``shared.up``, ``shared.down``), with ``shared_gate`` (a local tensor
 name, [1, W]) times the sigmoid of one number per token; its result is a part of its own after the choices'.
 """
@@ -47,7 +49,8 @@ class RoutedExperts(FeedForward):
                  router_name: str = "router", expert_prefix: str = "e", init_std: float = 0.02, gated: bool = True,
                  activation: str = "relu_squared", router: str = "top_softmax", correction_name: str = "correction",
                  shared_ff: Optional[int] = None, up_shift: float = 1.0, renorm: bool = True, groups: int = 1,
-                 keep_groups: int = 1, identity: int = 0, shared_gate: Optional[str] = None):
+                 keep_groups: int = 1, identity: int = 0, shared_gate: Optional[str] = None, scores: str = "softmax",
+                 weights_on: str = "output"):
         super().__init__(rt)
         self.hidden_size, self.ff = int(hidden_size), int(intermediate_size)
         self.num_experts, self.top = int(num_experts), int(top)
@@ -73,6 +76,13 @@ class RoutedExperts(FeedForward):
         if self.identity and not self.gated:
             raise ValueError("identity experts go with gated experts")
         self.correction_name = correction_name
+        if scores not in ("softmax", "sigmoid") or weights_on not in ("input", "output"):
+            raise ValueError(f"scores {scores!r}, weights_on {weights_on!r}")
+        self.sigmoid_scores, self.weights_on = scores == "sigmoid", str(weights_on)
+        if self.router != "softmax_top" and (self.sigmoid_scores or correction_name is None):
+            raise ValueError("sigmoid scores and a missing correction go with the 'softmax_top' router")
+        if self.weights_on == "input" and not self.gated:
+            raise ValueError("weights on the experts' input go with gated experts")
         self.shared_ff = int(shared_ff) if shared_ff else 0
         self.shared_gate = str(shared_gate) if shared_gate else None
         if self.shared_gate and not (self.shared_ff and self.gated):
@@ -89,7 +99,8 @@ class RoutedExperts(FeedForward):
         init = ("normal", self.init_std)
         out = {self.router_name: WeightSpec((self.total, H), init)}
         if self.router == "softmax_top":
-            out[self.correction_name] = WeightSpec((self.total,), ("normal", 0.05), follows_compute_dtype=False)
+            if self.correction_name is not None:
+                out[self.correction_name] = WeightSpec((self.total,), ("normal", 0.05), follows_compute_dtype=False)
         elif self.router_bias:
             out[self.router_name + ".b"] = WeightSpec((E,), ("normal", 0.5), follows_compute_dtype=False)
         if self.shared_ff and self.gated:
@@ -113,7 +124,7 @@ class RoutedExperts(FeedForward):
         if self.shared_gate:                  # the shared expert's gate is one more row of the router's product
             self.w_router = torch.cat([self.w_router, tensors[self.shared_gate]], dim=0).contiguous()
         if self.router == "softmax_top":
-            self.b_router = tensors[self.correction_name].contiguous()
+            self.b_router = tensors[self.correction_name].contiguous() if self.correction_name is not None else None
         else:
             self.b_router = tensors[self.router_name + ".b"].contiguous() if self.router_bias else None
         dev, dt = self.w_router.device, self.w_router.dtype
@@ -141,7 +152,7 @@ class RoutedExperts(FeedForward):
         z = linear(x, self.w_router, out_dtype=torch.float32, kernels=self.rt.kernels)
         if self.router == "softmax_top":
             ids, weights = K.router_softmax_topk(z, self.b_router, self.top, self.groups, self.keep_groups, self.renorm,
-                                                 self.total)
+                                                 self.total, self.sigmoid_scores)
         else:
             ids, weights = K.router_topk(z, self.b_router, self.top)
         if self.gated:
@@ -149,7 +160,7 @@ class RoutedExperts(FeedForward):
             parts = torch.empty((self.top + bool(self.shared_ff), x.shape[0], self.hidden_size), dtype=torch.float32,
                                 device=x.device)
             out = K.moe_experts(x, ids, weights, self.w_gate_up, self.w_down, self.limit, self.alpha, self.up_shift,
-                                self.total, parts)
+                                self.total, parts, self.weights_on)
             if not extras:
                 return out
             shared = None
@@ -182,7 +193,7 @@ class RoutedExperts(FeedForward):
         if self.router == "softmax_top":
             program.op("core", "ia_router_softmax_topk", [z.tensor(), b, b_code, ids, wts, N, total, top,
                                                           int(self.w_router.shape[0]), self.groups, self.keep_groups,
-                                                          int(self.renorm), STREAM])
+                                                          int(self.renorm), int(self.sigmoid_scores), STREAM])
         else:
             program.op("core", "ia_router_topk", [z.tensor(), b, b_code, ids, wts, N, total, top, STREAM])
         program.op("core", "ia_moe_sort", [ids, offsets, perm, N * top, total, STREAM])
@@ -192,9 +203,10 @@ class RoutedExperts(FeedForward):
         first = K.moe_grouped_from_tokens(E, top, H, I, self.rt.dtype)
         grouped = Guard.between(N, first) if first > 0 else NEVER
         tiled = ~grouped
+        in_w, out_w = (wts, None) if self.weights_on == "input" else (None, wts)
         program.op("core", "ia_moe_gate_up", [program.x, self.w_gate_up, y, offsets, perm, program.act_code, N * top,
-                                              E, top, H, I, self.limit, self.alpha, self.up_shift, STREAM], tiled)
-        program.op("core", "ia_moe_down", [y, self.w_down, parts, wts, offsets, perm, program.act_code, N, E, top, H,
+                                              E, top, H, I, self.limit, self.alpha, self.up_shift, in_w, STREAM], tiled)
+        program.op("core", "ia_moe_down", [y, self.w_down, parts, out_w, offsets, perm, program.act_code, N, E, top, H,
                                            I, STREAM], tiled)
         if first > 0 and first <= T:
             # steps of many tokens: the grouped form of the LDS-tiled product (kernels.api.moe_experts)
@@ -203,9 +215,10 @@ class RoutedExperts(FeedForward):
             program.op("core", "ia_moe_gather", [program.x, perm, xs, N * top, top, H, STREAM], grouped)
             program.op("core", "ia_gemm_mfma_grouped", [xs, self.w_gate_up, gu, offsets, E, N * top, 2 * I, H, STREAM],
                        grouped)
-            program.op("core", "ia_moe_glu", [gu, y, N * top, I, self.limit, self.alpha, self.up_shift, STREAM], grouped)
+            program.op("core", "ia_moe_glu", [gu, y, N * top, I, self.limit, self.alpha, self.up_shift, perm, in_w, STREAM],
+                       grouped)
             program.op("core", "ia_gemm_mfma_grouped", [y, self.w_down, xs, offsets, E, N * top, H, I, STREAM], grouped)
-            program.op("core", "ia_moe_scatter", [xs, perm, wts, parts, offsets.at(E * 4) if self.identity else None, N, top, H,
+            program.op("core", "ia_moe_scatter", [xs, perm, out_w, parts, offsets.at(E * 4) if self.identity else None, N, top, H,
                                                   STREAM], grouped)
         if self.identity or self.shared_ff:
             self._native_extras(program, z.tensor(), ids, wts, parts)

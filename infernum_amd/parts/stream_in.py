@@ -7,6 +7,8 @@ into h first; the product's operands are rounded to the compute dtype like any p
 are fp32.  The embedding must have been made with ``keep_output``.
 
 ``add_embedding``: h <- h + e, nothing else.
+
+``pass_vector``: h <- h + r_t, a learned vector for every pass t of the repeated stretch.
 """
 from __future__ import annotations
 
@@ -37,8 +39,8 @@ class ConcatLinearStreamIn(Part):
         self.weight = tensors[self.name].contiguous()
         prepare_weights(self.rt, [(self.weight, None, False)])
 
-    def forward(self, h: torch.Tensor, pending: Any, ctx: StepContext) -> None:
-        """h [N, H] fp32, rewritten in place."""
+    def forward(self, h: torch.Tensor, pending: Any, ctx: StepContext, pass_index: int = 0) -> None:
+        """h [N, H] fp32, rewritten in place; ``pass_index``: the pass that begins."""
         e = ctx.extras.get(EMBEDDING_OUTPUT)
         if e is None:
             raise K.KernelError("concat_linear: the embedding did not keep its output (keep_output)")
@@ -76,7 +78,7 @@ class AddEmbeddingStreamIn(Part):
         super().__init__(rt)
         self.hidden_size = int(hidden_size)
 
-    def forward(self, h: torch.Tensor, pending: Any, ctx: StepContext) -> None:
+    def forward(self, h: torch.Tensor, pending: Any, ctx: StepContext, pass_index: int = 0) -> None:
         e = ctx.extras.get(EMBEDDING_OUTPUT_F32)
         if e is None:
             raise K.KernelError("add_embedding: the embedding did not keep its output (keep_output='fp32')")
@@ -96,5 +98,39 @@ class AddEmbeddingStreamIn(Part):
         program.op("core", "ia_stream_add", [program.h, kept, f32, 1, N, H, STREAM])
 
 
+class PassVectorStreamIn(Part):
+    """h <- h + table[t] in pass t (``CacheView.pass_index``): one vector for all tokens, kept as the file has it."""
+    category = "stream_in"
+    graph_safe = True
+
+    def __init__(self, rt: Runtime, hidden_size: int, passes: int, name: str = "weight", init_std: float = 0.02):
+        super().__init__(rt)
+        self.hidden_size, self.passes, self.name, self.init_std = int(hidden_size), int(passes), str(name), init_std
+        self.table: Optional[torch.Tensor] = None
+
+    def weights(self) -> Dict[str, WeightSpec]:
+        return {self.name: WeightSpec((self.passes, self.hidden_size), ("normal", self.init_std), follows_compute_dtype=False)}
+
+    def load(self, tensors: Dict[str, torch.Tensor]) -> None:
+        self.table = tensors[self.name].contiguous()
+
+    def forward(self, h: torch.Tensor, pending: Any, ctx: StepContext, pass_index: int = 0) -> None:
+        if pending is not None:
+            K.stream_add(h, pending)
+        K.add_vector(h, self.table[pass_index])
+
+    def native(self, program, view=None) -> None:
+        from ..engine.program import STREAM
+        H, N = self.hidden_size, program.N
+        for alt in (program.pending.alts if program.pending is not None else []):
+            code = K.DTYPE_CODE[torch.float32] if alt.splits else K.DTYPE_CODE[alt.dtype]
+            program.op("core", "ia_stream_add", [program.h, alt.where, code, alt.splits or 1, N, H, STREAM], alt.when)
+        program.pending = None
+        program.keep(self.table)
+        vector = self.table[view.pass_index if view is not None else 0]
+        program.op("core", "ia_add_vector", [program.h, vector, K.DTYPE_CODE[vector.dtype], N, H, STREAM])
+
+
+register_part("stream_in", "pass_vector", PassVectorStreamIn)
 register_part("stream_in", "concat_linear", ConcatLinearStreamIn)
 register_part("stream_in", "add_embedding", AddEmbeddingStreamIn)
