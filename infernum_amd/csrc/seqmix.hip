@@ -569,7 +569,7 @@ __device__ __forceinline__ void values_to_page(const bf16_t* __restrict__ rows, 
   const int t = (int)(w / groups) * 16 + (lane & 15), piece = (int)(w % groups) * 4 + (lane >> 4);
   if (t >= N || piece >= pieces) return;
   const int slot = slots[t], page = slot / page_size, off = slot - page * page_size;
-  if (page < 0 || page >= num_pages) return;
+  if (slot < 0 || page >= num_pages) return;
   const int col = piece * 8, g = col / dv, c = col - g * dv;
   const uint4 raw = *(const uint4*)(rows + (size_t)t * x_stride + col);
   const uint32_t rw[4] = {raw.x, raw.y, raw.z, raw.w};
@@ -601,7 +601,7 @@ __global__ __launch_bounds__(256) void qk_rows_prepare_kernel(
   const int n = blockIdx.x;
   const T* row = x + (size_t)n * x_stride;
   const int slot = slots[n], page = slot / page_size, off = slot - page * page_size;
-  const bool place = (unsigned)page < (unsigned)num_pages;            // a token without a place: its keys are not written
+  const bool place = slot >= 0 && page < num_pages;            // a token without a place: its keys are not written
 #pragma unroll
   for (int part = 0; part < 2; ++part) {
     const int cols = part ? nk : nq;

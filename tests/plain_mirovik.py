@@ -306,6 +306,10 @@ def random_weights(cfg: Mapping, seed: int = 0, store: torch.dtype = torch.bfloa
             t = rnd() / math.sqrt(shape[-1])
         elif last == "router":
             t = 2.0 * rnd() / math.sqrt(shape[-1])
+        elif name.endswith(".right.k"):
+            # a token's own key lies along its query: what a retention head reads is then no difference of nearly equal
+            # terms, which the division by its root mean square would blow up
+            t = 0.7 * out[name[:-1] + "q"].float() + 0.7 * rnd() / math.sqrt(shape[-1])
         else:
             t = rnd() / math.sqrt(shape[-1])
         out[name] = t.to(store)
