@@ -706,6 +706,61 @@ def pamazen_bench(a) -> int:
                               pamazen_active_params, batches)
 
 
+# ---- the Mirovik design beside the Llama decoder at equal sizes -------------------------------------------------
+# Four layers of one width that run twice (a loop over all of them: eight layer runs, a vector of the pass added before
+# each): attention with a bias by distance and gated values (16 or 32 heads of 128 over 4 or 8) beside retention (half as
+# many heads of 128), twice the selective scan (twice the width of channels, a state of 16), and the first kind again; a dense
+# feed-forward of two matrices in every other layer, sixteen experts with two chosen and a shared one in the others, each with
+# as many feed-forward weights a token as the twin has.  The Llama twin has eight layers of the same width, vocabulary and heads.
+MIROVIK_SIZES = {
+    "2k": dict(width=2048, runs=8, vocab=32000, ff=5504, heads=16, kv_heads=4, dim=128, ret_heads=8, inner=4096, state=16,
+               dt_rank=128, experts=16, top=2, expert_ff=1408, shared_ff=2688),
+    "4k": dict(width=4096, runs=8, vocab=32000, ff=9600, heads=32, kv_heads=8, dim=128, ret_heads=16, inner=8192, state=16,
+               dt_rank=256, experts=16, top=2, expert_ff=2432, shared_ff=4736),
+}
+
+
+def mirovik_configs(size: dict):
+    from infernum_amd.config import LlamaConfig
+    from infernum_amd.config.mirovik import MirovikConfig
+    d, R = size["dim"], size["ret_heads"]
+    side = {"left": {"heads": size["heads"], "kv_heads": size["kv_heads"], "dim": d, "vdim": d, "scale": d ** -0.5,
+                     "bias_max": 256, "buckets": 40},
+            "right": {"heads": R, "dim": d, "vdim": d, "decay": [1.0 - 2.0 ** (-5 - 4 * i / R) for i in range(R)],
+                      "rot": {"base": 10000.0, "dims": d}}, "left_scale": 1.0, "right_scale": 0.8}
+    scan = {"inner": size["inner"], "state": size["state"], "dt_rank": size["dt_rank"], "conv": 4}
+    dense = {"kind": "dense", "ff": size["ff"] * 3 // 2}
+    moe = {"kind": "moe", "expert": {"ff": size["expert_ff"]}, "shared": {"ff": size["shared_ff"]},
+           "router": {"experts": size["experts"], "top": size["top"]}}
+    layers = [("parallel", side, dense), ("mamba1", scan, moe), ("mamba1", scan, dense), ("parallel", side, moe)]
+    mir = MirovikConfig.from_dict({
+        "architecture": "Mirovik", "vocab": size["vocab"], "width": size["width"], "norm": {"eps": 1e-5},
+        "embedding": {"scale": size["width"] ** 0.5}, "loop": {"start": 0, "stop": 4, "times": size["runs"] // 4},
+        "layers": [{"type": k, "mixer": m, "mlp": f} for k, m, f in layers]})
+    llama = LlamaConfig.from_dict(dict(
+        model_type="llama", num_hidden_layers=size["runs"], hidden_size=size["width"],
+        num_attention_heads=size["heads"], num_key_value_heads=size["kv_heads"], intermediate_size=size["ff"],
+        vocab_size=size["vocab"], rope_theta=10000.0, rms_norm_eps=1e-5, tie_word_embeddings=True,
+        max_position_embeddings=8192))
+    return mir, llama
+
+
+def mirovik_active_params(size: dict) -> int:
+    """Weights that a token multiplies with in the Mirovik model of these sizes (every layer run and the head)."""
+    W, d, I = size["width"], size["dim"], size["inner"]
+    side = W * (3 * size["heads"] + 2 * size["kv_heads"]) * d + 5 * W * size["ret_heads"] * d
+    scan = 3 * W * I + I * (2 * size["dt_rank"] + 2 * size["state"])
+    dense = 2 * W * (size["ff"] * 3 // 2)
+    moe = W * size["experts"] + 3 * W * (size["top"] * size["expert_ff"] + size["shared_ff"])
+    return (size["runs"] // 4) * 2 * (side + scan + dense + moe) + size["vocab"] * W
+
+
+def mirovik_bench(a) -> int:
+    batches = [int(b) for b in a.mirovik_batches.split(",") if b]
+    return beside_llama_bench(a, "Mirovik", [(n, MIROVIK_SIZES[n]) for n in a.mirovik.split(",")], mirovik_configs,
+                              mirovik_active_params, batches)
+
+
 def beside_llama_bench(a, design, sizes, configs, active_params, batches) -> int:
     """Prefill of 2,048 tokens and decode steps at batch 8 and 64 of a design and of the Llama decoder at equal
     sizes, random weights, through the same engine and generation loop; one JSON line of its own."""
@@ -815,6 +870,11 @@ def main() -> int:
                          "mixed values, grouped experts with identities) beside the Llama decoder at equal sizes: names of "
                          + ", ".join(PAMAZEN_SIZES) + " with commas")
     ap.add_argument("--pamazen-batches", default="8,64", help="decode batches of --pamazen")
+    ap.add_argument("--mirovik", default="", metavar="SIZES",
+                    help="the Mirovik design (biased attention beside retention, a selective scan, sigmoid-routed experts, a "
+                         "repeated stretch) beside the Llama decoder at equal sizes; a JSON line of its own: "
+                         + ", ".join(MIROVIK_SIZES) + " with commas")
+    ap.add_argument("--mirovik-batches", default="8,64", help="decode batches of --mirovik")
     a = ap.parse_args()
     if a.gpus != 1:
         print(f"bench.py measures one GPU: this engine has no multi-GPU path (asked for --gpus {a.gpus})")
@@ -828,6 +888,8 @@ def main() -> int:
         return sikazen_bench(a)
     if a.pamazen:
         return pamazen_bench(a)
+    if a.mirovik:
+        return mirovik_bench(a)
     if a.rogizen:
         return rogizen_bench(a)
     if a.decode_kernels:

@@ -25,6 +25,7 @@ typedef float rt_f32x4 __attribute__((ext_vector_type(4)));
 #define RET_TILE 64       // rows of a tile
 #define RET_GS 68         // row stride of a tile's [L, L] matrix in LDS, floats
 #define RET_MAX_DIM 256   // head sizes of the chunks
+#define RET_GROUPS 4      // groups of four values whose loads a thread asks for together
 #define RET_STEP_MAX 1024 // head sizes of the step
 
 __global__ __launch_bounds__(256) void rotation_table_kernel(const int* __restrict__ positions, const void* __restrict__ freq,
@@ -190,24 +191,41 @@ __device__ __forceinline__ void ret_stage(const bf16_t* __restrict__ proj, const
     }
     return;
   }
-  const int quads = dim / 4;
-  for (int i = tid; i < RET_TILE * quads; i += threads) {
-    const int r = i / quads, c = (i - r * quads) * 4;
-    float4 o = make_float4(0.f, 0.f, 0.f, 0.f);
-    if (r < count) {
-      const size_t n = (size_t)(first + r);
+  // RET_GROUPS groups of four values of a thread, their loads all asked for before the first is used: rows past the last
+  // load the last one and are zeroed behind it, values that are not rotated load themselves as their partners
+  const int quads = dim / 4, total = RET_TILE * quads;
+  for (int i0 = tid; i0 < total; i0 += RET_GROUPS * threads) {
+    uint2 w[RET_GROUPS], u[RET_GROUPS];
+    float4 ca[RET_GROUPS], cb[RET_GROUPS];
+#pragma unroll
+    for (int k = 0; k < RET_GROUPS; ++k) {
+      const int i = i0 + k * threads < total ? i0 + k * threads : i0;
+      const int r = i / quads, c = (i - r * quads) * 4;
+      const size_t n = (size_t)(first + (r < count ? r : count - 1));
       const bf16_t* row = proj + n * P.proj_stride + col;
-      const uint2 w = *reinterpret_cast<const uint2*>(row + c);
-      float x[4] = {__uint_as_float(w.x << 16), __uint_as_float(w.x & 0xffff0000u), __uint_as_float(w.y << 16),
-                    __uint_as_float(w.y & 0xffff0000u)};
+      const bool low = c < half, turned = c < P.rot;
+      w[k] = *reinterpret_cast<const uint2*>(row + c);
+      u[k] = *reinterpret_cast<const uint2*>(row + (turned ? (low ? c + half : c - half) : c));
+      if (turned) {
+        const float4* cs = reinterpret_cast<const float4*>(P.table + (n * half + (low ? c : c - half)) * 2);
+        ca[k] = cs[0];
+        cb[k] = cs[1];
+      } else {
+        ca[k] = cb[k] = make_float4(1.f, 0.f, 1.f, 0.f);
+      }
+    }
+#pragma unroll
+    for (int k = 0; k < RET_GROUPS; ++k) {
+      const int i = i0 + k * threads;
+      if (i >= total) break;
+      const int r = i / quads, c = (i - r * quads) * 4;
+      float x[4] = {__uint_as_float(w[k].x << 16), __uint_as_float(w[k].x & 0xffff0000u), __uint_as_float(w[k].y << 16),
+                    __uint_as_float(w[k].y & 0xffff0000u)};
       if (c < P.rot) {
         const bool low = c < half;
-        const uint2 u = *reinterpret_cast<const uint2*>(row + (low ? c + half : c - half));
-        const float y[4] = {__uint_as_float(u.x << 16), __uint_as_float(u.x & 0xffff0000u), __uint_as_float(u.y << 16),
-                            __uint_as_float(u.y & 0xffff0000u)};
-        const float4* cs = reinterpret_cast<const float4*>(P.table + (n * half + (low ? c : c - half)) * 2);
-        const float4 a = cs[0], b = cs[1];
-        const float cv[4] = {a.x, a.z, b.x, b.z}, sv[4] = {a.y, a.w, b.y, b.w};
+        const float y[4] = {__uint_as_float(u[k].x << 16), __uint_as_float(u[k].x & 0xffff0000u), __uint_as_float(u[k].y << 16),
+                            __uint_as_float(u[k].y & 0xffff0000u)};
+        const float cv[4] = {ca[k].x, ca[k].z, cb[k].x, cb[k].z}, sv[4] = {ca[k].y, ca[k].w, cb[k].y, cb[k].w};
 #pragma unroll
         for (int e = 0; e < 4; ++e) {
           float lo, hi;
@@ -215,9 +233,9 @@ __device__ __forceinline__ void ret_stage(const bf16_t* __restrict__ proj, const
           x[e] = low ? lo : hi;
         }
       }
-      o = make_float4(x[0] * factor, x[1] * factor, x[2] * factor, x[3] * factor);
+      const float f = r < count ? factor : 0.f;
+      *reinterpret_cast<float4*>(dst + r * stride + c) = make_float4(x[0] * f, x[1] * f, x[2] * f, x[3] * f);
     }
-    *reinterpret_cast<float4*>(dst + r * stride + c) = o;
   }
 }
 
@@ -324,7 +342,7 @@ __device__ __forceinline__ void ret_rows(const float* __restrict__ qs, int kst, 
   const float* sp = S + (size_t)(4 * kk) * vdim + 16 * ct + l15;
 #pragma unroll
   for (int a = 0; a < RT; ++a) acc[a] = (rt_f32x4){0.f, 0.f, 0.f, 0.f};
-#pragma unroll 2
+#pragma unroll 4
   for (int n0 = 0; n0 < dim; n0 += 16) {
     float b[4];
 #pragma unroll
@@ -401,11 +419,19 @@ __global__ __launch_bounds__(512) void retention_rows_kernel(const bf16_t* __res
   constexpr int SPLIT = 4 / RT;
   const int ctiles = vdim / 16, jobs = ctiles * SPLIT;
   rt_f32x4 acc[JOBS][4];
+  bf16_t gates[JOBS][RT][4];                            // asked for before the products, needed behind them
 #pragma unroll
   for (int b = 0; b < JOBS; ++b) {
     const int job = wave + 8 * b;
     if (job >= jobs) break;
     const int ct = job / SPLIT, rt0 = (job - ct * SPLIT) * RT;
+#pragma unroll
+    for (int a = 0; a < RT; ++a)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int i = 16 * (rt0 + a) + 4 * kk + r;
+        gates[b][a][r] = proj[(size_t)(first + (i < count ? i : count - 1)) * P.proj_stride + P.g_col + hd * vdim + 16 * ct + l15];
+      }
     ret_rows<RT>(qs, kst, G, vs, vst, pw, S, dim, vdim, ct, rt0, lane, acc[b]);
 #pragma unroll
     for (int a = 0; a < RT; ++a)
@@ -437,8 +463,9 @@ __global__ __launch_bounds__(512) void retention_rows_kernel(const bf16_t* __res
         if (i >= count) continue;
         const size_t n = (size_t)(first + i);
         const int c = hd * vdim + 16 * ct + l15;
-        const float gate = to_float(proj[n * P.proj_stride + P.g_col + c]);
-        out[n * P.out_stride + c] = from_float<bf16_t>(acc[b][a][r] * inv[i] * (gate / (1.0f + expf(-gate))));
+        const float gate = to_float(gates[b][a][r]);
+        const float silu = gate * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-1.4426950408889634f * gate));
+        out[n * P.out_stride + c] = from_float<bf16_t>(acc[b][a][r] * inv[i] * silu);
       }
   }
   if (last) {

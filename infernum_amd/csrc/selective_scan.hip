@@ -7,7 +7,8 @@
 //
 //   ia_selective_scan   the rows of the requests first_request .. first_request + B - 1 of a step, each from its state slot,
 //                       which is left moved on.  A thread owns a channel with all its state values in registers; B and C of
-//                       a token are the same for all lanes of a wave and come through scalar loads.  A request of more rows
+//                       a token are the same for all channels and come from LDS, SEL_ROWS tokens at a time, every read
+//                       one address for all lanes.  A request of more rows
 //                       than `seg_len` is cut into segments of that many that run side by side: every segment but a
 //                       request's last first runs from a zero state and leaves what it adds and the sum of its dt; a second
 //                       kernel walks a request's segments, S <- exp(A sum dt) S + U, and leaves each the state before it;
@@ -17,24 +18,25 @@
 #include "common.h"
 
 #define SEL_TB 4          // tokens whose channel values are asked for together
+#define SEL_ROWS 32       // tokens whose B and C lie in LDS together (a multiple of SEL_TB)
+#define SEL_BLOCK 128     // channels of a workgroup
 
-__device__ __forceinline__ float sel_softplus(float z) { return z > 20.f ? z : log1pf(expf(z)); }
-
-// Two neighbouring values of a row that is the same for all lanes.
-template <typename T> struct SelPair;
-template <> struct SelPair<bf16_t> {
-  static __device__ __forceinline__ void get(const bf16_t* p, int i, float& a, float& b) {
-    const uint32_t w = reinterpret_cast<const uint32_t*>(p)[i];
-    a = __uint_as_float(w << 16);
-    b = __uint_as_float(w & 0xffff0000u);
-  }
-};
-template <> struct SelPair<float> {
-  static __device__ __forceinline__ void get(const float* p, int i, float& a, float& b) {
-    a = p[2 * i];
-    b = p[2 * i + 1];
-  }
-};
+// ln(1 + e^z) = max(z, 0) + ln(1 + w) with w = e^-|z| in (0, 1]; ln(1 + w) = 2 artanh(s), s = w / (2 + w) at most 1/3, by
+// the series s + s^3/3 + ... + s^15/15 (the next term is below 5e-9 of the first): no difference of nearly equal
+// numbers anywhere, so the result is good to a few units in the last place of fp32 for every z.
+__device__ __forceinline__ float sel_softplus(float z) {
+  const float w = __builtin_amdgcn_exp2f(-1.4426950408889634f * fabsf(z));
+  const float s = w * __builtin_amdgcn_rcpf(2.0f + w), q = s * s;
+  float p = 1.0f / 15.0f;
+  p = __builtin_fmaf(p, q, 1.0f / 13.0f);
+  p = __builtin_fmaf(p, q, 1.0f / 11.0f);
+  p = __builtin_fmaf(p, q, 1.0f / 9.0f);
+  p = __builtin_fmaf(p, q, 1.0f / 7.0f);
+  p = __builtin_fmaf(p, q, 1.0f / 5.0f);
+  p = __builtin_fmaf(p, q, 1.0f / 3.0f);
+  p = __builtin_fmaf(p, q, 1.0f);
+  return __builtin_fmaf(2.0f * s, p, fmaxf(z, 0.0f));
+}
 
 struct SelArgs {
   const float* dt_raw;           // rows of dt_stride values
@@ -50,13 +52,16 @@ struct SelArgs {
   int dt_stride, x_stride, z_stride, bc_stride, b_col, c_col, out_stride, C, Ns, seg_len, max_segs, first_request;
 };
 
-// grid (blocks of 64 channels, segments, requests), 64 threads.  KN: state values a thread holds, Ns of them real (B and C
-// have KN columns, those past Ns zero).  MODE 0: a request's rows from its slot; 1: what a segment adds; 2: a segment's rows.
+// grid (blocks of SEL_BLOCK channels, segments, requests), SEL_BLOCK threads.  KN: state values a thread holds, Ns of them
+// real (B and C have KN columns, those past Ns zero).  MODE 0: a request's rows from its slot; 1: what a segment adds; 2: a
+// segment's rows.
 template <typename T, int KN, int MODE>
-__global__ __launch_bounds__(64) void selective_scan_kernel(const T* __restrict__ x, const T* __restrict__ z,
-                                                            const T* __restrict__ bc, T* __restrict__ out, SelArgs P) {
-  const int r = blockIdx.z, s = P.first_request + r, seg = blockIdx.y;
-  const int c = blockIdx.x * 64 + threadIdx.x;
+__global__ __launch_bounds__(SEL_BLOCK) void selective_scan_kernel(const T* __restrict__ x, const T* __restrict__ z,
+                                                                   const T* __restrict__ bc, T* __restrict__ out, SelArgs P) {
+  constexpr int BC = MODE == 1 ? KN : 2 * KN;                    // floats of a token in LDS: B, and C where rows are written
+  __shared__ __attribute__((aligned(16))) float s_bc[SEL_ROWS][BC];
+  const int r = blockIdx.z, s = P.first_request + r, seg = blockIdx.y, tid = threadIdx.x;
+  const int c = blockIdx.x * SEL_BLOCK + tid;
   int first = P.seq_starts[s], count = P.seq_starts[s + 1] - first;
   bool last = true;
   if (MODE != 0) {
@@ -73,6 +78,20 @@ __global__ __launch_bounds__(64) void selective_scan_kernel(const T* __restrict_
   const size_t rec = (size_t)r * P.max_segs + seg;
   float* slot = P.state + (size_t)P.state_slots[s] * P.state_stride;
   float* R = MODE == 0 ? slot : P.records + rec * ((size_t)P.Ns * P.C);
+  const T* xp = x + (size_t)first * P.x_stride + cc;
+  const T* zp = z + (size_t)first * P.z_stride + cc;
+  const float* dp = P.dt_raw + (size_t)first * P.dt_stride + cc;
+  float xn[SEL_TB], zn[SEL_TB], dn[SEL_TB];
+  auto fetch = [&](int t0) {
+#pragma unroll
+    for (int k = 0; k < SEL_TB; ++k) {
+      const int t = t0 + k < count ? t0 + k : count - 1;
+      xn[k] = to_float(xp[(size_t)t * P.x_stride]);
+      if (MODE != 1) zn[k] = to_float(zp[(size_t)t * P.z_stride]);
+      dn[k] = dp[(size_t)t * P.dt_stride];
+    }
+  };
+  fetch(0);
   float S[KN], A[KN];
 #pragma unroll
   for (int n = 0; n < KN; ++n) {
@@ -81,51 +100,51 @@ __global__ __launch_bounds__(64) void selective_scan_kernel(const T* __restrict_
   }
   const float bias = P.dt_bias[cc], D = MODE == 1 ? 0.f : P.skip[cc];
   float total = 0.f;
-  float xn[SEL_TB], zn[SEL_TB], dn[SEL_TB];
-  auto fetch = [&](int t0) {
-#pragma unroll
-    for (int k = 0; k < SEL_TB; ++k) {
-      const int t = t0 + k < count ? t0 + k : count - 1;
-      const size_t row = (size_t)(first + t);
-      xn[k] = to_float(x[row * P.x_stride + cc]);
-      if (MODE != 1) zn[k] = to_float(z[row * P.z_stride + cc]);
-      dn[k] = P.dt_raw[row * P.dt_stride + cc];
+  for (int b0 = 0; b0 < count; b0 += SEL_ROWS) {
+    const int nb = count - b0 < SEL_ROWS ? count - b0 : SEL_ROWS;
+    __syncthreads();                                              // the tokens before are read to their end
+    for (int i = tid; i < nb * BC; i += SEL_BLOCK) {
+      const int t = i / BC, n = i - t * BC;
+      s_bc[t][n] = to_float(bc[(size_t)(first + b0 + t) * P.bc_stride + (n < KN ? P.b_col + n : P.c_col + (n - KN))]);
     }
-  };
-  fetch(0);
-  for (int t0 = 0; t0 < count; t0 += SEL_TB) {
-    float xv[SEL_TB], zv[SEL_TB], dt[SEL_TB];
+    __syncthreads();
+    for (int t0 = 0; t0 < nb; t0 += SEL_TB) {
+      float xv[SEL_TB], zv[SEL_TB], dt[SEL_TB];
 #pragma unroll
-    for (int k = 0; k < SEL_TB; ++k) {
-      xv[k] = xn[k];
-      if (MODE != 1) zv[k] = zn[k];
-      dt[k] = sel_softplus(dn[k] + bias);
-    }
-    if (t0 + SEL_TB < count) fetch(t0 + SEL_TB);
-#pragma unroll
-    for (int k = 0; k < SEL_TB; ++k) {
-      if (t0 + k >= count) break;                                  // the same for all lanes
-      const T* br = bc + (size_t)(first + t0 + k) * P.bc_stride + P.b_col;
-      const T* cr = bc + (size_t)(first + t0 + k) * P.bc_stride + P.c_col;
-      const float d = dt[k], dx = d * xv[k];
-      float y0 = 0.f, y1 = 0.f;
-#pragma unroll
-      for (int n = 0; n < KN; n += 2) {
-        float b0, b1, c0, c1;
-        SelPair<T>::get(br, n / 2, b0, b1);
-        S[n] = __builtin_fmaf(__builtin_amdgcn_exp2f(d * A[n]), S[n], dx * b0);
-        S[n + 1] = __builtin_fmaf(__builtin_amdgcn_exp2f(d * A[n + 1]), S[n + 1], dx * b1);
-        if (MODE != 1) {
-          SelPair<T>::get(cr, n / 2, c0, c1);
-          y0 = __builtin_fmaf(S[n], c0, y0);
-          y1 = __builtin_fmaf(S[n + 1], c1, y1);
-        }
+      for (int k = 0; k < SEL_TB; ++k) {
+        xv[k] = xn[k];
+        if (MODE != 1) zv[k] = zn[k];
+        dt[k] = sel_softplus(dn[k] + bias);
       }
-      if (MODE == 1) {
-        total += d;
-      } else if (live) {
-        const float y = __builtin_fmaf(D, xv[k], y0 + y1);
-        out[(size_t)(first + t0 + k) * P.out_stride + c] = from_float<T>(y * (zv[k] / (1.0f + expf(-zv[k]))));
+      if (b0 + t0 + SEL_TB < count) fetch(b0 + t0 + SEL_TB);
+#pragma unroll
+      for (int k = 0; k < SEL_TB; ++k) {
+        if (t0 + k >= nb) break;                                   // the same for all lanes
+        const float4* bt = reinterpret_cast<const float4*>(&s_bc[t0 + k][0]);
+        const float d = dt[k], dx = d * xv[k];
+        float y0 = 0.f, y1 = 0.f;
+#pragma unroll
+        for (int n = 0; n < KN; n += 4) {
+          const float4 bv = bt[n / 4];
+          S[n] = __builtin_fmaf(__builtin_amdgcn_exp2f(d * A[n]), S[n], dx * bv.x);
+          S[n + 1] = __builtin_fmaf(__builtin_amdgcn_exp2f(d * A[n + 1]), S[n + 1], dx * bv.y);
+          S[n + 2] = __builtin_fmaf(__builtin_amdgcn_exp2f(d * A[n + 2]), S[n + 2], dx * bv.z);
+          S[n + 3] = __builtin_fmaf(__builtin_amdgcn_exp2f(d * A[n + 3]), S[n + 3], dx * bv.w);
+          if (MODE != 1) {
+            const float4 cv = bt[(KN + n) / 4];
+            y0 = __builtin_fmaf(S[n], cv.x, y0);
+            y1 = __builtin_fmaf(S[n + 1], cv.y, y1);
+            y0 = __builtin_fmaf(S[n + 2], cv.z, y0);
+            y1 = __builtin_fmaf(S[n + 3], cv.w, y1);
+          }
+        }
+        if (MODE == 1) {
+          total += d;
+        } else if (live) {
+          const float y = __builtin_fmaf(D, xv[k], y0 + y1), zz = zv[k];
+          const float gate = zz * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-1.4426950408889634f * zz));
+          out[(size_t)(first + b0 + t0 + k) * P.out_stride + c] = from_float<T>(y * gate);
+        }
       }
     }
   }
@@ -177,8 +196,8 @@ extern "C" int ia_selective_columns(int Ns) {
 }
 
 // x, z, bc: rows of the activations' type (code): the channels behind their convolution, the gates' logits, and a row that
-// holds ia_selective_columns(Ns) values of B from b_col and as many of C from c_col (even columns, even bc_stride; values
-// past Ns zero).  dt_raw fp32.  a2 fp32 [Ns, C]: A log2(e).  out: rows of out_stride values.  max_rows: at least the rows of
+// holds ia_selective_columns(Ns) values of B from b_col and as many of C from c_col (values past Ns
+// zero).  dt_raw fp32.  a2 fp32 [Ns, C]: A log2(e).  out: rows of out_stride values.  max_rows: at least the rows of
 // the longest of the requests; with more than seg_len: records fp32 [B, ceil(max_rows / seg_len), Ns, C] and sums
 // [B, ceil(max_rows / seg_len), C].
 extern "C" int ia_selective_scan(const void* x, int code, int x_stride, const void* z, int z_stride, const void* bc,
@@ -195,15 +214,14 @@ extern "C" int ia_selective_scan(const void* x, int code, int x_stride, const vo
   const int kn = ia_selective_columns(Ns);
   if (kn == 0) return IA_ERR_UNSUPPORTED;
   if (b_col < 0 || c_col < 0 || bc_stride < b_col + kn || bc_stride < c_col + kn) return IA_ERR_BAD_ARG;
-  if ((b_col | c_col | bc_stride) & 1 || ((uintptr_t)bc & 3)) return IA_ERR_UNSUPPORTED;
   const int segs = (max_rows + seg_len - 1) / seg_len;
   if (segs > 65535) return IA_ERR_UNSUPPORTED;
   if (segs > 1 && (!records || !sums)) return IA_ERR_BAD_ARG;
   const SelArgs P{dt_raw, dt_bias, a2, skip, state, state_stride, seq_starts, state_slots, records, sums,
                   dt_stride, x_stride, z_stride, bc_stride, b_col, c_col, out_stride, C, Ns, seg_len, segs, first_request};
-  const unsigned blocks = (unsigned)((C + 63) / 64);
+  const unsigned blocks = (unsigned)((C + SEL_BLOCK - 1) / SEL_BLOCK);
 #define IA_SEL(T, KN, MODE, SEGS)                                                                                     \
-  selective_scan_kernel<T, KN, MODE><<<dim3(blocks, (unsigned)(SEGS), (unsigned)B), 64, 0, stream>>>(                   \
+  selective_scan_kernel<T, KN, MODE><<<dim3(blocks, (unsigned)(SEGS), (unsigned)B), SEL_BLOCK, 0, stream>>>(            \
       (const T*)x, (const T*)z, (const T*)bc, (T*)out, P)
 #define IA_SEL_K(T, MODE, SEGS)                   \
   do {                                            \

@@ -1272,16 +1272,32 @@ extern "C" int ia_stream_add2(float* h, const void* a, int a_code, int a_splits,
 }
 
 // h [N, H] fp32 += v [H], the same vector for every row
-__global__ __launch_bounds__(256) void add_vector_kernel(float* __restrict__ h, const void* __restrict__ v, int v_code, size_t n, int H) {
-  const size_t i = (size_t)blockIdx.x * 256 + threadIdx.x;
-  if (i < n) h[i] += load_as_float(v, v_code, i % H);
+// grid (pieces of 256 values of a row, or of 1,024 with VEC, rows)
+template <bool VEC>
+__global__ __launch_bounds__(256) void add_vector_kernel(float* __restrict__ h, const void* __restrict__ v, int v_code, int H) {
+  const int i = (blockIdx.x * 256 + threadIdx.x) * (VEC ? 4 : 1);
+  if (i >= H) return;
+  float* p = h + (size_t)blockIdx.y * H + i;
+  if (VEC) {
+    float4 a = *reinterpret_cast<const float4*>(p);
+    a.x += load_as_float(v, v_code, i);
+    a.y += load_as_float(v, v_code, i + 1);
+    a.z += load_as_float(v, v_code, i + 2);
+    a.w += load_as_float(v, v_code, i + 3);
+    *reinterpret_cast<float4*>(p) = a;
+  } else {
+    p[0] += load_as_float(v, v_code, i);
+  }
 }
 
 extern "C" int ia_add_vector(float* h, const void* v, int v_code, int N, int H, hipStream_t stream) {
   if (N == 0) return IA_OK;
   if (!h || !v || N < 0 || H <= 0 || (v_code != IA_F32 && v_code != IA_BF16)) return IA_ERR_BAD_ARG;
-  const size_t n = (size_t)N * H;
-  add_vector_kernel<<<(unsigned)((n + 255) / 256), 256, 0, stream>>>(h, v, v_code, n, H);
+  if (N > 65535) return IA_ERR_UNSUPPORTED;
+  if (H % 4 == 0 && !((uintptr_t)h & 15))
+    add_vector_kernel<true><<<dim3((unsigned)((H + 1023) / 1024), (unsigned)N), 256, 0, stream>>>(h, v, v_code, H);
+  else
+    add_vector_kernel<false><<<dim3((unsigned)((H + 255) / 256), (unsigned)N), 256, 0, stream>>>(h, v, v_code, H);
   IA_LAUNCH_CHECK();
   return IA_OK;
 }
