@@ -47,10 +47,18 @@ struct SelArgs {
   long state_stride;
   const int* seq_starts;
   const int* state_slots;
-  float* records;                // [requests, max_segs, Ns, C]
-  float* sums;                   // [requests, max_segs, C]
-  int dt_stride, x_stride, z_stride, bc_stride, b_col, c_col, out_stride, C, Ns, seg_len, max_segs, first_request;
+  float* records;                // [segments of all requests, Ns, C]
+  float* sums;                   // [segments of all requests, C]
+  int dt_stride, x_stride, z_stride, bc_stride, b_col, c_col, out_stride, C, Ns, seg_len, first_request;
 };
+
+// The record of a request's first segment: the segments in the order of the requests.
+__device__ __forceinline__ size_t sel_record(const SelArgs& P, int r) {
+  int before = 0;
+  for (int i = P.first_request; i < P.first_request + r; ++i)
+    before += (P.seq_starts[i + 1] - P.seq_starts[i] + P.seg_len - 1) / P.seg_len;
+  return (size_t)before;
+}
 
 // grid (blocks of SEL_BLOCK channels, segments, requests), SEL_BLOCK threads.  KN: state values a thread holds, Ns of them
 // real (B and C have KN columns, those past Ns zero).  MODE 0: a request's rows from its slot; 1: what a segment adds; 2: a
@@ -75,7 +83,7 @@ __global__ __launch_bounds__(SEL_BLOCK) void selective_scan_kernel(const T* __re
   if (count <= 0) return;
   const bool live = c < P.C;
   const int cc = live ? c : P.C - 1;
-  const size_t rec = (size_t)r * P.max_segs + seg;
+  const size_t rec = MODE == 0 ? 0 : sel_record(P, r) + seg;
   float* slot = P.state + (size_t)P.state_slots[s] * P.state_stride;
   float* R = MODE == 0 ? slot : P.records + rec * ((size_t)P.Ns * P.C);
   const T* xp = x + (size_t)first * P.x_stride + cc;
@@ -169,8 +177,9 @@ __global__ __launch_bounds__(256) void selective_chain_kernel(SelArgs P) {
   const int c = e % P.C;
   const float a = P.a2[e];
   float S = P.state[(size_t)P.state_slots[s] * P.state_stride + e];
-  float* R = P.records + (size_t)r * P.max_segs * size + e;
-  const float* Q = P.sums + (size_t)r * P.max_segs * P.C + c;
+  const size_t rec = sel_record(P, r);
+  float* R = P.records + rec * size + e;
+  const float* Q = P.sums + rec * P.C + c;
   for (int j0 = 0; j0 < count; j0 += SEL_AHEAD) {
     float U[SEL_AHEAD], T[SEL_AHEAD];
 #pragma unroll
@@ -198,8 +207,8 @@ extern "C" int ia_selective_columns(int Ns) {
 // x, z, bc: rows of the activations' type (code): the channels behind their convolution, the gates' logits, and a row that
 // holds ia_selective_columns(Ns) values of B from b_col and as many of C from c_col (values past Ns
 // zero).  dt_raw fp32.  a2 fp32 [Ns, C]: A log2(e).  out: rows of out_stride values.  max_rows: at least the rows of
-// the longest of the requests; with more than seg_len: records fp32 [B, ceil(max_rows / seg_len), Ns, C] and sums
-// [B, ceil(max_rows / seg_len), C].
+// the longest of the requests; with more than seg_len: records fp32 [segments, Ns, C] and sums [segments, C] for the
+// segments of all requests (ceil(rows / seg_len) each).
 extern "C" int ia_selective_scan(const void* x, int code, int x_stride, const void* z, int z_stride, const void* bc,
                                  int bc_stride, int b_col, int c_col, const float* dt_raw, int dt_stride,
                                  const float* dt_bias, const float* a2, const float* skip, float* state, long state_stride,
@@ -218,7 +227,7 @@ extern "C" int ia_selective_scan(const void* x, int code, int x_stride, const vo
   if (segs > 65535) return IA_ERR_UNSUPPORTED;
   if (segs > 1 && (!records || !sums)) return IA_ERR_BAD_ARG;
   const SelArgs P{dt_raw, dt_bias, a2, skip, state, state_stride, seq_starts, state_slots, records, sums,
-                  dt_stride, x_stride, z_stride, bc_stride, b_col, c_col, out_stride, C, Ns, seg_len, segs, first_request};
+                  dt_stride, x_stride, z_stride, bc_stride, b_col, c_col, out_stride, C, Ns, seg_len, first_request};
   const unsigned blocks = (unsigned)((C + SEL_BLOCK - 1) / SEL_BLOCK);
 #define IA_SEL(T, KN, MODE, SEGS)                                                                                     \
   selective_scan_kernel<T, KN, MODE><<<dim3(blocks, (unsigned)(SEGS), (unsigned)B), SEL_BLOCK, 0, stream>>>(            \

@@ -142,22 +142,13 @@ class Mamba1Mixer(Mixer):
                 ssm, stride, y, I, program.seq_starts, program.state_slots]
         program.op("core", "ia_selective_scan", [*same, 0, program.ND, I, self.Ns, 1, 1, None, None, STREAM],
                    Guard.between(program.ND, 1))
-        # the segments of a step: never more than one a request and as many again as the rows are cut into at the least
-        slots = int(state.shape[0])
-        most_rows = lambda ctx: max(ctx.q_lens[ctx.num_decode:], default=1)            # noqa: E731
-
-        def segment(ctx: StepContext) -> int:
-            rows = ctx.q_lens[ctx.num_decode:]
-            if not rows:
-                return 1
-            seg, longest = K.selective_segment(rows, I, dev), max(rows)
-            # every request's records lie as far apart as the longest one's: no cut when that would not fit the arena
-            return seg if len(rows) * -(-longest // seg) <= limit else longest
-        limit = min(4 * K.SELECTIVE_WAVES // max(1, -(-I // 64)) + 2 * slots, max(1, T // 32) + slots)
-        records = program.buffer("mamba1.records", limit * self.Ns * I * 4)
-        sums = program.buffer("mamba1.sums", limit * I * 4)
-        longest = program.scalar("mamba1: rows of the longest portion", most_rows)
-        seg = program.scalar(("mamba1: rows of a segment", I, slots), segment)
+        # a request holds a state slot, and a segment but a request's last so many rows: so many segments a step has at most
+        most = T // K.SELECTIVE_SEGMENTS[0] + int(state.shape[0])
+        records = program.buffer("mamba1.records", most * self.Ns * I * 4)
+        sums = program.buffer("mamba1.sums", most * I * 4)
+        longest = program.scalar("mamba1: rows of the longest portion", lambda ctx: max(ctx.q_lens[ctx.num_decode:], default=1))
+        seg = program.scalar(("mamba1: rows of a segment", I),
+                             lambda ctx: K.selective_segment(ctx.q_lens[ctx.num_decode:], I, dev))
         program.op("core", "ia_selective_scan", [*same, program.ND, program.NP, I, self.Ns, longest, seg, records, sums, STREAM],
                    Guard.between(program.NP, 1))
         program.pending = emit_linear(program, y, N, self.w_o, rt.dtype, None, True, "mamba1.out", "mamba1.o")

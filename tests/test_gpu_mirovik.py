@@ -396,9 +396,11 @@ def test_where_rows_are_cut_into_segments():
     from infernum_amd.kernels import api as K
     assert K.selective_segment([40], 4096) == 40                               # short: in one piece
     assert K.selective_segment([256] * 64, 4096) == 256                        # many requests fill the GPU by themselves
-    seg = K.selective_segment([8192], 4096)
-    assert 32 <= seg <= 512 and seg % 16 == 0                                  # one long one is cut
-    assert K.selective_segment([5000], 64) >= 32
+    assert K.selective_segment([128] * 64, 4096) == 128
+    assert K.selective_segment([8192], 4096) == 64                             # one long one is cut
+    assert K.selective_segment([8000] + [3] * 60, 4096) == 64                  # also among many short ones
+    assert K.selective_segment([300], 4096) == 32 and K.selective_segment([5000], 64) == 32
+    assert K.selective_segment([], 64) == 1
 
 
 # ------------------------------------------------------------------------------------ the mixers alone
